@@ -2,9 +2,10 @@
 //
 // They replace separate elementwise launches of the reference's HF layer
 // (/root/reference/utils/shard_loader.py:66-74 -> LlamaDecoderLayer):
-//   EPI_STORE   y -> bf16 out (optionally act(y + bias): GPT-2 c_fc + gelu_new)
+//   EPI_STORE   y -> bf16 out (optionally act(y + bias): GPT-2 c_fc + gelu_new), or fp32 out32
 //   EPI_RESID   out = resid + y (+ bias)        (o_proj / down_proj + residual add)
-//   EPI_SWIGLU  out = silu(gate) * up           (gate/up fused GEMM, tiles interleaved)
+//   EPI_SWIGLU  out = silu(gate) * up           (gate/up fused GEMM, tiles interleaved), or the
+//               clipped GLU of glu() when glu_limit > 0
 //   EPI_QKV     half-split RoPE on q/k + direct write of k/v into the static KV cache
 //               (replaces apply_rotary_pos_emb + DynamicCache.update's torch.cat); with
 //               cos_t == nullptr (GPT-2: learned absolute positions) no rotation and the
@@ -47,9 +48,23 @@ struct EpiArgs {
   const float* ss_in;
   int ss_n;
   float ss_eps;
+  float* out32;             // STORE: fp32 output [M][ldo] instead of out (null: bf16 to out)
+  float glu_alpha;          // SWIGLU with glu_limit > 0: see glu()
+  float glu_limit;
+  float glu_shift;
 };
 
 LSA_DEVICE float silu(float g) { return g / (1.0f + __expf(-g)); }
+
+// The gated unit of an EPI_SWIGLU GEMM: silu(g) * u, or with glu_limit L > 0 the clipped unit
+//   g' = min(g, L), u' = clamp(u, -L, L):  g' * sigmoid(alpha * g') * (u' + shift)
+LSA_DEVICE float glu(const EpiArgs& ep, float g, float u) {
+  if (ep.glu_limit > 0.f) {
+    const float gc = fminf(g, ep.glu_limit), uc = fminf(fmaxf(u, -ep.glu_limit), ep.glu_limit);
+    return gc / (1.0f + __expf(-ep.glu_alpha * gc)) * (uc + ep.glu_shift);
+  }
+  return silu(g) * u;
+}
 
 // 0.5 x (1 + tanh(sqrt(2/pi) (x + 0.044715 x^3))), tanh(u) = 1 - 2 / (exp(2u) + 1)
 LSA_DEVICE float gelu_tanh(float x) {
@@ -58,6 +73,13 @@ LSA_DEVICE float gelu_tanh(float x) {
 }
 
 LSA_DEVICE float epi_bias(const EpiArgs& ep, int col) { return ep.bias ? ep.bias[col] : 0.f; }
+// One finished element of an EPI_STORE GEMM
+LSA_DEVICE void epi_store1(const EpiArgs& ep, int m, int col, float v) {
+  v += ep.bias ? ep.bias[col] : 0.f;
+  if (ep.act == 1) v = gelu_tanh(v);
+  if (ep.out32) ep.out32[(size_t)m * ep.ldo + col] = v;
+  else ep.out[(size_t)m * ep.ldo + col] = f2bf(v);
+}
 LSA_DEVICE float epi_act(const EpiArgs& ep, float v) { return ep.act == 1 ? gelu_tanh(v) : v; }
 
 // Store one finished element (row m, packed column n) of an EPI_QKV GEMM. `vp` is the value
@@ -204,6 +226,13 @@ LSA_DEVICE void epi_row16(const EpiArgs& ep, int m, int c0, float* v) {
     if (ep.act == 1) {
 #pragma unroll
       for (int j = 0; j < 16; ++j) v[j] = gelu_tanh(v[j]);
+    }
+    if (ep.out32) {
+      float* o32 = ep.out32 + (size_t)m * ep.ldo + c0;
+#pragma unroll
+      for (int q = 0; q < 4; ++q)
+        *reinterpret_cast<f32x4_t*>(o32 + 4 * q) = f32x4_t{v[4 * q], v[4 * q + 1], v[4 * q + 2], v[4 * q + 3]};
+      return;
     }
     bf16_raw* o = ep.out + (size_t)m * ep.ldo + c0;
     st16(o, pack8(v));

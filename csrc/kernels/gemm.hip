@@ -187,7 +187,7 @@ __global__ __launch_bounds__(GTHR) void gemm_packed_kernel(const bf16_raw* __res
       const int gm = m0 + rb * 16 + (lane >> 4) * 4 + r;
       if (EPI == EPI_SWIGLU) {
         const float g = acc[rb][0][r], u = acc[rb][1][r];
-        if (gm < M) ep.out[(size_t)gm * ep.ldo + (ntile0 / 2) * 16 + n] = f2bf(silu(g) * u);
+        if (gm < M) ep.out[(size_t)gm * ep.ldo + (ntile0 / 2) * 16 + n] = f2bf(glu(ep, g, u));
       } else {
 #pragma unroll
         for (int tn = 0; tn < TN; ++tn) {
@@ -199,7 +199,7 @@ __global__ __launch_bounds__(GTHR) void gemm_packed_kernel(const bf16_raw* __res
               epi_qkv_store(ep, gm, col, v + epi_bias(ep, col), vp + epi_bias(ep, col ^ 8), ep.pos[gm], ep.slot[gm]);
           } else if (gm < M) {
             if (EPI == EPI_STORE)
-              ep.out[(size_t)gm * ep.ldo + col] = f2bf(epi_act(ep, v + epi_bias(ep, col)));
+              epi_store1(ep, gm, col, v);
             else if (EPI == EPI_RESID)
               ep.out[(size_t)gm * ep.ldo + col] = f2bf(bf2f(ep.resid[(size_t)gm * ep.ldr + col]) + v + epi_bias(ep, col));
           }

@@ -534,7 +534,7 @@ struct Kern {
             epi_bias16(ep, c0, g);
             epi_bias16(ep, c0 + 16, uu);
 #pragma unroll
-            for (int q = 0; q < 16; ++q) v[q] = silu(g[q]) * uu[q];
+            for (int q = 0; q < 16; ++q) v[q] = glu(ep, g[q], uu[q]);
             bf16_raw* o = ep.out + (size_t)m * ep.ldo + (c0 >> 1);
             st16(o, pack8(v));
             st16(o + 8, pack8(v + 8));
@@ -791,7 +791,7 @@ extern "C" int lsa_gemm_sk(const void* a, int lda, const void* wp, int M, int N,
   if (grid < 1 || grid > 1024 || group_m < 1) return LSA_BAD_SHAPE;
   if (epi == EPI_RESID && !ep->resid) return LSA_BAD_SHAPE;
   if (epi == EPI_QKV && (!ep->k_cache || !ep->v_cache || !ep->slot || !ep->pos)) return LSA_BAD_SHAPE;
-  if (epi == EPI_ARGMAX ? (!ep->keys || bn == 192) : !ep->out) return LSA_BAD_SHAPE;
+  if (epi == EPI_ARGMAX ? (!ep->keys || bn == 192) : !(ep->out || (epi == EPI_STORE && ep->out32))) return LSA_BAD_SHAPE;
   if (ep->ss_out && (epi != EPI_RESID || bn == 192 || N % 64 || ep->ss_n != N / 64)) return LSA_BAD_SHAPE;
   if (ep->ss_in && ((epi != EPI_QKV && epi != EPI_SWIGLU) || ep->ss_n < 4 || ep->ss_n % 4 || K != 64 * ep->ss_n))
     return LSA_BAD_SHAPE;

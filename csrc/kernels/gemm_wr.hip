@@ -262,7 +262,7 @@ LSA_DEVICE void gemm_wr_body(unsigned char* smem, const bf16_raw* __restrict__ A
         if (m < M) {
           const float rsc = ep.ss_in ? s_rs[row] : 1.f;
 #pragma unroll
-          for (int q = 0; q < 16; ++q) g[q] = silu(g[q] * rsc) * (up[q] * rsc);
+          for (int q = 0; q < 16; ++q) g[q] = glu(ep, g[q] * rsc, up[q] * rsc);
           bf16_raw* o = ep.out + (size_t)m * ep.ldo + col_base / 2 + jp * 16;
           st16(o, pack8(g));
           st16(o + 8, pack8(g + 8));
@@ -332,7 +332,7 @@ extern "C" int lsa_gemm_wr(const void* a, int lda, const void* wp, int M, int N,
   if (N % bn) return LSA_BAD_SHAPE;
   if (epi != EPI_STORE && epi != EPI_QKV && epi != EPI_SWIGLU) return LSA_UNSUPPORTED;
   if (epi == EPI_SWIGLU && bn == 192) return LSA_UNSUPPORTED;  // 3 tiles per wave: no whole gate/up pairs
-  if (epi == EPI_STORE && (!ep->out || ep->ldo < N || ep->ldo % 8)) return LSA_BAD_SHAPE;
+  if (epi == EPI_STORE && ((!ep->out && !ep->out32) || ep->ldo < N || ep->ldo % 8)) return LSA_BAD_SHAPE;
   if (epi == EPI_SWIGLU && (!ep->out || ep->ldo < N / 2 || ep->ldo % 8 || ep->act || ep->bias)) return LSA_BAD_SHAPE;
   if (epi == EPI_QKV && (!ep->k_cache || !ep->v_cache || !ep->slot || !ep->pos || !ep->out)) return LSA_BAD_SHAPE;
   if (ep->ss_out) return LSA_BAD_SHAPE;

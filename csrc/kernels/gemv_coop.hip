@@ -490,7 +490,7 @@ __global__ __launch_bounds__(NW * KW * 64) void gemv_coop_kernel(
       load16(2 * tp, mm, r, gg);
       load16(2 * tp + 1, mm, r, uu);
 #pragma unroll
-      for (int j = 0; j < 16; ++j) gg[j] = silu(gg[j]) * uu[j];
+      for (int j = 0; j < 16; ++j) gg[j] = glu(ep, gg[j], uu[j]);
       bf16_raw* o = ep.out + (size_t)mm * ep.ldo + (ntg0 / 2 + tp) * 16;
       st16(o, pack8(gg));
       st16(o + 8, pack8(gg + 8));
@@ -607,6 +607,74 @@ int dispatch(int mb, int tnw, int nw, int kf, int kw, int d, bool norm, const bf
   return LSA_UNSUPPORTED;
 }
 
+}  // namespace
+
+// One launch, as the entry points hand it to the epilogue's object.
+struct CoopCall {
+  int mb, tnw, nw, kf, kw, d;
+  bool norm;
+  const bf16_raw* x;
+  int ldx;
+  const int* a_rows;
+  const bf16_raw* wp;
+  int M, N, K, SK;
+  float eps;
+  const EpiArgs* ep;
+  float* slab;
+  unsigned* cnt;
+  const float* wscale;
+  hipStream_t stream;
+};
+
+// The kernels of one (epilogue, weight format) are the slowest code of the library to compile,
+// so csrc/build.py compiles this file once per unit, side by side: LSA_COOP_UNIT = EPI_* (bf16
+// weights), LSA_COOP_UNIT_FP8 (every epilogue with fp8 weights) or LSA_COOP_UNIT_ENTRY (the
+// extern "C" entry points). Without LSA_COOP_UNIT the one object holds everything. A library
+// linked without a unit answers LSA_UNSUPPORTED for it (weak references).
+#define LSA_COOP_UNIT_FP8 6
+#define LSA_COOP_UNIT_ENTRY 7
+#ifdef LSA_COOP_UNIT
+#define COOP_HAS(U) (LSA_COOP_UNIT == (U))
+#else
+#define COOP_HAS(U) 1
+#endif
+#define LSA_COOP_EPIS(X) X(EPI_STORE, store) X(EPI_RESID, resid) X(EPI_SWIGLU, swiglu) X(EPI_QKV, qkv) \
+  X(EPI_ARGMAX, argmax) X(EPI_PARTIAL, partial)
+#define LSA_COOP_DECL(E, name)                                                     \
+  __attribute__((weak)) int lsa_coop_unit_##name(const CoopCall& c);               \
+  __attribute__((weak)) int lsa_coop_unit_fp8_##name(const CoopCall& c);
+LSA_COOP_EPIS(LSA_COOP_DECL)
+#define LSA_COOP_DEF(E, FP8, fn)                                                                                       \
+  int fn(const CoopCall& c) {                                                                                          \
+    return dispatch<E, FP8>(c.mb, c.tnw, c.nw, c.kf, c.kw, c.d, c.norm, c.x, c.ldx, c.a_rows, c.wp, c.M, c.N, c.K,     \
+                            c.SK, c.eps, *c.ep, c.slab, c.cnt, c.wscale, c.stream);                                    \
+  }
+#if COOP_HAS(0)
+LSA_COOP_DEF(EPI_STORE, false, lsa_coop_unit_store)
+#endif
+#if COOP_HAS(1)
+LSA_COOP_DEF(EPI_RESID, false, lsa_coop_unit_resid)
+#endif
+#if COOP_HAS(2)
+LSA_COOP_DEF(EPI_SWIGLU, false, lsa_coop_unit_swiglu)
+#endif
+#if COOP_HAS(3)
+LSA_COOP_DEF(EPI_QKV, false, lsa_coop_unit_qkv)
+#endif
+#if COOP_HAS(4)
+LSA_COOP_DEF(EPI_ARGMAX, false, lsa_coop_unit_argmax)
+#endif
+#if COOP_HAS(5)
+LSA_COOP_DEF(EPI_PARTIAL, false, lsa_coop_unit_partial)
+#endif
+#if COOP_HAS(LSA_COOP_UNIT_FP8)
+#define LSA_COOP_DEF_FP8(E, name) LSA_COOP_DEF(E, true, lsa_coop_unit_fp8_##name)
+LSA_COOP_EPIS(LSA_COOP_DEF_FP8)
+#endif
+
+#if COOP_HAS(LSA_COOP_UNIT_ENTRY)
+namespace {
+
 // K is split into 32*kf-k chunks, spread over the SK splits as evenly as possible.
 // Workspace: slab >= SK*N*16*MB*4 + SK*(N/16/(nw*tnw))*16*MB*4 bytes (only when SK > 1);
 // counters: N/16/(nw*tnw) zero-initialised uint32 (reset by the kernel itself).
@@ -629,19 +697,16 @@ int coop_entry(const void* x, int ldx, const int* a_rows, const void* wp, int M,
   }
   if (epi == EPI_SWIGLU && tg % 2) return LSA_BAD_SHAPE;  // gate / up tile pairs stay in one workgroup
   if (sk > 1 && (!slab || !counters)) return LSA_BAD_SHAPE;
-  const bf16_raw* xx = static_cast<const bf16_raw*>(x);
-  const bf16_raw* w = static_cast<const bf16_raw*>(wp);
-  const bool n = norm != 0;
-#define LSA_D(E) dispatch<E, FP8>(mb, tnw, nw, kf, kw, d, n, xx, ldx, a_rows, w, M, N, K, sk, eps, *ep, slab, counters, wscale, stream)
+  const CoopCall c{mb, tnw, nw, kf, kw, d, norm != 0, static_cast<const bf16_raw*>(x), ldx, a_rows,
+                   static_cast<const bf16_raw*>(wp), M, N, K, sk, eps, ep, slab, counters, wscale, stream};
+  int (*unit)(const CoopCall&) = nullptr;
+#define LSA_D(E, name)                                              \
+  case E: unit = FP8 ? lsa_coop_unit_fp8_##name : lsa_coop_unit_##name; break;
   switch (epi) {
-    case EPI_STORE: return LSA_D(EPI_STORE);
-    case EPI_RESID: return LSA_D(EPI_RESID);
-    case EPI_SWIGLU: return LSA_D(EPI_SWIGLU);
-    case EPI_QKV: return LSA_D(EPI_QKV);
-    case EPI_ARGMAX: return LSA_D(EPI_ARGMAX);
-    case EPI_PARTIAL: return LSA_D(EPI_PARTIAL);
+    LSA_COOP_EPIS(LSA_D)
     default: return LSA_UNSUPPORTED;
   }
+  return unit ? unit(c) : LSA_UNSUPPORTED;
 #undef LSA_D
 }
 
@@ -673,3 +738,4 @@ extern "C" int lsa_gemv_coop_fp8(const void* x, int ldx, const int* a_rows, cons
   return coop_entry<true>(x, ldx, a_rows, wq, M, N, K, norm, eps, epi, ep, tnw, nw, kf, sk, 1, 3, slab, counters,
                           wscale, stream);
 }
+#endif  // COOP_HAS(LSA_COOP_UNIT_ENTRY)

@@ -170,7 +170,7 @@ __global__ __launch_bounds__(NW * 64) void gemv_fp8_kernel(
       if (mm >= M) continue;
       const float r = rstd(mm);
       const float g = rsum(2 * tp, mm, n) * r, u = rsum(2 * tp + 1, mm, n) * r;
-      ep.out[(size_t)mm * ep.ldo + (nt0 / 2 + tp) * 16 + n] = f2bf(silu(g) * u);
+      ep.out[(size_t)mm * ep.ldo + (nt0 / 2 + tp) * 16 + n] = f2bf(glu(ep, g, u));
     }
   } else {
     for (int e = tid; e < TN * MR * 16; e += NTHR) {
@@ -180,7 +180,7 @@ __global__ __launch_bounds__(NW * 64) void gemv_fp8_kernel(
       const float v = rsum(t, mm, n) * r;
       const int col = (nt0 + t) * 16 + n;
       if (EPI == EPI_STORE) {
-        ep.out[(size_t)mm * ep.ldo + col] = f2bf(epi_act(ep, v + epi_bias(ep, col)));
+        epi_store1(ep, mm, col, v);
       } else if (EPI == EPI_RESID) {
         ep.out[(size_t)mm * ep.ldo + col] = f2bf(bf2f(ep.resid[(size_t)mm * ep.ldr + col]) + v + epi_bias(ep, col));
       } else if (EPI == EPI_QKV) {

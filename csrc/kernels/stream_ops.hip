@@ -1,0 +1,164 @@
+// Kernels of a decoder whose residual stream is fp32 and whose norms sit on the sublayers' OUTPUTS
+// (the sublayers read the stream itself):
+//   lsa_stream_embed     x = table[id] * scale in fp32, plus the copy the projections read
+//   lsa_stream_add_norm  x += rms(y) * gain: a sublayer's result, RMS-normed, joins the stream (gain
+//                        = norm weight times layer scale, fp32), plus the copy the projections read
+//   lsa_stream_norm      rms(x) * gain -> the head projection's input
+//   lsa_logits_argmax    argmax keys of fp32 logits (the fp32 engine; the bf16 one fuses this
+//                        into the head GEMM)
+//   lsa_cast_rows        fp32 rows -> the projections' type (a stage's input stream)
+// T is the projections' type (bf16, or fp32 for the fp32 engine). Rows of the copies may be wider
+// than the stream (GEMM padding): those columns are left as they are (zero).
+#include "elem.h"
+
+namespace {
+
+template <typename T>
+__global__ __launch_bounds__(256) void stream_embed_kernel(const int* __restrict__ ids, const T* __restrict__ table,
+                                                           int ldt, float scale, int W, float* __restrict__ x, int ldx,
+                                                           T* __restrict__ xc, int ldc) {
+  const int row = blockIdx.x;
+  const T* src = table + (size_t)ids[row] * ldt;
+  for (int c = threadIdx.x; c < W; c += 256) {
+    const float v = ld1(src + c) * scale;
+    x[(size_t)row * ldx + c] = v;
+    st1(xc + (size_t)row * ldc + c, v);
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void cast_rows_kernel(const float* __restrict__ x, int ldx, int W, T* __restrict__ xc,
+                                                        int ldc) {
+  const int row = blockIdx.x;
+  for (int c = threadIdx.x; c < W; c += 256) st1(xc + (size_t)row * ldc + c, x[(size_t)row * ldx + c]);
+}
+
+// ADD: x += rms(y) * gain and xc = x; else xc = rms(y) * gain. One workgroup per row; a row of up
+// to 256 * 4 * NV values stays in registers (NV > 0), longer ones are read twice.
+template <typename T, bool ADD, int NV>
+__global__ __launch_bounds__(256) void norm_rows_kernel(const float* __restrict__ y, int ldy,
+                                                        const float* __restrict__ gain, float eps, int W,
+                                                        float* __restrict__ x, int ldx, T* __restrict__ xc, int ldc) {
+  __shared__ float s_part[4];
+  const int row = blockIdx.x, tid = threadIdx.x;
+  const float* yr = y + (size_t)row * ldy;
+  float* xr = ADD ? x + (size_t)row * ldx : nullptr;
+  T* cr = xc + (size_t)row * ldc;
+  float s = 0.f;
+  if constexpr (NV > 0) {  // W % 4 == 0, every pointer 16-B aligned
+    f32x4_t v[NV], xv[NV];
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int c = (tid + j * 256) * 4;
+      v[j] = c < W ? *reinterpret_cast<const f32x4_t*>(yr + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+      if (ADD) xv[j] = c < W ? *reinterpret_cast<const f32x4_t*>(xr + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+    }
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+#pragma unroll
+      for (int k = 0; k < 4; ++k) s += v[j][k] * v[j][k];
+    s = wave_sum(s);
+    if ((tid & 63) == 0) s_part[tid >> 6] = s;
+    __syncthreads();
+    const float rs = 1.f / sqrtf((s_part[0] + s_part[1] + s_part[2] + s_part[3]) / (float)W + eps);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int c = (tid + j * 256) * 4;
+      if (c >= W) break;
+      const f32x4_t g = *reinterpret_cast<const f32x4_t*>(gain + c);
+      f32x4_t o;
+#pragma unroll
+      for (int k = 0; k < 4; ++k) o[k] = (ADD ? xv[j][k] : 0.f) + v[j][k] * rs * g[k];
+      if (ADD) *reinterpret_cast<f32x4_t*>(xr + c) = o;
+      st4(cr + c, o);
+    }
+  } else {
+    for (int c = tid; c < W; c += 256) s += yr[c] * yr[c];
+    s = wave_sum(s);
+    if ((tid & 63) == 0) s_part[tid >> 6] = s;
+    __syncthreads();
+    const float rs = 1.f / sqrtf((s_part[0] + s_part[1] + s_part[2] + s_part[3]) / (float)W + eps);
+    for (int c = tid; c < W; c += 256) {
+      const float o = (ADD ? xr[c] : 0.f) + yr[c] * rs * gain[c];
+      if (ADD) xr[c] = o;
+      st1(cr + c, o);
+    }
+  }
+}
+
+template <typename T, bool ADD>
+void launch_norm(const float* y, int ldy, const float* gain, float eps, int rows, int W, float* x, int ldx, T* xc,
+                 int ldc, hipStream_t s) {
+  const bool vec = W % 4 == 0 && ldy % 4 == 0 && ldc % 4 == 0 && (!ADD || ldx % 4 == 0) &&
+                   ((uintptr_t)y | (uintptr_t)gain | (uintptr_t)x | (uintptr_t)xc) % 16 == 0;
+  const int nv = vec ? (W + 1023) / 1024 : 0;
+#define LSA_N(NV) norm_rows_kernel<T, ADD, NV><<<rows, 256, 0, s>>>(y, ldy, gain, eps, W, x, ldx, xc, ldc)
+  if (nv >= 1 && nv <= 2) LSA_N(2);
+  else if (nv >= 3 && nv <= 4) LSA_N(4);
+  else if (nv >= 5 && nv <= 8) LSA_N(8);
+  else LSA_N(0);
+#undef LSA_N
+}
+
+// grid (rows, blocks): every workgroup one stretch of the vocabulary
+__global__ __launch_bounds__(256) void logits_argmax_kernel(const float* __restrict__ lg, int ldl, int V, int offset,
+                                                            unsigned long long* __restrict__ keys) {
+  __shared__ unsigned long long s_key;
+  if (threadIdx.x == 0) s_key = 0ull;
+  __syncthreads();
+  unsigned long long best = 0ull;
+  for (int c = blockIdx.y * 256 + threadIdx.x; c < V; c += gridDim.y * 256) {
+    const unsigned long long k = argmax_key(lg[(size_t)blockIdx.x * ldl + c], (unsigned)(c + offset));
+    best = k > best ? k : best;
+  }
+  atomicMax(&s_key, best);
+  __syncthreads();
+  if (threadIdx.x == 0) atomicMax(keys + blockIdx.x, s_key);
+}
+
+}  // namespace
+
+extern "C" int lsa_stream_embed(int f32, const int* ids, int rows, const void* table, int ldt, float scale, int W,
+                                float* x, int ldx, void* xc, int ldc, hipStream_t s) {
+  if (rows < 1 || W < 1 || ldt < W || ldx < W || ldc < W) return LSA_BAD_SHAPE;
+  if (f32)
+    stream_embed_kernel<float><<<rows, 256, 0, s>>>(ids, (const float*)table, ldt, scale, W, x, ldx, (float*)xc, ldc);
+  else
+    stream_embed_kernel<bf16_raw><<<rows, 256, 0, s>>>(ids, (const bf16_raw*)table, ldt, scale, W, x, ldx, (bf16_raw*)xc, ldc);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+extern "C" int lsa_cast_rows(int f32, const float* x, int ldx, int rows, int W, void* xc, int ldc, hipStream_t s) {
+  if (rows < 1 || W < 1 || ldx < W || ldc < W) return LSA_BAD_SHAPE;
+  if (f32) cast_rows_kernel<float><<<rows, 256, 0, s>>>(x, ldx, W, (float*)xc, ldc);
+  else cast_rows_kernel<bf16_raw><<<rows, 256, 0, s>>>(x, ldx, W, (bf16_raw*)xc, ldc);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+extern "C" int lsa_stream_add_norm(int f32, const float* y, int ldy, const float* gain, float eps, int rows, int W,
+                                   float* x, int ldx, void* xc, int ldc, hipStream_t s) {
+  if (rows < 1 || W < 1 || ldy < W || ldx < W || ldc < W || !x) return LSA_BAD_SHAPE;
+  if (f32) launch_norm<float, true>(y, ldy, gain, eps, rows, W, x, ldx, (float*)xc, ldc, s);
+  else launch_norm<bf16_raw, true>(y, ldy, gain, eps, rows, W, x, ldx, (bf16_raw*)xc, ldc, s);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+extern "C" int lsa_stream_norm(int f32, const float* y, int ldy, const float* gain, float eps, int rows, int W, void* xc,
+                               int ldc, hipStream_t s) {
+  if (rows < 1 || W < 1 || ldy < W || ldc < W) return LSA_BAD_SHAPE;
+  if (f32) launch_norm<float, false>(y, ldy, gain, eps, rows, W, nullptr, 0, (float*)xc, ldc, s);
+  else launch_norm<bf16_raw, false>(y, ldy, gain, eps, rows, W, nullptr, 0, (bf16_raw*)xc, ldc, s);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+extern "C" int lsa_logits_argmax(const float* lg, int ldl, int rows, int V, int offset, unsigned long long* keys,
+                                 hipStream_t s) {
+  if (rows < 1 || V < 1 || ldl < V || !keys) return LSA_BAD_SHAPE;
+  logits_argmax_kernel<<<dim3(rows, (V + 4095) / 4096), 256, 0, s>>>(lg, ldl, V, offset, keys);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}

@@ -19,9 +19,11 @@ import time
 import torch
 
 sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
-from llm_sharding_amd.config import LlamaConfig, get_preset  # noqa: E402
+from llm_sharding_amd.config import get_preset  # noqa: E402
 from llm_sharding_amd.models.tokenizer import SyntheticByteTokenizer, load_tokenizer  # noqa: E402
-from llm_sharding_amd.runtime.engine import DecodeGraph, RandomSource, ShardFolderSource, StageEngine  # noqa: E402
+from llm_sharding_amd.runtime.engine import DecodeGraph  # noqa: E402
+from llm_sharding_amd.runtime.registry import (compute_dtype, folder_source, load_config,  # noqa: E402
+                                              make_engine, random_source)
 
 
 def main():
@@ -31,18 +33,21 @@ def main():
     ap.add_argument("--prompt", default="Write a poem about the blue sky.")
     ap.add_argument("--max-new-tokens", type=int, default=128)
     ap.add_argument("--device", default="cuda:0" if torch.cuda.is_available() else "cpu")
+    ap.add_argument("--dtype", default="bfloat16", help="compute type on a GPU (float32 where the model has it)")
     ap.add_argument("--hf-compare", default="", help="HF checkpoint dir: also run transformers' greedy generate "
                                                      "(the reference inference.py's path, fp32 CPU) and compare tokens")
     a = ap.parse_args()
     if a.shards:
-        cfg = LlamaConfig.from_pretrained(a.shards)
-        src, tok = ShardFolderSource(a.shards, cfg), load_tokenizer(a.shards)
+        cfg = load_config(a.shards)
+        src, tok = folder_source(a.shards, cfg), load_tokenizer(a.shards)
     else:
         cfg = get_preset(a.random or "tiny")
-        src, tok = RandomSource(cfg), SyntheticByteTokenizer(cfg.vocab_size)
-    dt = torch.bfloat16 if a.device.startswith("cuda") else torch.float32
+        src, tok = random_source(cfg), SyntheticByteTokenizer(cfg.vocab_size)
+    dt = torch.float32
+    if a.device.startswith("cuda"):
+        dt = compute_dtype(cfg, torch.device(a.device), getattr(torch, a.dtype))
     t0 = time.perf_counter()
-    eng = StageEngine(cfg, 0, cfg.num_hidden_layers, a.device, dt, has_embed=True, has_head=True, source=src,
+    eng = make_engine(cfg, 0, cfg.num_hidden_layers, a.device, dt, has_embed=True, has_head=True, source=src,
                       max_seq=min(cfg.max_position_embeddings, 4096))
     ids = tok(a.prompt, return_tensors="pt")["input_ids"][0]
     print(f"[INFO] loaded in {time.perf_counter() - t0:.1f}s; prompt tokens {ids.numel()}")

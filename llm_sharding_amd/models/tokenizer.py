@@ -125,5 +125,6 @@ def load_tokenizer(path: str):
     cp = os.path.join(path, "config.json")
     if os.path.exists(cp):
         with open(cp) as f:
-            vocab = json.load(f).get("vocab_size", vocab)
+            d = json.load(f)
+        vocab = d.get("vocab_size", d.get("vocab", vocab))
     return SyntheticByteTokenizer(vocab)

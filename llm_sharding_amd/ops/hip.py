@@ -42,10 +42,22 @@ class EpiArgs(ctypes.Structure):
         ("n_kv", ctypes.c_int), ("head_dim", ctypes.c_int), ("t_max", ctypes.c_int),
         ("col_offset", ctypes.c_int), ("act", ctypes.c_int),
         ("ss_out", ctypes.c_void_p), ("ss_in", ctypes.c_void_p), ("ss_n", ctypes.c_int), ("ss_eps", ctypes.c_float),
+        ("out32", ctypes.c_void_p), ("glu_alpha", ctypes.c_float), ("glu_limit", ctypes.c_float),
+        ("glu_shift", ctypes.c_float),
     ]
 
 
 _lib = None
+_family = ""
+
+
+def use_family(name: str) -> None:
+    """Load the library of one model family's kernels (csrc/build.py FAMILIES) instead of the full
+    one. Calling a kernel of another family raises."""
+    global KERNELS_SO, _family
+    if _lib is not None:
+        raise RuntimeError("the kernel library is loaded already")
+    KERNELS_SO, _family = os.path.join(NATIVE_DIR, f"liblsa_kernels-{name}.so"), name
 
 
 def available() -> bool:
@@ -70,32 +82,36 @@ def load_library(path: str, mode: int = ctypes.RTLD_LOCAL) -> ctypes.CDLL:
     kernels; scripts/slp_kernel_diff.py runs every kernel of a step from both)."""
     L = ctypes.CDLL(path, mode=mode)
     vp, i, f = ctypes.c_void_p, ctypes.c_int, ctypes.c_float
-    L.lsa_gemv.argtypes = [vp, i, vp, vp, i, i, i, i, f, i, ctypes.POINTER(EpiArgs), i, i, i, vp]
-    L.lsa_gemv_coop.argtypes = [vp, i, vp, vp, i, i, i, i, f, i, ctypes.POINTER(EpiArgs), i, i, i, i, i, i, vp, vp, vp]
-    L.lsa_gemv_fp8.argtypes = [vp, i, vp, vp, vp, i, i, i, i, f, i, ctypes.POINTER(EpiArgs), i, i, i, vp]
-    L.lsa_dequant_fp8_packed.argtypes = [vp, vp, vp, i, i, vp]
-    L.lsa_gemv_coop_fp8.argtypes = [vp, i, vp, vp, vp, i, i, i, i, f, i, ctypes.POINTER(EpiArgs), i, i, i, i, vp, vp, vp]
-    L.lsa_gemm.argtypes = [vp, i, vp, i, i, i, i, ctypes.POINTER(EpiArgs), i, i, vp, vp, vp]
-    L.lsa_attn_decode.argtypes = [vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, f, i, i, vp, vp, vp, i, vp, vp]
-    L.lsa_attn_prefill.argtypes = [vp, i, vp, vp, vp, i, i, i, i, i, f, i, vp, i, vp]
-    L.lsa_attn_decode_mfma.argtypes = [vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, f, vp, i, i, vp]
-    L.lsa_embed.argtypes = [vp, i, vp, i, vp, i, vp]
-    L.lsa_rmsnorm.argtypes = [vp, i, vp, i, i, f, vp, i, vp]
-    L.lsa_layernorm.argtypes = [vp, i, vp, vp, vp, vp, i, i, f, vp, i, vp]
-    L.lsa_resid_rmsnorm_partials.argtypes = [vp, i, vp, i, ctypes.c_longlong, i, vp, i, i, f, vp, i, vp]
-    L.lsa_row_ss.argtypes = [vp, i, i, i, vp, vp]
-    L.lsa_argmax_finalize.argtypes = [vp, i, vp, vp, i, vp, i, i, vp, vp]
-    L.lsa_pos_advance.argtypes = [vp, i, i, vp]
-    L.lsa_gemm_wr.argtypes = [vp, i, vp, i, i, i, i, ctypes.POINTER(EpiArgs), i, i, vp]
-    L.lsa_gemm_sk.argtypes = [vp, i, vp, i, i, i, i, ctypes.POINTER(EpiArgs), i, i, i, i, i, i, i, vp, vp, ctypes.c_longlong, i,
-                              vp]
-    L.lsa_attn_oproj.argtypes = [vp, i, vp, vp, vp, vp, vp, i, i, i, i, f, vp, vp, i, i, ctypes.POINTER(EpiArgs), vp, i,
-                                 vp]
-    for name in ("lsa_gemv", "lsa_gemv_coop", "lsa_attn_oproj", "lsa_gemv_fp8", "lsa_dequant_fp8_packed", "lsa_gemv_coop_fp8", "lsa_gemm",
-                 "lsa_gemm_sk", "lsa_gemm_wr", "lsa_attn_decode", "lsa_attn_prefill", "lsa_embed", "lsa_rmsnorm", "lsa_layernorm",
-                 "lsa_resid_rmsnorm_partials", "lsa_row_ss",
-                 "lsa_argmax_finalize", "lsa_pos_advance", "lsa_version"):
-        getattr(L, name).restype = ctypes.c_int
+    sig = {
+        "lsa_gemv": [vp, i, vp, vp, i, i, i, i, f, i, ctypes.POINTER(EpiArgs), i, i, i, vp],
+        "lsa_gemv_coop": [vp, i, vp, vp, i, i, i, i, f, i, ctypes.POINTER(EpiArgs), i, i, i, i, i, i, vp, vp, vp],
+        "lsa_gemv_fp8": [vp, i, vp, vp, vp, i, i, i, i, f, i, ctypes.POINTER(EpiArgs), i, i, i, vp],
+        "lsa_dequant_fp8_packed": [vp, vp, vp, i, i, vp],
+        "lsa_gemv_coop_fp8": [vp, i, vp, vp, vp, i, i, i, i, f, i, ctypes.POINTER(EpiArgs), i, i, i, i, vp, vp, vp],
+        "lsa_gemm": [vp, i, vp, i, i, i, i, ctypes.POINTER(EpiArgs), i, i, vp, vp, vp],
+        "lsa_attn_decode": [vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, f, i, i, vp, vp, vp, i, vp, vp],
+        "lsa_attn_prefill": [vp, i, vp, vp, vp, i, i, i, i, i, f, i, vp, i, vp],
+        "lsa_attn_decode_mfma": [vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, f, vp, i, i, vp],
+        "lsa_embed": [vp, i, vp, i, vp, i, vp],
+        "lsa_rmsnorm": [vp, i, vp, i, i, f, vp, i, vp],
+        "lsa_layernorm": [vp, i, vp, vp, vp, vp, i, i, f, vp, i, vp],
+        "lsa_resid_rmsnorm_partials": [vp, i, vp, i, ctypes.c_longlong, i, vp, i, i, f, vp, i, vp],
+        "lsa_row_ss": [vp, i, i, i, vp, vp],
+        "lsa_argmax_finalize": [vp, i, vp, vp, i, vp, i, i, vp, vp],
+        "lsa_pos_advance": [vp, i, i, vp],
+        "lsa_gemm_wr": [vp, i, vp, i, i, i, i, ctypes.POINTER(EpiArgs), i, i, vp],
+        "lsa_gemm_sk": [vp, i, vp, i, i, i, i, ctypes.POINTER(EpiArgs), i, i, i, i, i, i, i, vp, vp, ctypes.c_longlong, i, vp],
+        "lsa_attn_oproj": [vp, i, vp, vp, vp, vp, vp, i, i, i, i, f, vp, vp, i, i, ctypes.POINTER(EpiArgs), vp, i, vp],
+        "lsa_version": [],
+    }
+    for name, args in sig.items():
+        if _family and not hasattr(L, name):
+            continue
+        fn = getattr(L, name)
+        fn.argtypes, fn.restype = args, ctypes.c_int
+    if hasattr(L, "lsa_latent_append"):
+        from . import latent
+        latent.declare(L)
     if os.environ.get("LSA_ATTN_SMALL_MAX_WGS"):  # A/B runs of the small-grid decode attention's range
         L.lsa_attn_set_small_max_wgs.argtypes = [i]
         _check(L.lsa_attn_set_small_max_wgs(int(os.environ["LSA_ATTN_SMALL_MAX_WGS"])), "lsa_attn_set_small_max_wgs")
@@ -129,17 +145,21 @@ ACT_NONE, ACT_GELU = 0, 1  # EpiArgs.act (EPI_STORE): identity / tanh-GELU (GPT-
 
 def make_epi(out=None, resid=None, k_cache=None, v_cache=None, slot=None, pos=None, cos=None,
              sin=None, keys=None, ldo=0, ldr=0, n_heads=0, n_kv=0, head_dim=0, t_max=0,
-             col_offset=0, bias=None, act=ACT_NONE, ss_out=None, ss_in=None, ss_eps=0.0) -> EpiArgs:
+             col_offset=0, bias=None, act=ACT_NONE, ss_out=None, ss_in=None, ss_eps=0.0, out32=None,
+             glu_alpha=0.0, glu_limit=0.0, glu_shift=0.0) -> EpiArgs:
     """Epilogue arguments. ``bias``: optional fp32 [N] added to every output column (in packed
     column order); ``cos=None`` with EPI_QKV: no RoPE, natural q|k|v column order.
     ``ss_out`` / ``ss_in`` (gemm_sk): fp32 [>= M, H/64] row partial sums of squares - a RESID
     GEMM writes them for its outputs, a QKV / SWIGLU GEMM reading the raw residual stream as A
-    applies the RMSNorm scale from them (the norm weight is folded into its W)."""
+    applies the RMSNorm scale from them (the norm weight is folded into its W). ``out32``: fp32
+    output of an EPI_STORE GEMM instead of ``out``. ``glu_limit`` > 0: EPI_SWIGLU computes the
+    clipped gated unit with these constants instead of silu(g) * u (epilogue.h glu)."""
+    _req(out32 is None or out32.dtype == torch.float32, "epilogue: out32 must be fp32")
     if bias is not None:
         _req(bias.dtype == torch.float32 and bias.is_contiguous(), "epilogue bias: contiguous fp32")
     # vectorised epilogues store 16-B runs: rows must start 16-B aligned
     _req(ldo % 8 == 0 and ldr % 8 == 0, f"epilogue: ldo/ldr ({ldo}, {ldr}) must be multiples of 8")
-    for t in (out, resid, bias):
+    for t in (out, resid, bias, out32):
         _req(t is None or t.data_ptr() % 16 == 0, "epilogue: out/resid/bias must be 16-byte aligned")
     _req(head_dim == 0 or (head_dim & (head_dim - 1)) == 0, f"epilogue: head_dim {head_dim} not a power of two")
     ssb = ss_in if ss_in is not None else ss_out
@@ -147,7 +167,8 @@ def make_epi(out=None, resid=None, k_cache=None, v_cache=None, slot=None, pos=No
         _req(t is None or (t.dtype == torch.float32 and t.dim() == 2 and t.is_contiguous()), "epilogue: ss fp32 [M, H/64]")
     return EpiArgs(_p(out), _p(resid), _p(k_cache), _p(v_cache), _p(slot), _p(pos), _p(cos), _p(sin),
                    _p(keys), _p(bias), ldo, ldr, n_heads, n_kv, head_dim, t_max, col_offset, int(act),
-                   _p(ss_out), _p(ss_in), 0 if ssb is None else ssb.shape[1], float(ss_eps))
+                   _p(ss_out), _p(ss_in), 0 if ssb is None else ssb.shape[1], float(ss_eps), _p(out32),
+                   float(glu_alpha), float(glu_limit), float(glu_shift))
 
 
 # ------------------------------------------------------------------------------ projections

@@ -28,7 +28,8 @@ from typing import Optional
 import torch
 
 from ..config import get_preset
-from ..runtime.engine import DecodeGraph, EagerDecode, RandomSource, StageEngine
+from ..runtime.engine import DecodeGraph, EagerDecode, StageEngine
+from ..runtime.registry import compute_dtype, make_engine, random_source
 from ..utils import tracing
 from .scheduler import plan_stages, scratch_bytes, stage_memory
 
@@ -245,7 +246,7 @@ class PipelineStage:
         self.device = torch.device(device)
         self.gpu = self.device.type == "cuda"
         self.use_graph = use_graph and self.gpu
-        self.dtype = torch.bfloat16 if self.gpu else dtype
+        self.dtype = compute_dtype(cfg, self.device, dtype)
         # Split lm_head (GPU pipelines of >= 2 stages): the last stage covers vocab [0, V1), the
         # first stage [V1, V). The ring back-edge then carries the raw final hidden + partial
         # argmax keys instead of token ids, and the first stage completes the argmax at the
@@ -266,13 +267,13 @@ class PipelineStage:
                 raise ValueError("PipelineStage: the shared engine does not match this stage")
             self.eng = engine
         else:
-            self.eng = StageEngine(cfg, start, end, device, self.dtype, has_embed=self.first,
+            self.eng = make_engine(cfg, start, end, device, self.dtype, has_embed=self.first,
                                    has_head=self.last or (self.split and self.first), source=source,
                                    max_slots=batch * microbatches, max_seq=max_seq,
                                    max_prefill_rows=max(max_prefill_rows, batch), head_cols=head_cols,
                                    weight_dtype=weight_dtype)
         H = cfg.hidden_size
-        self.h_out = [torch.zeros((batch, H), dtype=self.dtype, device=self.device) for _ in range(microbatches)]
+        self.h_out = [torch.zeros((batch, H), dtype=self.eng.hidden_dtype, device=self.device) for _ in range(microbatches)]
         self.tok_out = [torch.zeros(batch, dtype=torch.int32, device=self.device) for _ in range(microbatches)]
         if self.split:
             self.keys_out = [torch.zeros(batch, dtype=torch.int64, device=self.device) for _ in range(microbatches)]
@@ -333,7 +334,7 @@ class PipelineStage:
         if self.first:
             h = eng.embed(prompts[mb].reshape(-1).to(self.device))
         else:
-            h = torch.empty((B * P, H), dtype=self.dtype, device=self.device)
+            h = torch.empty((B * P, H), dtype=eng.hidden_dtype, device=self.device)
             self._recv(h, self.rank - 1)
         with self.tl.span("prefill", mb=mb, rows=B * P):
             h = eng.forward(h, slot, pos)
@@ -362,7 +363,7 @@ class PipelineStage:
 
     def recv_first_token(self, mb: int = 0) -> torch.Tensor:
         if self.split:
-            hf = torch.zeros((self.B, self.cfg.hidden_size), dtype=self.dtype, device=self.device)
+            hf = torch.zeros((self.B, self.cfg.hidden_size), dtype=self.eng.hidden_dtype, device=self.device)
             keys = torch.zeros(self.B, dtype=torch.int64, device=self.device)
             self._recv(hf, self.world - 1)
             self._recv(keys, self.world - 1)
@@ -421,7 +422,7 @@ class PipelineStage:
                 and os.environ.get("LSA_GRAPH_COMM", "1") == "1"):
             return False
         H = self.cfg.hidden_size
-        probe = [torch.empty((self.B, H), dtype=self.dtype, device=self.device),
+        probe = [torch.empty((self.B, H), dtype=self.eng.hidden_dtype, device=self.device),
                  torch.empty(self.B, dtype=torch.int64, device=self.device),
                  torch.empty(self.B, dtype=torch.int32, device=self.device)]
         return all(self.p2p.fits(t) for t in probe)
@@ -860,7 +861,7 @@ def run_decode_benchmark(model: str = "llama2-7b", n_gpus: int = 1, steps: int =
               f"edges {topology['edges']}", flush=True)
     t0 = time.perf_counter()
     stage = PipelineStage(cfg, srank, pp, st.start, st.end, dev, batch, M, max_seq,
-                          RandomSource(cfg, seed), use_graph=use_graph,
+                          random_source(cfg, seed), use_graph=use_graph,
                           max_prefill_rows=batch * prompt_len, weight_dtype=weight_dtype, streams=streams,
                           dtype=torch.bfloat16 if gpu else torch.float32, p2p=p2p)
     if dp > 1:  # trace files are named by rank: use the global one

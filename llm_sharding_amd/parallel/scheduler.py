@@ -68,7 +68,10 @@ class Plan:
 
 
 def default_costs(cfg: LlamaConfig, elem_bytes: int = 2) -> tuple:
-    layer = [float(cfg.layer_bytes(elem_bytes))] * cfg.num_hidden_layers
+    if hasattr(cfg, "layer_costs"):  # a stack: layers of different sizes
+        layer = cfg.layer_costs(elem_bytes)
+    else:
+        layer = [float(cfg.layer_bytes(elem_bytes))] * cfg.num_hidden_layers
     head = float((cfg.vocab_size * cfg.hidden_size + cfg.hidden_size) * elem_bytes)
     embed = float(cfg.hidden_size * elem_bytes)  # one row gathered per token
     return layer, embed, head
@@ -179,6 +182,8 @@ def scratch_bytes(cfg: LlamaConfig, rows: int, sets: int = 1, max_seq: int = 409
     StageEngine._alloc_runtime / decode_scratch: activations, attention split partials and
     their tickets, the coop-GEMV workspace, the gemm_sk slabs and split-K partials (> 128 rows)."""
     from ..ops import packing
+    if hasattr(cfg, "scratch_bytes"):
+        return float(sets * cfg.scratch_bytes(max(rows, packing.GEMV_MAX_ROWS)))
     H, I, nh, hd = cfg.hidden_size, cfg.intermediate_size, cfg.num_attention_heads, cfg.head_dim
     dmr = packing.GEMV_MAX_ROWS
     R = max(rows, dmr)

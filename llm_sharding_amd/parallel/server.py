@@ -43,6 +43,7 @@ from typing import Callable, Dict, List, Optional
 import torch
 
 from ..runtime.engine import DecodeGraph, StageEngine
+from ..runtime.registry import compute_dtype, make_engine
 from ..utils import tracing
 from .pipeline import DistP2P, _percentile
 
@@ -112,7 +113,11 @@ class PipelineServer:
     def __init__(self, cfg, source, rank: int = 0, world: int = 1, start: int = 0, end: Optional[int] = None,
                  device="cpu", batch: int = 8, microbatches: int = 1, max_seq: int = 2048,
                  prefill_budget: int = 2048, use_graph: bool = True, dtype=torch.bfloat16,
-                 ctrl_group=None, p2p=None, causal: bool = True, verbose: bool = False, streams: int = 1):
+                 ctrl_group=None, p2p=None, causal: bool = True, verbose: bool = False, streams: int = 1,
+                 cache_tokens: Optional[int] = None):
+        """``cache_tokens`` (models with a paged cache): tokens the cache holds over all slots; requests
+        wait until the pages of their prompt and all their new tokens are free (default: every
+        slot's longest sequence)."""
         self.cfg, self.rank, self.world = cfg, rank, world
         end = cfg.num_hidden_layers if end is None else end
         self.first, self.last = rank == 0, rank == world - 1
@@ -120,10 +125,10 @@ class PipelineServer:
         self.device = torch.device(device)
         self.gpu = self.device.type == "cuda"
         self.graph_mode = use_graph and self.gpu
-        self.dtype = torch.bfloat16 if self.gpu else dtype
+        self.dtype = compute_dtype(cfg, self.device, dtype)
         self.budget = int(prefill_budget)
         self.verbose = verbose
-        self.source, self.causal, self.max_seq = source, causal, max_seq
+        self.source, self.causal, self.max_seq, self.cache_tokens = source, causal, max_seq, cache_tokens
         self.start, self.end = start, end
         self.eng = self._build_engine(start, end)
         self.p2p = p2p if p2p is not None else DistP2P()
@@ -158,9 +163,10 @@ class PipelineServer:
 
     # ------------------------------------------------------------------ engine (re)build
     def _build_engine(self, start: int, end: int) -> StageEngine:
-        return StageEngine(self.cfg, start, end, self.device, self.dtype, has_embed=self.first, has_head=self.last,
+        extra = {} if self.cache_tokens is None else {"cache_tokens": self.cache_tokens}
+        return make_engine(self.cfg, start, end, self.device, self.dtype, has_embed=self.first, has_head=self.last,
                            source=self.source, max_slots=self.B * self.M, max_seq=self.max_seq,
-                           max_prefill_rows=max(self.budget, self.B), causal=self.causal)
+                           max_prefill_rows=max(self.budget, self.B), causal=self.causal, **extra)
 
     def _build_graphs(self) -> None:
         for k in range(1, self.S):
@@ -237,7 +243,19 @@ class PipelineServer:
         self.eng.seq_len[slot] = p
         if self.graph_mode:
             mb, i = divmod(slot, self.B)
-            self.graphs[mb].pos[i] = p
+            self.graphs[mb].set_pos(i, p)
+
+    def _clear(self, slot: int) -> None:
+        """A finished sequence's slot: position 0, its cache memory given back."""
+        self._set_pos(slot, 0)
+        self.eng.reset([slot])
+
+    def _cache_fits(self, r: "Request") -> bool:
+        """Room in a shared cache for all of ``r``, beside what the live requests may still grow to."""
+        if self.eng.cache_budget is None:
+            return True
+        held = sum(self.eng.cache_need(len(q.input_ids) + q.max_new_tokens) for q in self.by_slot.values())
+        return held + self.eng.cache_need(len(r.input_ids) + r.max_new_tokens) <= self.eng.cache_budget
 
     def _to_host(self, t: torch.Tensor):
         """Token ids -> host without serialising the host behind later GPU work: a pinned
@@ -289,10 +307,12 @@ class PipelineServer:
     def _exec_body(self, cmd, mb, items, resets, ids=None):
         eng, H = self.eng, self.cfg.hidden_size
         for s in resets:
-            self._set_pos(s, 0)
+            self._clear(s)
         if cmd == CMD_PREFILL:
             slot, pos, emit_rows = [], [], []
             for (s, p0, n, emit) in items:
+                if p0 == 0:
+                    eng.reset([s])  # a new sequence: whatever the slot's last one held is free
                 eng.seq_len[s] = p0
                 slot += [s] * n
                 pos += list(range(p0, p0 + n))
@@ -302,7 +322,7 @@ class PipelineServer:
             if self.first:
                 h = eng.embed(torch.tensor(ids, dtype=torch.int64))
             else:
-                h = torch.empty((rows, H), dtype=self.dtype, device=self.device)
+                h = torch.empty((rows, H), dtype=eng.hidden_dtype, device=self.device)
                 self.p2p.recv(h, self.rank - 1)
             h = eng.forward(h, slot, pos)
             for (s, p0, n, emit) in items:
@@ -337,7 +357,7 @@ class PipelineServer:
             if self.first:
                 h = eng.embed(torch.tensor(ids, dtype=torch.int64))
             else:
-                h = torch.empty((n, H), dtype=self.dtype, device=self.device)
+                h = torch.empty((n, H), dtype=eng.hidden_dtype, device=self.device)
                 self.p2p.recv(h, self.rank - 1)
             pos = [it[1] for it in items]
             for s, p in zip(slots, pos):
@@ -367,6 +387,8 @@ class PipelineServer:
         if len(ids) + max_new_tokens > self.eng.max_seq:
             raise ValueError(f"prompt ({len(ids)}) + max_new_tokens ({max_new_tokens}) exceeds max_seq "
                              f"{self.eng.max_seq}")
+        if self.eng.cache_budget is not None and self.eng.cache_need(len(ids) + max_new_tokens) > self.eng.cache_budget:
+            raise ValueError(f"prompt ({len(ids)}) + max_new_tokens ({max_new_tokens}) exceeds the cache")
         with self._lock:
             rid = self._next_id
             self._next_id += 1
@@ -468,7 +490,7 @@ class PipelineServer:
         resets = self.pending_resets[mb]
         # admission: waiting requests into free slots (held back while a re-plan drains)
         for s in self._free_slots(mb):
-            if not self.waiting or self._replan is not None:
+            if not self.waiting or self._replan is not None or not self._cache_fits(self.waiting[0]):
                 break
             r = self.waiting.pop(0)
             r.slot, r.state, r.prefilled = s, PREFILLING, 0
@@ -513,7 +535,7 @@ class PipelineServer:
         if not run:
             with self._mb_ctx(mb):
                 for s in resets:
-                    self._set_pos(s, 0)
+                    self._clear(s)
             return
         local = self._exec(cmd, mb, items, resets, ids=ids)
         self.outstanding[mb] = (cmd, info, local)
@@ -571,7 +593,7 @@ class PipelineServer:
                 break
             if cmd == 0:
                 for s in resets:
-                    self._set_pos(s, 0)
+                    self._clear(s)
                 continue
             self._exec(cmd, mb, items, resets)
         self._flush_sends()

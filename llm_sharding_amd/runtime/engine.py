@@ -30,6 +30,7 @@ import torch
 import torch.nn.functional as F
 
 from ..config import LlamaConfig, ceil_div
+from ..models import deretar as DT
 from ..models import gpt2 as G2
 from ..models import weights as W
 from ..models.rope import rope_table
@@ -128,6 +129,52 @@ class RandomSource(WeightSource):
         return G2.random_ln_f(self.cfg, dtype, device, self.seed)[1] if self.cfg.is_gpt2 else None
 
 
+class StackFolderSource(WeightSource):
+    """A stack design's checkpoint folder (config.json + model.safetensors, models/deretar.py)."""
+
+    def __init__(self, path: str, cfg):
+        self.path, self.cfg = path, cfg
+        self.tensors = DT.DeretarTensors(path)
+
+    def layer(self, i, device, dtype):
+        o = self.cfg.layers[i].owner
+        shapes = DT.layer_shapes(self.cfg, o)
+        t = self.tensors.get({k: f"l{o}.{k}" for k in shapes}, device, dtype)
+        for k, shp in shapes.items():
+            if tuple(t[k].shape) != shp:
+                raise ValueError(f"l{o}.{k} has shape {tuple(t[k].shape)}, config.json says {shp}")
+        return t
+
+    def embedding(self, device, dtype):
+        t = self.tensors.get({"w": "embed"}, device, dtype)["w"]
+        if tuple(t.shape) != (self.cfg.vocab_size, self.cfg.hidden_size):
+            raise ValueError(f"embed has shape {tuple(t.shape)}")
+        return t
+
+    def final_norm(self, device, dtype):
+        return self.tensors.get({"w": "final.norm"}, device, dtype)["w"]
+
+    lm_head = embedding  # tied
+
+
+class StackRandomSource(WeightSource):
+    """Deterministic random tensors of a stack design, made on the target device."""
+
+    def __init__(self, cfg, seed: int = 0):
+        self.cfg, self.seed = cfg, seed
+
+    def layer(self, i, device, dtype):
+        return DT.random_layer(self.cfg, i, dtype, device, self.seed)
+
+    def embedding(self, device, dtype):
+        return DT.random_embedding(self.cfg, dtype, device, self.seed)
+
+    def final_norm(self, device, dtype):
+        return DT.random_final_norm(self.cfg, dtype, device, self.seed)
+
+    lm_head = embedding
+
+
 @dataclass
 class LayerWeights:
     qkv: torch.Tensor      # packed (GPU) or fused-unpacked (CPU) [qkv, H]
@@ -186,6 +233,8 @@ class StageEngine:
     # launches (profiles/r6_attn_oproj.md); LSA_ATTN_OPROJ=1 turns it on
     ATTN_OPROJ = os.environ.get("LSA_ATTN_OPROJ", "0") == "1"
 
+    GPU_DTYPES = (torch.bfloat16,)  # compute types of the HIP path
+
     def __init__(self, cfg: LlamaConfig, start: int, end: int, device="cpu",
                  dtype=torch.bfloat16, *, has_embed: bool = False, has_head: bool = False,
                  source: Optional[WeightSource] = None, max_slots: int = 1, max_seq: int = 2048,
@@ -196,13 +245,11 @@ class StageEngine:
         self.cfg = cfg
         self.start, self.end = start, end
         self.n_layers = end - start
-        if "LSA_GEMV_MAX_ROWS" not in os.environ:  # the class value (env / tests) bounds the route table's
-            from ..ops import routes
-            self.GEMV_MAX_ROWS = min(type(self).GEMV_MAX_ROWS, routes.gemv_max_rows(self.proj_shapes(cfg)))
+        self._init_routes()
         self.device = torch.device(device)
         self.gpu = _is_gpu(self.device)
-        if self.gpu and dtype != torch.bfloat16:
-            raise ValueError("the HIP path computes in bfloat16 (pass dtype=torch.bfloat16)")
+        if self.gpu and dtype not in self.GPU_DTYPES:
+            raise ValueError(f"this model's HIP path computes in {self.GPU_DTYPES}, not {dtype}")
         self.dtype = dtype
         self.has_embed, self.has_head = has_embed, has_head
         if weight_dtype not in ("bf16", "fp8"):
@@ -237,6 +284,16 @@ class StageEngine:
             _hip.lib()
         if load:
             self.load()
+
+    @property
+    def hidden_dtype(self) -> torch.dtype:
+        """Type of the rows stages hand each other (the residual stream)."""
+        return self.dtype
+
+    def _init_routes(self) -> None:
+        if "LSA_GEMV_MAX_ROWS" not in os.environ:  # the class value (env / tests) bounds the route table's
+            from ..ops import routes
+            self.GEMV_MAX_ROWS = min(type(self).GEMV_MAX_ROWS, routes.gemv_max_rows(self.proj_shapes(self.cfg)))
 
     # ------------------------------------------------------------------------- loading
     @staticmethod
@@ -482,6 +539,16 @@ class StageEngine:
         for s in (range(self.max_slots) if slots is None else slots):
             self.seq_len[s] = 0
 
+    # Cache memory that sequences share (paged engines): units in all, units a sequence of ``tokens``
+    # takes, and room for a slot's next decoded token. A static cache has no shared budget.
+    cache_budget: Optional[int] = None
+
+    def cache_need(self, tokens: int) -> int:
+        return 0
+
+    def grow(self, slot: int, tokens: int) -> None:
+        """Make sure a live ``slot`` has room for its first ``tokens`` tokens."""
+
     # ------------------------------------------------------------------------- helpers
     def _i32(self, x) -> torch.Tensor:
         if isinstance(x, torch.Tensor):
@@ -501,6 +568,11 @@ class StageEngine:
             hip.embed(self._i32(ids), self.embed_w, out)
             return out
         return F.embedding(ids.to(self.device, torch.long), self.embed_w)
+
+    def embed_into(self, ids: torch.Tensor, h: torch.Tensor) -> None:
+        """ids (int32) -> the rows of ``h``, without allocating (decode graphs)."""
+        from ..ops import hip
+        hip.embed(ids, self.embed_w, h)
 
     def forward(self, h: torch.Tensor, slot, pos, kv_len=None) -> torch.Tensor:
         """Run this stage's layers on ``h`` [rows, H]. Row r is a token of the sequence in
@@ -617,6 +689,14 @@ class StageEngine:
             c = min(self.DECODE_MAX_ROWS, n - c0)
             hip.argmax_finalize(keys[c0:c0 + c], c, out[c0:c0 + c])
         return out
+
+    def logits(self, h: torch.Tensor, rows_idx=None) -> torch.Tensor:
+        """fp32 logits of the selected rows over this stage's part of the vocabulary."""
+        if self.gpu:
+            raise NotImplementedError("this model's GPU head returns tokens only (head, head_keys)")
+        hs = h if rows_idx is None else h[torch.as_tensor(rows_idx, dtype=torch.long)]
+        lg = self.logits_torch(hs)
+        return lg[:, :min(self.head_v1, self.cfg.vocab_size) - self.head_v0]
 
     def logits_torch(self, hs: torch.Tensor) -> torch.Tensor:
         from ..models.reference import rmsnorm
@@ -953,7 +1033,8 @@ class DecodeGraph:
         self.pos = torch.tensor([eng.seq_len[s] for s in self.slots], dtype=torch.int32, device=dev)
         self.tokens = torch.zeros(rows, dtype=torch.int32, device=dev)
         self.keys = torch.zeros(rows, dtype=torch.int64, device=dev)
-        self.h_in = torch.zeros((rows, eng.cfg.hidden_size), dtype=torch.bfloat16, device=dev)
+        self.h_in = torch.zeros((rows, eng.cfg.hidden_size), dtype=eng.hidden_dtype, device=dev)
+        self._host_pos = [eng.seq_len[s] for s in self.slots]  # paged caches: where the next tokens go
         self.history = torch.zeros((max(1, history_len), rows), dtype=torch.int32, device=dev) if history_len else None
         self.step_ctr = torch.zeros(1, dtype=torch.int32, device=dev)
         self.graph = None
@@ -969,7 +1050,7 @@ class DecodeGraph:
         if split_head:
             if mode not in ("first", "last"):
                 raise ValueError("split_head needs mode 'first' or 'last'")
-            self.h_fin = torch.zeros((rows, eng.cfg.hidden_size), dtype=torch.bfloat16, device=dev)
+            self.h_fin = torch.zeros((rows, eng.cfg.hidden_size), dtype=eng.hidden_dtype, device=dev)
             self.keys_in = torch.zeros(rows, dtype=torch.int64, device=dev)
 
     def _body(self) -> None:
@@ -985,7 +1066,7 @@ class DecodeGraph:
             hip.argmax_finalize(self.keys, rows, self.tokens, None, 1, self.history,
                                 self.step_ctr if self.history is not None else None)
         if self.mode in ("full", "first"):
-            hip.embed(self.tokens, eng.embed_w, h)
+            eng.embed_into(self.tokens, h)
         else:
             h.copy_(self.h_in)
         eng._forward_hip(h, self.slot, self.pos, None, rows, nsplit=eng.decode_nsplit(rows))
@@ -1034,10 +1115,20 @@ class DecodeGraph:
         return self
 
     def replay(self) -> None:
+        if self.eng.cache_budget is not None:
+            for i, s in enumerate(self.slots):
+                self.eng.grow(s, self._host_pos[i] + 1)
+                self._host_pos[i] += 1
         self.graph.replay()
+
+    def set_pos(self, i: int, p: int) -> None:
+        """Row ``i``'s next token goes to position ``p``."""
+        self.pos[i] = p
+        self._host_pos[i] = p
 
     def set_positions(self) -> None:
         self.pos.copy_(torch.tensor([self.eng.seq_len[s] for s in self.slots], dtype=torch.int32))
+        self._host_pos = [self.eng.seq_len[s] for s in self.slots]
 
     def sync_positions(self) -> None:
         p = self.pos.tolist()
@@ -1054,13 +1145,13 @@ class EagerDecode:
         self.eng, self.rows, self.mode = eng, rows, mode
         self.slots = list(range(rows)) if slots is None else list(slots)
         self.tokens = torch.zeros(rows, dtype=torch.int32)
-        self.h_in = torch.zeros((rows, eng.cfg.hidden_size), dtype=eng.dtype)
+        self.h_in = torch.zeros((rows, eng.cfg.hidden_size), dtype=eng.hidden_dtype)
         self.history = torch.zeros((history_len, rows), dtype=torch.int32) if history_len else None
         self.step = 0
         self._out = None
         self.split_head = split_head
         self.keys = torch.zeros(rows, dtype=torch.int64)
-        self.h_fin = torch.zeros((rows, eng.cfg.hidden_size), dtype=eng.dtype)
+        self.h_fin = torch.zeros((rows, eng.cfg.hidden_size), dtype=eng.hidden_dtype)
         self.keys_in = torch.zeros(rows, dtype=torch.int64)
 
     def _body(self) -> None:

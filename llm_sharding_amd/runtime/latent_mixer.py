@@ -1,0 +1,244 @@
+"""Latent attention as a layer mixer of :class:`.stack_engine.StackEngine`: weights and forward.
+
+``Weights`` is loaded once per owner layer and shared by every layer that uses its tensors; the cache
+belongs to the layer. One forward of a row batch (any mix of sequences, prompt portions beside
+single decoded tokens) is
+
+    input projection   x -> [query latent | key latent, rotated key part | gate]      one GEMM
+    append             both latents normed, rotated part turned, key side into the cache
+    query projection   query latent -> q                                              one GEMM
+    attention          per row in the absorbed form, or for long portions expanded (below)
+    output projection  gated heads -> fp32
+
+Rows are dealt to the two attention forms by run (consecutive positions of one sequence): a run of
+at least ``expand_min`` rows multiplies keys and values of its visible tokens out once and runs the
+flash kernel; everything else attends over the latents themselves.
+"""
+from __future__ import annotations
+
+from typing import Optional
+
+import torch
+import torch.nn.functional as F
+
+from ..models.stack import LatentSpec, pad_to
+
+
+def rotation_tables(spec: LatentSpec, n: int, device) -> tuple:
+    """cos, sin [n, rot_dims / 2] fp32 of p * base^(-2i / dims)."""
+    i = torch.arange(spec.rot_dims // 2, dtype=torch.float64)
+    ang = torch.outer(torch.arange(n, dtype=torch.float64), spec.rot_base ** (-2.0 * i / spec.rot_dims))
+    return ang.cos().float().to(device).contiguous(), ang.sin().float().to(device).contiguous()
+
+
+def _head_pad(w: torch.Tensor, heads: int, parts) -> torch.Tensor:
+    """Rows [heads][sum of sizes] -> [heads][sum of padded sizes], zeros behind every part.
+    ``parts``: [(size, padded size), ...]."""
+    v = w.view(heads, sum(s for s, _ in parts), w.shape[1])
+    out, o = [], 0
+    for s, p in parts:
+        out.append(F.pad(v[:, o:o + s], (0, 0, 0, p - s)))
+        o += s
+    return torch.cat(out, 1).reshape(-1, w.shape[1])
+
+
+class Weights:
+    """One owner layer's mixer tensors, laid out for the kernels (GPU) or as they are (CPU)."""
+
+    def __init__(self, spec: LatentSpec, t: dict, gpu: bool):
+        self.spec = spec
+        self.gpu = gpu
+        if not gpu:
+            self.raw = t
+            return
+        from ..ops import latent as L
+        s, H = spec, spec.heads
+        self.raw = None
+        self.f32 = t["dq"].dtype == torch.float32
+        # input projection: query latent at column 0, key latent + rotated part at ok, gate at og
+        self.ok = pad_to(s.q_rank, 16)
+        self.og = self.ok + pad_to(s.kv_rank + s.rot_dim, 16)
+        win = torch.zeros((self.og + H * s.dvp, t["dq"].shape[1]), dtype=t["dq"].dtype, device=t["dq"].device)
+        win[:s.q_rank] = t["dq"]
+        win[self.ok:self.ok + s.kv_rank + s.rot_dim] = t["dkv"]
+        win[self.og:] = _head_pad(t["g"], H, [(s.vdim, s.dvp)])
+        self.inp = L.Linear(win)
+        self.uq = L.Linear(_head_pad(t["uq"], H, [(s.dim, s.dkp), (s.rot_dim, s.rp)]))
+        self.out = L.Linear(_head_pad(t["o"].t().contiguous(), H, [(s.vdim, s.dvp)]).t().contiguous())
+        self.gq = t["dq.norm"].float().contiguous()
+        self.gk = t["dkv.norm"].float().contiguous()
+        uk = _head_pad(t["uk"], H, [(s.dim, s.dkp)])             # [H dkp, kv_rank]
+        uv = _head_pad(t["uv"], H, [(s.vdim, s.dvp)])
+        uk, uv = (F.pad(w, (0, s.krp - s.kv_rank)).view(H, -1, s.krp) for w in (uk, uv))
+        self.tuned = L.tuned_size(s) and not self.f32            # MFMA kernels of the absorbed form
+        self.expand = L.expand_size(s) and self.tuned            # MFMA kernel of the expanded form
+        if self.tuned:
+            self.wk = L.pack_heads(uk.transpose(1, 2))           # N = latent, K = key dimension
+            self.wv = L.pack_heads(uv)                           # N = value dimension, K = latent
+        else:
+            self.wk = uk.contiguous()                            # [H, dkp, krp]
+            self.wv = uv.transpose(1, 2).contiguous()            # [H, krp, dvp]
+        self.kv = L.Linear(torch.cat([uk, uv], 1).reshape(-1, s.krp), k=s.krp) if self.expand else None
+
+    def tensors(self) -> list:
+        if not self.gpu:
+            return list(self.raw.values())
+        ts = [self.wk, self.wv, self.gq, self.gk]
+        for lin in (self.inp, self.uq, self.out, self.kv):
+            ts += lin.tensors() if lin is not None else []
+        return ts
+
+    # ------------------------------------------------------------------ GPU
+    def forward(self, eng, x: torch.Tensor, y: torch.Tensor, cache: torch.Tensor, slot, pos, rows: int, plan) -> None:
+        """``x`` [rows, padded width] -> ``y`` fp32 [rows, padded width]; appends to ``cache``."""
+        from ..ops import latent as L
+        s = self.spec
+        inp, cq = eng.scratch_view("inp", rows, self.inp.n), eng.scratch_view("cq", rows, self.uq.k)
+        q, ao = eng.scratch_view("q", rows, self.uq.n), eng.scratch_view("attn", rows, self.out.k)
+        cos, sin = eng.rotation(s)
+        table = eng.pool.table
+        a = L.make_args(s, cache, table, slot, pos, cos, sin, eng.cfg.norm_eps)
+        eng.project(self.inp, x, rows, inp)
+        L.append(a, rows, inp, 0, self.ok, self.gq, self.gk, cq)
+        eng.project(self.uq, cq, rows, q)
+        gate = inp[:, self.og:]
+        if plan.n_absorbed(self):
+            idx = plan.absorbed_index(self)
+            n = plan.n_absorbed(self)
+            b = a if idx is None else L.make_args(s, cache, table, slot, pos, cos, sin, eng.cfg.norm_eps, index=idx)
+            qt, po, pm, cap = eng.attend_scratch(s, n)
+            ns = max(1, min(plan.nsplit(eng, self), cap // n))
+            if self.tuned:
+                L.absorb_mfma(b, n, q, self.wk, qt)
+                L.attend_mfma(b, n, qt, ns, po, pm)
+                L.value_mfma(b, n, po, pm, ns, self.wv, gate, ao)
+            else:
+                L.absorb(b, n, q, self.wk, qt)
+                L.attend(b, n, qt, ns, po, pm)
+                L.value(b, n, po, pm, ns, self.wv, gate, ao)
+        for g in plan.expanded_groups(self):
+            lat, kv = eng.expand_scratch(s, g.tokens, self.kv.n)
+            L.gather(a, g.src, g.tokens, lat)
+            eng.project(self.kv, lat, g.tokens, kv)
+            L.prefill(a, g.tiles, g.tiles_host, q, kv, lat, gate, ao, rows, g.tokens)
+        eng.project(self.out, ao, rows, y)
+
+    # ------------------------------------------------------------------ CPU
+    def forward_torch(self, eng, x, cache, slot, pos) -> torch.Tensor:
+        """The same mixer on a CPU engine (absorbed form); cache [pages, 64, kv_rank + rot_dim]."""
+        s, w, H = self.spec, {k: v.float() for k, v in self.raw.items()}, self.spec.heads
+        eps, dt = eng.cfg.norm_eps, eng.dtype
+        cos, sin = eng.rotation(s)
+        half = s.rot_dims // 2
+
+        def rms(v, g):
+            return v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * g
+
+        def turn(v, p):
+            c, sn = cos[p], sin[p]
+            if v.dim() == 3:
+                c, sn = c[:, None], sn[:, None]
+            u, z, rest = v[..., :half], v[..., half:2 * half], v[..., 2 * half:]
+            return torch.cat([u * c - z * sn, z * c + u * sn, rest], -1)
+
+        d = F.linear(x, w["dkv"])
+        entry = torch.cat([rms(d[:, :s.kv_rank], w["dkv.norm"]), turn(d[:, s.kv_rank:], pos)], -1)
+        page = eng.pool.table[slot, pos // 64].long()
+        cache[page, pos % 64] = entry.to(dt)
+        q = F.linear(rms(F.linear(x, w["dq"]), w["dq.norm"]), w["uq"]).view(-1, H, s.dim + s.rot_dim)
+        qt = torch.cat([torch.einsum("nhd,hdk->nhk", q[..., :s.dim], w["uk"].view(H, s.dim, s.kv_rank)),
+                        turn(q[..., s.dim:], pos)], -1)
+        o = torch.empty((x.shape[0], H, s.kv_rank))
+        for i in range(x.shape[0]):
+            n = int(pos[i]) + 1
+            keys = cache[eng.pool.table[slot[i], :-(-n // 64)].long()].reshape(-1, cache.shape[-1])[:n].float()
+            p = torch.softmax(qt[i] @ keys.t() * s.scale, -1)
+            o[i] = p @ keys[:, :s.kv_rank]
+        v = torch.einsum("nhk,hvk->nhv", o, w["uv"].view(H, s.vdim, s.kv_rank)).reshape(x.shape[0], -1)
+        return F.linear(v * torch.sigmoid(F.linear(x, w["g"])), w["o"])
+
+
+class Group:
+    """Runs expanded together: their tokens (cache entries to gather) and query tiles."""
+
+    def __init__(self, runs, tile_rows: int, device):
+        src, tiles, kv0 = [], [], 0
+        for (row0, n, slot, p0) in runs:
+            total = p0 + n
+            src.append(torch.stack([torch.full((total,), slot), torch.arange(total)], 1))
+            for r in range(0, n, tile_rows):
+                m = min(tile_rows, n - r)
+                tiles.append([row0 + r, m, kv0, p0 + r, p0 + r + m, 0, 0, 0])
+            kv0 += total
+        tiles.sort(key=lambda t: -t[4])
+        self.tokens = kv0
+        self.src = torch.cat(src).to(torch.int32).to(device)
+        self.tiles_host = torch.tensor(tiles, dtype=torch.int32)
+        self.tiles = self.tiles_host.to(device)
+
+
+class Plan:
+    """How one row batch's attention runs: built once per forward, used by every layer."""
+
+    GROUP_TOKENS = 1 << 16  # expanded tokens at a time (bounds the expanded keys' and values' memory)
+
+    def __init__(self, eng, rows: int, runs: Optional[list], nsplit: Optional[int] = None):
+        """``runs``: [(first row, rows, slot, first position)] covering the batch, or None when only
+        the device knows (a decode graph): everything absorbed."""
+        self.eng, self.rows, self.runs, self._ns = eng, rows, runs, nsplit
+        self._cache: dict = {}
+
+    @staticmethod
+    def find_runs(slot: list, pos: list) -> list:
+        runs, r, n = [], 0, len(slot)
+        while r < n:
+            e = r + 1
+            while e < n and slot[e] == slot[r] and pos[e] == pos[e - 1] + 1:
+                e += 1
+            runs.append((r, e - r, slot[r], pos[r]))
+            r = e
+        return runs
+
+    def _split(self, w: Weights):
+        key = w.spec if w.expand else None
+        if key not in self._cache:
+            if self.runs is None or not w.expand:
+                self._cache[key] = (self.rows, None, [])
+            else:
+                long = [r for r in self.runs if r[1] >= self.eng.expand_min]
+                if not long:
+                    self._cache[key] = (self.rows, None, [])
+                else:
+                    from ..ops import latent as L
+                    idx = [i for r in self.runs if r[1] < self.eng.expand_min for i in range(r[0], r[0] + r[1])]
+                    groups, cur, tok = [], [], 0
+                    rows = L.prefill_tile_rows(sum(r[1] for r in long), w.spec.heads)
+                    for r in long:
+                        if cur and tok + r[1] + r[3] > self.GROUP_TOKENS:
+                            groups.append(Group(cur, rows, self.eng.device))
+                            cur, tok = [], 0
+                        cur.append(r)
+                        tok += r[1] + r[3]
+                    groups.append(Group(cur, rows, self.eng.device))
+                    dev = torch.tensor(idx, dtype=torch.int32).to(self.eng.device) if idx else None
+                    self._cache[key] = (len(idx), dev, groups)
+        return self._cache[key]
+
+    def n_absorbed(self, w) -> int:
+        return self._split(w)[0]
+
+    def absorbed_index(self, w):
+        return self._split(w)[1]
+
+    def expanded_groups(self, w) -> list:
+        return self._split(w)[2]
+
+    def nsplit(self, eng, w) -> int:
+        """Splits of a row's keys, so that a small batch still fills the chip."""
+        if self._ns is None:
+            longest = max(p0 + n for _, n, _, p0 in self.runs)
+            return eng.latent_nsplit(w.spec, self.n_absorbed(w), longest)
+        return self._ns
+
+
+__all__ = ["Weights", "Plan", "Group", "rotation_tables"]

@@ -1,0 +1,402 @@
+"""StackEngine: a pipeline stage of a config-driven layer stack (:class:`..models.stack.StackConfig`).
+
+The same step function, sequence API, decode graphs and serving as :class:`.engine.StageEngine`, for
+decoders that differ from Llama / GPT-2 in what a layer is made of:
+
+* the residual stream is fp32 (rows of ``hidden_dtype``), every sublayer reads it in the projections'
+  type and its result joins it through a norm of its own (stream_ops.hip, one launch);
+* mixers and feed-forwards come from the layer's spec; layers may share tensors;
+* the cache is paged (:mod:`.paging`): one pool for all slots, one page table for all layers;
+* projections run the framework's GEMV / GEMM kernels on padded weights (ops/latent.Linear); fp32
+  engines run every product in true fp32.
+"""
+from __future__ import annotations
+
+from typing import Optional
+
+import torch
+import torch.nn.functional as F
+
+from ..config import ceil_div
+from ..models.stack import StackConfig, pad_to
+from .engine import StageEngine, WeightSource
+from .latent_mixer import Plan, Weights, rotation_tables
+from .paging import PagePool
+
+PAGE = 64
+
+
+class _Layer:
+    def __init__(self, spec, mixer, mlp, gain1, gain2):
+        self.spec, self.mixer, self.mlp, self.gain1, self.gain2 = spec, mixer, mlp, gain1, gain2
+
+
+class _Glu:
+    """Gate / up / down projection of a clipped gated unit."""
+
+    def __init__(self, spec, t: dict, gpu: bool):
+        self.spec = spec
+        self.raw = None if gpu else t
+        if gpu:
+            from ..ops import latent as L
+            self.gate_up, self.down = L.Linear.glu(t["gate"], t["up"]), L.Linear(t["down"])
+
+    def tensors(self) -> list:
+        return list(self.raw.values()) if self.raw is not None else self.gate_up.tensors() + self.down.tensors()
+
+    def forward(self, eng, x, y, rows: int) -> None:
+        act = eng.scratch_view("act", rows, self.down.k)
+        eng.project(self.gate_up, x, rows, act, glu=self.spec)
+        eng.project(self.down, act, rows, y)
+
+    def forward_torch(self, x) -> torch.Tensor:
+        w, s = {k: v.float() for k, v in self.raw.items()}, self.spec
+        g = F.linear(x, w["gate"]).clamp(max=s.limit)
+        u = F.linear(x, w["up"]).clamp(-s.limit, s.limit)
+        return F.linear(g * torch.sigmoid(s.alpha * g) * (u + s.shift), w["down"])
+
+
+class StackEngine(StageEngine):
+    GPU_DTYPES = (torch.bfloat16, torch.float32)
+    SCRATCH_ATTRS = ("buf_h", "buf_x", "buf_y", "flat", "qt", "part_o", "part_ml", "coop_ws", "sk_ws", "keys", "tokens",
+                     "_x_ready")
+    # rows from which a run of one sequence's consecutive positions attends in the expanded form: below,
+    # multiplying keys and values out costs more than the wider products of the absorbed form
+    expand_min = 64
+
+    def __init__(self, cfg: StackConfig, start: int, end: int, device="cpu", dtype=torch.bfloat16, *,
+                 has_embed: bool = False, has_head: bool = False, source: Optional[WeightSource] = None,
+                 max_slots: int = 1, max_seq: int = 2048, max_prefill_rows: int = 2048, causal: bool = True,
+                 load: bool = True, verbose: bool = False, head_cols: Optional[tuple] = None,
+                 weight_dtype: str = "bf16", cache_tokens: Optional[int] = None):
+        """``cache_tokens``: tokens the page pool holds (default: every slot's longest sequence)."""
+        if not causal:
+            raise ValueError("stack engines attend causally")
+        if weight_dtype != "bf16":
+            raise ValueError("stack engines keep their weights in the compute type (weight_dtype='bf16')")
+        pages = ceil_div(min(max_seq, cfg.max_position_embeddings), PAGE) * max_slots
+        self.cache_pages = pages if cache_tokens is None else ceil_div(cache_tokens, PAGE)
+        self._rot: dict = {}
+        self._expand_bufs: dict = {}
+        super().__init__(cfg, start, end, device, dtype, has_embed=has_embed, has_head=has_head, source=source,
+                         max_slots=max_slots, max_seq=max_seq, max_prefill_rows=max_prefill_rows, causal=causal,
+                         load=load, verbose=verbose, head_cols=head_cols, weight_dtype=weight_dtype)
+
+    # ------------------------------------------------------------------------- loading
+    def _init_routes(self) -> None:
+        pass
+
+    @property
+    def hidden_dtype(self) -> torch.dtype:
+        return torch.float32
+
+    @property
+    def head_vocab(self) -> int:
+        """Vocabulary entries this stage's part of the head covers."""
+        return min(self.head_v1, self.cfg.vocab_size) - self.head_v0
+
+    @property
+    def width_p(self) -> int:
+        return pad_to(self.cfg.hidden_size, 128)
+
+    def load(self) -> None:
+        cfg, dev, dt = self.cfg, self.device, self.dtype
+        if self.source is None:
+            raise ValueError("StackEngine needs a WeightSource")
+        self.layers, shared = [], {}
+        for i in range(self.start, self.end):
+            spec = cfg.layers[i]
+            if spec.owner not in shared:
+                self._log(f"[INFO] loading layer {i}")
+                shared[spec.owner] = self._prepare(spec, self.source.layer(i, dev, dt))
+            self.layers.append(_Layer(spec, *shared[spec.owner]))
+        table = None
+        if self.has_embed or self.has_head:
+            table = self.source.embedding(dev, dt).contiguous()
+        if self.has_embed:
+            self.embed_w = table
+        if self.has_head:
+            self.final_norm = (self.source.final_norm(dev, dt).float() + cfg.norm_offset).contiguous()
+            head = F.pad(table, (0, 0, 0, cfg.head_rows - cfg.vocab_size))[self.head_v0:self.head_v1]
+            if self.gpu:
+                from ..ops import latent as L
+                self.lm_head = L.Linear(head)
+            else:
+                self.lm_head = head.contiguous()
+            n = self.lm_head.n if self.gpu else head.shape[0]
+            if n > self.head_vocab:  # padding rows must not win the argmax
+                self.head_bias = torch.zeros(n, dtype=torch.float32, device=dev)
+                self.head_bias[self.head_vocab:] = -3.0e38
+        self._alloc_runtime()
+
+    def _prepare(self, spec, t: dict) -> tuple:
+        def part(p):
+            return {k[len(p):]: v for k, v in t.items() if k.startswith(p)}
+
+        def gain(n):  # norm weight times layer scale, fp32
+            return ((t[f"norm{n}"].float() + self.cfg.norm_offset) * t[f"ls{n}"].float()).contiguous()
+
+        mixer = Weights(spec.mixer, part("mix."), self.gpu)
+        if spec.mlp is None:
+            return mixer, None, gain(1), None
+        return mixer, _Glu(spec.mlp, part("mlp."), self.gpu), gain(1), gain(2)
+
+    # ------------------------------------------------------------------------- memory
+    def _alloc_runtime(self) -> None:
+        cfg, dev, dt = self.cfg, self.device, self.dtype
+        self.pool = PagePool(self.cache_pages, self.max_slots, self.max_seq, PAGE, dev)
+
+        def width(spec):
+            return spec.mixer.cache_width if self.gpu else spec.mixer.kv_rank + spec.mixer.rot_dim
+
+        self.k_cache = [torch.zeros((self.cache_pages, PAGE, width(l.spec)), dtype=dt, device=dev) for l in self.layers]
+        self.v_cache = []
+        for l in self.layers:
+            m = l.spec.mixer
+            if (m.rot_base, m.rot_dims) not in self._rot:
+                self._rot[(m.rot_base, m.rot_dims)] = rotation_tables(m, self.pool.max_pages * PAGE, dev)
+        self.cos = self.sin = None
+        if self.gpu:
+            # widest row of every intermediate over the layers
+            mx = {"inp": 0, "cq": 0, "q": 0, "attn": 0, "act": 0}
+            for l in self.layers:
+                w = l.mixer
+                for k, n in (("inp", w.inp.n), ("cq", w.uq.k), ("q", w.uq.n), ("attn", w.out.k),
+                             ("act", l.mlp.down.k if l.mlp is not None else 0)):
+                    mx[k] = max(mx[k], n)
+            self._widths = mx
+            for k, v in self._scratch_set(max(self.max_prefill_rows, self.DECODE_MAX_ROWS)).items():
+                setattr(self, k, v)
+
+    def _projections(self) -> list:
+        out = []
+        for l in self.layers:
+            out += [(p.n, p.k, False) for p in (l.mixer.inp, l.mixer.uq, l.mixer.out)]
+            if l.mlp is not None:
+                out += [(l.mlp.gate_up.n, l.mlp.gate_up.k, True), (l.mlp.down.n, l.mlp.down.k, False)]
+        if self.has_head:
+            out.append((self.lm_head.n, self.lm_head.k, False))
+        return sorted(set(out))
+
+    def _scratch_set(self, R: int) -> dict:
+        """Everything a forward of up to R rows writes besides the cache."""
+        from ..ops import hip, packing
+        dev, dt, W = self.device, self.dtype, self.width_p
+        out = {"buf_h": torch.zeros((R, self.cfg.hidden_size), dtype=torch.float32, device=dev),
+               "buf_x": torch.zeros((R, W), dtype=dt, device=dev),
+               "buf_y": torch.zeros((R, W), dtype=torch.float32, device=dev),
+               "flat": {k: torch.zeros(R * n, dtype=dt, device=dev) for k, n in self._widths.items() if n},
+               "keys": torch.zeros(R, dtype=torch.int64, device=dev),
+               "tokens": torch.zeros(R, dtype=torch.int32, device=dev), "_x_ready": False, "coop_ws": None, "sk_ws": None}
+        # absorbed attention: queries, and split partials of up to max(rows, ATTEND_ITEMS) (row, split)s
+        items = max(R, self.ATTEND_ITEMS)
+        qn = max(l.spec.mixer.heads * l.spec.mixer.cache_width for l in self.layers)
+        on = max(l.spec.mixer.heads * l.spec.mixer.krp for l in self.layers)
+        hn = max(l.spec.mixer.heads for l in self.layers)
+        out["qt"] = torch.zeros(R * qn, dtype=dt, device=dev)
+        out["part_o"] = torch.zeros(items * on, dtype=torch.float32, device=dev)
+        out["part_ml"] = torch.zeros(items * hn * 2, dtype=torch.float32, device=dev)
+        if dt == torch.bfloat16:
+            shapes = self._projections()
+            floats, groups = packing.coop_workspace_need([(n, k) for n, k, _ in shapes], self.DECODE_MAX_ROWS,
+                                                         even_n=[(n, k) for n, k, even in shapes if even])
+            out["coop_ws"] = hip.CoopWorkspace(dev, slab_floats=max(floats, 1 << 20), groups=max(groups, 4096))
+            out["sk_ws"] = hip.SkWorkspace(dev)
+        return out
+
+    ATTEND_ITEMS = 1024  # (row, split) pairs the partial buffers hold at least
+
+    def decode_scratch(self, k: int, rows: Optional[int] = None) -> dict:
+        if k == 0:
+            return {a: getattr(self, a) for a in self.SCRATCH_ATTRS}
+        R = max(self.DECODE_MAX_ROWS, rows or 0)
+        if k in self._scratch and self._scratch[k]["buf_h"].shape[0] < R:
+            raise ValueError(f"scratch set {k} was allocated for fewer than {R} rows")
+        if k not in self._scratch:
+            self._scratch[k] = self._scratch_set(R)
+        return self._scratch[k]
+
+    def scratch_view(self, name: str, rows: int, n: int) -> torch.Tensor:
+        return self.flat[name][:rows * n].view(rows, n)
+
+    def attend_scratch(self, s, n: int) -> tuple:
+        """(absorbed queries, partial sums, partial max / sum, (row, split) pairs they hold)."""
+        cap = min(self.part_o.numel() // (s.heads * s.krp), self.part_ml.numel() // (2 * s.heads))
+        return self.qt, self.part_o, self.part_ml, cap
+
+    def expand_scratch(self, s, tokens: int, n: int) -> tuple:
+        """Gathered latents and expanded keys / values (grown on demand: long portions run eagerly;
+        one set per stream of concurrent micro-batches)."""
+        key = torch.cuda.current_stream(self.device).cuda_stream
+        lat, kv = self._expand_bufs.get(key, (None, None))
+        if lat is None or lat.numel() < tokens * s.cache_width or kv.numel() < tokens * n:
+            m = max(l.spec.mixer.cache_width for l in self.layers)
+            kn = max(l.mixer.kv.n for l in self.layers if l.mixer.kv is not None)
+            t = pad_to(tokens, 1024)
+            lat = torch.empty(t * m, dtype=self.dtype, device=self.device)
+            kv = torch.empty(t * kn, dtype=self.dtype, device=self.device)
+            self._expand_bufs[key] = (lat, kv)
+        return lat[:tokens * s.cache_width].view(tokens, -1), kv[:tokens * n].view(tokens, n)
+
+    def rotation(self, s) -> tuple:
+        return self._rot[(s.rot_base, s.rot_dims)]
+
+    def memory_bytes(self) -> int:
+        ts = [self.embed_w, self.final_norm] + self.k_cache
+        ts += (self.lm_head.tensors() if self.gpu else [self.lm_head]) if self.has_head else []
+        for l in self.layers:
+            ts += l.mixer.tensors() + (l.mlp.tensors() if l.mlp is not None else []) + [l.gain1, l.gain2]
+        seen, n = set(), 0
+        for t in ts:
+            if t is not None and t.data_ptr() not in seen:
+                seen.add(t.data_ptr())
+                n += t.numel() * t.element_size()
+        return n
+
+    # ------------------------------------------------------------------------- sequences and pages
+    @property
+    def cache_budget(self) -> int:
+        return self.pool.pages
+
+    def cache_need(self, tokens: int) -> int:
+        return self.pool.pages_for(tokens)
+
+    def grow(self, slot: int, tokens: int) -> None:
+        if self.pool.held[slot] and tokens <= self.max_seq:
+            self.pool.ensure(slot, tokens)
+
+    def reset(self, slots=None) -> None:
+        for s in (range(self.max_slots) if slots is None else slots):
+            self.seq_len[s] = 0
+            self.pool.release(s)
+
+    def prefill_rows(self, slot_ids: list, lengths: list) -> tuple:
+        out = super().prefill_rows(slot_ids, lengths)
+        for s, n in zip(slot_ids, lengths):
+            self.pool.ensure(s, self.seq_len[s] + n)
+        return out
+
+    # ------------------------------------------------------------------------- forward
+    def project(self, lin, x, rows: int, out, glu=None) -> None:
+        lin(x, rows, out, ws=self.coop_ws, sk_ws=self.sk_ws, glu=glu)
+
+    def embed_into(self, ids: torch.Tensor, h: torch.Tensor) -> None:
+        if self.embed_w is None:
+            raise RuntimeError("[ERROR] this stage has no embedding layer")
+        rows = ids.numel()
+        if not self.gpu:
+            h.copy_(F.embedding(ids.long(), self.embed_w).float() * self.cfg.embed_scale)
+            return
+        from ..ops import latent as L
+        fits = rows <= self.buf_x.shape[0]
+        xc = self.buf_x if fits else torch.empty((rows, self.width_p), dtype=self.dtype, device=self.device)
+        L.stream_embed(ids, self.embed_w, self.cfg.embed_scale, h, xc, rows)
+        self._x_ready = h.data_ptr() == self.buf_h.data_ptr()  # buf_x holds buf_h's copy
+
+    def embed(self, ids: torch.Tensor) -> torch.Tensor:
+        ids = ids.reshape(-1)
+        h = torch.empty((ids.numel(), self.cfg.hidden_size), dtype=torch.float32, device=self.device)
+        self.embed_into(self._i32(ids), h)
+        return h
+
+    def forward(self, h: torch.Tensor, slot, pos, kv_len=None) -> torch.Tensor:
+        if kv_len is not None:
+            raise ValueError("stack engines attend causally (no kv_len)")
+        rows = h.shape[0]
+        sl, ps = ([int(v) for v in (t.tolist() if torch.is_tensor(t) else t)] for t in (slot, pos))
+        if len(sl) != rows or len(ps) != rows:
+            raise ValueError("forward: one slot and one position per row")
+        if min(sl) < 0 or max(sl) >= self.max_slots or min(ps) < 0 or max(ps) >= self.max_seq:
+            raise ValueError("forward: slot or position out of range")
+        need: dict = {}
+        for s, p in zip(sl, ps):
+            need[s] = max(need.get(s, 0), p + 1)
+        for s, n in need.items():
+            self.pool.ensure(s, n)
+        if not self.gpu:
+            return self._forward_stack_torch(h, torch.tensor(sl), torch.tensor(ps))
+        return self._forward_hip(h, self._i32(sl), self._i32(ps), None, rows, runs=Plan.find_runs(sl, ps))
+
+    def latent_nsplit(self, s, entries: int, longest: int) -> int:
+        """Key splits of the absorbed attention: enough workgroups for the chip, splits of at
+        least four pages."""
+        wgs = entries * max(1, ceil_div(s.heads, 16))
+        return int(max(1, min(16, ceil_div(512, wgs), ceil_div(longest, 4 * PAGE))))
+
+    def decode_nsplit(self, rows: int) -> int:
+        m = max((l.spec.mixer for l in self.layers), key=lambda m: m.heads)
+        return self.latent_nsplit(m, rows, self.max_seq)
+
+    def _forward_hip(self, h, slot, pos, kv_len, rows, nsplit: Optional[int] = None, tiles=None, runs=None):
+        from ..ops import latent as L
+        if rows > max(self.max_prefill_rows, self.DECODE_MAX_ROWS):
+            raise ValueError(f"{rows} rows exceed max_prefill_rows={self.max_prefill_rows}")
+        if h.dtype != torch.float32 or not h.is_contiguous():
+            h = h.to(torch.float32).contiguous()
+        hbuf, x, y = self.buf_h[:rows], self.buf_x[:rows], self.buf_y[:rows]
+        if not (self._x_ready and h.data_ptr() == hbuf.data_ptr()):
+            L.cast_rows(h, x, rows)
+        self._x_ready = False
+        if h.data_ptr() != hbuf.data_ptr():
+            hbuf.copy_(h)
+        if runs is None and nsplit is None:
+            nsplit = self.decode_nsplit(rows)
+        plan = Plan(self, rows, runs, nsplit)
+        eps = self.cfg.norm_eps
+        for i, l in enumerate(self.layers):
+            l.mixer.forward(self, x, y, self.k_cache[i], slot, pos, rows, plan)
+            L.stream_add_norm(y, l.gain1, eps, hbuf, x, rows)
+            if l.mlp is not None:
+                l.mlp.forward(self, x, y, rows)
+                L.stream_add_norm(y, l.gain2, eps, hbuf, x, rows)
+        return hbuf
+
+    def _forward_stack_torch(self, h, slot, pos) -> torch.Tensor:
+        def join(x, y, gain):
+            return x + y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + self.cfg.norm_eps) * gain
+
+        x = h.float()
+        for i, l in enumerate(self.layers):
+            x = join(x, l.mixer.forward_torch(self, x, self.k_cache[i], slot, pos), l.gain1)
+            if l.mlp is not None:
+                x = join(x, l.mlp.forward_torch(x), l.gain2)
+        return x
+
+    # ------------------------------------------------------------------------- head
+    def _normed(self, h, rows: int, a_rows=None) -> torch.Tensor:
+        """Final norm of the selected rows -> the head projection's input."""
+        from ..ops import latent as L
+        src = h[:rows] if a_rows is None else h.index_select(0, a_rows.long())
+        xn = self.buf_x[:rows] if rows <= self.buf_x.shape[0] else torch.zeros(
+            (rows, self.width_p), dtype=self.dtype, device=self.device)
+        L.stream_norm(src, self.final_norm, self.cfg.norm_eps, xn, rows)
+        return xn
+
+    def head_gemv(self, h: torch.Tensor, rows: int, keys: torch.Tensor, a_rows=None) -> None:
+        from ..ops import latent as L
+        xn = self._normed(h, rows, a_rows)
+        if self.dtype == torch.float32:
+            lg = torch.empty((rows, self.lm_head.n), dtype=torch.float32, device=self.device)
+            self.lm_head(xn, rows, lg)
+            L.logits_argmax(lg, rows, self.head_vocab, keys, offset=self.head_v0)
+            return
+        self.lm_head(xn, rows, None, ws=self.coop_ws, sk_ws=self.sk_ws, keys=keys, bias=self.head_bias,
+                     col_offset=self.head_v0)
+
+    def logits(self, h: torch.Tensor, rows_idx=None) -> torch.Tensor:
+        if not self.gpu:
+            return super().logits(h, rows_idx)
+        idx = None if rows_idx is None else self._i32(rows_idx)
+        rows = h.shape[0] if idx is None else idx.numel()
+        lg = torch.empty((rows, self.lm_head.n), dtype=torch.float32, device=self.device)
+        self.lm_head(self._normed(h, rows, idx), rows, lg, ws=self.coop_ws, sk_ws=self.sk_ws)
+        return lg[:, :self.head_vocab]
+
+    def logits_torch(self, hs: torch.Tensor) -> torch.Tensor:
+        x = hs.float()
+        x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + self.cfg.norm_eps) * self.final_norm
+        lg = F.linear(x, self.lm_head.float())
+        return lg if self.head_bias is None else lg + self.head_bias
+
+
+__all__ = ["StackEngine"]

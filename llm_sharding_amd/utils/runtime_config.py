@@ -16,8 +16,8 @@ BACKENDS = ("tcp", "rccl", "local")
 
 
 # Every LSA_* switch in the package, kernels and entry points, in one place.
-# kind: "env" (read at run time) or "define" (a -D compile flag of csrc/kernels, never set by
-# csrc/build.py: only probe builds under probe_bin/ use them). role: "product" (changes what a
+# kind: "env" (read at run time) or "define" (a -D compile flag of csrc/kernels; except for
+# LSA_COOP_UNIT only probe builds under probe_bin/ set them). role: "product" (changes what a
 # deployment runs or how it reports), "diagnostic" (A/B and ablation switches; the default is the
 # shipped behaviour, measured in the profile named), "test" (test harness only).
 # tests/test_runtime_config.py::test_every_lsa_knob_is_listed keeps this table complete.
@@ -53,6 +53,7 @@ KNOBS = {
     "LSA_COOP_ABLATE": ("define", "diagnostic", "0", "coop GEMV ablation builds"),
     "LSA_GEMM_SK_TUNING": ("env", "diagnostic", "", "path of a gemm_sk tuning table to use instead of ops/gemm_sk_tuning.json (A/B runs)"),
     "LSA_GEMV_TUNING": ("env", "diagnostic", "", "path of a decode-GEMV tuning table to use instead of ops/gemv_tuning.json (A/B runs)"),
+    "LSA_COOP_UNIT": ("define", "product", "", "which part of gemv_coop.hip an object holds (set by csrc/build.py: parallel compilation)"),
     "LSA_STREAM_ABLATE": ("define", "diagnostic", "0", "gemv_stream probe ablation builds (scripts/probes/build_gemv_stream.sh)"),
     "LSA_GEMM_STAMPS": ("define", "diagnostic", "", "gemm_sk per-phase s_memrealtime stamps"),
     "LSA_COOP_STAMPS": ("define", "diagnostic", "", "coop GEMV per-phase stamps"),
@@ -81,6 +82,7 @@ class RuntimeConfig:
     streams: int = 1              # one GPU: micro-batches on this many concurrent HIP streams
     max_seq: int = 2048
     prefill_budget: int = 2048    # prompt tokens per prefill command (longer prompts are chunked)
+    cache_tokens: int = 0         # paged caches: tokens over all slots (0 = every slot's max_seq)
     max_new_tokens: int = 128
     use_graph: bool = True        # hipGraph-captured decode
     causal: bool = True           # False = the reference's unmasked prefill
@@ -129,20 +131,25 @@ class RuntimeConfig:
             return torch.device(self.device)
         return torch.device("cuda", local_rank) if torch.cuda.is_available() else torch.device("cpu")
 
-    def torch_dtype(self, device: Optional[torch.device] = None) -> torch.dtype:
-        if device is not None and device.type == "cuda":
-            return torch.bfloat16  # the HIP path computes in bf16
-        return getattr(torch, self.dtype)
+    def torch_dtype(self, device: Optional[torch.device] = None, cfg=None) -> torch.dtype:
+        """The compute type: on a GPU one the model's HIP path has (bfloat16 unless ``cfg`` says so)."""
+        want = getattr(torch, self.dtype)
+        if device is None or device.type != "cuda":
+            return want
+        if cfg is None:
+            return torch.bfloat16
+        from ..runtime.registry import compute_dtype
+        return compute_dtype(cfg, device, want)
 
     def model_and_source(self):
-        """(LlamaConfig, WeightSource) for the shards folder or the random-init preset."""
-        from ..config import LlamaConfig, get_preset
-        from ..runtime.engine import RandomSource, ShardFolderSource
+        """(model configuration, WeightSource) for the shards folder or the random-init preset."""
+        from ..config import get_preset
+        from ..runtime.registry import folder_source, load_config, random_source
         if self.shards:
-            cfg = LlamaConfig.from_pretrained(self.shards)
-            return cfg, ShardFolderSource(self.shards, cfg)
+            cfg = load_config(self.shards)
+            return cfg, folder_source(self.shards, cfg)
         cfg = get_preset(self.model)
-        return cfg, RandomSource(cfg, self.seed)
+        return cfg, random_source(cfg, self.seed)
 
 
 __all__ = ["RuntimeConfig", "BACKENDS"]
