@@ -87,6 +87,15 @@ def parse():
                          "runs it in a fresh child and can restart it once, see --no-fallback)")
     ap.add_argument("--no-fallback", dest="fallback", action="store_false",
                     help="N > 1: do not restart with --transport ipc when the RCCL ring preflight fails")
+    ap.add_argument("--compare", default="",
+                    help="instead of the headline: prefill and decode throughput of Deretar stacks of these sizes "
+                         "(2k,4k,8k: layers like a 2048-wide model's, Llama-2-7B's, Llama-2-70B's; random weights) "
+                         "beside Llama layers of the same width, heads and ff")
+    ap.add_argument("--compare-points", default="prefill:1x2048,prefill:4x2048,decode:1,decode:16,decode:64,decode:128",
+                    help="prefill:SEQUENCESxTOKENS and decode:BATCH points of --compare")
+    ap.add_argument("--compare-models", default="deretar,llama", help="which of the two --compare runs")
+    ap.add_argument("--compare-context", type=int, default=1024, help="cached tokens per sequence of a decode point")
+    ap.add_argument("--compare-layers", type=int, default=8)
     return ap.parse_args()
 
 
@@ -337,6 +346,78 @@ def extra_runs(spec: str, a) -> dict:
     return out
 
 
+def compare_designs(a) -> list:
+    """--compare: one record per (size, point, design), printed as JSON lines."""
+    import dataclasses
+    import statistics
+
+    import torch
+
+    from llm_sharding_amd.config import LlamaConfig, get_preset
+    from llm_sharding_amd.runtime.engine import DecodeGraph
+    from llm_sharding_amd.runtime.registry import is_stack, make_engine, random_source
+    kv_heads = {"2k": 16, "4k": 32, "8k": 8}
+    dev, out = torch.device("cuda", 0), []
+
+    def timed(fn, n, warm=2):
+        ts = []
+        for i in range(warm + n):
+            e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+            e0.record()
+            fn()
+            e1.record()
+            e1.synchronize()
+            if i >= warm:
+                ts.append(e0.elapsed_time(e1))
+        return statistics.median(ts)
+
+    for size in [x.strip() for x in a.compare.split(",") if x.strip()]:
+        st = get_preset(f"deretar-{size}")
+        st = dataclasses.replace(st, layers=st.layers[:a.compare_layers])
+        m, ff = st.layers[0].mixer, st.layers[0].mlp.ff
+        ll = LlamaConfig(hidden_size=st.hidden_size, intermediate_size=ff, num_hidden_layers=a.compare_layers,
+                         num_attention_heads=m.heads, num_key_value_heads=kv_heads[size], head_dim=128,
+                         vocab_size=st.vocab_size, max_position_embeddings=1 << 15, name=f"llama-{size}")
+        for cfg in (st, ll):
+            kind = "deretar" if is_stack(cfg) else "llama"
+            if kind not in a.compare_models.split(","):
+                continue
+            for point in [x.strip() for x in a.compare_points.split(",") if x.strip()]:
+                what, arg = point.split(":")
+                n, ctx = (int(v) for v in arg.split("x")) if what == "prefill" else (int(arg), a.compare_context)
+                rows = n * ctx if what == "prefill" else max(n, 128)
+                eng = make_engine(cfg, 0, a.compare_layers, dev, torch.bfloat16, has_embed=True, has_head=True,
+                                  source=random_source(cfg, a.seed), max_slots=n, max_seq=ctx + 128,
+                                  max_prefill_rows=rows)
+                if what == "prefill":
+                    ids = torch.randint(3, cfg.vocab_size, (n * ctx,), dtype=torch.int32).to(dev)
+
+                    def run():
+                        eng.reset()
+                        sl, po = eng.prefill_rows(list(range(n)), [ctx] * n)
+                        eng.head(eng.forward(eng.embed(ids), sl, po), [i * ctx + ctx - 1 for i in range(n)])
+                    ms, tokens = timed(run, 5), n * ctx
+                else:
+                    for s in range(n):
+                        eng.prefill_rows([s], [ctx])
+                        eng.seq_len[s] = ctx
+                    for c in eng.k_cache + eng.v_cache:
+                        c.normal_()
+                    g = DecodeGraph(eng, n, "full").capture()
+                    ms, tokens = timed(g.replay, 24, warm=4), n
+                rec = {"size": size, "design": kind, "point": point, "context": ctx, "layers": a.compare_layers,
+                       "ms": round(ms, 4), "tok_s": round(tokens / ms * 1e3, 1),
+                       "ms_per_layer": round(ms / a.compare_layers, 5),
+                       "layer_mb": round(cfg.layer_bytes() / 1e6, 1),
+                       "cache_bytes_per_token_layer": cfg.kv_bytes_per_token_per_layer()}
+                print(json.dumps(rec), flush=True)
+                out.append(rec)
+                g = None
+                del eng
+                torch.cuda.empty_cache()
+    return out
+
+
 def main():
     _die_with_parent()  # a child of spawn_ranks / supervise: die with that parent
     a = parse()
@@ -347,6 +428,9 @@ def main():
         raise SystemExit(spawn_ranks(a.gpus))
     if world > 1 and os.environ.get("LSA_BENCH_ROLE") != "worker" and a.supervise:
         raise SystemExit(supervise(a, sys.argv[1:]))
+    if a.compare:
+        compare_designs(a)
+        return
     if a.trace:
         os.environ["LSA_TRACE"] = a.trace
     from llm_sharding_amd.parallel.pipeline import run_decode_benchmark

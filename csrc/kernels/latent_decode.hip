@@ -1,0 +1,356 @@
+// Latent attention in the absorbed form on MFMA (latent.h): decode rows and short portions, bf16.
+//
+//   lsa_latent_absorb_mfma  q~^T[latent][row] = W_uk^h^T . q_h^T per head; rotated part behind it
+//   lsa_latent_attend_mfma  one workgroup per (row, group of HT x 16 heads, split): every cached
+//       entry is read from memory ONCE for all heads of the group and once from LDS per use:
+//       * a 64-token page arrives by LDS-DMA into a double buffer (the next page is in flight
+//         while this one is computed), chunk-swizzled on the source address
+//       * S^T[key][head] = C . q~^T: the four waves take 16 keys each (A = page rows by ds_read_b128,
+//         B = the group's queries, in registers for the whole launch)
+//       * softmax: column maxima meet in LDS, every lane then works on its own keys in fp32
+//       * O^T[latent][head] += C^T . P^T: the waves take a quarter of the latent each, C^T by the
+//         hardware-transposed LDS read of the same page image, P^T (bf16) through LDS
+//   lsa_latent_value_mfma   merge of the splits, then W_uv^h per head, output gate in the epilogue
+#include "latent.h"
+
+namespace {
+
+typedef short v4s_t __attribute__((ext_vector_type(4)));
+
+// chunk swizzle of row r in a page image of NCH 16-B chunks per row: both the 16-lane ds_read_b128
+// groups (rows l16) and the transposed reads hit distinct bank slots. NCH = 8 (mod 16): odd rows
+// start half a bank row later, so (r >> 1) & 7 completes the sixteen slots.
+template <int NCH>
+LSA_DEVICE int swz(int r) {
+  if constexpr (NCH % 16 == 0) return ((r & 3) << 2) ^ (((r >> 2) & 3) << 1);
+  else return (r >> 1) & 7;
+}
+
+LSA_DEVICE void glds16(const void* src, unsigned char* lds_base) {
+  __builtin_amdgcn_global_load_lds(src, (__attribute__((address_space(3))) void*)lds_base, 16, 0, 0);
+}
+
+constexpr int RP = 64;   // rotated part of a cache entry
+constexpr int NW = 4;    // waves
+
+template <int KRP, int HT>
+__global__ __launch_bounds__(NW * 64, 1) void attend_mfma_kernel(LatentArgs a, const bf16_raw* __restrict__ qt, int ns,
+                                                                 float* __restrict__ po, float* __restrict__ pm) {
+  constexpr int CW = KRP + RP, NCH = CW / 8, KF = CW / 32, DTW = KRP / 16 / NW;
+  constexpr int BLK = LAT_PAGE * CW * 2, PPW = BLK / 1024 / NW;
+  static_assert(PPW * NW * 1024 == BLK && DTW >= 1, "geometry");
+  __shared__ __attribute__((aligned(16))) unsigned char smem[2 * BLK];
+  __shared__ __attribute__((aligned(16))) unsigned char spt[HT * 2 * 64 * 16];  // P^T fragments
+  __shared__ float smax[NW][HT * 16];
+
+  const int e = blockIdx.x, h0 = blockIdx.y * (HT * 16), sp = blockIdx.z;
+  const int row = a.index ? a.index[e] : e;
+  const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l16 = lane & 15;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int slot = a.slot[row];
+  const int len = __builtin_amdgcn_readfirstlane(lat_keys(a, row));
+  const int nb = (len + LAT_PAGE - 1) / LAT_PAGE, b0 = nb * sp / ns, b1 = nb * (sp + 1) / ns;
+  const bf16_raw* cache = static_cast<const bf16_raw*>(a.cache);
+  const float sl2 = a.scale * 1.4426950408889634f;
+
+  u32x4_t qf[HT][KF];
+#pragma unroll
+  for (int t = 0; t < HT; ++t) {
+    const int h = h0 + t * 16 + l16;
+    const bf16_raw* q = qt + ((size_t)e * a.heads + (h < a.heads ? h : 0)) * CW;
+#pragma unroll
+    for (int kf = 0; kf < KF; ++kf) qf[t][kf] = h < a.heads ? ld16(q + kf * 32 + g * 8) : u32x4_t{0u, 0u, 0u, 0u};
+  }
+
+  auto stage = [&](int page, int buf) {
+    const bf16_raw* src = cache + (size_t)page * LAT_PAGE * CW;
+#pragma unroll
+    for (int s = 0; s < PPW; ++s) {
+      const int pc = w * PPW + s, lin = pc * 64 + lane, r = lin / NCH, c = lin % NCH;
+      glds16(src + (size_t)r * CW + (c ^ swz<NCH>(r)) * 8, smem + buf * BLK + pc * 1024);
+    }
+  };
+
+  f32x4_t o[HT][DTW];
+  float m_run[HT], l_run[HT];
+#pragma unroll
+  for (int t = 0; t < HT; ++t) {
+    m_run[t] = -INFINITY;
+    l_run[t] = 0.f;
+#pragma unroll
+    for (int d = 0; d < DTW; ++d) o[t][d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  }
+  // per-lane offsets into a page image: key row 16 w + l16 (its swizzle depends on l16 alone), and
+  // the transposed reads' row 4 g + l16 / 4 (+ 16, + 32: same swizzle)
+  const int krow = (w * 16 + l16) * (CW * 2), ksw = swz<NCH>(l16);
+  const int vlo = 4 * g + (l16 >> 2), vrow = vlo * (CW * 2), vsw = swz<NCH>(vlo);
+
+  int page_next = 0;
+  if (b0 < b1) {
+    stage(lat_page(a, slot, b0), 0);
+    page_next = b0 + 1 < b1 ? lat_page(a, slot, b0 + 1) : 0;
+  }
+  for (int b = b0; b < b1; ++b) {
+    const unsigned char* img = smem + ((b - b0) & 1) * BLK;
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's part of page b has landed
+    __syncthreads();  // every wave's, and every wave is done with the other buffer and with spt
+    if (b + 1 < b1) {
+      stage(page_next, (b + 1 - b0) & 1);
+      page_next = b + 2 < b1 ? lat_page(a, slot, b + 2) : 0;
+    }
+
+    f32x4_t s[HT], s2[HT];
+#pragma unroll
+    for (int t = 0; t < HT; ++t) s[t] = s2[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int kf = 0; kf < KF; ++kf) {
+      const u32x4_t k = *reinterpret_cast<const u32x4_t*>(img + krow + (((kf * 4 + g) ^ ksw) << 4));
+#pragma unroll
+      for (int t = 0; t < HT; ++t) {
+        if (HT <= 2 && (kf & 1)) s2[t] = mfma16(k, qf[t][kf], s2[t]);  // two chains where one would stall
+        else s[t] = mfma16(k, qf[t][kf], s[t]);
+      }
+    }
+    float mx[HT];
+#pragma unroll
+    for (int t = 0; t < HT; ++t) {
+      mx[t] = -INFINITY;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = b * LAT_PAGE + w * 16 + g * 4 + r;
+        const float v = key < len ? (s[t][r] + s2[t][r]) * sl2 : -INFINITY;
+        s[t][r] = v;
+        mx[t] = fmaxf(mx[t], v);
+      }
+      mx[t] = fmaxf(mx[t], __shfl_xor(mx[t], 16, 64));
+      mx[t] = fmaxf(mx[t], __shfl_xor(mx[t], 32, 64));
+      if (g == 0) smax[w][t * 16 + l16] = mx[t];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < HT; ++t) {
+      const int c = t * 16 + l16;
+      // page b holds at least one visible key, so the new maximum is finite
+      const float mn = fmaxf(m_run[t], fmaxf(fmaxf(smax[0][c], smax[1][c]), fmaxf(smax[2][c], smax[3][c])));
+      const float alpha = __builtin_amdgcn_exp2f(m_run[t] - mn);
+      float ps = 0.f;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        s[t][r] = __builtin_amdgcn_exp2f(s[t][r] - mn);
+        ps += s[t][r];
+      }
+      l_run[t] = l_run[t] * alpha + ps;  // this lane's keys; summed at the end
+      if (__builtin_amdgcn_ballot_w64(mn != m_run[t])) {
+#pragma unroll
+        for (int d = 0; d < DTW; ++d) o[t][d] *= alpha;
+      }
+      m_run[t] = mn;
+      // fragment f2 = w / 2 of the 32-key PV step, this wave's half of its eight keys per lane
+      st4(reinterpret_cast<bf16_raw*>(spt + (((t * 2 + (w >> 1)) * 64 + lane) << 4) + ((w & 1) << 3)), s[t]);
+    }
+    __syncthreads();
+#pragma unroll
+    for (int f2 = 0; f2 < 2; ++f2) {
+      u32x4_t p[HT];
+#pragma unroll
+      for (int t = 0; t < HT; ++t) p[t] = *reinterpret_cast<const u32x4_t*>(spt + (((t * 2 + f2) * 64 + lane) << 4));
+#pragma unroll
+      for (int d = 0; d < DTW; ++d) {
+        const int dt = w * DTW + d;
+        const unsigned char* v = img + f2 * 32 * (CW * 2) + vrow + (((2 * dt + ((l16 & 3) >> 1)) ^ vsw) << 4) + 8 * (l16 & 1);
+        const v4s_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s_t*)v);
+        const v4s_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+            (__attribute__((address_space(3))) v4s_t*)(v + 16 * (CW * 2)));
+        u32x4_t c;
+        c[0] = __builtin_bit_cast(u32x2_t, lo)[0];
+        c[1] = __builtin_bit_cast(u32x2_t, lo)[1];
+        c[2] = __builtin_bit_cast(u32x2_t, hi)[0];
+        c[3] = __builtin_bit_cast(u32x2_t, hi)[1];
+#pragma unroll
+        for (int t = 0; t < HT; ++t) o[t][d] = mfma16(c, p[t], o[t][d]);
+      }
+    }
+  }
+
+  __syncthreads();  // the last page's maxima have been read
+#pragma unroll
+  for (int t = 0; t < HT; ++t) {
+    l_run[t] += __shfl_xor(l_run[t], 16, 64);
+    l_run[t] += __shfl_xor(l_run[t], 32, 64);
+    if (g == 0) smax[w][t * 16 + l16] = l_run[t];
+  }
+  __syncthreads();
+#pragma unroll
+  for (int t = 0; t < HT; ++t) {
+    const int h = h0 + t * 16 + l16;
+    if (h >= a.heads) continue;
+    const size_t out = ((size_t)e * a.heads + h) * ns + sp;
+#pragma unroll
+    for (int d = 0; d < DTW; ++d)
+      *reinterpret_cast<f32x4_t*>(po + out * KRP + (w * DTW + d) * 16 + 4 * g) = o[t][d];
+    if (w == 0 && g == 0) {
+      const int c = t * 16 + l16;
+      pm[out * 2] = m_run[t];
+      pm[out * 2 + 1] = smax[0][c] + smax[1][c] + smax[2][c] + smax[3][c];
+    }
+  }
+}
+
+// wk: per head the packed [krp][dkp] matrix (common.h fragment order). Grid (16-entry tiles, heads,
+// 16-tile stretches of the latent); every wave up to 4 latent tiles.
+__global__ __launch_bounds__(256) void absorb_mfma_kernel(LatentArgs a, int n, const bf16_raw* __restrict__ q, int ldq,
+                                                          const bf16_raw* __restrict__ wk, bf16_raw* __restrict__ qt) {
+  const int h = blockIdx.y, e0 = blockIdx.x * 16;
+  const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l16 = lane & 15, w = tid >> 6;
+  const int kf_n = a.dkp / 32, nt_n = a.krp / 16, cw = a.krp + a.rp;
+  const int e = e0 + l16;
+  const bool ok = e < n;
+  const int row = ok ? (a.index ? a.index[e] : e) : 0;
+  const bf16_raw* qh = q + (size_t)row * ldq + (size_t)h * (a.dkp + a.rp);
+  const int t0 = blockIdx.z * 16 + w * 4;
+  const bf16_raw* wh = wk + ((size_t)h * nt_n + t0) * kf_n * 512;
+  f32x4_t acc[4];
+#pragma unroll
+  for (int t = 0; t < 4; ++t) acc[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int kf = 0; kf < kf_n; ++kf) {
+    const u32x4_t b = ok ? ld16(qh + kf * 32 + g * 8) : u32x4_t{0u, 0u, 0u, 0u};
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+      if (t0 + t < nt_n) acc[t] = mfma16(ld16(wh + ((size_t)t * kf_n + kf) * 512 + lane * 8), b, acc[t]);
+  }
+  if (ok) {
+    bf16_raw* o = qt + ((size_t)e * a.heads + h) * cw;
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+      if (t0 + t < nt_n) st4(o + (t0 + t) * 16 + 4 * g, acc[t]);
+  }
+  if (blockIdx.z == 0) {
+    for (int i = tid; i < 16 * a.rp; i += 256) {
+      const int ee = e0 + i / a.rp, j = i % a.rp;
+      if (ee >= n) break;
+      const int rr = a.index ? a.index[ee] : ee;
+      const bf16_raw* qr = q + (size_t)rr * ldq + (size_t)h * (a.dkp + a.rp) + a.dkp;
+      const bool live = j < a.rot_dim && lat_keys(a, rr) > 0;
+      st1(qt + ((size_t)ee * a.heads + h) * cw + a.krp + j, live ? lat_rot(a, qr, j, a.pos[rr]) : 0.f);
+    }
+  }
+}
+
+// wv: per head the packed [dvp][krp] matrix. Grid (16-entry tiles, heads, 4-tile stretches of the
+// value); one 16-wide value tile per wave.
+template <int KRP>
+__global__ __launch_bounds__(256) void value_mfma_kernel(LatentArgs a, int n, const float* __restrict__ po,
+                                                         const float* __restrict__ pm, int ns,
+                                                         const bf16_raw* __restrict__ wv, const bf16_raw* __restrict__ gate,
+                                                         int ldg, bf16_raw* __restrict__ out, int ldo) {
+  constexpr int KF = KRP / 32, LD = KRP + 8;
+  __shared__ __attribute__((aligned(16))) bf16_raw so[16 * LD];
+  __shared__ float wgt[16][64];
+  const int h = blockIdx.y, e0 = blockIdx.x * 16;
+  const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l16 = lane & 15, w = tid >> 6;
+  if (tid < 16) {
+    const int e = e0 + tid;
+    if (e < n) {
+      const float* p = pm + ((size_t)e * a.heads + h) * ns * 2;
+      float M = -INFINITY, L = 0.f;
+      for (int s = 0; s < ns; ++s) M = fmaxf(M, p[2 * s]);
+      if (M == -INFINITY) M = 0.f;
+      for (int s = 0; s < ns; ++s) {
+        const float f = __builtin_amdgcn_exp2f(p[2 * s] - M);
+        wgt[tid][s] = f;
+        L += p[2 * s + 1] * f;
+      }
+      const float inv = L > 0.f ? 1.f / L : 0.f;
+      for (int s = 0; s < ns; ++s) wgt[tid][s] *= inv;
+    }
+  }
+  __syncthreads();
+  for (int i = tid; i < 16 * (KRP / 4); i += 256) {
+    const int r = i / (KRP / 4), c = (i % (KRP / 4)) * 4, e = e0 + r;
+    f32x4_t v = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    if (e < n) {
+      const float* p = po + ((size_t)e * a.heads + h) * ns * KRP + c;
+      for (int s = 0; s < ns; ++s) v += *reinterpret_cast<const f32x4_t*>(p + (size_t)s * KRP) * wgt[r][s];
+    }
+    st4(so + r * LD + c, v);
+  }
+  __syncthreads();
+  const int t = blockIdx.z * NW + w, e = e0 + l16;
+  if (t * 16 >= a.dvp) return;
+  const bf16_raw* wh = wv + ((size_t)h * (a.dvp / 16) + t) * KF * 512;
+  f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int kf = 0; kf < KF; ++kf)
+    acc = mfma16(ld16(wh + (size_t)kf * 512 + lane * 8), ld16(so + l16 * LD + kf * 32 + g * 8), acc);
+  if (e >= n) return;
+  const int row = a.index ? a.index[e] : e, col = h * a.dvp + t * 16 + 4 * g;
+  if (gate) {
+    const bf16_raw* gp = gate + (size_t)row * ldg + col;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) acc[r] *= sigmoid(bf2f(gp[r]));
+  }
+  st4(out + (size_t)row * ldo + col, acc);
+}
+
+bool size_ok(const LatentArgs* a, int n) {
+  return a && n >= 1 && a->cache && a->table && a->slot && a->pos && a->max_pages >= 1 && a->n_pages >= 1 && a->heads >= 1 &&
+         a->dim >= 1 && a->dim <= a->dkp && a->dkp % 64 == 0 && a->rp == RP && a->rot_dim >= 2 && a->rot_dim <= RP &&
+         a->rot_dims >= 2 && a->rot_dims % 2 == 0 && a->rot_dims <= a->rot_dim && a->vdim >= 1 && a->vdim <= a->dvp &&
+         a->dvp % 64 == 0 && a->kv_rank >= 1 && a->kv_rank <= a->krp && a->cos_t && a->sin_t &&
+         (a->krp == 64 || a->krp == 128 || a->krp == 256 || a->krp == 512);
+}
+
+}  // namespace
+
+extern "C" int lsa_latent_absorb_mfma(const LatentArgs* a, int n, const void* q, int ldq, const void* wk, void* qt,
+                                      hipStream_t s) {
+  if (!size_ok(a, n) || ldq < a->heads * (a->dkp + a->rp) || ldq % 8 || (uintptr_t)q % 16 || (uintptr_t)qt % 16)
+    return LSA_BAD_SHAPE;
+  dim3 grid((n + 15) / 16, a->heads, (a->krp / 16 + 15) / 16);
+  absorb_mfma_kernel<<<grid, 256, 0, s>>>(*a, n, (const bf16_raw*)q, ldq, (const bf16_raw*)wk, (bf16_raw*)qt);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+extern "C" int lsa_latent_attend_mfma(const LatentArgs* a, int n, const void* qt, int ns, float* po, float* pm,
+                                      hipStream_t s) {
+  if (!size_ok(a, n) || ns < 1 || ns > 64 || (uintptr_t)qt % 16 || (uintptr_t)po % 16) return LSA_BAD_SHAPE;
+  // head tiles per workgroup; four tiles of 512-wide latents do not fit the register file
+  const int tiles = (a->heads + 15) / 16, ht = tiles >= 3 ? (a->krp == 512 ? 2 : 4) : tiles;
+  dim3 grid(n, (tiles + ht - 1) / ht, ns);
+#define LSA_A(K, T) attend_mfma_kernel<K, T><<<grid, NW * 64, 0, s>>>(*a, (const bf16_raw*)qt, ns, po, pm)
+#define LSA_K(K)                                 \
+  if (ht == 1) LSA_A(K, 1);                      \
+  else if (ht == 2) LSA_A(K, 2);                 \
+  else if constexpr (K < 512) LSA_A(K, 4);
+  switch (a->krp) {
+    case 64: LSA_K(64) break;
+    case 128: LSA_K(128) break;
+    case 256: LSA_K(256) break;
+    case 512: LSA_K(512) break;
+    default: return LSA_UNSUPPORTED;
+  }
+#undef LSA_K
+#undef LSA_A
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+extern "C" int lsa_latent_value_mfma(const LatentArgs* a, int n, const float* po, const float* pm, int ns, const void* wv,
+                                     const void* gate, int ldg, void* out, int ldo, hipStream_t s) {
+  if (!size_ok(a, n) || ns < 1 || ns > 64 || ldo < a->heads * a->dvp || ldo % 4 || (uintptr_t)out % 8 || (uintptr_t)po % 16)
+    return LSA_BAD_SHAPE;
+  dim3 grid((n + 15) / 16, a->heads, a->dvp / 64);
+#define LSA_V(K)                                                                                                       \
+  case K:                                                                                                              \
+    value_mfma_kernel<K><<<grid, 256, 0, s>>>(*a, n, po, pm, ns, (const bf16_raw*)wv, (const bf16_raw*)gate, ldg,      \
+                                              (bf16_raw*)out, ldo);                                                    \
+    break;
+  switch (a->krp) {
+    LSA_V(64) LSA_V(128) LSA_V(256) LSA_V(512)
+    default: return LSA_UNSUPPORTED;
+  }
+#undef LSA_V
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}

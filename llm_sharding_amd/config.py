@@ -229,7 +229,23 @@ def tiny_gpt2(layers: int = 4, hidden: int = 256, heads: int = 4, vocab: int = 5
                        bos_token_id=vocab - 1, eos_token_id=vocab - 1, model_type="gpt2", name="tiny-gpt2")
 
 
+def _deretar(width: int, heads: int, ff: int, layers: int, vocab: int, kv_rank: int, q_rank: int, dim: int = 128,
+             rot: int = 64, vdim: int = 128, max_pos: int = 1 << 17, name: str = "deretar"):
+    """A Deretar stack of equal layers (random-init presets)."""
+    from .models.deretar import layer_entry, make_config
+    cfg = make_config(width, vocab, [layer_entry(heads, dim, rot, vdim, kv_rank, q_rank, ff) for _ in range(layers)],
+                      name=name)
+    cfg.max_position_embeddings = max_pos
+    return cfg
+
+
 PRESETS = {
+    # Deretar with the layer sizes of Llama-2-7B / a 2048-wide model / Llama-2-70B
+    "deretar-4k": lambda: _deretar(4096, 32, 11008, 32, 32000, 512, 1536, name="deretar-4k"),
+    "deretar-2k": lambda: _deretar(2048, 16, 8192, 24, 32000, 256, 768, name="deretar-2k"),
+    "deretar-8k": lambda: _deretar(8192, 64, 28672, 80, 32000, 512, 1536, name="deretar-8k"),
+    "tiny-deretar": lambda: _deretar(160, 5, 208, 4, 330, 56, 88, dim=24, rot=16, vdim=40, max_pos=1024,
+                                     name="tiny-deretar"),
     "llama2-7b": llama2_7b,
     "llama2-13b": llama2_13b,
     "llama2-70b": llama2_70b,

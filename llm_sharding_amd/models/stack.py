@@ -160,9 +160,9 @@ class StackConfig:
         inter = part = 0
         for l in self.layers:
             m = l.mixer
-            inter = max(inter, m.q_rank * 2 + m.kv_rank + m.rot_dim + m.heads * (2 * m.dvp + m.dkp + m.rp + m.cache_width)
+            inter = max(inter, m.q_rank * 2 + m.kv_rank + m.rot_dim + m.heads * (2 * m.dvp + m.dkp + m.rp)
                         + (l.mlp.ff if l.mlp is not None else 0) + 5 * 128)
-            part = max(part, max(rows, 1024) * m.heads * (m.krp + 2) * 4)
+            part = max(part, 1024 * m.heads * ((m.krp + 2) * 4 + m.cache_width * elem_bytes))
         return n + rows * inter * elem_bytes + part + (1 << 26) + 2 * 256 * 256 * 256 * 4
 
     def stream_bytes(self) -> int:

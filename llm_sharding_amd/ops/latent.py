@@ -126,11 +126,26 @@ def logits_argmax(lg, rows: int, vocab: int, keys, offset: int = 0) -> None:
 
 # ------------------------------------------------------------------------------ latent attention
 def tuned_size(s) -> bool:
-    return False
+    """The MFMA kernels of the absorbed form take this size (others run the plain kernels)."""
+    return s.krp in (64, 128, 256, 512) and s.rp == 64
 
 
 def expand_size(s) -> bool:
-    return False
+    """The MFMA kernel of the expanded form takes this size."""
+    return s.rp == 64 and s.dkp in (64, 128) and s.dvp in (64, 128)
+
+
+def pack_heads(w: torch.Tensor) -> torch.Tensor:
+    """Per-head matrices [H, N, K] (N % 16, K % 32) in MFMA fragment order, head after head."""
+    return pack_b(w.reshape(-1, w.shape[2])).contiguous()
+
+
+def prefill_tile_rows(rows: int, heads: int) -> int:
+    """Query rows per tile of the expanded form: 128, halved while the chip would idle."""
+    t = 128
+    while t > 16 and -(-rows // t) * heads < hip.N_CU:
+        t //= 2
+    return t
 
 
 def make_args(spec, cache, table, slot, pos, cos, sin, eps: float, index=None) -> LatentArgs:
@@ -183,6 +198,68 @@ def value(a: LatentArgs, n: int, po, pm, ns: int, wv, gate, out) -> None:
            "lsa_latent_value")
 
 
+def absorb_mfma(a: LatentArgs, n: int, q, wk, qt) -> None:
+    """As :func:`absorb` in bf16; ``wk``: pack_heads of [heads, krp, dkp]."""
+    _req(q.dtype == wk.dtype == qt.dtype == torch.bfloat16 and wk.numel() == a.heads * a.dkp * a.krp
+         and qt.numel() >= n * a.heads * (a.krp + a.rp) and qt.is_contiguous(), "absorb_mfma: shapes")
+    _check(lib().lsa_latent_absorb_mfma(ctypes.byref(a), n, _p(q), q.stride(0), _p(wk), _p(qt), _stream()),
+           "lsa_latent_absorb_mfma")
+
+
+def attend_mfma(a: LatentArgs, n: int, qt, ns: int, po, pm) -> None:
+    e = n * a.heads * ns
+    _req(qt.dtype == torch.bfloat16 and qt.numel() >= n * a.heads * (a.krp + a.rp), "attend_mfma: query shape")
+    _req(po.dtype == pm.dtype == torch.float32 and po.numel() >= e * a.krp and pm.numel() >= 2 * e,
+         "attend_mfma: workspace")
+    _check(lib().lsa_latent_attend_mfma(ctypes.byref(a), n, _p(qt), ns, _p(po), _p(pm), _stream()),
+           "lsa_latent_attend_mfma")
+
+
+def value_mfma(a: LatentArgs, n: int, po, pm, ns: int, wv, gate, out) -> None:
+    """As :func:`value` in bf16; ``wv``: pack_heads of [heads, dvp, krp]."""
+    e = n * a.heads * ns
+    _req(po.numel() >= e * a.krp and pm.numel() >= 2 * e and wv.numel() == a.heads * a.krp * a.dvp
+         and out.shape[1] >= a.heads * a.dvp and wv.dtype == out.dtype == torch.bfloat16, "value_mfma: shapes")
+    _req(gate is None or (gate.dtype == out.dtype and gate.shape[1] >= a.heads * a.dvp), "value_mfma: gate")
+    _check(lib().lsa_latent_value_mfma(ctypes.byref(a), n, _p(po), _p(pm), ns, _p(wv), _p(gate),
+                                       0 if gate is None else gate.stride(0), _p(out), out.stride(0), _stream()),
+           "lsa_latent_value_mfma")
+
+
+def gather(a: LatentArgs, src, n: int, out) -> None:
+    """Cached entries of the (slot, position) pairs ``src`` int32 [n, 2] -> rows of ``out`` (bf16)."""
+    _req(src.dtype == torch.int32 and src.is_contiguous() and src.numel() >= 2 * n and out.dtype == torch.bfloat16
+         and out.shape[0] >= n and out.shape[1] == a.krp + a.rp and out.is_contiguous(), "gather: shapes")
+    _check(lib().lsa_latent_gather(ctypes.byref(a), _p(src), n, _p(out), _stream()), "lsa_latent_gather")
+
+
+_TILES_OK = None  # the last tile table prefill() validated: a forward checks its table once, not per layer
+
+
+def prefill(a: LatentArgs, tiles, tiles_host, q, kv, lat, gate, out, rows: int, tokens: int) -> None:
+    """Attention of the query tiles [row0, nrows, kv0, pos0, kvlen, 0, 0, 0] over expanded keys and
+    values ``kv`` [tokens, heads (dkp + dvp)] and the gathered entries ``lat`` [tokens, krp + rp]."""
+    _req(all(t.dtype == torch.bfloat16 for t in (q, kv, lat, out)) and tiles.dtype == torch.int32
+         and tiles.shape == tiles_host.shape and tiles.shape[1] == 8 and tiles.is_contiguous(), "prefill: types")
+    _req(min(q.shape[0], out.shape[0]) >= rows and out.shape[1] >= a.heads * a.dvp
+         and min(kv.shape[0], lat.shape[0]) >= tokens and kv.shape[1] >= a.heads * (a.dkp + a.dvp)
+         and lat.shape[1] == a.krp + a.rp and lat.is_contiguous(), "prefill: shapes")
+    _req(gate is None or (gate.dtype == torch.bfloat16 and gate.shape[0] >= rows
+                          and gate.shape[1] >= a.heads * a.dvp), "prefill: gate")
+    global _TILES_OK
+    key = (tiles.data_ptr(), rows, tokens, a.max_pages)
+    if not (_TILES_OK is not None and _TILES_OK[0] is tiles_host and _TILES_OK[1] == key):
+        r0, nr, k0, p0, kl = (tiles_host[:, i] for i in range(5))
+        _req(bool((nr >= 1).all() and (nr <= 128).all() and (r0 >= 0).all()) and int((r0 + nr).max()) <= rows,
+             "prefill: tile rows")
+        _req(bool((k0 >= 0).all() and (kl >= 1).all() and (p0 >= 0).all()) and int((k0 + kl).max()) <= tokens
+             and bool((p0 + nr <= kl).all()) and int(kl.max()) <= a.max_pages * PAGE, "prefill: tile keys")
+        _TILES_OK = (tiles_host, key)
+    _check(lib().lsa_latent_prefill(ctypes.byref(a), _p(tiles), tiles.shape[0], _p(q), q.stride(0), _p(kv), kv.stride(0),
+                                    _p(lat), _p(gate), 0 if gate is None else gate.stride(0), _p(out), out.stride(0),
+                                    _stream()), "lsa_latent_prefill")
+
+
 def declare(L: ctypes.CDLL) -> None:
     """Signatures of these entry points (called by hip.load_library)."""
     vp, i, f = ctypes.c_void_p, ctypes.c_int, ctypes.c_float
@@ -198,6 +275,10 @@ def declare(L: ctypes.CDLL) -> None:
         "lsa_latent_absorb": [i, la, i, vp, i, vp, vp, vp],
         "lsa_latent_attend": [i, la, i, vp, i, vp, vp, vp],
         "lsa_latent_value": [i, la, i, vp, vp, i, vp, vp, i, vp, i, vp],
+        "lsa_latent_absorb_mfma": [la, i, vp, i, vp, vp, vp],
+        "lsa_latent_attend_mfma": [la, i, vp, i, vp, vp, vp],
+        "lsa_latent_value_mfma": [la, i, vp, vp, i, vp, vp, i, vp, i, vp],
+        "lsa_latent_prefill": [la, vp, i, vp, i, vp, i, vp, vp, i, vp, i, vp],
         "lsa_latent_gather": [la, vp, i, vp, vp],
     }
     for name, args in sig.items():

@@ -29,7 +29,7 @@ import torch
 
 from ..config import get_preset
 from ..runtime.engine import DecodeGraph, EagerDecode, StageEngine
-from ..runtime.registry import compute_dtype, make_engine, random_source
+from ..runtime.registry import compute_dtype, is_stack, make_engine, random_source
 from ..utils import tracing
 from .scheduler import plan_stages, scratch_bytes, stage_memory
 
@@ -772,7 +772,10 @@ def run_decode_benchmark(model: str = "llama2-7b", n_gpus: int = 1, steps: int =
     cfg = get_preset(model)
     if stage_layers:
         import dataclasses
-        cfg = dataclasses.replace(cfg, num_hidden_layers=stage_layers)
+        if is_stack(cfg):
+            cfg = dataclasses.replace(cfg, layers=cfg.layers[:stage_layers])
+        else:
+            cfg = dataclasses.replace(cfg, num_hidden_layers=stage_layers)
     world = int(os.environ.get("WORLD_SIZE", "1"))
     rank = int(os.environ.get("RANK", "0"))
     if n_gpus != world:
@@ -835,7 +838,7 @@ def run_decode_benchmark(model: str = "llama2-7b", n_gpus: int = 1, steps: int =
     if ipc_only:
         from .ipc_ring import IpcRingP2P
         edges = [(r[i], r[(i + 1) % pp]) for r in rings for i in range(pp)]
-        p2p = IpcRingP2P(rank, slot_bytes=batch * cfg.hidden_size * 2, slots=min(64, max(2, M)),
+        p2p = IpcRingP2P(rank, slot_bytes=batch * (cfg.stream_bytes() if is_stack(cfg) else cfg.hidden_size * 2), slots=min(64, max(2, M)),
                          ranks=rings[replica], edges=edges)
     else:
         p2p = DistP2P(ranks=rings[replica], rings=rings)

@@ -102,20 +102,15 @@ class Weights:
         L.append(a, rows, inp, 0, self.ok, self.gq, self.gk, cq)
         eng.project(self.uq, cq, rows, q)
         gate = inp[:, self.og:]
-        if plan.n_absorbed(self):
-            idx = plan.absorbed_index(self)
-            n = plan.n_absorbed(self)
+        absorb, attend, value = ((L.absorb_mfma, L.attend_mfma, L.value_mfma) if self.tuned
+                                 else (L.absorb, L.attend, L.value))
+        for idx, n in plan.absorbed_chunks(self):
             b = a if idx is None else L.make_args(s, cache, table, slot, pos, cos, sin, eng.cfg.norm_eps, index=idx)
-            qt, po, pm, cap = eng.attend_scratch(s, n)
-            ns = max(1, min(plan.nsplit(eng, self), cap // n))
-            if self.tuned:
-                L.absorb_mfma(b, n, q, self.wk, qt)
-                L.attend_mfma(b, n, qt, ns, po, pm)
-                L.value_mfma(b, n, po, pm, ns, self.wv, gate, ao)
-            else:
-                L.absorb(b, n, q, self.wk, qt)
-                L.attend(b, n, qt, ns, po, pm)
-                L.value(b, n, po, pm, ns, self.wv, gate, ao)
+            qt, po, pm = eng.attend_scratch()
+            ns = max(1, min(plan.nsplit(eng, self), eng.ATTEND_ITEMS // n))
+            absorb(b, n, q, self.wk, qt)
+            attend(b, n, qt, ns, po, pm)
+            value(b, n, po, pm, ns, self.wv, gate, ao)
         for g in plan.expanded_groups(self):
             lat, kv = eng.expand_scratch(s, g.tokens, self.kv.n)
             L.gather(a, g.src, g.tokens, lat)
@@ -227,8 +222,16 @@ class Plan:
     def n_absorbed(self, w) -> int:
         return self._split(w)[0]
 
-    def absorbed_index(self, w):
-        return self._split(w)[1]
+    def absorbed_chunks(self, w) -> list:
+        """[(row indices or None for all rows, count)] of the absorbed form, at most
+        ``ATTEND_ITEMS`` at a time (its buffers)."""
+        n, idx, _ = self._split(w)
+        cap = self.eng.ATTEND_ITEMS
+        if idx is None and n <= cap:
+            return [(None, n)] if n else []
+        if idx is None:
+            idx = torch.arange(n, dtype=torch.int32, device=self.eng.device)
+        return [(idx[c:c + cap], min(cap, n - c)) for c in range(0, n, cap)]
 
     def expanded_groups(self, w) -> list:
         return self._split(w)[2]

@@ -188,12 +188,12 @@ class StackEngine(StageEngine):
                "flat": {k: torch.zeros(R * n, dtype=dt, device=dev) for k, n in self._widths.items() if n},
                "keys": torch.zeros(R, dtype=torch.int64, device=dev),
                "tokens": torch.zeros(R, dtype=torch.int32, device=dev), "_x_ready": False, "coop_ws": None, "sk_ws": None}
-        # absorbed attention: queries, and split partials of up to max(rows, ATTEND_ITEMS) (row, split)s
-        items = max(R, self.ATTEND_ITEMS)
+        # absorbed attention: queries and split partials of up to ATTEND_ITEMS (row, split) pairs at a time
+        items = self.ATTEND_ITEMS
         qn = max(l.spec.mixer.heads * l.spec.mixer.cache_width for l in self.layers)
         on = max(l.spec.mixer.heads * l.spec.mixer.krp for l in self.layers)
         hn = max(l.spec.mixer.heads for l in self.layers)
-        out["qt"] = torch.zeros(R * qn, dtype=dt, device=dev)
+        out["qt"] = torch.zeros(items * qn, dtype=dt, device=dev)
         out["part_o"] = torch.zeros(items * on, dtype=torch.float32, device=dev)
         out["part_ml"] = torch.zeros(items * hn * 2, dtype=torch.float32, device=dev)
         if dt == torch.bfloat16:
@@ -204,7 +204,7 @@ class StackEngine(StageEngine):
             out["sk_ws"] = hip.SkWorkspace(dev)
         return out
 
-    ATTEND_ITEMS = 1024  # (row, split) pairs the partial buffers hold at least
+    ATTEND_ITEMS = 1024  # (row, split) pairs of one absorbed-attention launch
 
     def decode_scratch(self, k: int, rows: Optional[int] = None) -> dict:
         if k == 0:
@@ -219,10 +219,9 @@ class StackEngine(StageEngine):
     def scratch_view(self, name: str, rows: int, n: int) -> torch.Tensor:
         return self.flat[name][:rows * n].view(rows, n)
 
-    def attend_scratch(self, s, n: int) -> tuple:
-        """(absorbed queries, partial sums, partial max / sum, (row, split) pairs they hold)."""
-        cap = min(self.part_o.numel() // (s.heads * s.krp), self.part_ml.numel() // (2 * s.heads))
-        return self.qt, self.part_o, self.part_ml, cap
+    def attend_scratch(self) -> tuple:
+        """(absorbed queries, partial sums, partial max / sum)."""
+        return self.qt, self.part_o, self.part_ml
 
     def expand_scratch(self, s, tokens: int, n: int) -> tuple:
         """Gathered latents and expanded keys / values (grown on demand: long portions run eagerly;

@@ -8,13 +8,13 @@ import socket
 import pytest
 import torch
 
-from llm_sharding_amd.config import tiny, tiny_gpt2
+from llm_sharding_amd.config import get_preset, tiny, tiny_gpt2
 from llm_sharding_amd.parallel.pipeline import run_pipeline_generate
 from llm_sharding_amd.parallel.scheduler import plan_stages
-from llm_sharding_amd.runtime.engine import RandomSource
+from llm_sharding_amd.runtime.registry import random_source
 
 M, B, P, NEW = 2, 2, 5, 6
-MODELS = {"llama": lambda: tiny(layers=5), "gpt2": lambda: tiny_gpt2(layers=5)}
+MODELS = {"llama": lambda: tiny(layers=5), "gpt2": lambda: tiny_gpt2(layers=5), "deretar": lambda: get_preset("tiny-deretar")}
 
 
 def _free_port() -> int:
@@ -36,7 +36,7 @@ def _worker(rank, world, port, q, model="llama"):
     dist.init_process_group("gloo", init_method=f"tcp://127.0.0.1:{port}", rank=rank, world_size=world)
     try:
         cfg = MODELS[model]()
-        out = run_pipeline_generate(cfg, RandomSource(cfg, seed=7), _prompts(cfg) if rank == 0 else None, NEW,
+        out = run_pipeline_generate(cfg, random_source(cfg, 7), _prompts(cfg) if rank == 0 else None, NEW,
                                     rank, world, batch=B, microbatches=M, max_seq=64)
         if rank == 0:
             q.put(out.tolist())
@@ -65,7 +65,7 @@ def _run_world(world, model="llama"):
 
 def _single(model):
     cfg = MODELS[model]()
-    out = run_pipeline_generate(cfg, RandomSource(cfg, seed=7), _prompts(cfg), NEW, 0, 1, batch=B,
+    out = run_pipeline_generate(cfg, random_source(cfg, 7), _prompts(cfg), NEW, 0, 1, batch=B,
                                 microbatches=M, max_seq=64)
     return out.tolist()
 
@@ -92,6 +92,13 @@ def test_gpt2_pipeline_matches_single():
     assert _run_world(2, "gpt2") == ref
 
 
+def test_stack_pipeline_matches_single():
+    """A Deretar stack (fp32 residual stream handed over, paged cache per stage) over 2 gloo ranks."""
+    ref = _single("deretar")
+    assert len(set(sum(sum(ref, []), []))) > 3
+    assert _run_world(2, "deretar") == ref
+
+
 def test_plan_covers_all_layers():
     cfg = tiny(layers=5)
     for n in (1, 2, 3, 5):
@@ -107,7 +114,7 @@ def test_local_multistage_matches_single(n_stages, single):
     """N stages in one process over the in-process device-copy transport (CPU)."""
     from llm_sharding_amd.parallel.pipeline import drive_local_pipeline
     cfg = tiny(layers=5)
-    out = drive_local_pipeline(cfg, RandomSource(cfg, seed=7), _prompts(cfg), NEW, n_stages, "cpu",
+    out = drive_local_pipeline(cfg, random_source(cfg, 7), _prompts(cfg), NEW, n_stages, "cpu",
                                batch=B, microbatches=M, max_seq=64, dtype=torch.float32)
     assert out.tolist() == single
 
