@@ -27,34 +27,91 @@ LSA_DEVICE float block_max(float v, float* part) {
   return fmaxf(fmaxf(part[0], part[1]), fmaxf(part[2], part[3]));
 }
 
-// in: row of the fused input projection, query latent at column oq, [key latent | rotated part] at ok
-template <typename T>
+// (a, b) summed over the 256 threads of a workgroup
+LSA_DEVICE void block_sum2(float& a, float& b, float (*part)[4]) {
+  a = wave_sum(a);
+  b = wave_sum(b);
+  if ((threadIdx.x & 63) == 0) {
+    part[0][threadIdx.x >> 6] = a;
+    part[1][threadIdx.x >> 6] = b;
+  }
+  __syncthreads();
+  a = part[0][0] + part[0][1] + part[0][2] + part[0][3];
+  b = part[1][0] + part[1][1] + part[1][2] + part[1][3];
+}
+
+LSA_DEVICE void ld8(const float* p, float* f) {
+#pragma unroll
+  for (int k = 0; k < 8; ++k) f[k] = p[k];
+}
+LSA_DEVICE void ld8(const bf16_raw* p, float* f) { unpack8(ld16(p), f); }
+LSA_DEVICE void st8(float* p, const float* f) {
+#pragma unroll
+  for (int k = 0; k < 8; ++k) p[k] = f[k];
+}
+LSA_DEVICE void st8(bf16_raw* p, const float* f) { st16(p, pack8(f)); }
+
+// in: row of the fused input projection, query latent at column oq, [key latent | rotated part] at
+// ok. VEC: 8 values at a time (ranks and offsets multiples of 8), the first of a thread's stretches
+// kept in registers between the sums and the scaling.
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void append_kernel(LatentArgs a, const T* __restrict__ in, int ldi, int oq, int ok,
                                                      const float* __restrict__ gq, const float* __restrict__ gk,
                                                      T* __restrict__ cq, int ldc) {
-  __shared__ float part[4];
+  __shared__ float part[2][4];
+  constexpr int S = VEC ? 8 : 1;
   const int row = blockIdx.x, tid = threadIdx.x;
   const T* q = in + (size_t)row * ldi + oq;
   const T* k = in + (size_t)row * ldi + ok;
-  float sq = 0.f, sk = 0.f;
-  for (int c = tid; c < a.q_rank; c += 256) {
-    const float v = ld1(q + c);
-    sq += v * v;
+  const int nq = a.q_rank / S, n = nq + a.kv_rank / S;  // stretches of both latents
+  float sq = 0.f, sk = 0.f, first[S];
+  auto load = [&](int c, float* f) {
+    const T* src = c < nq ? q + c * S : k + (c - nq) * S;
+    if constexpr (VEC) ld8(src, f);
+    else f[0] = ld1(src);
+  };
+  for (int c = tid; c < n; c += 256) {
+    float f[S], ss = 0.f;
+    load(c, f);
+#pragma unroll
+    for (int j = 0; j < S; ++j) {
+      ss += f[j] * f[j];
+      if (c == tid) first[j] = f[j];
+    }
+    if (c < nq) sq += ss;
+    else sk += ss;
   }
-  for (int c = tid; c < a.kv_rank; c += 256) {
-    const float v = ld1(k + c);
-    sk += v * v;
-  }
-  sq = block_sum(sq, part);
-  sk = block_sum(sk, part);
-  const float rq = 1.f / sqrtf(sq / (float)a.q_rank + a.eps), rk = 1.f / sqrtf(sk / (float)a.kv_rank + a.eps);
-  for (int c = tid; c < a.q_rank; c += 256) st1(cq + (size_t)row * ldc + c, ld1(q + c) * rq * gq[c]);
-  if (lat_keys(a, row) == 0) return;  // uniform over the workgroup
+  const bool live = lat_keys(a, row) > 0;  // uniform over the workgroup
   const int p = a.pos[row];
-  T* dst = static_cast<T*>(a.cache) +
-           ((size_t)lat_page(a, a.slot[row], p / LAT_PAGE) * LAT_PAGE + p % LAT_PAGE) * (a.krp + a.rp);
-  for (int c = tid; c < a.krp; c += 256) st1(dst + c, c < a.kv_rank ? ld1(k + c) * rk * gk[c] : 0.f);
-  for (int c = tid; c < a.rp; c += 256) st1(dst + a.krp + c, c < a.rot_dim ? lat_rot(a, k + a.kv_rank, c, p) : 0.f);
+  T* dst = nullptr;
+  if (live) {
+    dst = static_cast<T*>(a.cache) +
+          ((size_t)lat_page(a, a.slot[row], p / LAT_PAGE) * LAT_PAGE + p % LAT_PAGE) * (a.krp + a.rp);
+    for (int c = tid; c < a.rp; c += 256) st1(dst + a.krp + c, c < a.rot_dim ? lat_rot(a, k + a.kv_rank, c, p) : 0.f);
+  }
+  block_sum2(sq, sk, part);
+  const float rq = 1.f / sqrtf(sq / (float)a.q_rank + a.eps), rk = 1.f / sqrtf(sk / (float)a.kv_rank + a.eps);
+  for (int c = tid; c < n; c += 256) {
+    float f[S];
+    if (c == tid) {
+#pragma unroll
+      for (int j = 0; j < S; ++j) f[j] = first[j];
+    } else {
+      load(c, f);
+    }
+    const bool isq = c < nq;
+    const int o = (isq ? c : c - nq) * S;
+    const float* g = (isq ? gq : gk) + o;
+    const float r = isq ? rq : rk;
+#pragma unroll
+    for (int j = 0; j < S; ++j) f[j] *= r * g[j];
+    if (!isq && !live) continue;
+    T* d = isq ? cq + (size_t)row * ldc + o : dst + o;
+    if constexpr (VEC) st8(d, f);
+    else st1(d, f[0]);
+  }
+  if (live)
+    for (int c = a.kv_rank + tid; c < a.krp; c += 256) st1(dst + c, 0.f);
 }
 
 // wk: [heads][dkp][krp] (row d = the key's dimension d); qt: [entries][heads][krp + rp]
@@ -182,8 +239,13 @@ extern "C" int lsa_latent_append(int f32, const LatentArgs* a, int rows, const v
   if (!args_ok(a, rows) || a->index || oq < 0 || ok < 0 || ldi < oq + a->q_rank || ldi < ok + a->kv_rank + a->rot_dim ||
       ldc < a->q_rank)
     return LSA_BAD_SHAPE;
-  if (f32) append_kernel<float><<<rows, 256, 0, s>>>(*a, (const float*)in, ldi, oq, ok, gq, gk, (float*)cq, ldc);
-  else append_kernel<bf16_raw><<<rows, 256, 0, s>>>(*a, (const bf16_raw*)in, ldi, oq, ok, gq, gk, (bf16_raw*)cq, ldc);
+  const bool vec = !f32 && !((a->q_rank | a->kv_rank | oq | ok | ldi | ldc) % 8) && !(((uintptr_t)in | (uintptr_t)cq) % 16);
+  if (f32)
+    append_kernel<float, false><<<rows, 256, 0, s>>>(*a, (const float*)in, ldi, oq, ok, gq, gk, (float*)cq, ldc);
+  else if (vec)
+    append_kernel<bf16_raw, true><<<rows, 256, 0, s>>>(*a, (const bf16_raw*)in, ldi, oq, ok, gq, gk, (bf16_raw*)cq, ldc);
+  else
+    append_kernel<bf16_raw, false><<<rows, 256, 0, s>>>(*a, (const bf16_raw*)in, ldi, oq, ok, gq, gk, (bf16_raw*)cq, ldc);
   LSA_CHECK_LAUNCH();
   return LSA_OK;
 }

@@ -5,10 +5,10 @@
 //       entry is read from memory ONCE for all heads of the group and once from LDS per use:
 //       * a 64-token page arrives by LDS-DMA into a double buffer (the next page is in flight
 //         while this one is computed), chunk-swizzled on the source address
-//       * S^T[key][head] = C . q~^T: the four waves take 16 keys each (A = page rows by ds_read_b128,
-//         B = the group's queries, in registers for the whole launch)
+//       * S^T[key][head] = C . q~^T: a wave takes 16 keys and all or half of the head tiles (A = page
+//         rows by ds_read_b128, B = its queries, in registers for the whole launch)
 //       * softmax: column maxima meet in LDS, every lane then works on its own keys in fp32
-//       * O^T[latent][head] += C^T . P^T: the waves take a quarter of the latent each, C^T by the
+//       * O^T[latent][head] += C^T . P^T: the waves take equal parts of the latent, C^T by the
 //         hardware-transposed LDS read of the same page image, P^T (bf16) through LDS
 //   lsa_latent_value_mfma   merge of the splits, then W_uv^h per head, output gate in the epilogue
 #include "latent.h"
@@ -31,36 +31,41 @@ LSA_DEVICE void glds16(const void* src, unsigned char* lds_base) {
 }
 
 constexpr int RP = 64;   // rotated part of a cache entry
-constexpr int NW = 4;    // waves
+
+// Workgroup barrier for LDS traffic alone: the page DMA in flight stays in flight (a fence of
+// __syncthreads would drain it).
+LSA_DEVICE void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
+
+// waves: four key groups, and with two or more head tiles two head groups in the score step
+template <int KRP, int HT>
+constexpr int attend_waves() { return HT >= 2 && KRP >= 128 ? 8 : 4; }
 
 template <int KRP, int HT>
-__global__ __launch_bounds__(NW * 64, 1) void attend_mfma_kernel(LatentArgs a, const bf16_raw* __restrict__ qt, int ns,
-                                                                 float* __restrict__ po, float* __restrict__ pm) {
+__global__ __launch_bounds__((attend_waves<KRP, HT>() * 64), (attend_waves<KRP, HT>() / 4)) void attend_mfma_kernel(
+    LatentArgs a, const bf16_raw* __restrict__ qt, int ns, float* __restrict__ po, float* __restrict__ pm) {
+  constexpr int NW = attend_waves<KRP, HT>(), HG = NW / 4, QT = HT / HG;  // QT: head tiles per wave's scores
   constexpr int CW = KRP + RP, NCH = CW / 8, KF = CW / 32, DTW = KRP / 16 / NW;
-  constexpr int BLK = LAT_PAGE * CW * 2, PPW = BLK / 1024 / NW;
-  static_assert(PPW * NW * 1024 == BLK && DTW >= 1, "geometry");
-  __shared__ __attribute__((aligned(16))) unsigned char smem[2 * BLK];
-  __shared__ __attribute__((aligned(16))) unsigned char spt[HT * 2 * 64 * 16];  // P^T fragments
-  __shared__ float smax[NW][HT * 16];
+  constexpr int BLK = LAT_PAGE * CW * 2, PPW = BLK / 1024 / NW, C1 = HT * 16;
+  static_assert(PPW * NW * 1024 == BLK && DTW >= 1 && QT * HG == HT, "geometry");
+  // ONE array: with several, the compiler tells their accesses apart and drains the page DMA before
+  // the first read of the other page
+  __shared__ __attribute__((aligned(16))) unsigned char smem[2 * BLK + HT * 2 * 64 * 16 + 4 * HT * 16 * 4];
+  unsigned char* spt = smem + 2 * BLK;                                       // P^T fragments
+  float* smax = reinterpret_cast<float*>(smem + 2 * BLK + HT * 2 * 64 * 16);  // [4 key groups][HT * 16]
 
   const int e = blockIdx.x, h0 = blockIdx.y * (HT * 16), sp = blockIdx.z;
   const int row = a.index ? a.index[e] : e;
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l16 = lane & 15;
-  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int slot = a.slot[row];
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6), kg = w & 3, t0 = (w >> 2) * QT;
+  const int slot = __builtin_amdgcn_readfirstlane(a.slot[row]);
   const int len = __builtin_amdgcn_readfirstlane(lat_keys(a, row));
   const int nb = (len + LAT_PAGE - 1) / LAT_PAGE, b0 = nb * sp / ns, b1 = nb * (sp + 1) / ns;
   const bf16_raw* cache = static_cast<const bf16_raw*>(a.cache);
   const float sl2 = a.scale * 1.4426950408889634f;
-
-  u32x4_t qf[HT][KF];
-#pragma unroll
-  for (int t = 0; t < HT; ++t) {
-    const int h = h0 + t * 16 + l16;
-    const bf16_raw* q = qt + ((size_t)e * a.heads + (h < a.heads ? h : 0)) * CW;
-#pragma unroll
-    for (int kf = 0; kf < KF; ++kf) qf[t][kf] = h < a.heads ? ld16(q + kf * 32 + g * 8) : u32x4_t{0u, 0u, 0u, 0u};
-  }
 
   auto stage = [&](int page, int buf) {
     const bf16_raw* src = cache + (size_t)page * LAT_PAGE * CW;
@@ -70,85 +75,122 @@ __global__ __launch_bounds__(NW * 64, 1) void attend_mfma_kernel(LatentArgs a, c
       glds16(src + (size_t)r * CW + (c ^ swz<NCH>(r)) * 8, smem + buf * BLK + pc * 1024);
     }
   };
+  // lane i holds the page of block pb + i: no memory access (whose wait would drain the DMA) in the loop
+  int pb = b0;
+  int pages = b0 + lane < b1 ? lat_page(a, slot, b0 + lane) : 0;
+  if (b0 < b1) stage(__builtin_amdgcn_readlane(pages, 0), 0);
+
+  u32x4_t qf[QT][KF];
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    const int h = h0 + (t0 + t) * 16 + l16;
+    const bf16_raw* q = qt + ((size_t)e * a.heads + min(h, a.heads - 1)) * CW;  // surplus columns are not stored
+#pragma unroll
+    for (int kf = 0; kf < KF; ++kf) qf[t][kf] = ld16(q + kf * 32 + g * 8);
+  }
+  // the queries have arrived here, not at their first use inside the loop (whose wait would also
+  // drain the next page's DMA, every time around)
+#pragma unroll
+  for (int t = 0; t < QT; ++t)
+#pragma unroll
+    for (int kf = 0; kf < KF; ++kf) asm volatile("" : "+v"(qf[t][kf]));
 
   f32x4_t o[HT][DTW];
-  float m_run[HT], l_run[HT];
+  float m_run[HT], l_run[QT];
 #pragma unroll
   for (int t = 0; t < HT; ++t) {
     m_run[t] = -INFINITY;
-    l_run[t] = 0.f;
+    if (t < QT) l_run[t] = 0.f;
 #pragma unroll
     for (int d = 0; d < DTW; ++d) o[t][d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   }
-  // per-lane offsets into a page image: key row 16 w + l16 (its swizzle depends on l16 alone), and
+  // per-lane offsets into a page image: key row 16 kg + l16 (its swizzle depends on l16 alone), and
   // the transposed reads' row 4 g + l16 / 4 (+ 16, + 32: same swizzle)
-  const int krow = (w * 16 + l16) * (CW * 2), ksw = swz<NCH>(l16);
+  const int krow = (kg * 16 + l16) * (CW * 2), ksw = swz<NCH>(l16);
   const int vlo = 4 * g + (l16 >> 2), vrow = vlo * (CW * 2), vsw = swz<NCH>(vlo);
 
-  int page_next = 0;
-  if (b0 < b1) {
-    stage(lat_page(a, slot, b0), 0);
-    page_next = b0 + 1 < b1 ? lat_page(a, slot, b0 + 1) : 0;
-  }
   for (int b = b0; b < b1; ++b) {
     const unsigned char* img = smem + ((b - b0) & 1) * BLK;
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's part of page b has landed
-    __syncthreads();  // every wave's, and every wave is done with the other buffer and with spt
+    lds_barrier();  // every wave's, and every wave is done with the other buffer and with spt
     if (b + 1 < b1) {
-      stage(page_next, (b + 1 - b0) & 1);
-      page_next = b + 2 < b1 ? lat_page(a, slot, b + 2) : 0;
+      if (b + 1 - pb == 64) {
+        pb += 64;
+        pages = pb + lane < b1 ? lat_page(a, slot, pb + lane) : 0;
+      }
+      stage(__builtin_amdgcn_readlane(pages, b + 1 - pb), (b + 1 - b0) & 1);
     }
 
-    f32x4_t s[HT], s2[HT];
+    f32x4_t s[QT], s2[QT];
 #pragma unroll
-    for (int t = 0; t < HT; ++t) s[t] = s2[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int t = 0; t < QT; ++t) s[t] = s2[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int kf = 0; kf < KF; ++kf) {
       const u32x4_t k = *reinterpret_cast<const u32x4_t*>(img + krow + (((kf * 4 + g) ^ ksw) << 4));
 #pragma unroll
-      for (int t = 0; t < HT; ++t) {
-        if (HT <= 2 && (kf & 1)) s2[t] = mfma16(k, qf[t][kf], s2[t]);  // two chains where one would stall
+      for (int t = 0; t < QT; ++t) {
+        if (QT <= 2 && (kf & 1)) s2[t] = mfma16(k, qf[t][kf], s2[t]);  // two chains where one would stall
         else s[t] = mfma16(k, qf[t][kf], s[t]);
       }
     }
-    float mx[HT];
+    // four reads ahead of the MFMAs
+    __builtin_amdgcn_sched_group_barrier(0x100, KF < 4 ? KF : 4, 0);
 #pragma unroll
-    for (int t = 0; t < HT; ++t) {
-      mx[t] = -INFINITY;
+    for (int kf = 4; kf < KF; ++kf) {
+      __builtin_amdgcn_sched_group_barrier(0x008, QT, 0);
+      __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+    }
+    __builtin_amdgcn_sched_group_barrier(0x008, QT * (KF < 4 ? KF : 4), 0);
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+      float mx = -INFINITY;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int key = b * LAT_PAGE + w * 16 + g * 4 + r;
+        const int key = b * LAT_PAGE + kg * 16 + g * 4 + r;
         const float v = key < len ? (s[t][r] + s2[t][r]) * sl2 : -INFINITY;
         s[t][r] = v;
-        mx[t] = fmaxf(mx[t], v);
+        mx = fmaxf(mx, v);
       }
-      mx[t] = fmaxf(mx[t], __shfl_xor(mx[t], 16, 64));
-      mx[t] = fmaxf(mx[t], __shfl_xor(mx[t], 32, 64));
-      if (g == 0) smax[w][t * 16 + l16] = mx[t];
+      mx = fmaxf(mx, lane_xor<16>(mx));
+      mx = fmaxf(mx, lane_xor<32>(mx));
+      if (g == 0) smax[kg * C1 + (t0 + t) * 16 + l16] = mx;
     }
-    __syncthreads();
+    lds_barrier();
+    float mn[HT];
 #pragma unroll
     for (int t = 0; t < HT; ++t) {
       const int c = t * 16 + l16;
       // page b holds at least one visible key, so the new maximum is finite
-      const float mn = fmaxf(m_run[t], fmaxf(fmaxf(smax[0][c], smax[1][c]), fmaxf(smax[2][c], smax[3][c])));
-      const float alpha = __builtin_amdgcn_exp2f(m_run[t] - mn);
+      mn[t] = fmaxf(m_run[t], fmaxf(fmaxf(smax[c], smax[C1 + c]), fmaxf(smax[2 * C1 + c], smax[3 * C1 + c])));
+    }
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+      const int ta = t0 + t;
+      float mt = mn[t], mo = m_run[t];
+      if (HG == 2) {  // this wave's head group (wave-uniform)
+        mt = t0 ? mn[HT - QT + t] : mt;
+        mo = t0 ? m_run[HT - QT + t] : mo;
+      }
       float ps = 0.f;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        s[t][r] = __builtin_amdgcn_exp2f(s[t][r] - mn);
+        s[t][r] = __builtin_amdgcn_exp2f(s[t][r] - mt);
         ps += s[t][r];
       }
-      l_run[t] = l_run[t] * alpha + ps;  // this lane's keys; summed at the end
-      if (__builtin_amdgcn_ballot_w64(mn != m_run[t])) {
+      l_run[t] = l_run[t] * __builtin_amdgcn_exp2f(mo - mt) + ps;  // this lane's keys; summed at the end
+      // fragment f2 = kg / 2 of the 32-key PV step, this wave's half of its eight keys per lane
+      st4(reinterpret_cast<bf16_raw*>(spt + (((ta * 2 + (kg >> 1)) * 64 + lane) << 4) + ((kg & 1) << 3)), s[t]);
+    }
+#pragma unroll
+    for (int t = 0; t < HT; ++t) {
+      if (__builtin_amdgcn_ballot_w64(mn[t] != m_run[t])) {
+        const float alpha = __builtin_amdgcn_exp2f(m_run[t] - mn[t]);
 #pragma unroll
         for (int d = 0; d < DTW; ++d) o[t][d] *= alpha;
       }
-      m_run[t] = mn;
-      // fragment f2 = w / 2 of the 32-key PV step, this wave's half of its eight keys per lane
-      st4(reinterpret_cast<bf16_raw*>(spt + (((t * 2 + (w >> 1)) * 64 + lane) << 4) + ((w & 1) << 3)), s[t]);
+      m_run[t] = mn[t];
     }
-    __syncthreads();
+    lds_barrier();
 #pragma unroll
     for (int f2 = 0; f2 < 2; ++f2) {
       u32x4_t p[HT];
@@ -170,16 +212,24 @@ __global__ __launch_bounds__(NW * 64, 1) void attend_mfma_kernel(LatentArgs a, c
         for (int t = 0; t < HT; ++t) o[t][d] = mfma16(c, p[t], o[t][d]);
       }
     }
+    // both P fragments and the first latent tiles are read ahead of the MFMAs
+    __builtin_amdgcn_sched_group_barrier(0x100, 2 * HT + 4, 0);
+#pragma unroll
+    for (int i = 2; i < 2 * DTW; ++i) {
+      __builtin_amdgcn_sched_group_barrier(0x008, HT, 0);
+      __builtin_amdgcn_sched_group_barrier(0x100, 2, 0);
+    }
+    __builtin_amdgcn_sched_group_barrier(0x008, 2 * HT, 0);
   }
 
-  __syncthreads();  // the last page's maxima have been read
+  lds_barrier();  // the last page's maxima have been read
 #pragma unroll
-  for (int t = 0; t < HT; ++t) {
-    l_run[t] += __shfl_xor(l_run[t], 16, 64);
-    l_run[t] += __shfl_xor(l_run[t], 32, 64);
-    if (g == 0) smax[w][t * 16 + l16] = l_run[t];
+  for (int t = 0; t < QT; ++t) {
+    l_run[t] += lane_xor<16>(l_run[t]);
+    l_run[t] += lane_xor<32>(l_run[t]);
+    if (g == 0) smax[kg * C1 + (t0 + t) * 16 + l16] = l_run[t];
   }
-  __syncthreads();
+  lds_barrier();
 #pragma unroll
   for (int t = 0; t < HT; ++t) {
     const int h = h0 + t * 16 + l16;
@@ -191,55 +241,64 @@ __global__ __launch_bounds__(NW * 64, 1) void attend_mfma_kernel(LatentArgs a, c
     if (w == 0 && g == 0) {
       const int c = t * 16 + l16;
       pm[out * 2] = m_run[t];
-      pm[out * 2 + 1] = smax[0][c] + smax[1][c] + smax[2][c] + smax[3][c];
+      pm[out * 2 + 1] = smax[c] + smax[C1 + c] + smax[2 * C1 + c] + smax[3 * C1 + c];
     }
   }
 }
 
 // wk: per head the packed [krp][dkp] matrix (common.h fragment order). Grid (16-entry tiles, heads,
-// 16-tile stretches of the latent); every wave up to 4 latent tiles.
+// 16-tile stretches of the latent + 1): every wave up to 4 latent tiles; the last z turns the
+// rotated parts beside them.
 __global__ __launch_bounds__(256) void absorb_mfma_kernel(LatentArgs a, int n, const bf16_raw* __restrict__ q, int ldq,
                                                           const bf16_raw* __restrict__ wk, bf16_raw* __restrict__ qt) {
   const int h = blockIdx.y, e0 = blockIdx.x * 16;
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l16 = lane & 15, w = tid >> 6;
   const int kf_n = a.dkp / 32, nt_n = a.krp / 16, cw = a.krp + a.rp;
-  const int e = e0 + l16;
-  const bool ok = e < n;
-  const int row = ok ? (a.index ? a.index[e] : e) : 0;
-  const bf16_raw* qh = q + (size_t)row * ldq + (size_t)h * (a.dkp + a.rp);
-  const int t0 = blockIdx.z * 16 + w * 4;
-  const bf16_raw* wh = wk + ((size_t)h * nt_n + t0) * kf_n * 512;
-  f32x4_t acc[4];
-#pragma unroll
-  for (int t = 0; t < 4; ++t) acc[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  for (int kf = 0; kf < kf_n; ++kf) {
-    const u32x4_t b = ok ? ld16(qh + kf * 32 + g * 8) : u32x4_t{0u, 0u, 0u, 0u};
-#pragma unroll
-    for (int t = 0; t < 4; ++t)
-      if (t0 + t < nt_n) acc[t] = mfma16(ld16(wh + ((size_t)t * kf_n + kf) * 512 + lane * 8), b, acc[t]);
-  }
-  if (ok) {
-    bf16_raw* o = qt + ((size_t)e * a.heads + h) * cw;
-#pragma unroll
-    for (int t = 0; t < 4; ++t)
-      if (t0 + t < nt_n) st4(o + (t0 + t) * 16 + 4 * g, acc[t]);
-  }
-  if (blockIdx.z == 0) {
+  if (blockIdx.z == gridDim.z - 1) {
     for (int i = tid; i < 16 * a.rp; i += 256) {
       const int ee = e0 + i / a.rp, j = i % a.rp;
       if (ee >= n) break;
       const int rr = a.index ? a.index[ee] : ee;
       const bf16_raw* qr = q + (size_t)rr * ldq + (size_t)h * (a.dkp + a.rp) + a.dkp;
-      const bool live = j < a.rot_dim && lat_keys(a, rr) > 0;
-      st1(qt + ((size_t)ee * a.heads + h) * cw + a.krp + j, live ? lat_rot(a, qr, j, a.pos[rr]) : 0.f);
+      const int p = a.pos[rr];
+      const bool live = j < a.rot_dim && p >= 0 && p < a.max_pages * LAT_PAGE;
+      st1(qt + ((size_t)ee * a.heads + h) * cw + a.krp + j, live ? lat_rot(a, qr, j, p) : 0.f);
     }
+    return;
+  }
+  const int e = min(e0 + l16, n - 1);  // surplus columns repeat the last entry and are not stored
+  const int row = a.index ? a.index[e] : e;
+  const bf16_raw* qh = q + (size_t)row * ldq + (size_t)h * (a.dkp + a.rp);
+  const int t0 = blockIdx.z * 16 + w * 4;
+  if (t0 >= nt_n) return;  // krp % 64 == 0: whole groups of four tiles
+  const bf16_raw* wh = wk + ((size_t)h * nt_n + t0) * kf_n * 512 + lane * 8;
+  f32x4_t acc[4];
+#pragma unroll
+  for (int t = 0; t < 4; ++t) acc[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < kf_n; k0 += 2) {  // dkp % 64 == 0
+    u32x4_t wt[2][4], b[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+#pragma unroll
+      for (int t = 0; t < 4; ++t) wt[u][t] = ld16(wh + ((size_t)t * kf_n + k0 + u) * 512);
+      b[u] = ld16(qh + (k0 + u) * 32 + g * 8);
+    }
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+      for (int t = 0; t < 4; ++t) acc[t] = mfma16(wt[u][t], b[u], acc[t]);
+  }
+  if (e0 + l16 < n) {
+    bf16_raw* o = qt + ((size_t)e * a.heads + h) * cw;
+#pragma unroll
+    for (int t = 0; t < 4; ++t) st4(o + (t0 + t) * 16 + 4 * g, acc[t]);
   }
 }
 
-// wv: per head the packed [dvp][krp] matrix. Grid (16-entry tiles, heads, 4-tile stretches of the
-// value); one 16-wide value tile per wave.
+// wv: per head the packed [dvp][krp] matrix. Grid (16-entry tiles, heads, 8-tile stretches of the
+// value); eight waves, one 16-wide value tile each, whose weights are requested before the merge.
 template <int KRP>
-__global__ __launch_bounds__(256) void value_mfma_kernel(LatentArgs a, int n, const float* __restrict__ po,
+__global__ __launch_bounds__(512) void value_mfma_kernel(LatentArgs a, int n, const float* __restrict__ po,
                                                          const float* __restrict__ pm, int ns,
                                                          const bf16_raw* __restrict__ wv, const bf16_raw* __restrict__ gate,
                                                          int ldg, bf16_raw* __restrict__ out, int ldo) {
@@ -248,7 +307,15 @@ __global__ __launch_bounds__(256) void value_mfma_kernel(LatentArgs a, int n, co
   __shared__ float wgt[16][64];
   const int h = blockIdx.y, e0 = blockIdx.x * 16;
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, l16 = lane & 15, w = tid >> 6;
-  if (tid < 16) {
+  const int t = blockIdx.z * 8 + w;
+  const bool work = t * 16 < a.dvp;
+  u32x4_t wf[KF];
+  {
+    const bf16_raw* wh = wv + ((size_t)h * (a.dvp / 16) + (work ? t : 0)) * KF * 512 + lane * 8;
+#pragma unroll
+    for (int kf = 0; kf < KF; ++kf) wf[kf] = ld16(wh + (size_t)kf * 512);
+  }
+  if (ns > 1 && tid < 16) {
     const int e = e0 + tid;
     if (e < n) {
       const float* p = pm + ((size_t)e * a.heads + h) * ns * 2;
@@ -265,29 +332,42 @@ __global__ __launch_bounds__(256) void value_mfma_kernel(LatentArgs a, int n, co
     }
   }
   __syncthreads();
-  for (int i = tid; i < 16 * (KRP / 4); i += 256) {
+  for (int i = tid; i < 16 * (KRP / 4); i += 512) {
     const int r = i / (KRP / 4), c = (i % (KRP / 4)) * 4, e = e0 + r;
     f32x4_t v = f32x4_t{0.f, 0.f, 0.f, 0.f};
     if (e < n) {
-      const float* p = po + ((size_t)e * a.heads + h) * ns * KRP + c;
-      for (int s = 0; s < ns; ++s) v += *reinterpret_cast<const f32x4_t*>(p + (size_t)s * KRP) * wgt[r][s];
+      const size_t b = ((size_t)e * a.heads + h) * ns;
+      const float* p = po + b * KRP + c;
+      if (ns == 1) {
+        const float L = pm[b * 2 + 1];
+        v = *reinterpret_cast<const f32x4_t*>(p) * (L > 0.f ? 1.f / L : 0.f);
+      } else {
+        int s = 0;
+        for (; s + 4 <= ns; s += 4) {
+          f32x4_t x[4];
+#pragma unroll
+          for (int u = 0; u < 4; ++u) x[u] = *reinterpret_cast<const f32x4_t*>(p + (size_t)(s + u) * KRP);
+#pragma unroll
+          for (int u = 0; u < 4; ++u) v += x[u] * wgt[r][s + u];
+        }
+        for (; s < ns; ++s) v += *reinterpret_cast<const f32x4_t*>(p + (size_t)s * KRP) * wgt[r][s];
+      }
     }
     st4(so + r * LD + c, v);
   }
   __syncthreads();
-  const int t = blockIdx.z * NW + w, e = e0 + l16;
-  if (t * 16 >= a.dvp) return;
-  const bf16_raw* wh = wv + ((size_t)h * (a.dvp / 16) + t) * KF * 512;
+  const int e = e0 + l16;
   f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-  for (int kf = 0; kf < KF; ++kf)
-    acc = mfma16(ld16(wh + (size_t)kf * 512 + lane * 8), ld16(so + l16 * LD + kf * 32 + g * 8), acc);
-  if (e >= n) return;
+  for (int kf = 0; kf < KF; ++kf) acc = mfma16(wf[kf], ld16(so + l16 * LD + kf * 32 + g * 8), acc);
+  if (!work || e >= n) return;
   const int row = a.index ? a.index[e] : e, col = h * a.dvp + t * 16 + 4 * g;
   if (gate) {
-    const bf16_raw* gp = gate + (size_t)row * ldg + col;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) acc[r] *= sigmoid(bf2f(gp[r]));
+    const u32x2_t gb = *reinterpret_cast<const u32x2_t*>(gate + (size_t)row * ldg + col);
+    acc[0] *= sigmoid(__uint_as_float(gb[0] << 16));
+    acc[1] *= sigmoid(__uint_as_float(gb[0] & 0xffff0000u));
+    acc[2] *= sigmoid(__uint_as_float(gb[1] << 16));
+    acc[3] *= sigmoid(__uint_as_float(gb[1] & 0xffff0000u));
   }
   st4(out + (size_t)row * ldo + col, acc);
 }
@@ -306,7 +386,7 @@ extern "C" int lsa_latent_absorb_mfma(const LatentArgs* a, int n, const void* q,
                                       hipStream_t s) {
   if (!size_ok(a, n) || ldq < a->heads * (a->dkp + a->rp) || ldq % 8 || (uintptr_t)q % 16 || (uintptr_t)qt % 16)
     return LSA_BAD_SHAPE;
-  dim3 grid((n + 15) / 16, a->heads, (a->krp / 16 + 15) / 16);
+  dim3 grid((n + 15) / 16, a->heads, (a->krp / 16 + 15) / 16 + 1);
   absorb_mfma_kernel<<<grid, 256, 0, s>>>(*a, n, (const bf16_raw*)q, ldq, (const bf16_raw*)wk, (bf16_raw*)qt);
   LSA_CHECK_LAUNCH();
   return LSA_OK;
@@ -318,7 +398,7 @@ extern "C" int lsa_latent_attend_mfma(const LatentArgs* a, int n, const void* qt
   // head tiles per workgroup; four tiles of 512-wide latents do not fit the register file
   const int tiles = (a->heads + 15) / 16, ht = tiles >= 3 ? (a->krp == 512 ? 2 : 4) : tiles;
   dim3 grid(n, (tiles + ht - 1) / ht, ns);
-#define LSA_A(K, T) attend_mfma_kernel<K, T><<<grid, NW * 64, 0, s>>>(*a, (const bf16_raw*)qt, ns, po, pm)
+#define LSA_A(K, T) attend_mfma_kernel<K, T><<<grid, (attend_waves<K, T>() * 64), 0, s>>>(*a, (const bf16_raw*)qt, ns, po, pm)
 #define LSA_K(K)                                 \
   if (ht == 1) LSA_A(K, 1);                      \
   else if (ht == 2) LSA_A(K, 2);                 \
@@ -340,10 +420,11 @@ extern "C" int lsa_latent_value_mfma(const LatentArgs* a, int n, const float* po
                                      const void* gate, int ldg, void* out, int ldo, hipStream_t s) {
   if (!size_ok(a, n) || ns < 1 || ns > 64 || ldo < a->heads * a->dvp || ldo % 4 || (uintptr_t)out % 8 || (uintptr_t)po % 16)
     return LSA_BAD_SHAPE;
-  dim3 grid((n + 15) / 16, a->heads, a->dvp / 64);
+  if (gate && (ldg % 4 || (uintptr_t)gate % 8)) return LSA_BAD_SHAPE;
+  dim3 grid((n + 15) / 16, a->heads, (a->dvp + 127) / 128);
 #define LSA_V(K)                                                                                                       \
   case K:                                                                                                              \
-    value_mfma_kernel<K><<<grid, 256, 0, s>>>(*a, n, po, pm, ns, (const bf16_raw*)wv, (const bf16_raw*)gate, ldg,      \
+    value_mfma_kernel<K><<<grid, 512, 0, s>>>(*a, n, po, pm, ns, (const bf16_raw*)wv, (const bf16_raw*)gate, ldg,      \
                                               (bf16_raw*)out, ldo);                                                    \
     break;
   switch (a->krp) {

@@ -35,7 +35,7 @@ LSA_DEVICE void glds16(const void* src, unsigned char* lds_base) {
 }
 
 template <int DK, int DV>
-__global__ __launch_bounds__(NTHR) void latent_prefill_kernel(LatentArgs a, const LatTile* __restrict__ tiles,
+__global__ __launch_bounds__(NTHR, 4) void latent_prefill_kernel(LatentArgs a, const LatTile* __restrict__ tiles,
                                                               const bf16_raw* __restrict__ q, int ldq,
                                                               const bf16_raw* __restrict__ kv, int ldkv,
                                                               const bf16_raw* __restrict__ lat,
@@ -80,6 +80,10 @@ __global__ __launch_bounds__(NTHR) void latent_prefill_kernel(LatentArgs a, cons
       }
       qf[kf] = pack8(v);
     }
+    // the query has arrived here, not at its first use inside the block loop (whose wait would also
+    // drain the next block's DMA, every time around)
+#pragma unroll
+    for (int kf = 0; kf < KF; ++kf) asm volatile("" : "+v"(qf[kf]));
   }
   const int lim = min(tile.pos0 + tile.nrows, tile.kvlen);
   const int my_lim = min(my_pos + 1, tile.kvlen);
@@ -121,8 +125,9 @@ __global__ __launch_bounds__(NTHR) void latent_prefill_kernel(LatentArgs a, cons
 
   if (nkb > 0) stage(0, 0);
   for (int kb = 0; kb < nkb; ++kb) {
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    __syncthreads();
+    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
     if (kb + 1 < nkb) stage(kb + 1, (kb + 1) & 1);
     if (kb * BKV >= wave_lim) continue;
     const unsigned char* ks = smem + (kb & 1) * (KBLK + VBLK);

@@ -25,12 +25,42 @@ __global__ __launch_bounds__(256) void stream_embed_kernel(const int* __restrict
     st1(xc + (size_t)row * ldc + c, v);
   }
 }
-
-template <typename T>
-__global__ __launch_bounds__(256) void cast_rows_kernel(const float* __restrict__ x, int ldx, int W, T* __restrict__ xc,
-                                                        int ldc) {
+// bf16, 8 values per thread and step
+__global__ __launch_bounds__(256) void stream_embed8_kernel(const int* __restrict__ ids, const bf16_raw* __restrict__ table,
+                                                            int ldt, float scale, int W, float* __restrict__ x, int ldx,
+                                                            bf16_raw* __restrict__ xc, int ldc) {
   const int row = blockIdx.x;
-  for (int c = threadIdx.x; c < W; c += 256) st1(xc + (size_t)row * ldc + c, x[(size_t)row * ldx + c]);
+  const bf16_raw* src = table + (size_t)ids[row] * ldt;
+  for (int c = threadIdx.x * 8; c < W; c += 2048) {
+    float f[8];
+    unpack8(ld16(src + c), f);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) f[k] *= scale;
+    float* d = x + (size_t)row * ldx + c;
+    *reinterpret_cast<f32x4_t*>(d) = f32x4_t{f[0], f[1], f[2], f[3]};
+    *reinterpret_cast<f32x4_t*>(d + 4) = f32x4_t{f[4], f[5], f[6], f[7]};
+    st16(xc + (size_t)row * ldc + c, pack8(f));
+  }
+}
+
+// x -> its copy xc and, where given, x2 (the engine's own stream buffer)
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void cast_rows_kernel(const float* __restrict__ x, int ldx, int W, T* __restrict__ xc,
+                                                        int ldc, float* __restrict__ x2, int ldx2) {
+  const int row = blockIdx.x;
+  const float* s = x + (size_t)row * ldx;
+  if constexpr (VEC) {
+    for (int c = threadIdx.x * 4; c < W; c += 1024) {
+      const f32x4_t v = *reinterpret_cast<const f32x4_t*>(s + c);
+      st4(xc + (size_t)row * ldc + c, v);
+      if (x2) *reinterpret_cast<f32x4_t*>(x2 + (size_t)row * ldx2 + c) = v;
+    }
+  } else {
+    for (int c = threadIdx.x; c < W; c += 256) {
+      st1(xc + (size_t)row * ldc + c, s[c]);
+      if (x2) x2[(size_t)row * ldx2 + c] = s[c];
+    }
+  }
 }
 
 // ADD: x += rms(y) * gain and xc = x; else xc = rms(y) * gain. One workgroup per row; a row of up
@@ -123,16 +153,24 @@ extern "C" int lsa_stream_embed(int f32, const int* ids, int rows, const void* t
   if (rows < 1 || W < 1 || ldt < W || ldx < W || ldc < W) return LSA_BAD_SHAPE;
   if (f32)
     stream_embed_kernel<float><<<rows, 256, 0, s>>>(ids, (const float*)table, ldt, scale, W, x, ldx, (float*)xc, ldc);
+  else if (!((W | ldt | ldx | ldc) % 8) && !(((uintptr_t)table | (uintptr_t)x | (uintptr_t)xc) % 16))
+    stream_embed8_kernel<<<rows, 256, 0, s>>>(ids, (const bf16_raw*)table, ldt, scale, W, x, ldx, (bf16_raw*)xc, ldc);
   else
     stream_embed_kernel<bf16_raw><<<rows, 256, 0, s>>>(ids, (const bf16_raw*)table, ldt, scale, W, x, ldx, (bf16_raw*)xc, ldc);
   LSA_CHECK_LAUNCH();
   return LSA_OK;
 }
 
-extern "C" int lsa_cast_rows(int f32, const float* x, int ldx, int rows, int W, void* xc, int ldc, hipStream_t s) {
-  if (rows < 1 || W < 1 || ldx < W || ldc < W) return LSA_BAD_SHAPE;
-  if (f32) cast_rows_kernel<float><<<rows, 256, 0, s>>>(x, ldx, W, (float*)xc, ldc);
-  else cast_rows_kernel<bf16_raw><<<rows, 256, 0, s>>>(x, ldx, W, (bf16_raw*)xc, ldc);
+extern "C" int lsa_cast_rows(int f32, const float* x, int ldx, int rows, int W, void* xc, int ldc, float* x2, int ldx2,
+                             hipStream_t s) {
+  if (rows < 1 || W < 1 || ldx < W || ldc < W || (x2 && ldx2 < W)) return LSA_BAD_SHAPE;
+  const bool vec = !((W | ldx | ldc | ldx2) % 4) && !(((uintptr_t)x | (uintptr_t)xc | (uintptr_t)x2) % 16);
+#define LSA_R(T, V) cast_rows_kernel<T, V><<<rows, 256, 0, s>>>(x, ldx, W, (T*)xc, ldc, x2, ldx2)
+  if (f32 && vec) LSA_R(float, true);
+  else if (f32) LSA_R(float, false);
+  else if (vec) LSA_R(bf16_raw, true);
+  else LSA_R(bf16_raw, false);
+#undef LSA_R
   LSA_CHECK_LAUNCH();
   return LSA_OK;
 }

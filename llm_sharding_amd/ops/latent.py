@@ -94,11 +94,13 @@ def stream_embed(ids, table, scale: float, x, xc, rows: int) -> None:
                                   x.stride(0), _p(xc), xc.stride(0), _stream()), "lsa_stream_embed")
 
 
-def cast_rows(x, xc, rows: int) -> None:
+def cast_rows(x, xc, rows: int, x2=None) -> None:
+    """xc = x in the projections' type; ``x2`` (fp32): a copy as it is."""
     _req(x.dtype == torch.float32 and x.stride(1) == 1 and xc.shape[1] >= x.shape[1]
          and min(x.shape[0], xc.shape[0]) >= rows, "cast_rows: shapes")
-    _check(lib().lsa_cast_rows(is_f32(xc.dtype), _p(x), x.stride(0), rows, x.shape[1], _p(xc), xc.stride(0), _stream()),
-           "lsa_cast_rows")
+    _req(x2 is None or (x2.dtype == torch.float32 and x2.shape[0] >= rows and x2.shape[1] >= x.shape[1]), "cast_rows: x2")
+    _check(lib().lsa_cast_rows(is_f32(xc.dtype), _p(x), x.stride(0), rows, x.shape[1], _p(xc), xc.stride(0), _p(x2),
+                               0 if x2 is None else x2.stride(0), _stream()), "lsa_cast_rows")
 
 
 def stream_add_norm(y, gain, eps: float, x, xc, rows: int) -> None:
@@ -133,6 +135,14 @@ def tuned_size(s) -> bool:
 def expand_size(s) -> bool:
     """The MFMA kernel of the expanded form takes this size."""
     return s.rp == 64 and s.dkp in (64, 128) and s.dvp in (64, 128)
+
+
+def head_groups(s) -> int:
+    """Workgroups per (row, split) of attend_mfma: head tiles of 16, 1 / 2 / 4 to a workgroup (at
+    most 2 with 512-wide latents)."""
+    tiles = -(-s.heads // 16)
+    per = tiles if tiles < 3 else (2 if s.krp == 512 else 4)
+    return -(-tiles // per)
 
 
 def pack_heads(w: torch.Tensor) -> torch.Tensor:
@@ -266,7 +276,7 @@ def declare(L: ctypes.CDLL) -> None:
     la = ctypes.POINTER(LatentArgs)
     sig = {
         "lsa_stream_embed": [i, vp, i, vp, i, f, i, vp, i, vp, i, vp],
-        "lsa_cast_rows": [i, vp, i, i, i, vp, i, vp],
+        "lsa_cast_rows": [i, vp, i, i, i, vp, i, vp, i, vp],
         "lsa_stream_add_norm": [i, vp, i, vp, f, i, i, vp, i, vp, i, vp],
         "lsa_stream_norm": [i, vp, i, vp, f, i, i, vp, i, vp],
         "lsa_logits_argmax": [vp, i, i, i, i, vp, vp],

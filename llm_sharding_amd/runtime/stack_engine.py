@@ -204,7 +204,7 @@ class StackEngine(StageEngine):
             out["sk_ws"] = hip.SkWorkspace(dev)
         return out
 
-    ATTEND_ITEMS = 1024  # (row, split) pairs of one absorbed-attention launch
+    ATTEND_ITEMS = 1024  # (row, key split) pairs of one absorbed-attention launch
 
     def decode_scratch(self, k: int, rows: Optional[int] = None) -> dict:
         if k == 0:
@@ -317,10 +317,11 @@ class StackEngine(StageEngine):
         return self._forward_hip(h, self._i32(sl), self._i32(ps), None, rows, runs=Plan.find_runs(sl, ps))
 
     def latent_nsplit(self, s, entries: int, longest: int) -> int:
-        """Key splits of the absorbed attention: enough workgroups for the chip, splits of at
-        least four pages."""
-        wgs = entries * max(1, ceil_div(s.heads, 16))
-        return int(max(1, min(16, ceil_div(512, wgs), ceil_div(longest, 4 * PAGE))))
+        """Key splits of the absorbed attention: about one workgroup per CU (each fills a CU's
+        LDS with its two pages), no more splits than pages."""
+        from ..ops import hip
+        from ..ops import latent as L
+        return int(max(1, min(64, hip.N_CU // max(1, entries * L.head_groups(s)), ceil_div(longest, PAGE))))
 
     def decode_nsplit(self, rows: int) -> int:
         m = max((l.spec.mixer for l in self.layers), key=lambda m: m.heads)
@@ -333,11 +334,10 @@ class StackEngine(StageEngine):
         if h.dtype != torch.float32 or not h.is_contiguous():
             h = h.to(torch.float32).contiguous()
         hbuf, x, y = self.buf_h[:rows], self.buf_x[:rows], self.buf_y[:rows]
-        if not (self._x_ready and h.data_ptr() == hbuf.data_ptr()):
-            L.cast_rows(h, x, rows)
+        own = h.data_ptr() == hbuf.data_ptr()
+        if not (own and self._x_ready):
+            L.cast_rows(h, x, rows, x2=None if own else hbuf)
         self._x_ready = False
-        if h.data_ptr() != hbuf.data_ptr():
-            hbuf.copy_(h)
         if runs is None and nsplit is None:
             nsplit = self.decode_nsplit(rows)
         plan = Plan(self, rows, runs, nsplit)
