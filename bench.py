@@ -291,12 +291,12 @@ def ttft_probe(model: str, lengths: list, seed: int = 0, repeats: int = 3) -> di
     import torch
 
     from llm_sharding_amd.config import get_preset
-    from llm_sharding_amd.runtime.engine import RandomSource, StageEngine
+    from llm_sharding_amd.runtime.registry import make_engine, random_source
 
     cfg = get_preset(model)
     dev = torch.device("cuda", 0)
-    eng = StageEngine(cfg, 0, cfg.num_hidden_layers, dev, torch.bfloat16, has_embed=True, has_head=True,
-                      source=RandomSource(cfg, seed), max_slots=1, max_seq=max(lengths) + 8,
+    eng = make_engine(cfg, 0, cfg.num_hidden_layers, dev, torch.bfloat16, has_embed=True, has_head=True,
+                      source=random_source(cfg, seed), max_slots=1, max_seq=max(lengths) + 8,
                       max_prefill_rows=max(lengths))
     g = torch.Generator().manual_seed(seed)
     out = {}

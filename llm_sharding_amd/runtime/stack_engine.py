@@ -26,6 +26,16 @@ from .paging import PagePool
 PAGE = 64
 
 
+def embed_rows(cfg: StackConfig, table: torch.Tensor, ids: torch.Tensor) -> torch.Tensor:
+    """Rows of the stream for ``ids`` [n], without an engine (an ingress that holds the table only)."""
+    h = torch.empty((ids.numel(), cfg.hidden_size), dtype=torch.float32, device=table.device)
+    if table.device.type != "cuda":
+        return h.copy_(F.embedding(ids.long(), table).float() * cfg.embed_scale)
+    from ..ops import latent as L
+    L.stream_embed(ids.to(torch.int32), table, cfg.embed_scale, h, torch.empty_like(h, dtype=table.dtype), ids.numel())
+    return h
+
+
 class _Layer:
     def __init__(self, spec, mixer, mlp, gain1, gain2):
         self.spec, self.mixer, self.mlp, self.gain1, self.gain2 = spec, mixer, mlp, gain1, gain2

@@ -39,6 +39,7 @@ from dataclasses import replace
 from typing import List, Optional, Sequence
 
 from ..config import LlamaConfig
+from ..runtime.registry import load_config
 from ..parallel.scheduler import DeviceSpec, Plan, build_chain_configs, plan_stages
 from ..parallel.transport import PushSocket
 from .config_sender import ConfigSender
@@ -56,7 +57,7 @@ class MasterNode:
 
     @classmethod
     def from_shards(cls, shards_path: str, devices: Sequence[DeviceSpec], kv_tokens: int = 4096) -> "MasterNode":
-        return cls(LlamaConfig.from_pretrained(shards_path), devices, kv_tokens)
+        return cls(load_config(shards_path), devices, kv_tokens)
 
     @staticmethod
     def speed_from_profiles(profiles: Sequence[dict]) -> list:

@@ -39,6 +39,7 @@ from typing import Optional
 import torch
 
 from ..config import LlamaConfig
+from ..runtime.registry import folder_source, load_config, make_engine
 from ..models.tokenizer import load_tokenizer
 from .node_worker import NodeWorker
 
@@ -79,12 +80,12 @@ def profile_stage_costs(cfg: LlamaConfig, source, device, batch: int = 1, contex
     tokens at 1 and n layers. Returns ms: ``layer_decode_ms``, ``embed_decode_ms``,
     ``head_decode_ms``, ``stage_overhead_ms``, ``layer_prefill_ms``, ``prefill_overhead_ms``
     plus the geometry."""
-    from ..runtime.engine import DecodeGraph, EagerDecode, StageEngine
+    from ..runtime.engine import DecodeGraph, EagerDecode
     dev = torch.device(device)
     gpu = dev.type == "cuda"
     n = max(2, min(int(n_layers), cfg.num_hidden_layers))
     max_seq = -(-(context + 4 * (replays + 4) + prefill_len + 8) // 64) * 64
-    eng = StageEngine(cfg, 0, n, dev, dtype if gpu else torch.float32, has_embed=True, has_head=True,
+    eng = make_engine(cfg, 0, n, dev, dtype if gpu else torch.float32, has_embed=True, has_head=True,
                       source=source, max_slots=batch, max_seq=max_seq,
                       max_prefill_rows=max(prefill_len, batch))
     layers = eng.layers
@@ -95,6 +96,8 @@ def profile_stage_costs(cfg: LlamaConfig, source, device, batch: int = 1, contex
         eng.layers = layers[:j]
         try:
             for s_ in slots:
+                eng.seq_len[s_] = 0
+                eng.prefill_rows([s_], [context + 1])  # a paged cache: room for what the steps attend to
                 eng.seq_len[s_] = context
             if gpu:
                 g = DecodeGraph(eng, batch, mode, slots=slots)
@@ -193,7 +196,7 @@ class NodeProfiler:
         self.device = torch.device(device)
         self.dtype = dtype
         self.backend = backend
-        self.config = LlamaConfig.from_pretrained(shards_path)
+        self.config = load_config(shards_path)
         self.layer_num = self.config.num_hidden_layers
         self.plot_dir = plot_dir
         self.verbose = verbose
@@ -219,8 +222,7 @@ class NodeProfiler:
         """Graph-replay cost model of the deployed pipeline engine on this device, from this
         node's shard folder (:func:`profile_stage_costs`); what ``MasterNode.deploy_pipeline
         (profiles=...)`` plans with."""
-        from ..runtime.engine import ShardFolderSource
-        res = profile_stage_costs(self.config, ShardFolderSource(self.shards_path, self.config), self.device,
+        res = profile_stage_costs(self.config, folder_source(self.shards_path, self.config), self.device,
                                   batch=batch, context=context, n_layers=n_layers, prefill_len=prefill_len,
                                   replays=replays, dtype=self.dtype)
         self._log(f"[INFO] stage costs (batch {batch}, context {context}): layer {res['layer_decode_ms']:.4f} ms, "
@@ -677,12 +679,11 @@ class NodeProfiler:
     def go_through_every_shards_only_by_profiler(self, out_token_num: int = 50, request: str = "Write a poem "
                                                  "about the blue sky.", input_ids=None) -> list:
         """One engine per layer, no networking (the reference's golden forward, C8j)."""
-        from ..runtime.engine import ShardFolderSource, StageEngine
         cfg, dev = self.config, self.device
         dt = torch.bfloat16 if dev.type == "cuda" else self.dtype
-        src = ShardFolderSource(self.shards_path, cfg)
+        src = folder_source(self.shards_path, cfg)
         L = self.layer_num
-        self.shards = [StageEngine(cfg, i, i + 1, dev, dt, has_embed=(i == 0), has_head=(i == L - 1), source=src,
+        self.shards = [make_engine(cfg, i, i + 1, dev, dt, has_embed=(i == 0), has_head=(i == L - 1), source=src,
                                    max_seq=2048) for i in range(L)]
         tok = load_tokenizer(self.shards_path)
         ids = tok(request, return_tensors="pt")["input_ids"][0] if input_ids is None else input_ids.reshape(-1)

@@ -49,13 +49,13 @@ from typing import Optional
 
 import torch
 
-from ..config import LlamaConfig
 from ..models.rope import full_cos_sin
 from ..models.tokenizer import load_tokenizer
 from ..parallel import protocol
 from ..parallel.communicator import Again, Communicator
 from ..parallel.transport import PullSocket, PushSocket, local_ip
-from ..runtime.engine import DecodeGraph, ShardFolderSource, StageEngine, WeightSource
+from ..runtime.engine import DecodeGraph, StageEngine, WeightSource
+from ..runtime.registry import compute_dtype, folder_source, is_stack, load_config, make_engine
 from .forwarding_utils import build_position_ids  # noqa: F401 - re-exported as in the reference module
 
 
@@ -88,16 +88,14 @@ class NodeWorker:
         self.can_receive_user_request = can_receive_user_request
         self.shards_path = shards_path
         self.device = torch.device(device)
-        if self.device.type == "cuda" and dtype != torch.bfloat16:
-            if verbose:
-                _log(f"[INFO] {dtype} requested on {self.device}: the MI355X kernels compute in torch.bfloat16")
-            dtype = torch.bfloat16
-        self.dtype = dtype
-        self.config = LlamaConfig.from_pretrained(shards_path)
+        self.config = load_config(shards_path)
+        self.dtype = compute_dtype(self.config, self.device, dtype)
+        if self.dtype != dtype and verbose:
+            _log(f"[INFO] {dtype} requested on {self.device}: the MI355X kernels compute in {self.dtype}")
         self.layer_num = self.config.num_hidden_layers
         self.max_batch, self.max_seq = max_batch, max_seq
         self.noncausal_prefill = noncausal_prefill
-        self.source = source or ShardFolderSource(shards_path, self.config)
+        self.source = source or folder_source(shards_path, self.config)
         self.verbose = verbose
         self.ship_rope = ship_rope  # send real cos/sin tables in next_state_info (reference wire parity)
         # GPU decode steps (seq_len 1) replay a captured hipGraph of the stage (one per batch
@@ -142,7 +140,7 @@ class NodeWorker:
             torch.cuda.empty_cache()
         if self.verbose:
             _log(f"[INFO] loading hidden layer {start}~{end}(end excluded)...")
-        self.engine = StageEngine(self.config, start, end, self.device, self.dtype,
+        self.engine = make_engine(self.config, start, end, self.device, self.dtype,
                                   has_embed=False, has_head=(end == self.layer_num), source=self.source,
                                   max_slots=self.max_batch, max_seq=self.max_seq,
                                   causal=not self.noncausal_prefill)
@@ -156,6 +154,9 @@ class NodeWorker:
     # ------------------------------------------------------------------ helpers
     def _embed(self, ids: torch.Tensor) -> torch.Tensor:
         ids = ids.to(self.device)
+        if is_stack(self.config):  # the fp32 stream, scaled
+            from ..runtime.stack_engine import embed_rows
+            return embed_rows(self.config, self.embed_tokens, ids.reshape(-1)).reshape(*ids.shape, -1)
         if self.device.type == "cuda":
             from ..ops import hip
             flat = ids.reshape(-1).to(torch.int32)
@@ -216,7 +217,7 @@ class NodeWorker:
         else:
             slot, pos = eng.prefill_rows(slots, [S] * B)
             kv_len = [past + S] * (B * S) if (self.noncausal_prefill and S > 1) else None
-            h = eng.forward(hs.reshape(B * S, H).to(self.device, eng.dtype), slot, pos, kv_len=kv_len)
+            h = eng.forward(hs.reshape(B * S, H).to(self.device, eng.hidden_dtype), slot, pos, kv_len=kv_len)
             eng.advance(slots, [S] * B)
             out = eng.head(h, [b * S + S - 1 for b in range(B)]) if self.end == self.layer_num else h
         if self.end == self.layer_num:
@@ -251,7 +252,7 @@ class NodeWorker:
         want = [int(eng.seq_len[r]) for r in range(B)]
         if self._graph_pos[B] != want:
             g.set_positions()
-        g.h_in.copy_(hs.reshape(B, H).to(self.device, eng.dtype))
+        g.h_in.copy_(hs.reshape(B, H).to(self.device, eng.hidden_dtype))
         g.replay()
         eng.advance(list(range(B)), [1] * B)
         self._graph_pos[B] = [p + 1 for p in want]
@@ -480,8 +481,8 @@ class NodeController:
         if self.node_worker is not None:
             self.node_worker.close()
             self.node_worker = None
-        mcfg = LlamaConfig.from_pretrained(self.shards_path)
-        source = ShardFolderSource(self.shards_path, mcfg)
+        mcfg = load_config(self.shards_path)
+        source = folder_source(self.shards_path, mcfg)
         ctrl = dist.new_group(backend="gloo")  # rank 0's command headers (never blocks a GPU)
         self.server = PipelineServer(mcfg, source, r, n, int(cfg["shards_start"]), int(cfg["shards_end"]),
                                      self.device, batch=int(cfg.get("batch", 8)),

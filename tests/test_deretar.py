@@ -159,6 +159,47 @@ def test_pipeline_generates(model):
         assert out.permute(1, 2, 0).reshape(4, -1)[i].tolist() == want, gaps  # out: [new, micro-batch, row]
 
 
+def test_reference_style_chain(tmp_path, model):
+    """Two nodes of the TCP chain (ingress + head) pass one request through by hand."""
+    import socket
+
+    from llm_sharding_amd.utils.node_worker import NodeWorker
+    cfg, t = model
+    folder = D.write_random_checkpoint(cfg, str(tmp_path / "m"), seed=0)
+    ports = []
+    for _ in range(2):
+        with socket.socket() as sk:
+            sk.bind(("127.0.0.1", 0))
+            ports.append(sk.getsockname()[1])
+    nodes = [NodeWorker(f"tcp://*:{ports[i]}", f"tcp://127.0.0.1:{ports[1 - i]}", i == 0, folder, dtype=torch.float32,
+                        max_batch=1, max_seq=128, verbose=False) for i in range(2)]
+    try:
+        nodes[0].load_shards(0, 2)
+        nodes[1].load_shards(2, 6)
+        prompt = _ids(9, seed=6)
+        want, _ = P.greedy(cfg.to_dict(), t, prompt, 4)
+        state = nodes[0].receive_user_request(input_ids=torch.tensor([prompt]))
+        got = []
+        for _ in range(4):
+            tok = nodes[1].pass_through_shard(nodes[0].pass_through_shard(state))
+            got.append(int(tok))
+            _, state = nodes[0].receive_next_token(tok)
+        assert got == want
+    finally:
+        for n in nodes:
+            n.close()
+
+
+def test_placement_knows_the_layers():
+    from llm_sharding_amd.parallel.scheduler import kv_slots_for_memory, plan_stages, scratch_bytes, stage_memory
+    cfg = get_preset("deretar-4k")
+    plan = plan_stages(cfg, 4, kv_tokens=4096 * 32)
+    assert [s.n_layers for s in plan.stages] == [8, 8, 8, 8]
+    assert kv_slots_for_memory(cfg, 8, 4096, 288e9, plan.stages[0].weight_bytes) == 128
+    m = stage_memory(cfg, 8, slots=32, max_seq=4096, prefill_rows=2048)
+    assert m["kv"] == 8 * 32 * 4096 * 576 * 2 and m["scratch"] == scratch_bytes(cfg, 2048)
+
+
 def test_trace_replay_needs_a_gpu(tmp_path):
     if torch.cuda.is_available():
         pytest.skip("a GPU is there")

@@ -470,6 +470,29 @@ def test_graph_replays_equal_eager_steps(ordinary):
         g.tokens.copy_(tok)
 
 
+def test_stages_on_one_gpu(ordinary):
+    """Two and three pipeline stages (split head, captured graphs, fp32 stream between them) give the
+    single engine's tokens."""
+    from llm_sharding_amd.parallel.pipeline import drive_local_pipeline, run_pipeline_generate
+    from llm_sharding_amd.config import get_preset
+    cfg = get_preset("tiny-deretar")
+    src = M.NamedSource(cfg, 3)
+    prompts = torch.randint(3, cfg.vocab_size, (2, 2, 70), generator=_gen(4))
+    kw = dict(batch=2, microbatches=2, max_seq=128, dtype=F32)
+    one = run_pipeline_generate(cfg, src, prompts, 6, 0, 1, device=DEV, **kw)
+    want, _ = P.greedy(cfg.to_dict(), M.tensors(cfg, 3), prompts[1, 0].tolist(), 6)
+    assert one[:, 1, 0].tolist() == want
+    for n in (2, 3):
+        assert torch.equal(drive_local_pipeline(cfg, src, prompts, 6, n, DEV, **kw), one), n
+
+
+def test_stage_costs_are_measured(ordinary):
+    from llm_sharding_amd.utils.node_profiler import profile_stage_costs
+    cfg, _ = ordinary
+    r = profile_stage_costs(cfg, M.NamedSource(cfg, 0), DEV, batch=2, context=70, n_layers=3, prefill_len=80, replays=4)
+    assert r["layer_decode_ms"] > 0 and r["layer_prefill_ms"] > 0
+
+
 def test_trace_replay(ordinary, tmp_path):
     cfg, _ = ordinary
     folder = D.write_random_checkpoint(cfg, str(tmp_path / "m"), seed=0)
