@@ -40,78 +40,91 @@ LSA_DEVICE void block_sum2(float& a, float& b, float (*part)[4]) {
   b = part[1][0] + part[1][1] + part[1][2] + part[1][3];
 }
 
-LSA_DEVICE void ld8(const float* p, float* f) {
-#pragma unroll
-  for (int k = 0; k < 8; ++k) f[k] = p[k];
-}
-LSA_DEVICE void ld8(const bf16_raw* p, float* f) { unpack8(ld16(p), f); }
-LSA_DEVICE void st8(float* p, const float* f) {
-#pragma unroll
-  for (int k = 0; k < 8; ++k) p[k] = f[k];
-}
-LSA_DEVICE void st8(bf16_raw* p, const float* f) { st16(p, pack8(f)); }
-
-// in: row of the fused input projection, query latent at column oq, [key latent | rotated part] at
-// ok. VEC: 8 values at a time (ranks and offsets multiples of 8), the first of a thread's stretches
-// kept in registers between the sums and the scaling.
-template <typename T, bool VEC>
+// in: row of the fused input projection, query latent at column oq, [key latent | rotated part] at ok
+template <typename T>
 __global__ __launch_bounds__(256) void append_kernel(LatentArgs a, const T* __restrict__ in, int ldi, int oq, int ok,
                                                      const float* __restrict__ gq, const float* __restrict__ gk,
                                                      T* __restrict__ cq, int ldc) {
   __shared__ float part[2][4];
-  constexpr int S = VEC ? 8 : 1;
   const int row = blockIdx.x, tid = threadIdx.x;
   const T* q = in + (size_t)row * ldi + oq;
   const T* k = in + (size_t)row * ldi + ok;
-  const int nq = a.q_rank / S, n = nq + a.kv_rank / S;  // stretches of both latents
-  float sq = 0.f, sk = 0.f, first[S];
-  auto load = [&](int c, float* f) {
-    const T* src = c < nq ? q + c * S : k + (c - nq) * S;
-    if constexpr (VEC) ld8(src, f);
-    else f[0] = ld1(src);
-  };
-  for (int c = tid; c < n; c += 256) {
-    float f[S], ss = 0.f;
-    load(c, f);
-#pragma unroll
-    for (int j = 0; j < S; ++j) {
-      ss += f[j] * f[j];
-      if (c == tid) first[j] = f[j];
-    }
-    if (c < nq) sq += ss;
-    else sk += ss;
+  float sq = 0.f, sk = 0.f;
+  for (int c = tid; c < a.q_rank; c += 256) {
+    const float v = ld1(q + c);
+    sq += v * v;
   }
-  const bool live = lat_keys(a, row) > 0;  // uniform over the workgroup
-  const int p = a.pos[row];
-  T* dst = nullptr;
-  if (live) {
-    dst = static_cast<T*>(a.cache) +
-          ((size_t)lat_page(a, a.slot[row], p / LAT_PAGE) * LAT_PAGE + p % LAT_PAGE) * (a.krp + a.rp);
-    for (int c = tid; c < a.rp; c += 256) st1(dst + a.krp + c, c < a.rot_dim ? lat_rot(a, k + a.kv_rank, c, p) : 0.f);
+  for (int c = tid; c < a.kv_rank; c += 256) {
+    const float v = ld1(k + c);
+    sk += v * v;
   }
   block_sum2(sq, sk, part);
   const float rq = 1.f / sqrtf(sq / (float)a.q_rank + a.eps), rk = 1.f / sqrtf(sk / (float)a.kv_rank + a.eps);
-  for (int c = tid; c < n; c += 256) {
-    float f[S];
-    if (c == tid) {
+  for (int c = tid; c < a.q_rank; c += 256) st1(cq + (size_t)row * ldc + c, ld1(q + c) * rq * gq[c]);
+  if (lat_keys(a, row) == 0) return;  // uniform over the workgroup
+  const int p = a.pos[row];
+  T* dst = static_cast<T*>(a.cache) +
+           ((size_t)lat_page(a, a.slot[row], p / LAT_PAGE) * LAT_PAGE + p % LAT_PAGE) * (a.krp + a.rp);
+  for (int c = tid; c < a.krp; c += 256) st1(dst + c, c < a.kv_rank ? ld1(k + c) * rk * gk[c] : 0.f);
+  for (int c = tid; c < a.rp; c += 256) st1(dst + a.krp + c, c < a.rot_dim ? lat_rot(a, k + a.kv_rank, c, p) : 0.f);
+}
+
+// The same in bf16 with one wave per row (no barrier), both latents in registers: NV stretches of 8
+// values per lane (ranks and column offsets multiples of 8, (q_rank + kv_rank) / 8 <= 64 NV).
+template <int NV>
+__global__ __launch_bounds__(256) void append_wave_kernel(LatentArgs a, int rows, const bf16_raw* __restrict__ in, int ldi,
+                                                          int oq, int ok, const float* __restrict__ gq,
+                                                          const float* __restrict__ gk, bf16_raw* __restrict__ cq, int ldc) {
+  const int row = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (row >= rows) return;
+  const bf16_raw* q = in + (size_t)row * ldi + oq;
+  const bf16_raw* k = in + (size_t)row * ldi + ok;
+  const int nq = a.q_rank / 8, n = nq + a.kv_rank / 8;
+  u32x4_t v[NV];
 #pragma unroll
-      for (int j = 0; j < S; ++j) f[j] = first[j];
-    } else {
-      load(c, f);
-    }
-    const bool isq = c < nq;
-    const int o = (isq ? c : c - nq) * S;
-    const float* g = (isq ? gq : gk) + o;
-    const float r = isq ? rq : rk;
-#pragma unroll
-    for (int j = 0; j < S; ++j) f[j] *= r * g[j];
-    if (!isq && !live) continue;
-    T* d = isq ? cq + (size_t)row * ldc + o : dst + o;
-    if constexpr (VEC) st8(d, f);
-    else st1(d, f[0]);
+  for (int j = 0; j < NV; ++j) {
+    const int c = lane + 64 * j;
+    v[j] = c < n ? ld16(c < nq ? q + c * 8 : k + (c - nq) * 8) : u32x4_t{0u, 0u, 0u, 0u};
   }
-  if (live)
-    for (int c = a.kv_rank + tid; c < a.krp; c += 256) st1(dst + c, 0.f);
+  const int p = a.pos[row];
+  bf16_raw* dst = nullptr;
+  if (lat_keys(a, row) > 0) {  // uniform over the wave
+    dst = static_cast<bf16_raw*>(a.cache) +
+          ((size_t)lat_page(a, a.slot[row], p / LAT_PAGE) * LAT_PAGE + p % LAT_PAGE) * (a.krp + a.rp);
+    for (int c = lane; c < a.rp; c += 64) st1(dst + a.krp + c, c < a.rot_dim ? lat_rot(a, k + a.kv_rank, c, p) : 0.f);
+    for (int c = a.kv_rank + lane; c < a.krp; c += 64) st1(dst + c, 0.f);
+  }
+  float sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    float f[8], s = 0.f;
+    unpack8(v[j], f);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) s += f[i] * f[i];
+    if (lane + 64 * j < nq) sq += s;
+    else sk += s;
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  const float rq = 1.f / sqrtf(sq / (float)a.q_rank + a.eps), rk = 1.f / sqrtf(sk / (float)a.kv_rank + a.eps);
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = lane + 64 * j;
+    const bool isq = c < nq;
+    if (c >= n || (!isq && !dst)) continue;
+    const int o = (isq ? c : c - nq) * 8;
+    const float* g = (isq ? gq : gk) + o;
+    const f32x4_t g0 = *reinterpret_cast<const f32x4_t*>(g), g1 = *reinterpret_cast<const f32x4_t*>(g + 4);
+    const float r = isq ? rq : rk;
+    float f[8];
+    unpack8(v[j], f);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      f[i] *= r * g0[i];
+      f[4 + i] *= r * g1[i];
+    }
+    st16(isq ? cq + (size_t)row * ldc + o : dst + o, pack8(f));
+  }
 }
 
 // wk: [heads][dkp][krp] (row d = the key's dimension d); qt: [entries][heads][krp + rp]
@@ -239,13 +252,19 @@ extern "C" int lsa_latent_append(int f32, const LatentArgs* a, int rows, const v
   if (!args_ok(a, rows) || a->index || oq < 0 || ok < 0 || ldi < oq + a->q_rank || ldi < ok + a->kv_rank + a->rot_dim ||
       ldc < a->q_rank)
     return LSA_BAD_SHAPE;
-  const bool vec = !f32 && !((a->q_rank | a->kv_rank | oq | ok | ldi | ldc) % 8) && !(((uintptr_t)in | (uintptr_t)cq) % 16);
-  if (f32)
-    append_kernel<float, false><<<rows, 256, 0, s>>>(*a, (const float*)in, ldi, oq, ok, gq, gk, (float*)cq, ldc);
-  else if (vec)
-    append_kernel<bf16_raw, true><<<rows, 256, 0, s>>>(*a, (const bf16_raw*)in, ldi, oq, ok, gq, gk, (bf16_raw*)cq, ldc);
-  else
-    append_kernel<bf16_raw, false><<<rows, 256, 0, s>>>(*a, (const bf16_raw*)in, ldi, oq, ok, gq, gk, (bf16_raw*)cq, ldc);
+  const int n8 = (a->q_rank + a->kv_rank) / 8;
+  const bool wave = !f32 && n8 <= 512 && !((a->q_rank | a->kv_rank | oq | ok | ldi | ldc) % 8) &&
+                    !(((uintptr_t)in | (uintptr_t)cq | (uintptr_t)gq | (uintptr_t)gk) % 16);
+  const int wpg = rows >= 2048 ? 4 : 1;  // few rows: one to a CU
+#define LSA_W(NV)                                                                                                  \
+  append_wave_kernel<NV><<<(rows + wpg - 1) / wpg, wpg * 64, 0, s>>>(*a, rows, (const bf16_raw*)in, ldi, oq, ok,  \
+                                                                    gq, gk, (bf16_raw*)cq, ldc)
+  if (wave && n8 <= 128) LSA_W(2);
+  else if (wave && n8 <= 320) LSA_W(5);
+  else if (wave) LSA_W(8);
+  else if (f32) append_kernel<float><<<rows, 256, 0, s>>>(*a, (const float*)in, ldi, oq, ok, gq, gk, (float*)cq, ldc);
+  else append_kernel<bf16_raw><<<rows, 256, 0, s>>>(*a, (const bf16_raw*)in, ldi, oq, ok, gq, gk, (bf16_raw*)cq, ldc);
+#undef LSA_W
   LSA_CHECK_LAUNCH();
   return LSA_OK;
 }

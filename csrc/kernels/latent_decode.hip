@@ -315,20 +315,14 @@ __global__ __launch_bounds__(512) void value_mfma_kernel(LatentArgs a, int n, co
 #pragma unroll
     for (int kf = 0; kf < KF; ++kf) wf[kf] = ld16(wh + (size_t)kf * 512);
   }
-  if (ns > 1 && tid < 16) {
-    const int e = e0 + tid;
-    if (e < n) {
-      const float* p = pm + ((size_t)e * a.heads + h) * ns * 2;
-      float M = -INFINITY, L = 0.f;
-      for (int s = 0; s < ns; ++s) M = fmaxf(M, p[2 * s]);
+  if (ns > 1) {  // weights of the splits (ns <= 64): a wave per entry, a lane per split
+    for (int r = w; r < 16 && e0 + r < n; r += 8) {
+      const float* p = pm + ((size_t)(e0 + r) * a.heads + h) * ns * 2;
+      const float m = lane < ns ? p[2 * lane] : -INFINITY, l = lane < ns ? p[2 * lane + 1] : 0.f;
+      float M = wave_max(m);
       if (M == -INFINITY) M = 0.f;
-      for (int s = 0; s < ns; ++s) {
-        const float f = __builtin_amdgcn_exp2f(p[2 * s] - M);
-        wgt[tid][s] = f;
-        L += p[2 * s + 1] * f;
-      }
-      const float inv = L > 0.f ? 1.f / L : 0.f;
-      for (int s = 0; s < ns; ++s) wgt[tid][s] *= inv;
+      const float f = __builtin_amdgcn_exp2f(m - M), L = wave_sum(l * f);
+      wgt[r][lane] = L > 0.f ? f / L : 0.f;
     }
   }
   __syncthreads();
@@ -343,14 +337,13 @@ __global__ __launch_bounds__(512) void value_mfma_kernel(LatentArgs a, int n, co
         v = *reinterpret_cast<const f32x4_t*>(p) * (L > 0.f ? 1.f / L : 0.f);
       } else {
         int s = 0;
-        for (; s + 4 <= ns; s += 4) {
-          f32x4_t x[4];
+        for (; s < ns; s += 8) {  // eight reads in flight (past the last split: its value again, times 0)
+          f32x4_t x[8];
 #pragma unroll
-          for (int u = 0; u < 4; ++u) x[u] = *reinterpret_cast<const f32x4_t*>(p + (size_t)(s + u) * KRP);
+          for (int u = 0; u < 8; ++u) x[u] = *reinterpret_cast<const f32x4_t*>(p + (size_t)min(s + u, ns - 1) * KRP);
 #pragma unroll
-          for (int u = 0; u < 4; ++u) v += x[u] * wgt[r][s + u];
+          for (int u = 0; u < 8; ++u) v += x[u] * (s + u < ns ? wgt[r][s + u] : 0.f);
         }
-        for (; s < ns; ++s) v += *reinterpret_cast<const f32x4_t*>(p + (size_t)s * KRP) * wgt[r][s];
       }
     }
     st4(so + r * LD + c, v);

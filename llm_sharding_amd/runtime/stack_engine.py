@@ -181,7 +181,7 @@ class StackEngine(StageEngine):
     def _projections(self) -> list:
         out = []
         for l in self.layers:
-            out += [(p.n, p.k, False) for p in (l.mixer.inp, l.mixer.uq, l.mixer.out)]
+            out += [(p.n, p.k, False) for p in (l.mixer.inp, l.mixer.uq, l.mixer.out, l.mixer.kv) if p is not None]
             if l.mlp is not None:
                 out += [(l.mlp.gate_up.n, l.mlp.gate_up.k, True), (l.mlp.down.n, l.mlp.down.k, False)]
         if self.has_head:

@@ -278,9 +278,10 @@ def test_expanded_attention(name):
 
 
 @pytest.mark.parametrize("dtype", [BF, F32])
-def test_append_norms_turns_and_places(dtype):
+@pytest.mark.parametrize("name", ["small", "two_tiles", "r128", "r512", "wave_wide"])
+def test_append_norms_turns_and_places(dtype, name):
     from llm_sharding_amd.ops import latent as L
-    s = SIZES["small"]
+    s = LatentSpec(2, 32, 16, 32, 504, 3080, 1e4, 16, 0.2) if name == "wave_wide" else SIZES[name]
     case = Case(s, [130, 70], dtype)
     slot, pos = [0, 1, 0, 0, 1], [129, 64, 63, 0, 127]
     w = case.w
@@ -413,6 +414,19 @@ def test_other_sizes_and_values_that_often_coincide():
         eng = M.engine(cfg, DEV, dtype)
         got = torch.cat([M.feed(eng, [(0, p)]) for p in M.cut(ids, [100, 1, 49])])
         assert M.rel(got, want) < tol, dtype
+
+
+def test_layers_of_a_real_width():
+    """Wide heads and latents: portions on every projection kernel (1..16, 17..128, more rows), absorbed
+    and expanded attention, groups of heads."""
+    cfg = D.make_config(512, 260, [D.layer_entry(40, 128, 64, 128, 512, 256, ff=600),
+                                   D.layer_entry(16, 128, 64, 128, 256, 128)])
+    t = M.tensors(cfg)
+    ids = _ids(350, vocab=260)
+    want = P.run(cfg.to_dict(), t, ids, dtype=torch.float32)
+    eng = M.engine(cfg, DEV, BF)
+    got = torch.cat([M.feed(eng, [(0, p)]) for p in M.cut(ids, [100, 1, 20, 64, 129, 2, 34])])
+    assert M.rel(got, want) < TOL[BF]
 
 
 # ------------------------------------------------------------------------------ generation
