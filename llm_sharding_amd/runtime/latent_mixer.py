@@ -184,15 +184,13 @@ class Plan:
         self._cache: dict = {}
 
     @staticmethod
-    def find_runs(slot: list, pos: list) -> list:
-        runs, r, n = [], 0, len(slot)
-        while r < n:
-            e = r + 1
-            while e < n and slot[e] == slot[r] and pos[e] == pos[e - 1] + 1:
-                e += 1
-            runs.append((r, e - r, slot[r], pos[r]))
-            r = e
-        return runs
+    def find_runs(slot, pos) -> list:
+        """Stretches of one slot's consecutive positions in int64 tensors (host)."""
+        new = torch.ones(slot.numel(), dtype=torch.bool)
+        new[1:] = (slot[1:] != slot[:-1]) | (pos[1:] != pos[:-1] + 1)
+        at = new.nonzero().flatten()
+        ends = torch.cat([at[1:], torch.tensor([slot.numel()])])
+        return list(zip(at.tolist(), (ends - at).tolist(), slot[at].tolist(), pos[at].tolist()))
 
     def _split(self, w: Weights):
         key = w.spec if w.expand else None

@@ -312,19 +312,17 @@ class StackEngine(StageEngine):
         if kv_len is not None:
             raise ValueError("stack engines attend causally (no kv_len)")
         rows = h.shape[0]
-        sl, ps = ([int(v) for v in (t.tolist() if torch.is_tensor(t) else t)] for t in (slot, pos))
-        if len(sl) != rows or len(ps) != rows:
+        sl, ps = (torch.as_tensor(t, dtype=torch.int64).cpu().reshape(-1) for t in (slot, pos))
+        if sl.numel() != rows or ps.numel() != rows or rows < 1:
             raise ValueError("forward: one slot and one position per row")
-        if min(sl) < 0 or max(sl) >= self.max_slots or min(ps) < 0 or max(ps) >= self.max_seq:
+        if int(sl.min()) < 0 or int(sl.max()) >= self.max_slots or int(ps.min()) < 0 or int(ps.max()) >= self.max_seq:
             raise ValueError("forward: slot or position out of range")
-        need: dict = {}
-        for s, p in zip(sl, ps):
-            need[s] = max(need.get(s, 0), p + 1)
-        for s, n in need.items():
-            self.pool.ensure(s, n)
+        runs = Plan.find_runs(sl, ps)
+        for _, n, s, p in runs:
+            self.pool.ensure(s, p + n)
         if not self.gpu:
-            return self._forward_stack_torch(h, torch.tensor(sl), torch.tensor(ps))
-        return self._forward_hip(h, self._i32(sl), self._i32(ps), None, rows, runs=Plan.find_runs(sl, ps))
+            return self._forward_stack_torch(h, sl, ps)
+        return self._forward_hip(h, self._i32(sl), self._i32(ps), None, rows, runs=runs)
 
     def latent_nsplit(self, s, entries: int, longest: int) -> int:
         """Key splits of the absorbed attention: about one workgroup per CU (each fills a CU's
