@@ -107,7 +107,9 @@ struct Pull {
     if (it == conns.end()) return;
     Conn& c = it->second;
     char tmp[1 << 16];
-    for (;;) {
+    // a bounded burst, then back to epoll (level-triggered): a sender that never pauses must not
+    // hold its messages back, starve other connections or keep shutdown() waiting
+    for (int burst = 0; burst < 16 && !stop.load(); ++burst) {
       ssize_t n = ::recv(fd, tmp, sizeof(tmp), 0);
       if (n > 0) {
         c.buf.append(tmp, (size_t)n);
