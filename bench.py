@@ -402,7 +402,8 @@ def compare_designs(a) -> list:
                         eng.prefill_rows([s], [ctx])
                         eng.seq_len[s] = ctx
                     for c in eng.k_cache + eng.v_cache:
-                        c.normal_()
+                        if c is not None:
+                            c.normal_()
                     g = DecodeGraph(eng, n, "full").capture()
                     ms, tokens = timed(g.replay, 24, warm=4), n
                 rec = {"size": size, "design": kind, "point": point, "context": ctx, "layers": a.compare_layers,

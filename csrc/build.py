@@ -35,6 +35,8 @@ COOP_UNITS = tuple(range(8))
 FAMILIES = {
     "latent": ("elementwise.hip", "gemm_sk.hip", "gemv.hip", "gemv_coop.hip-0", "gemv_coop.hip-2", "gemv_coop.hip-4",
                "gemv_coop.hip-7", "latent", "linear_f32.hip", "stream_ops.hip"),
+    "hybrid": ("elementwise.hip", "gemm_sk.hip", "gemv.hip", "gemv_coop.hip-0", "gemv_coop.hip-4", "gemv_coop.hip-7",
+               "linear_f32.hip", "stream_ops.hip", "paged_attn", "delta", "moe"),
 }
 
 

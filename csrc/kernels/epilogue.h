@@ -2,7 +2,8 @@
 //
 // They replace separate elementwise launches of the reference's HF layer
 // (/root/reference/utils/shard_loader.py:66-74 -> LlamaDecoderLayer):
-//   EPI_STORE   y -> bf16 out (optionally act(y + bias): GPT-2 c_fc + gelu_new), or fp32 out32
+//   EPI_STORE   y -> bf16 out (optionally act(y + bias): GPT-2 c_fc + gelu_new), or fp32 out32, or some
+//               columns to either; or out32 += sigmoid(gate) * y (a result joins an fp32 stream)
 //   EPI_RESID   out = resid + y (+ bias)        (o_proj / down_proj + residual add)
 //   EPI_SWIGLU  out = silu(gate) * up           (gate/up fused GEMM, tiles interleaved), or the
 //               clipped GLU of glu() when glu_limit > 0
@@ -14,7 +15,7 @@
 //   EPI_ARGMAX  greedy argmax over the vocab via 64-bit atomicMax keys
 //               (lm_head + torch.argmax, node_worker.py:262-264, fused)
 #pragma once
-#include "common.h"
+#include "elem.h"
 
 // EPI_PARTIAL (gemm_sk only): every K-split workgroup stores its fp32 partial tile to
 // ((float*)out)[split][M][ldo]; the following norm kernel adds the partials to the residual
@@ -52,7 +53,25 @@ struct EpiArgs {
   float glu_alpha;          // SWIGLU with glu_limit > 0: see glu()
   float glu_limit;
   float glu_shift;
+  // STORE of several parts: columns from col32 on (a multiple of 16; 0 without ``out``) go to
+  // out32[m][n - col32] (rows of ldo32), act applies to columns of ``out`` from act_from on
+  const void* gate;         // STORE to out32 alone: out32[m][n] += sigmoid(gate[m][n]) * y for n < cols
+  int ldg;                  // (gate: bf16 in the bf16 GEMMs, fp32 in linear_f32)
+  int col32;
+  int ldo32;
+  int act_from;
+  int cols;
 };
+
+// Host check of an EPI_STORE product's outputs
+static inline bool bad_store(const EpiArgs& e, int N) {
+  if (!e.out && !e.out32) return true;
+  if (e.out && e.ldo < (e.out32 ? e.col32 : N)) return true;
+  if (!e.out32) return false;
+  if (e.col32 < 0 || e.col32 % 16 || e.col32 > N || (!e.out && e.col32)) return true;
+  if (e.gate) return e.out || e.act || e.cols < 1 || e.cols % 16 || e.cols > N || e.ldo32 < e.cols || e.ldg < e.cols;
+  return e.ldo32 < N - e.col32;
+}
 
 LSA_DEVICE float silu(float g) { return g / (1.0f + __expf(-g)); }
 
@@ -72,13 +91,23 @@ LSA_DEVICE float gelu_tanh(float x) {
   return 0.5f * x * (2.0f - 2.0f / (__expf(2.0f * u) + 1.0f));
 }
 
+// act applies to columns from act_from on, up to those that go to out32 beside out
+LSA_DEVICE bool epi_acts(const EpiArgs& ep, int col) { return col >= ep.act_from && !(ep.out && ep.out32 && col >= ep.col32); }
 LSA_DEVICE float epi_bias(const EpiArgs& ep, int col) { return ep.bias ? ep.bias[col] : 0.f; }
 // One finished element of an EPI_STORE GEMM
 LSA_DEVICE void epi_store1(const EpiArgs& ep, int m, int col, float v) {
   v += ep.bias ? ep.bias[col] : 0.f;
-  if (ep.act == 1) v = gelu_tanh(v);
-  if (ep.out32) ep.out32[(size_t)m * ep.ldo + col] = v;
-  else ep.out[(size_t)m * ep.ldo + col] = f2bf(v);
+  if (ep.act == 1 && epi_acts(ep, col)) v = gelu_tanh(v);
+  if (ep.out32 && col >= ep.col32) {
+    float* o = ep.out32 + (size_t)m * ep.ldo32 + (col - ep.col32);
+    if (ep.gate) {
+      if (col < ep.cols) *o += sigmoid(bf2f(((const bf16_raw*)ep.gate)[(size_t)m * ep.ldg + col])) * v;
+    } else {
+      *o = v;
+    }
+  } else {
+    ep.out[(size_t)m * ep.ldo + col] = f2bf(v);
+  }
 }
 LSA_DEVICE float epi_act(const EpiArgs& ep, float v) { return ep.act == 1 ? gelu_tanh(v) : v; }
 
@@ -223,12 +252,25 @@ LSA_DEVICE void epi_row16(const EpiArgs& ep, int m, int c0, float* v) {
   if (EPI == EPI_QKV) {
     epi_qkv_row16(ep, m, c0, v);
   } else if (EPI == EPI_STORE) {
-    if (ep.act == 1) {
+    if (ep.act == 1 && epi_acts(ep, c0)) {
 #pragma unroll
       for (int j = 0; j < 16; ++j) v[j] = gelu_tanh(v[j]);
     }
-    if (ep.out32) {
-      float* o32 = ep.out32 + (size_t)m * ep.ldo + c0;
+    if (ep.out32 && c0 >= ep.col32) {
+      float* o32 = ep.out32 + (size_t)m * ep.ldo32 + (c0 - ep.col32);
+      if (ep.gate) {
+        if (c0 >= ep.cols) return;
+        const bf16_raw* gp = (const bf16_raw*)ep.gate + (size_t)m * ep.ldg + c0;
+        float g[16];
+        unpack8(ld16(gp), g);
+        unpack8(ld16(gp + 8), g + 8);
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+          const f32x4_t o = *reinterpret_cast<const f32x4_t*>(o32 + 4 * q);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) v[4 * q + j] = o[j] + sigmoid(g[4 * q + j]) * v[4 * q + j];
+        }
+      }
 #pragma unroll
       for (int q = 0; q < 4; ++q)
         *reinterpret_cast<f32x4_t*>(o32 + 4 * q) = f32x4_t{v[4 * q], v[4 * q + 1], v[4 * q + 2], v[4 * q + 3]};

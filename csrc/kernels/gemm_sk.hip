@@ -795,6 +795,7 @@ extern "C" int lsa_gemm_sk(const void* a, int lda, const void* wp, int M, int N,
   if (ep->ss_out && (epi != EPI_RESID || bn == 192 || N % 64 || ep->ss_n != N / 64)) return LSA_BAD_SHAPE;
   if (ep->ss_in && ((epi != EPI_QKV && epi != EPI_SWIGLU) || ep->ss_n < 4 || ep->ss_n % 4 || K != 64 * ep->ss_n))
     return LSA_BAD_SHAPE;
+  if (epi == EPI_STORE && bad_store(*ep, N)) return LSA_BAD_SHAPE;
   if (epi == EPI_PARTIAL && (split < 1 || ep->ldo < N || ep->ldo % 4)) return LSA_BAD_SHAPE;
   SkParams prm;
   prm.M = M;

@@ -8,6 +8,19 @@ namespace {
 
 constexpr int TM = 64, TN = 64, TK = 16;
 
+// epi_store1 with fp32 in the place of bf16 (ep.out, ep.gate)
+LSA_DEVICE void store_f32(const EpiArgs& ep, int m, int n, float v) {
+  v += epi_bias(ep, n);
+  if (ep.act == 1 && epi_acts(ep, n)) v = gelu_tanh(v);
+  if (!ep.out32 || n < ep.col32) {
+    ((float*)ep.out)[(size_t)m * ep.ldo + n] = v;
+    return;
+  }
+  float* o = ep.out32 + (size_t)m * ep.ldo32 + (n - ep.col32);
+  if (!ep.gate) *o = v;
+  else if (n < ep.cols) *o += sigmoid(((const float*)ep.gate)[(size_t)m * ep.ldg + n]) * v;
+}
+
 template <bool GLU>
 __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict__ A, int lda,
                                                          const float* __restrict__ W, int M, int N, int K, EpiArgs ep) {
@@ -61,7 +74,7 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const int n = n0 + tx + 16 * j;
-        if (n < N) ep.out32[(size_t)m * ep.ldo + n] = acc[i][j] + epi_bias(ep, n);
+        if (n < N) store_f32(ep, m, n, acc[i][j]);
       }
     }
   }
@@ -71,14 +84,14 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict
 
 extern "C" int lsa_linear_f32(const float* a, int lda, const float* w, int M, int N, int K, int epi, const EpiArgs* ep,
                               hipStream_t stream) {
-  if (M < 1 || N < 1 || K < 16 || K % 16 || lda < K || lda % 4 || !ep || !ep->out32) return LSA_BAD_SHAPE;
+  if (M < 1 || N < 1 || K < 16 || K % 16 || lda < K || lda % 4 || !ep || !(ep->out32 || ep->out)) return LSA_BAD_SHAPE;
   if (((uintptr_t)a | (uintptr_t)w) % 16) return LSA_BAD_SHAPE;
   dim3 grid((N + TN - 1) / TN, (M + TM - 1) / TM);
   if (epi == EPI_SWIGLU) {
-    if (N % 32 || ep->ldo < N / 2) return LSA_BAD_SHAPE;
+    if (N % 32 || ep->ldo < N / 2 || !ep->out32) return LSA_BAD_SHAPE;
     linear_f32_kernel<true><<<grid, 256, 0, stream>>>(a, lda, w, M, N, K, *ep);
   } else if (epi == EPI_STORE) {
-    if (ep->ldo < N) return LSA_BAD_SHAPE;
+    if (bad_store(*ep, N)) return LSA_BAD_SHAPE;
     linear_f32_kernel<false><<<grid, 256, 0, stream>>>(a, lda, w, M, N, K, *ep);
   } else {
     return LSA_UNSUPPORTED;

@@ -1,0 +1,274 @@
+// Mixture of experts (moe.h): routing, grouping and the expert products (bf16 on MFMA, and plain fp32
+// for the fp32 engine).
+#include "moe.h"
+
+namespace {
+
+// one wave per row: ``top`` times the largest logit left (ties: the smaller index), softmax over them
+constexpr int MAX_E = 1024;
+__global__ __launch_bounds__(256) void route_kernel(const float* __restrict__ logits, int ldl, int rows, int E, int top,
+                                                    int* __restrict__ expert, float* __restrict__ weight) {
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (row >= rows) return;
+  const float* z = logits + (size_t)row * ldl;
+  float v[MAX_E / 64];
+#pragma unroll
+  for (int j = 0; j < MAX_E / 64; ++j) {
+    const int e = j * 64 + lane;
+    v[j] = e < E ? z[e] : 0.f;
+  }
+  unsigned taken = 0;  // bit j: this lane's logit j is chosen
+  float first = 0.f, sum = 0.f, mine = 0.f;
+  for (int k = 0; k < top; ++k) {
+    unsigned long long best = 0ull;
+#pragma unroll
+    for (int j = 0; j < MAX_E / 64; ++j) {
+      const int e = j * 64 + lane;
+      if (e < E && !(taken >> j & 1)) {
+        const unsigned long long key = argmax_key(v[j], (unsigned)e);
+        best = key > best ? key : best;
+      }
+    }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const unsigned long long x = __shfl_xor(best, o, 64);
+      best = x > best ? x : best;
+    }
+    const int e = min((int)argmax_key_index(best), E - 1);
+    const float val = z[e];
+    if ((e & 63) == lane) taken |= 1u << (e >> 6);
+    if (k == 0) first = val;
+    const float w = expf(val - first);
+    sum += w;
+    if (lane == (k & 63)) mine = w;
+    if (lane == 0) expert[(size_t)row * top + k] = e;
+    if ((k & 63) == 63 || k == top - 1) {  // unnormalised; the sum is known at the end
+      const int kk = (k & ~63) + lane;
+      if (kk <= k) weight[(size_t)row * top + kk] = mine;
+    }
+  }
+  const float inv = 1.f / sum;
+  for (int k = lane; k < top; k += 64) weight[(size_t)row * top + k] *= inv;  // this lane's own stores
+}
+
+// one workgroup: counting sort of the pairs by expert, and the tile table
+__global__ __launch_bounds__(1024) void group_kernel(const int* __restrict__ expert, int pairs, int E, int tile_rows,
+                                                     int max_tiles, int* __restrict__ order, int* __restrict__ place,
+                                                     MoeTile* __restrict__ tiles) {
+  __shared__ int s_cnt[MAX_E], s_off[MAX_E], s_tile[MAX_E], s_n[1], s_w[2][16];
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+  s_cnt[tid] = 0;
+  __syncthreads();
+  for (int i = tid; i < pairs; i += 1024) place[i] = atomicAdd(&s_cnt[expert[i]], 1);  // rank within its expert
+  __syncthreads();
+  // exclusive sums over experts of pairs and of tiles
+  const int c = tid < E ? s_cnt[tid] : 0, nt = (c + tile_rows - 1) / tile_rows;
+  int a = c, b = nt;
+#pragma unroll
+  for (int o = 1; o < 64; o <<= 1) {
+    const int x = __shfl_up(a, o, 64), y = __shfl_up(b, o, 64);
+    if (lane >= o) {
+      a += x;
+      b += y;
+    }
+  }
+  if (lane == 63) {
+    s_w[0][w] = a;
+    s_w[1][w] = b;
+  }
+  __syncthreads();
+  int ba = 0, bb = 0;
+  for (int x = 0; x < w; ++x) {
+    ba += s_w[0][x];
+    bb += s_w[1][x];
+  }
+  s_off[tid] = ba + a - c;
+  s_tile[tid] = bb + b - nt;
+  if (tid == 1023) s_n[0] = bb + b;
+  __syncthreads();
+  if (tid < E)
+    for (int t = 0; t < nt; ++t)
+      if (s_tile[tid] + t < max_tiles)
+        tiles[s_tile[tid] + t] = MoeTile{tid, s_off[tid] + t * tile_rows, min(tile_rows, c - t * tile_rows), 0};
+  for (int t = s_n[0] + tid; t < max_tiles; t += 1024) tiles[t] = MoeTile{-1, 0, 0, 0};
+  for (int i = tid; i < pairs; i += 1024) {  // this thread's own ranks
+    const int at = s_off[expert[i]] + place[i];
+    place[i] = at;
+    order[at] = i;
+  }
+}
+
+// One tile of MT x 16 pairs x 64 columns of one expert's product; four waves share K and meet in LDS.
+// GLU: the columns are gate / up 16-tiles in turn and the output is silu(gate) * up (32 columns);
+// the rows of A are then the pairs' rows of h, else the sorted pairs themselves.
+template <int MT, bool GLU>
+__global__ __launch_bounds__(256) void moe_small_kernel(const MoeTile* __restrict__ tiles, const int* __restrict__ order,
+                                                        int top, const bf16_raw* __restrict__ A, int lda,
+                                                        const bf16_raw* __restrict__ W, int N, int K,
+                                                        bf16_raw* __restrict__ out, int ldo) {
+  constexpr int NT = 4;
+  __shared__ __attribute__((aligned(16))) float s_acc[4][MT * 16][NT * 16 + 4];
+  const MoeTile tile = tiles[blockIdx.y];
+  if (tile.expert < 0) return;
+  const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, q4 = lane >> 4;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int nt0 = blockIdx.x * NT, KT = K / 32, ntn = min(NT, N / 16 - nt0);
+  const bf16_raw* ar[MT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+    const int i = tile.start + min(m * 16 + l16, tile.count - 1);  // rows past the count are not stored
+    ar[m] = A + (size_t)(GLU ? order[i] / top : i) * lda + q4 * 8;
+  }
+  const bf16_raw* wp = W + (size_t)tile.expert * N * K + ((size_t)nt0 * KT * 64 + lane) * 8;
+  f32x4_t acc[MT][NT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int n = 0; n < NT; ++n) acc[m][n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const int k1 = KT * (w + 1) / 4;
+#pragma unroll 4
+  for (int kt = KT * w / 4; kt < k1; ++kt) {
+    u32x4_t b[NT], x[MT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) b[n] = ld16(wp + ((size_t)min(n, ntn - 1) * KT + kt) * 512);
+#pragma unroll
+    for (int m = 0; m < MT; ++m) x[m] = ld16(ar[m] + kt * 32);
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+      for (int n = 0; n < NT; ++n) acc[m][n] = mfma16(x[m], b[n], acc[m][n]);
+  }
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int n = 0; n < NT; ++n)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) s_acc[w][m * 16 + q4 * 4 + r][n * 16 + l16] = acc[m][n][r];
+  __syncthreads();
+  const int cols = GLU ? ntn * 8 : ntn * 16;  // output columns of this workgroup
+  for (int t = tid; t < tile.count * (cols / 4); t += 256) {
+    const int m = t / (cols / 4), c = (t % (cols / 4)) * 4;
+    f32x4_t v = {0.f, 0.f, 0.f, 0.f}, u = {0.f, 0.f, 0.f, 0.f};
+    const int cc = GLU ? (c / 16) * 32 + c % 16 : c;
+#pragma unroll
+    for (int x = 0; x < 4; ++x) {
+      v += *reinterpret_cast<const f32x4_t*>(&s_acc[x][m][cc]);
+      if (GLU) u += *reinterpret_cast<const f32x4_t*>(&s_acc[x][m][cc + 16]);
+    }
+    if (GLU)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = v[j] / (1.f + __expf(-v[j])) * u[j];
+    st4(out + (size_t)(tile.start + m) * ldo + (GLU ? nt0 * 8 : nt0 * 16) + c, v);
+  }
+}
+
+// true fp32: tiles of at most 64 pairs x 64 columns, 16-deep K steps through LDS (as linear_f32.hip)
+template <bool GLU>
+__global__ __launch_bounds__(256) void moe_f32_kernel(const MoeTile* __restrict__ tiles, const int* __restrict__ order,
+                                                      int top, const float* __restrict__ A, int lda,
+                                                      const float* __restrict__ W, int N, int K,
+                                                      float* __restrict__ out, int ldo) {
+  __shared__ float sa[16][68], sw[16][68];
+  const MoeTile tile = tiles[blockIdx.y];
+  if (tile.expert < 0) return;
+  const int tid = threadIdx.x, n0 = blockIdx.x * 64, tx = tid & 15, ty = tid >> 4, lr = tid >> 2, lk = (tid & 3) * 4;
+  float acc[4][4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = 0.f;
+  const int at = tile.start + min(lr, tile.count - 1);
+  const float* ar = A + (size_t)(GLU ? order[at] / top : at) * lda;
+  const float* wr = W + ((size_t)tile.expert * N + min(n0 + lr, N - 1)) * K;
+  for (int k0 = 0; k0 < K; k0 += 16) {
+    const f32x4_t x = *reinterpret_cast<const f32x4_t*>(ar + k0 + lk);
+    const f32x4_t y = *reinterpret_cast<const f32x4_t*>(wr + k0 + lk);
+    __syncthreads();
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      sa[lk + q][lr] = x[q];
+      sw[lk + q][lr] = y[q];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < 16; ++k) {
+      float av[4], wv[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        av[i] = sa[k][ty + 16 * i];
+        wv[i] = sw[k][tx + 16 * i];
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = fmaf(av[i], wv[j], acc[i][j]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int m = ty + 16 * i;
+    if (m >= tile.count) continue;
+    float* o = out + (size_t)(tile.start + m) * ldo;
+    if constexpr (GLU) {
+#pragma unroll
+      for (int p = 0; p < 2; ++p) {
+        const int c = n0 + 32 * p;
+        const float g = acc[i][2 * p];
+        if (c < N) o[c / 2 + tx] = g / (1.f + expf(-g)) * acc[i][2 * p + 1];
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (n0 + tx + 16 * j < N) o[n0 + tx + 16 * j] = acc[i][j];
+    }
+  }
+}
+
+}  // namespace
+
+extern "C" int lsa_moe_route(const float* logits, int ldl, int rows, int E, int top, int* expert, float* weight,
+                             hipStream_t s) {
+  if (rows < 1 || E < 1 || E > MAX_E || top < 1 || top > E || ldl < E) return LSA_BAD_SHAPE;
+  route_kernel<<<(rows + 3) / 4, 256, 0, s>>>(logits, ldl, rows, E, top, expert, weight);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+// max_tiles >= min(E, pairs) + pairs / tile_rows
+extern "C" int lsa_moe_group(const int* expert, int pairs, int E, int tile_rows, int max_tiles, int* order, int* place,
+                             void* tiles, hipStream_t s) {
+  if (pairs < 1 || E < 1 || E > MAX_E || tile_rows < 1 || max_tiles < (E < pairs ? E : pairs) + pairs / tile_rows)
+    return LSA_BAD_SHAPE;
+  group_kernel<<<1, 1024, 0, s>>>(expert, pairs, E, tile_rows, max_tiles, order, place, (MoeTile*)tiles);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+// up (glu = 1): A = h rows, out [pairs][ldo >= N / 2]; down: A = act [pairs], out [pairs][ldo >= N]
+extern "C" int lsa_moe_gemm(int f32, int glu, const void* tiles, int max_tiles, int tile_rows, const int* order, int top,
+                            const void* A, int lda, const void* W, int N, int K, void* out, int ldo, hipStream_t s) {
+  if (max_tiles < 1 || max_tiles > 65535 || top < 1 || N < 32 || N % 32 || K < 32 || K % 32 || lda < K || lda % 8 ||
+      ldo < (glu ? N / 2 : N) || ldo % 4 || ((uintptr_t)A | (uintptr_t)W | (uintptr_t)out) % 16)
+    return LSA_BAD_SHAPE;
+  const dim3 grid((N + 63) / 64, max_tiles);
+  const MoeTile* t = (const MoeTile*)tiles;
+  if (f32) {
+    if (tile_rows > 64) return LSA_UNSUPPORTED;
+    if (glu) moe_f32_kernel<true><<<grid, 256, 0, s>>>(t, order, top, (const float*)A, lda, (const float*)W, N, K, (float*)out, ldo);
+    else moe_f32_kernel<false><<<grid, 256, 0, s>>>(t, order, top, (const float*)A, lda, (const float*)W, N, K, (float*)out, ldo);
+    LSA_CHECK_LAUNCH();
+    return LSA_OK;
+  }
+#define LSA_M(MT)                                                                                                       \
+  if (tile_rows == MT * 16) {                                                                                           \
+    if (glu) moe_small_kernel<MT, true><<<grid, 256, 0, s>>>(t, order, top, (const bf16_raw*)A, lda, (const bf16_raw*)W, \
+                                                             N, K, (bf16_raw*)out, ldo);                                \
+    else moe_small_kernel<MT, false><<<grid, 256, 0, s>>>(t, order, top, (const bf16_raw*)A, lda, (const bf16_raw*)W, N, \
+                                                          K, (bf16_raw*)out, ldo);                                      \
+    LSA_CHECK_LAUNCH();                                                                                                 \
+    return LSA_OK;                                                                                                      \
+  }
+  LSA_M(1) LSA_M(2) LSA_M(4)
+#undef LSA_M
+  return LSA_UNSUPPORTED;
+}

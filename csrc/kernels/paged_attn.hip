@@ -1,0 +1,206 @@
+// Paged grouped-query attention (paged_attn.h): cache append, the merge of key splits, and a plain
+// kernel for any size and both types (the fp32 engine; head parts above 256).
+#include "paged_attn.h"
+
+namespace {
+
+// ---- append: one workgroup per row (decoded tokens)
+template <typename T>
+__global__ __launch_bounds__(256) void append_rows_kernel(AttnArgs a, const T* __restrict__ in, int ldi, int ok, int ov) {
+  const int row = a.index ? a.index[blockIdx.x] : blockIdx.x;
+  const int p = att_pos(a, row);
+  if (p < 0) return;
+  const size_t page = (size_t)att_page(a, a.slot[row], p / ATT_PAGE) * a.kv_heads;
+  const int r = p % ATT_PAGE, vi = att_vidx(r);
+  const T* src = in + (size_t)row * ldi;
+  T* k = (T*)a.k;
+  T* v = (T*)a.v;
+  for (int c = threadIdx.x; c < a.kv_heads * a.dkp; c += 256) {
+    const int g = c / a.dkp, d = c % a.dkp;
+    k[((page + g) * ATT_PAGE + r) * a.dkp + d] = src[ok + c];
+  }
+  for (int c = threadIdx.x; c < a.kv_heads * a.dvp; c += 256)  // c = g * dvp + d: value row
+    v[(page * a.dvp + c) * ATT_PAGE + vi] = src[ov + c];
+}
+
+struct AttTile {  // query tile: nrows rows of one slot from row0 on, at positions pos0 ..
+  int row0, nrows, slot, pos0;
+};
+
+// ---- append: the rows of the tiles, 32 positions of one value channel per thread
+template <typename T>
+__global__ __launch_bounds__(256) void append_tiles_kernel(AttnArgs a, const AttTile* __restrict__ tiles,
+                                                           const T* __restrict__ in, int ldi, int ok, int ov) {
+  const AttTile t = tiles[blockIdx.x];
+  const int b0 = t.pos0 / 32 + blockIdx.y;  // 32-position stretch
+  const int lo = max(b0 * 32, t.pos0), hi = min(b0 * 32 + 32, t.pos0 + t.nrows);
+  if (lo >= hi) return;
+  const int pg = b0 / 2 < a.max_pages ? a.table[(size_t)t.slot * a.max_pages + b0 / 2] : -1;
+  if (pg < 0 || pg >= a.n_pages) return;
+  const size_t page = (size_t)pg * a.kv_heads;
+  const T* src = in + (size_t)(t.row0 - t.pos0) * ldi;  // row of position p: src + p ldi
+  T* k = (T*)a.k;
+  T* v = (T*)a.v;
+  constexpr int VN = 16 / sizeof(T);
+  const int kc = a.kv_heads * a.dkp / VN;
+  for (int i = blockIdx.z * 256 + threadIdx.x; i < kc * (hi - lo); i += gridDim.z * 256) {
+    const int p = lo + i / kc, c = (i % kc) * VN, g = c / a.dkp, d = c % a.dkp;
+    st16(k + ((page + g) * ATT_PAGE + p % ATT_PAGE) * a.dkp + d, ld16(src + (size_t)p * ldi + ok + c));
+  }
+  for (int c = blockIdx.z * 256 + threadIdx.x; c < a.kv_heads * a.dvp; c += gridDim.z * 256) {
+    T* row = v + (page * a.dvp + c) * ATT_PAGE;
+    if (hi - lo == 32 && sizeof(T) == 2) {
+      unsigned short e[32];
+#pragma unroll
+      for (int r = 0; r < 32; ++r)
+        e[att_vidx(r)] = *reinterpret_cast<const unsigned short*>(src + (size_t)(lo + r) * ldi + ov + c);
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        u32x4_t w;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) w[j] = e[8 * q + 2 * j] | ((unsigned)e[8 * q + 2 * j + 1] << 16);
+        st16(row + (lo % ATT_PAGE) + 8 * q, w);
+      }
+    } else {
+      for (int p = lo; p < hi; ++p) row[att_vidx(p % ATT_PAGE)] = src[(size_t)p * ldi + ov + c];
+    }
+  }
+}
+
+// ---- one workgroup per (row, head), a page of keys at a time
+template <typename T>
+__global__ __launch_bounds__(256) void attend_plain_kernel(AttnArgs a, const T* __restrict__ q, int ldq,
+                                                           const T* __restrict__ gate, int ldg, T* __restrict__ out,
+                                                           int ldo) {
+  extern __shared__ float smem[];
+  float* sq = smem;             // [dkp]
+  float* so = smem + a.dkp;     // [dvp]
+  __shared__ float sp[ATT_PAGE];
+  const int row = a.index ? a.index[blockIdx.x] : blockIdx.x, h = blockIdx.y, g = h / (a.heads / a.kv_heads);
+  const int tid = threadIdx.x, p = att_pos(a, row);
+  T* o = out + (size_t)row * ldo + (size_t)h * a.dvp;
+  if (p < 0) {
+    for (int d = tid; d < a.dvp; d += 256) st1(o + d, 0.f);
+    return;
+  }
+  for (int d = tid; d < a.dkp; d += 256) sq[d] = ld1(q + (size_t)row * ldq + (size_t)h * a.dkp + d);
+  for (int d = tid; d < a.dvp; d += 256) so[d] = 0.f;
+  const float hs = a.hscale[h];
+  const int slot = a.slot[row];
+  float m = -INFINITY, l = 0.f;
+  const AttBlocks blocks(a, p, p);
+  for (int i = 0; i < blocks.n; ++i) {
+    const int b = blocks.at(i);
+    const size_t page = (size_t)att_page(a, slot, b) * a.kv_heads + g;
+    __syncthreads();
+    const int r = tid >> 2, key = b * ATT_PAGE + r;  // four threads per key
+    float s = 0.f;
+    const T* kr = (const T*)a.k + (page * ATT_PAGE + r) * a.dkp;
+    if (att_sees(a, p, key))
+      for (int d = tid & 3; d < a.dkp; d += 4) s = fmaf(sq[d], ld1(kr + d), s);
+    s += __shfl_xor(s, 1, 64);
+    s += __shfl_xor(s, 2, 64);
+    s *= hs;
+    if (a.softcap > 0.f) s = a.softcap * tanhf(s / a.softcap);
+    if (!att_sees(a, p, key)) s = -INFINITY;
+    if ((tid & 3) == 0) sp[r] = s;
+    __syncthreads();
+    float x = sp[tid & 63];
+    const float mn = fmaxf(m, wave_max(x));  // a block holds at least one visible key
+    x = expf(x - mn);
+    const float alpha = expf(m - mn), ps = wave_sum(x);
+    l = l * alpha + ps;
+    m = mn;
+    __syncthreads();
+    if (tid < 64) sp[tid] = x;
+    __syncthreads();
+    const T* vp = (const T*)a.v + page * a.dvp * ATT_PAGE;
+    for (int d = tid; d < a.dvp; d += 256) {
+      float acc = so[d] * alpha;
+      for (int e = 0; e < ATT_PAGE; ++e)
+        if (sp[e] != 0.f) acc = fmaf(sp[e], ld1(vp + (size_t)d * ATT_PAGE + att_vidx(e)), acc);
+      so[d] = acc;
+    }
+  }
+  const float f = (gate ? 1.f / (1.f + expf(-ld1(gate + (size_t)row * ldg + h))) : 1.f) / l;
+  for (int d = tid; d < a.dvp; d += 256) st1(o + d, so[d] * f);
+}
+
+// ---- partial sums of ns key splits -> the gated output; one wave per (entry, head)
+__global__ __launch_bounds__(64) void merge_kernel(AttnArgs a, const float* __restrict__ po, const float* __restrict__ pm,
+                                                   int ns, const bf16_raw* __restrict__ gate, int ldg,
+                                                   bf16_raw* __restrict__ out, int ldo) {
+  const int i = blockIdx.x, h = blockIdx.y, row = a.index ? a.index[i] : i, lane = threadIdx.x;
+  const size_t e = ((size_t)i * a.heads + h) * ns;
+  float m = -INFINITY;
+  for (int s = 0; s < ns; ++s) m = fmaxf(m, pm[2 * (e + s)]);
+  float l = 0.f;
+  for (int s = 0; s < ns; ++s) {
+    const float ms = pm[2 * (e + s)];
+    if (ms > -INFINITY) l += pm[2 * (e + s) + 1] * __builtin_amdgcn_exp2f(ms - m);
+  }
+  const float f = l > 0.f ? (gate ? sigmoid(bf2f(gate[(size_t)row * ldg + h])) : 1.f) / l : 0.f;
+  for (int d = lane; d < a.dvp; d += 64) {
+    float acc = 0.f;
+    for (int s = 0; s < ns; ++s) {
+      const float ms = pm[2 * (e + s)];
+      if (ms > -INFINITY) acc += po[(e + s) * a.dvp + d] * __builtin_amdgcn_exp2f(ms - m);
+    }
+    out[(size_t)row * ldo + (size_t)h * a.dvp + d] = f2bf(acc * f);
+  }
+}
+
+bool bad_args(const AttnArgs* a) {
+  return !a || !a->k || !a->v || !a->table || !a->hscale || a->max_pages < 1 || a->n_pages < 1 || a->heads < 1 ||
+         a->kv_heads < 1 || a->heads % a->kv_heads || a->dim < 1 || a->vdim < 1 || a->dkp < a->dim || a->dvp < a->vdim ||
+         a->dkp % 64 || a->dvp % 64 || a->window < 1 || a->keep < 0 || a->softcap < 0.f;
+}
+
+}  // namespace
+
+extern "C" int lsa_attn_append(int f32, const AttnArgs* a, int n, const void* in, int ldi, int ok, int ov, hipStream_t s) {
+  if (bad_args(a) || !a->slot || !a->pos || n < 1 || ok < 0 || ov < 0 || ldi < ok + a->kv_heads * a->dkp ||
+      ldi < ov + a->kv_heads * a->dvp)
+    return LSA_BAD_SHAPE;
+  if (f32) append_rows_kernel<float><<<n, 256, 0, s>>>(*a, (const float*)in, ldi, ok, ov);
+  else append_rows_kernel<bf16_raw><<<n, 256, 0, s>>>(*a, (const bf16_raw*)in, ldi, ok, ov);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+// tiles: n_tiles {row0, nrows <= 128, slot, pos0}
+extern "C" int lsa_attn_append_tiles(int f32, const AttnArgs* a, const void* tiles, int n_tiles, const void* in, int ldi,
+                                     int ok, int ov, hipStream_t s) {
+  if (bad_args(a) || n_tiles < 1 || ok < 0 || ov < 0 || ldi < ok + a->kv_heads * a->dkp ||
+      ldi < ov + a->kv_heads * a->dvp || ldi % 8 || ok % 8 || (uintptr_t)in % 16)
+    return LSA_BAD_SHAPE;
+  const dim3 grid(n_tiles, 5, max(1, min(4, a->kv_heads * a->dvp / 256)));
+  if (f32) append_tiles_kernel<float><<<grid, 256, 0, s>>>(*a, (const AttTile*)tiles, (const float*)in, ldi, ok, ov);
+  else append_tiles_kernel<bf16_raw><<<grid, 256, 0, s>>>(*a, (const AttTile*)tiles, (const bf16_raw*)in, ldi, ok, ov);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+extern "C" int lsa_attn_plain(int f32, const AttnArgs* a, int n, const void* q, int ldq, const void* gate, int ldg,
+                              void* out, int ldo, hipStream_t s) {
+  if (bad_args(a) || !a->slot || !a->pos || n < 1 || ldq < a->heads * a->dkp || ldo < a->heads * a->dvp ||
+      (gate && ldg < a->heads) || a->dkp + a->dvp > 8192)
+    return LSA_BAD_SHAPE;
+  const dim3 grid(n, a->heads);
+  const size_t lds = (size_t)(a->dkp + a->dvp) * 4;
+  if (f32)
+    attend_plain_kernel<float><<<grid, 256, lds, s>>>(*a, (const float*)q, ldq, (const float*)gate, ldg, (float*)out, ldo);
+  else
+    attend_plain_kernel<bf16_raw><<<grid, 256, lds, s>>>(*a, (const bf16_raw*)q, ldq, (const bf16_raw*)gate, ldg,
+                                                         (bf16_raw*)out, ldo);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+extern "C" int lsa_attn_merge(const AttnArgs* a, int n, const float* po, const float* pm, int ns, const void* gate,
+                              int ldg, void* out, int ldo, hipStream_t s) {
+  if (bad_args(a) || n < 1 || ns < 1 || ldo < a->heads * a->dvp || (gate && ldg < a->heads)) return LSA_BAD_SHAPE;
+  merge_kernel<<<dim3(n, a->heads), 64, 0, s>>>(*a, po, pm, ns, (const bf16_raw*)gate, ldg, (bf16_raw*)out, ldo);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}

@@ -1,0 +1,228 @@
+// Paged attention of prompt portions, bf16 on MFMA (paged_attn.h).
+//
+// The pipeline of the flash prefill kernel (attn_prefill.hip): one query tile of one sequence x one
+// head, eight waves of 16 rows, key and value pages by LDS-DMA into a double buffer, S^T = K Q^T,
+// per-lane online softmax, O^T += V^T P^T with P^T taken from the score accumulators. A page is
+// one block; only blocks that hold a visible key are visited (the kept first ones, then those from the
+// window's first on), page numbers sit in lanes (one load per 64 blocks), and values come transposed
+// from the cache, so both operands are plain 16-byte LDS reads.
+#include <limits.h>
+
+#include "paged_attn.h"
+
+namespace {
+
+constexpr int NWV = 8, NTHR = NWV * 64;
+
+struct AttTile {
+  int row0, nrows, slot, pos0;
+};
+
+template <int NC>
+LSA_DEVICE int swz(int r) {
+  if constexpr (NC == 16) return ((r & 3) << 2) ^ (((r >> 2) & 3) << 1);
+  else return NC == 8 ? (r & 7) : ((r & 7) << 1);
+}
+
+LSA_DEVICE void glds16(const void* src, unsigned char* lds_base) {
+  __builtin_amdgcn_global_load_lds(src, (__attribute__((address_space(3))) void*)lds_base, 16, 0, 0);
+}
+
+template <int DK, int DV>
+__global__ __launch_bounds__(NTHR, DK + DV <= 256 ? 4 : 2) void attn_tiles_kernel(
+    AttnArgs a, const AttTile* __restrict__ tiles, const bf16_raw* __restrict__ q, int ldq,
+    const bf16_raw* __restrict__ gate, int ldg, bf16_raw* __restrict__ out, int ldo) {
+  constexpr int KF = DK / 32, DT = DV / 16, NCK = DK / 8, NCV = ATT_PAGE / 8;
+  constexpr int KBLK = ATT_PAGE * DK * 2, VBLK = ATT_PAGE * DV * 2;
+  constexpr int KPW = KBLK / 1024 / NWV, VPW = VBLK / 1024 / NWV;  // DMA pieces per wave
+  static_assert(KPW * NWV * 1024 == KBLK && VPW * NWV * 1024 == VBLK, "geometry");
+  __shared__ __attribute__((aligned(16))) unsigned char smem[2 * (KBLK + VBLK)];
+
+  const int H = a.heads, n_tiles = gridDim.x / H;
+  int tix, head;
+  if (H % 8 == 0) {  // one XCD's workgroups share heads of one kv head: its pages stay in that L2
+    const int x = blockIdx.x % 8, j = blockIdx.x / 8, hx = H / 8;
+    tix = j / hx;
+    head = x * hx + j % hx;
+  } else {
+    tix = blockIdx.x % n_tiles;
+    head = blockIdx.x / n_tiles;
+  }
+  const AttTile tile = tiles[tix];
+  const int g = head / (H / a.kv_heads);
+  const int tid = threadIdx.x, lane = tid & 63, q4 = lane >> 4, l16 = lane & 15;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int my_row = w * 16 + l16;
+  const bool row_ok = my_row < tile.nrows;
+  const int my_pos = tile.pos0 + my_row;
+
+  u32x4_t qf[KF];
+  {
+    const bf16_raw* qr = q + (size_t)(tile.row0 + (row_ok ? my_row : 0)) * ldq + (size_t)head * DK;
+#pragma unroll
+    for (int kf = 0; kf < KF; ++kf) qf[kf] = ld16(qr + kf * 32 + q4 * 8);
+  }
+  const float cap = a.softcap, icap = cap > 0.f ? 2.f * 1.4426950408889634f / cap : 0.f;
+  float hs = a.hscale[head] * (cap > 0.f ? 1.f : 1.4426950408889634f);
+  const AttBlocks blocks(a, tile.pos0, tile.pos0 + tile.nrows - 1);
+  const int wp0 = tile.pos0 + w * 16, wp1 = tile.pos0 + min(w * 16 + 16, tile.nrows) - 1;  // this wave's positions
+  const int* tab = a.table + (size_t)tile.slot * a.max_pages;
+  int pages = 0;
+  auto load_pages = [&](int i0) {  // lane l: page of listed block i0 + l
+    const int i = i0 + lane;
+    const int pg = i < blocks.n ? tab[blocks.at(i)] : 0;
+    pages = pg < 0 || pg >= a.n_pages ? 0 : pg;
+  };
+  load_pages(0);
+  // what was loaded has arrived here, not at its first use inside the block loop (whose wait would also
+  // drain the next block's DMA, every time around)
+#pragma unroll
+  for (int kf = 0; kf < KF; ++kf) asm volatile("" : "+v"(qf[kf]));
+  asm volatile("" : "+v"(pages), "+v"(hs));
+
+  auto stage = [&](int i, int buf) {
+    unsigned char* kd = smem + buf * (KBLK + VBLK);
+    const size_t page = (size_t)__builtin_amdgcn_readlane(pages, i & 63) * a.kv_heads + g;
+    const bf16_raw* kp = (const bf16_raw*)a.k + page * ATT_PAGE * DK;
+    const bf16_raw* vp = (const bf16_raw*)a.v + page * ATT_PAGE * DV;
+#pragma unroll
+    for (int s = 0; s < KPW; ++s) {
+      const int pc = w * KPW + s, lin = pc * 64 + lane, r = lin / NCK, ch = (lin % NCK) ^ swz<NCK>(r);
+      glds16(kp + r * DK + ch * 8, kd + pc * 1024);
+    }
+#pragma unroll
+    for (int s = 0; s < VPW; ++s) {
+      const int pc = w * VPW + s, lin = pc * 64 + lane, r = lin / NCV, ch = (lin % NCV) ^ swz<NCV>(r);
+      glds16(vp + r * ATT_PAGE + ch * 8, kd + KBLK + pc * 1024);
+    }
+  };
+
+  f32x4_t o[DT];
+#pragma unroll
+  for (int d = 0; d < DT; ++d) o[d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float m_run = -INFINITY, l_run = 0.f;
+  int k_off[KF], v_off[2];
+#pragma unroll
+  for (int kf = 0; kf < KF; ++kf) k_off[kf] = l16 * (DK * 2) + (((kf * 4 + q4) ^ swz<NCK>(l16)) << 4);
+#pragma unroll
+  for (int f = 0; f < 2; ++f) v_off[f] = l16 * (ATT_PAGE * 2) + (((f * 4 + q4) ^ swz<NCV>(l16)) << 4);
+
+  stage(0, 0);
+  for (int i = 0; i < blocks.n; ++i) {
+    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+    if (i + 1 < blocks.n) {
+      if (((i + 1) & 63) == 0) {
+        load_pages(i + 1);
+        asm volatile("" : "+v"(pages));
+      }
+      stage(i + 1, (i + 1) & 1);
+    }
+    const int b0 = blocks.at(i) * ATT_PAGE;
+    // no row of this wave sees a key of the block
+    if (wp1 < wp0 || b0 > wp1 || (wp0 - (b0 + ATT_PAGE - 1) >= a.window && b0 >= a.keep)) continue;
+    const unsigned char* ks = smem + (i & 1) * (KBLK + VBLK);
+    const unsigned char* vs = ks + KBLK;
+    f32x4_t s[4];
+#pragma unroll
+    for (int kt = 0; kt < 4; ++kt) {
+      s[kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kf = 0; kf < KF; ++kf) {
+        const u32x4_t k = *reinterpret_cast<const u32x4_t*>(ks + kt * 16 * (DK * 2) + k_off[kf]);
+        s[kt] = mfma16(k, qf[kf], s[kt]);
+      }
+    }
+#pragma unroll
+    for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        float x = s[kt][r] * hs;
+        if (cap > 0.f) x = att_cap(x, cap, icap) * 1.4426950408889634f;
+        s[kt][r] = x;
+      }
+    if (b0 + ATT_PAGE - 1 > wp0 || wp1 - b0 >= a.window) {  // some row does not see some key
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (!att_sees(a, my_pos, b0 + kt * 16 + q4 * 4 + r)) s[kt][r] = -INFINITY;
+    }
+    float mx = -INFINITY;
+#pragma unroll
+    for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[kt][r]);
+    mx = fmaxf(mx, lane_xor<16>(mx));
+    mx = fmaxf(mx, lane_xor<32>(mx));
+    const float m_new = fmaxf(m_run, mx);
+    const float m_use = m_new == -INFINITY ? 0.f : m_new;
+    const float alpha = __builtin_amdgcn_exp2f(m_run - m_use);
+    float psum = 0.f;
+#pragma unroll
+    for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float p = __builtin_amdgcn_exp2f(s[kt][r] - m_use);
+        s[kt][r] = p;
+        psum += p;
+      }
+    l_run = l_run * alpha + psum;
+    if (__builtin_amdgcn_ballot_w64(m_new != m_run)) {
+#pragma unroll
+      for (int d = 0; d < DT; ++d) o[d] *= alpha;
+    }
+    m_run = m_new;
+#pragma unroll
+    for (int f = 0; f < 2; ++f) {
+      float pf[8];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        pf[r] = s[2 * f][r];
+        pf[4 + r] = s[2 * f + 1][r];
+      }
+      const u32x4_t b = pack8(pf);
+#pragma unroll
+      for (int d = 0; d < DT; ++d) {
+        const u32x4_t v = *reinterpret_cast<const u32x4_t*>(vs + d * 16 * (ATT_PAGE * 2) + v_off[f]);
+        o[d] = mfma16(v, b, o[d]);
+      }
+    }
+  }
+
+  l_run += lane_xor<16>(l_run);
+  l_run += lane_xor<32>(l_run);
+  if (!row_ok) return;
+  const size_t row = tile.row0 + my_row;
+  const float f = l_run > 0.f ? (gate ? sigmoid(bf2f(gate[row * ldg + head])) : 1.f) / l_run : 0.f;
+  bf16_raw* orow = out + row * ldo + (size_t)head * DV;
+#pragma unroll
+  for (int d = 0; d < DT; ++d) st4(orow + d * 16 + q4 * 4, o[d] * f);  // this lane: O[row][d * 16 + 4 q4 + r]
+}
+
+}  // namespace
+
+// tiles: n_tiles {row0, nrows <= 128, slot, pos0}; every position's page is in the table
+extern "C" int lsa_attn_tiles(const AttnArgs* a, const void* tiles, int n_tiles, const void* q, int ldq, const void* gate,
+                              int ldg, void* out, int ldo, hipStream_t s) {
+  if (!a || !a->k || !a->v || !a->table || !a->hscale || n_tiles < 1 || a->max_pages < 1 || a->n_pages < 1 ||
+      a->heads < 1 || a->kv_heads < 1 || a->heads % a->kv_heads || a->window < 1 || a->keep < 0 || a->softcap < 0.f ||
+      a->dkp < a->dim || a->dvp < a->vdim)
+    return LSA_BAD_SHAPE;
+  if (ldq < a->heads * a->dkp || ldq % 8 || ldo < a->heads * a->dvp || ldo % 4 || (gate && ldg < a->heads) ||
+      ((uintptr_t)q | (uintptr_t)a->k | (uintptr_t)a->v) % 16 || (uintptr_t)out % 8)
+    return LSA_BAD_SHAPE;
+  const dim3 grid(n_tiles * a->heads);
+#define LSA_T(K, V)                                                                                                   \
+  if (a->dkp == K && a->dvp == V) {                                                                                   \
+    attn_tiles_kernel<K, V><<<grid, NTHR, 0, s>>>(*a, (const AttTile*)tiles, (const bf16_raw*)q, ldq,                 \
+                                                  (const bf16_raw*)gate, ldg, (bf16_raw*)out, ldo);                   \
+    LSA_CHECK_LAUNCH();                                                                                               \
+    return LSA_OK;                                                                                                    \
+  }
+  LSA_T(64, 64) LSA_T(64, 128) LSA_T(128, 64) LSA_T(128, 128) LSA_T(64, 256) LSA_T(128, 256) LSA_T(256, 64)
+  LSA_T(256, 128) LSA_T(256, 256)
+#undef LSA_T
+  return LSA_UNSUPPORTED;
+}

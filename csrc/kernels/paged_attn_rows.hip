@@ -1,0 +1,173 @@
+// Paged attention of single rows (decoded tokens, short portions), bf16 on MFMA (paged_attn.h).
+//
+// One workgroup per (row, kv head, key split): the heads that share the kv head are the columns of
+// 16-wide score tiles, so a cached byte is read once for all of them. Four waves take pages in
+// turn; keys and values go straight from memory into MFMA operand registers (no LDS on the way),
+// the next page's keys being requested before this page's softmax. S^T = K Q^T leaves the weights in
+// the layout in which O^T += V^T P^T takes them. The waves' results meet in LDS at the end; with
+// several splits the workgroup leaves fp32 partials for lsa_attn_merge.
+#include <limits.h>
+
+#include "paged_attn.h"
+
+namespace {
+
+constexpr int NW = 4;
+
+template <int DK, int DV>
+__global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void attend_rows_kernel(
+    AttnArgs a, const bf16_raw* __restrict__ q, int ldq, const bf16_raw* __restrict__ gate, int ldg,
+    bf16_raw* __restrict__ out, int ldo, int ns, float* __restrict__ po, float* __restrict__ pm) {
+  constexpr int KF = DK / 32, DT = DV / 16, LDO = DV + 4;
+  __shared__ __attribute__((aligned(16))) float s_o[NW][16][LDO];
+  __shared__ float s_m[NW][16], s_l[NW][16];
+  const int i = blockIdx.x, row = a.index ? a.index[i] : i;
+  const int grp = a.heads / a.kv_heads, ht = (grp + 15) / 16;
+  const int g = blockIdx.y / ht, h0 = g * grp + (blockIdx.y % ht) * 16, nh = min(16, (g + 1) * grp - h0);
+  const int split = blockIdx.z, tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, q4 = lane >> 4;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int p = att_pos(a, row);
+  float m_run = -INFINITY, l_run = 0.f;
+  f32x4_t o[DT];
+#pragma unroll
+  for (int d = 0; d < DT; ++d) o[d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  if (p >= 0) {
+    const int head = h0 + min(l16, nh - 1), slot = a.slot[row];
+    u32x4_t qf[KF];
+    const bf16_raw* qr = q + (size_t)row * ldq + (size_t)head * DK;
+#pragma unroll
+    for (int kf = 0; kf < KF; ++kf) qf[kf] = ld16(qr + kf * 32 + q4 * 8);
+    const float cap = a.softcap, icap = cap > 0.f ? 2.f * 1.4426950408889634f / cap : 0.f;
+    const float hs = a.hscale[head] * (cap > 0.f ? 1.f : 1.4426950408889634f);  // exponents of two
+    const AttBlocks blocks(a, p, p);
+    const int step = ns * NW;
+    int bi = split * NW + w;
+    u32x4_t kr[4][KF];
+    auto load_k = [&](int b) {
+      const bf16_raw* kp = (const bf16_raw*)a.k + ((size_t)att_page(a, slot, b) * a.kv_heads + g) * ATT_PAGE * DK;
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int kf = 0; kf < KF; ++kf) kr[kt][kf] = ld16(kp + (kt * 16 + l16) * DK + kf * 32 + q4 * 8);
+    };
+    if (bi < blocks.n) load_k(blocks.at(bi));
+    for (; bi < blocks.n; bi += step) {
+      const int b = blocks.at(bi);
+      const bf16_raw* vp = (const bf16_raw*)a.v + ((size_t)att_page(a, slot, b) * a.kv_heads + g) * ATT_PAGE * DV;
+      u32x4_t vr[2][DT];
+#pragma unroll
+      for (int f = 0; f < 2; ++f)
+#pragma unroll
+        for (int d = 0; d < DT; ++d) vr[f][d] = ld16(vp + (d * 16 + l16) * ATT_PAGE + f * 32 + q4 * 8);
+      f32x4_t s[4];
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt) {
+        s[kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kf = 0; kf < KF; ++kf) s[kt] = mfma16(kr[kt][kf], qf[kf], s[kt]);
+      }
+      if (bi + step < blocks.n) load_k(blocks.at(bi + step));
+      float mx = -INFINITY;
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          float x = s[kt][r] * hs;
+          if (cap > 0.f) x = att_cap(x, cap, icap) * 1.4426950408889634f;
+          x = att_sees(a, p, b * ATT_PAGE + kt * 16 + q4 * 4 + r) ? x : -INFINITY;
+          s[kt][r] = x;
+          mx = fmaxf(mx, x);
+        }
+      mx = fmaxf(mx, lane_xor<16>(mx));
+      mx = fmaxf(mx, lane_xor<32>(mx));
+      const float mn = fmaxf(m_run, mx), mu = mn == -INFINITY ? 0.f : mn;
+      const float alpha = __builtin_amdgcn_exp2f(m_run - mu);
+      float ps = 0.f;
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float e = __builtin_amdgcn_exp2f(s[kt][r] - mu);
+          s[kt][r] = e;
+          ps += e;
+        }
+      l_run = l_run * alpha + ps;
+      m_run = mn;
+#pragma unroll
+      for (int d = 0; d < DT; ++d) o[d] *= alpha;
+#pragma unroll
+      for (int f = 0; f < 2; ++f) {
+        float pf[8];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          pf[r] = s[2 * f][r];
+          pf[4 + r] = s[2 * f + 1][r];
+        }
+        const u32x4_t b8 = pack8(pf);
+#pragma unroll
+        for (int d = 0; d < DT; ++d) o[d] = mfma16(vr[f][d], b8, o[d]);
+      }
+    }
+    l_run += lane_xor<16>(l_run);
+    l_run += lane_xor<32>(l_run);
+  }
+  // this lane: O[d * 16 + 4 q4 + r] of head l16
+#pragma unroll
+  for (int d = 0; d < DT; ++d) *reinterpret_cast<f32x4_t*>(&s_o[w][l16][d * 16 + q4 * 4]) = o[d];
+  if (q4 == 0) {
+    s_m[w][l16] = m_run;
+    s_l[w][l16] = l_run;
+  }
+  __syncthreads();
+  for (int t = tid; t < nh * (DV / 4); t += 256) {
+    const int hh = t / (DV / 4), d = (t % (DV / 4)) * 4, h = h0 + hh;
+    float m = s_m[0][hh];
+#pragma unroll
+    for (int x = 1; x < NW; ++x) m = fmaxf(m, s_m[x][hh]);
+    float l = 0.f;
+    f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int x = 0; x < NW; ++x) {
+      const float f = s_m[x][hh] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(s_m[x][hh] - m);
+      l += s_l[x][hh] * f;
+      v += *reinterpret_cast<const f32x4_t*>(&s_o[x][hh][d]) * f;
+    }
+    if (ns == 1) {
+      const float f = l > 0.f ? (gate ? sigmoid(bf2f(gate[(size_t)row * ldg + h])) : 1.f) / l : 0.f;
+      st4(out + (size_t)row * ldo + (size_t)h * DV + d, v * f);
+    } else {
+      const size_t e = ((size_t)i * a.heads + h) * ns + split;
+      *reinterpret_cast<f32x4_t*>(po + e * DV + d) = v;
+      if (d == 0) {
+        pm[2 * e] = m;
+        pm[2 * e + 1] = l;
+      }
+    }
+  }
+}
+
+}  // namespace
+
+extern "C" int lsa_attn_rows(const AttnArgs* a, int n, const void* q, int ldq, const void* gate, int ldg, void* out,
+                             int ldo, int ns, float* po, float* pm, hipStream_t s) {
+  if (!a || !a->k || !a->v || !a->table || !a->slot || !a->pos || !a->hscale || n < 1 || ns < 1 || ns > 1024 ||
+      a->max_pages < 1 || a->n_pages < 1 || a->heads < 1 || a->kv_heads < 1 || a->heads % a->kv_heads ||
+      a->window < 1 || a->keep < 0 || a->softcap < 0.f || a->dkp < a->dim || a->dvp < a->vdim)
+    return LSA_BAD_SHAPE;
+  if (ldq < a->heads * a->dkp || ldq % 8 || ldo < a->heads * a->dvp || ldo % 4 || (gate && ldg < a->heads) ||
+      (ns > 1 && (!po || !pm)) || ((uintptr_t)q | (uintptr_t)a->k | (uintptr_t)a->v) % 16 || (uintptr_t)out % 8)
+    return LSA_BAD_SHAPE;
+  const int grp = a->heads / a->kv_heads;
+  const dim3 grid(n, a->kv_heads * ((grp + 15) / 16), ns);
+#define LSA_R(K, V)                                                                                                  \
+  if (a->dkp == K && a->dvp == V) {                                                                                  \
+    attend_rows_kernel<K, V><<<grid, 256, 0, s>>>(*a, (const bf16_raw*)q, ldq, (const bf16_raw*)gate, ldg,           \
+                                                  (bf16_raw*)out, ldo, ns, po, pm);                                  \
+    LSA_CHECK_LAUNCH();                                                                                              \
+    return LSA_OK;                                                                                                   \
+  }
+  LSA_R(64, 64) LSA_R(64, 128) LSA_R(128, 64) LSA_R(128, 128) LSA_R(64, 256) LSA_R(128, 256) LSA_R(256, 64)
+  LSA_R(256, 128) LSA_R(256, 256)
+#undef LSA_R
+  return LSA_UNSUPPORTED;
+}

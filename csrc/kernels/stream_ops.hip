@@ -4,6 +4,9 @@
 //   lsa_stream_add_norm  x += rms(y) * gain: a sublayer's result, RMS-normed, joins the stream (gain
 //                        = norm weight times layer scale, fp32), plus the copy the projections read
 //   lsa_stream_norm      rms(x) * gain -> the head projection's input
+// and of one whose sublayers read a norm of the stream and join it through a sigmoid gate per element:
+//   lsa_stream_join      x += sigmoid(g1) * y1 + sigmoid(g2) * (y2, or the weighted sum of a row's expert
+//                        results), then (optionally) rms(x) * gain -> the next sublayers' input
 //   lsa_logits_argmax    argmax keys of fp32 logits (the fp32 engine; the bf16 one fuses this
 //                        into the head GEMM)
 //   lsa_cast_rows        fp32 rows -> the projections' type (a stage's input stream)
@@ -130,6 +133,133 @@ void launch_norm(const float* y, int ldy, const float* gain, float eps, int rows
 #undef LSA_N
 }
 
+struct JoinArgs {  // Mirrored by llm_sharding_amd/ops/stream.py::JoinArgs
+  const float* y1;       // [rows][ldy1] or null
+  const void* g1;        // gate logits of y1 / of the second result, in the projections' type
+  const void* g2;
+  const float* y2;       // [rows][ldy2] or null
+  const void* ye;        // [rows * top][ldye] expert results of the sorted pairs, or null
+  const float* weight;   // [rows * top]
+  const int* place;      // [rows * top] where a row's pair lies in ye
+  const float* gain;     // null: no norm
+  int ldy1, ldg1, ldg2, ldy2, ldye, top;
+  float eps;
+};
+
+template <typename T>
+LSA_DEVICE f32x4_t load4(const T* p) {
+  if constexpr (sizeof(T) == 4) {
+    return *reinterpret_cast<const f32x4_t*>(p);
+  } else {
+    const u32x2_t v = *reinterpret_cast<const u32x2_t*>(p);
+    return f32x4_t{__uint_as_float(v[0] << 16), __uint_as_float(v[0] & 0xffff0000u), __uint_as_float(v[1] << 16),
+                   __uint_as_float(v[1] & 0xffff0000u)};
+  }
+}
+
+// what the results add to x[row][c .. c + V)
+template <typename T, int V>
+LSA_DEVICE void join_at(const JoinArgs& a, int row, int c, float* x) {
+  auto get = [&](const auto* p, float* f) {
+    if constexpr (V == 4) {
+      const f32x4_t v = load4(p);
+#pragma unroll
+      for (int k = 0; k < 4; ++k) f[k] = v[k];
+    } else {
+      f[0] = ld1(p);
+    }
+  };
+  float y[V], g[V];
+  if (a.y1) {
+    get(a.y1 + (size_t)row * a.ldy1 + c, y);
+    get((const T*)a.g1 + (size_t)row * a.ldg1 + c, g);
+#pragma unroll
+    for (int k = 0; k < V; ++k) x[k] += sigmoid(g[k]) * y[k];
+  }
+  if (a.y2 || a.ye) {
+    get((const T*)a.g2 + (size_t)row * a.ldg2 + c, g);
+    if (a.y2) {
+      get(a.y2 + (size_t)row * a.ldy2 + c, y);
+    } else {
+#pragma unroll
+      for (int k = 0; k < V; ++k) y[k] = 0.f;
+      for (int e = 0; e < a.top; ++e) {
+        float z[V];
+        get((const T*)a.ye + (size_t)a.place[row * a.top + e] * a.ldye + c, z);
+        const float w = a.weight[row * a.top + e];
+#pragma unroll
+        for (int k = 0; k < V; ++k) y[k] = fmaf(w, z[k], y[k]);
+      }
+    }
+#pragma unroll
+    for (int k = 0; k < V; ++k) x[k] += sigmoid(g[k]) * y[k];
+  }
+}
+
+// NV > 0: rows of up to 1024 NV values in registers, four at a time; 0: any width
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void join_kernel(JoinArgs a, int W, float* __restrict__ x, int ldx, T* __restrict__ xc,
+                                                   int ldc) {
+  __shared__ float s_part[4];
+  const int row = blockIdx.x, tid = threadIdx.x;
+  float* xr = x + (size_t)row * ldx;
+  float s = 0.f;
+  f32x4_t v[NV > 0 ? NV : 1];
+  if constexpr (NV > 0) {
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int c = (tid + j * 256) * 4;
+      v[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      if (c >= W) continue;
+      float f[4];
+      const f32x4_t x4 = *reinterpret_cast<const f32x4_t*>(xr + c);
+#pragma unroll
+      for (int k = 0; k < 4; ++k) f[k] = x4[k];
+      join_at<T, 4>(a, row, c, f);
+      v[j] = f32x4_t{f[0], f[1], f[2], f[3]};
+      *reinterpret_cast<f32x4_t*>(xr + c) = v[j];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) s += f[k] * f[k];
+    }
+  } else {
+    for (int c = tid; c < W; c += 256) {
+      float f = xr[c];
+      join_at<T, 1>(a, row, c, &f);
+      xr[c] = f;
+      s += f * f;
+    }
+  }
+  if (!a.gain) return;
+  s = wave_sum(s);
+  if ((tid & 63) == 0) s_part[tid >> 6] = s;
+  __syncthreads();
+  const float rs = 1.f / sqrtf((s_part[0] + s_part[1] + s_part[2] + s_part[3]) / (float)W + a.eps);
+  T* cr = xc + (size_t)row * ldc;
+  if constexpr (NV > 0) {
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int c = (tid + j * 256) * 4;
+      if (c < W) st4(cr + c, v[j] * rs * *reinterpret_cast<const f32x4_t*>(a.gain + c));
+    }
+  } else {
+    for (int c = tid; c < W; c += 256) st1(cr + c, xr[c] * rs * a.gain[c]);  // this thread's own stores
+  }
+}
+
+template <typename T>
+void launch_join(const JoinArgs& a, int rows, int W, float* x, int ldx, T* xc, int ldc, hipStream_t s) {
+  const bool vec = !((W | ldx | ldc | a.ldy1 | a.ldg1 | a.ldg2 | a.ldy2 | a.ldye) % 4) &&
+                   !(((uintptr_t)x | (uintptr_t)xc | (uintptr_t)a.y1 | (uintptr_t)a.g1 | (uintptr_t)a.g2 |
+                      (uintptr_t)a.y2 | (uintptr_t)a.ye | (uintptr_t)a.gain) % 16);
+  const int nv = vec ? (W + 1023) / 1024 : 0;
+#define LSA_J(NV) join_kernel<T, NV><<<rows, 256, 0, s>>>(a, W, x, ldx, xc, ldc)
+  if (nv >= 1 && nv <= 2) LSA_J(2);
+  else if (nv >= 3 && nv <= 4) LSA_J(4);
+  else if (nv >= 5 && nv <= 8) LSA_J(8);
+  else LSA_J(0);
+#undef LSA_J
+}
+
 // grid (rows, blocks): every workgroup one stretch of the vocabulary
 __global__ __launch_bounds__(256) void logits_argmax_kernel(const float* __restrict__ lg, int ldl, int V, int offset,
                                                             unsigned long long* __restrict__ keys) {
@@ -189,6 +319,19 @@ extern "C" int lsa_stream_norm(int f32, const float* y, int ldy, const float* ga
   if (rows < 1 || W < 1 || ldy < W || ldc < W) return LSA_BAD_SHAPE;
   if (f32) launch_norm<float, false>(y, ldy, gain, eps, rows, W, nullptr, 0, (float*)xc, ldc, s);
   else launch_norm<bf16_raw, false>(y, ldy, gain, eps, rows, W, nullptr, 0, (bf16_raw*)xc, ldc, s);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+extern "C" int lsa_stream_join(int f32, const JoinArgs* a, int rows, int W, float* x, int ldx, void* xc, int ldc,
+                               hipStream_t s) {
+  if (!a || rows < 1 || W < 1 || ldx < W || !x || (a->gain && (!xc || ldc < W)) || (a->y2 && a->ye)) return LSA_BAD_SHAPE;
+  if (a->y1 && (a->ldy1 < W || !a->g1 || a->ldg1 < W)) return LSA_BAD_SHAPE;
+  if ((a->y2 || a->ye) && (!a->g2 || a->ldg2 < W)) return LSA_BAD_SHAPE;
+  if (a->y2 && a->ldy2 < W) return LSA_BAD_SHAPE;
+  if (a->ye && (a->ldye < W || a->top < 1 || !a->weight || !a->place)) return LSA_BAD_SHAPE;
+  if (f32) launch_join<float>(*a, rows, W, x, ldx, (float*)xc, ldc, s);
+  else launch_join<bf16_raw>(*a, rows, W, x, ldx, (bf16_raw*)xc, ldc, s);
   LSA_CHECK_LAUNCH();
   return LSA_OK;
 }

@@ -25,10 +25,7 @@ from .stack import GluSpec, LatentSpec, LayerSpec, StackConfig
 ARCHITECTURE = "Deretar"
 GLU_ALPHA, GLU_SHIFT = 1.702, 1.0   # fixed by the design
 NORM_OFFSET = 1.0                   # norm weights are stored around zero
-
-
-def is_deretar(d: dict) -> bool:
-    return d.get("architecture") == ARCHITECTURE
+TIED_HEAD = True                    # the head is the embedding table
 
 
 def _mixer(entry: dict) -> LatentSpec:
@@ -49,7 +46,8 @@ def _mlp(entry: dict) -> Optional[GluSpec]:
     return GluSpec(ff=int(m["ff"]), limit=float(m["limit"]), alpha=GLU_ALPHA, shift=GLU_SHIFT)
 
 
-def config_from_dict(d: dict, name: str = "deretar") -> StackConfig:
+def config_from_dict(d: dict, name: str = "deretar", shapes: Optional[dict] = None) -> StackConfig:
+    """``shapes`` (of a checkpoint's tensors) is not needed: config.json has every size."""
     entries = d["layers"]
     layers = []
     for i, e in enumerate(entries):
@@ -152,20 +150,5 @@ def write_random_checkpoint(cfg: StackConfig, folder: str, seed: int = 0, dtype=
     return folder
 
 
-class DeretarTensors:
-    """Named tensors of a checkpoint folder, read one at a time (memory-mapped)."""
-
-    def __init__(self, path: str):
-        self.file = os.path.join(path, "model.safetensors")
-        if not os.path.exists(self.file):
-            raise FileNotFoundError(self.file)
-
-    def get(self, names: dict, device, dtype) -> dict:
-        """{key: tensor name} -> {key: tensor}; shapes are checked by the caller."""
-        from safetensors import safe_open
-        with safe_open(self.file, framework="pt", device="cpu") as f:
-            return {k: f.get_tensor(n).to(device=device, dtype=dtype) for k, n in names.items()}
-
-
-__all__ = ["ARCHITECTURE", "is_deretar", "config_from_dict", "make_config", "layer_entry", "layer_shapes",
-           "random_layer", "random_embedding", "random_final_norm", "write_random_checkpoint", "DeretarTensors"]
+__all__ = ["ARCHITECTURE", "config_from_dict", "make_config", "layer_entry", "layer_shapes",
+           "random_layer", "random_embedding", "random_final_norm", "write_random_checkpoint"]

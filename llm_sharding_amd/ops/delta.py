@@ -1,0 +1,82 @@
+"""Bindings of the gated delta rule kernels (csrc/kernels/delta*.hip).
+
+The conventions of :mod:`.hip` hold: shapes are checked on the host, launches go to torch's current
+stream, nothing falls back to another implementation."""
+from __future__ import annotations
+
+import ctypes
+
+import torch
+
+from . import hip
+from .hip import _check, _p, _req, _stream, lib
+from .stream import is_f32
+
+
+class DeltaArgs(ctypes.Structure):
+    _fields_ = ([(n, ctypes.c_void_p) for n in ("inp", "in32", "z", "gate", "conv", "decay", "dt_bias", "norm", "state",
+                                                "ring", "runs", "slot", "pos", "table", "out")]
+                + [(n, ctypes.c_int) for n in ("ldi", "ld32", "ldz", "ldg", "ldo", "oq", "ok", "ov", "ob", "heads",
+                                               "kv_heads", "dim", "vdim", "taps", "dk", "dv", "max_pages", "n_pages")]
+                + [("q_scale", ctypes.c_float), ("unit_eps", ctypes.c_float), ("eps", ctypes.c_float)])
+
+
+def state_shapes(s, slots: int) -> tuple:
+    """(state, ring of convolution inputs) of one layer, fp32."""
+    return (slots, s.heads) + s.state_dims, (slots, s.taps, s.channels)
+
+
+def make_args(s, w: dict, state: tuple, inp, cols: tuple, in32, ob: int, z, gate, out, eps: float, table, n_pages: int,
+              slot=None, pos=None, runs=None) -> DeltaArgs:
+    """``w``: conv [channels, taps], decay [heads], dt_bias [heads dim], norm [vdim], fp32; ``cols``: first columns
+    of q, k and v in ``inp``; ``ob``: of the step sizes in ``in32``; ``runs`` int32 [n, 4] (row0, rows, slot,
+    pos0), checked by :func:`check_runs`, or ``slot`` / ``pos`` int32 [rows]."""
+    S, ring = state
+    rows = inp.shape[0]
+    _req(all(t.dtype == torch.float32 and t.is_contiguous() for t in (S, ring, *w.values())), "delta: fp32 state, weights")
+    _req(tuple(S.shape[1:]) == (s.heads,) + s.state_dims and tuple(ring.shape) == (S.shape[0], s.taps, s.channels),
+         "delta: state shapes")
+    _req(w["conv"].shape == (s.channels, s.taps) and w["decay"].numel() == s.heads and w["norm"].numel() == s.vdim
+         and w["dt_bias"].numel() == s.heads * s.dim, "delta: weights")
+    _req(in32.dtype == z.dtype == torch.float32 and gate.dtype == inp.dtype == out.dtype
+         and all(t.stride(1) == 1 and t.shape[0] >= rows for t in (inp, in32, z, gate, out)), "delta: inputs")
+    kc, vc = s.kv_heads * s.dim, s.heads * s.vdim
+    _req(inp.shape[1] >= max(cols[0] + kc, cols[1] + kc, cols[2] + vc) and in32.shape[1] >= ob + s.heads
+         and z.shape[1] >= s.heads * s.dim and min(gate.shape[1], out.shape[1]) >= vc, "delta: columns")
+    _req((runs is None) != (slot is None), "delta: runs or rows")
+    _req(table.dtype == torch.int32 and table.shape[0] <= S.shape[0], "delta: page table")
+    for t in (runs, slot, pos):
+        _req(t is None or (t.dtype == torch.int32 and t.is_contiguous()), "delta: int32 rows")
+    q = {n: _p(t) for n, t in (("runs", runs), ("slot", slot), ("pos", pos))}
+    dk, dv = s.state_dims
+    return DeltaArgs(_p(inp), _p(in32), _p(z), _p(gate), _p(w["conv"]), _p(w["decay"]), _p(w["dt_bias"]), _p(w["norm"]),
+                     _p(S), _p(ring), q["runs"], q["slot"], q["pos"], _p(table), _p(out), inp.stride(0), in32.stride(0),
+                     z.stride(0), gate.stride(0), out.stride(0), *cols, ob, s.heads, s.kv_heads, s.dim, s.vdim, s.taps,
+                     dk, dv, table.shape[1], n_pages, float(s.q_scale), float(s.unit_eps), float(eps))
+
+
+def check_runs(runs_host, rows: int, slots: int) -> None:
+    """Runs inside the batch, one per slot (a state has one writer)."""
+    r0, n, sl, p0 = (runs_host[:, i] for i in range(4))
+    _req(bool((n >= 1).all() and (r0 >= 0).all() and (p0 >= 0).all() and (sl >= 0).all()) and int((r0 + n).max()) <= rows
+         and int(sl.max()) < slots, "delta runs: rows")
+    _req(len(set(sl.tolist())) == sl.numel(), "delta runs: one run per slot and step")
+
+
+def steps(a: DeltaArgs, dtype, n: int, keep: bool) -> None:
+    """n runs step by step. ``keep``: all of one row, their inputs join the ring here (else :func:`ring` follows)."""
+    _check(lib().lsa_delta_steps(is_f32(dtype), ctypes.byref(a), n, int(keep), _stream()), "lsa_delta_steps")
+
+
+def ring(a: DeltaArgs, dtype, n: int) -> None:
+    _check(lib().lsa_delta_ring(is_f32(dtype), ctypes.byref(a), n, _stream()), "lsa_delta_ring")
+
+
+def declare(L: ctypes.CDLL) -> None:
+    """Signatures of these entry points (called by hip.load_library)."""
+    vp, i = ctypes.c_void_p, ctypes.c_int
+    da = ctypes.POINTER(DeltaArgs)
+    hip.set_signatures(L, {
+        "lsa_delta_steps": [i, da, i, i, vp],
+        "lsa_delta_ring": [i, da, i, vp],
+    })

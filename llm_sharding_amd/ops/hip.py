@@ -44,6 +44,8 @@ class EpiArgs(ctypes.Structure):
         ("ss_out", ctypes.c_void_p), ("ss_in", ctypes.c_void_p), ("ss_n", ctypes.c_int), ("ss_eps", ctypes.c_float),
         ("out32", ctypes.c_void_p), ("glu_alpha", ctypes.c_float), ("glu_limit", ctypes.c_float),
         ("glu_shift", ctypes.c_float),
+        ("gate", ctypes.c_void_p), ("ldg", ctypes.c_int), ("col32", ctypes.c_int), ("ldo32", ctypes.c_int),
+        ("act_from", ctypes.c_int), ("cols", ctypes.c_int),
     ]
 
 
@@ -104,18 +106,23 @@ def load_library(path: str, mode: int = ctypes.RTLD_LOCAL) -> ctypes.CDLL:
         "lsa_attn_oproj": [vp, i, vp, vp, vp, vp, vp, i, i, i, i, f, vp, vp, i, i, ctypes.POINTER(EpiArgs), vp, i, vp],
         "lsa_version": [],
     }
+    set_signatures(L, sig)
+    from . import delta, latent, moe, paged_attn, stream
+    for m in (stream, latent, paged_attn, delta, moe):
+        m.declare(L)
+    if os.environ.get("LSA_ATTN_SMALL_MAX_WGS"):  # A/B runs of the small-grid decode attention's range
+        L.lsa_attn_set_small_max_wgs.argtypes = [i]
+        _check(L.lsa_attn_set_small_max_wgs(int(os.environ["LSA_ATTN_SMALL_MAX_WGS"])), "lsa_attn_set_small_max_wgs")
+    return L
+
+
+def set_signatures(L: ctypes.CDLL, sig: dict) -> None:
+    """Argument types of entry points (a family's library has only its own)."""
     for name, args in sig.items():
         if _family and not hasattr(L, name):
             continue
         fn = getattr(L, name)
         fn.argtypes, fn.restype = args, ctypes.c_int
-    if hasattr(L, "lsa_latent_append"):
-        from . import latent
-        latent.declare(L)
-    if os.environ.get("LSA_ATTN_SMALL_MAX_WGS"):  # A/B runs of the small-grid decode attention's range
-        L.lsa_attn_set_small_max_wgs.argtypes = [i]
-        _check(L.lsa_attn_set_small_max_wgs(int(os.environ["LSA_ATTN_SMALL_MAX_WGS"])), "lsa_attn_set_small_max_wgs")
-    return L
 
 
 def _p(t: Optional[torch.Tensor]):
@@ -146,15 +153,24 @@ ACT_NONE, ACT_GELU = 0, 1  # EpiArgs.act (EPI_STORE): identity / tanh-GELU (GPT-
 def make_epi(out=None, resid=None, k_cache=None, v_cache=None, slot=None, pos=None, cos=None,
              sin=None, keys=None, ldo=0, ldr=0, n_heads=0, n_kv=0, head_dim=0, t_max=0,
              col_offset=0, bias=None, act=ACT_NONE, ss_out=None, ss_in=None, ss_eps=0.0, out32=None,
-             glu_alpha=0.0, glu_limit=0.0, glu_shift=0.0) -> EpiArgs:
+             glu_alpha=0.0, glu_limit=0.0, glu_shift=0.0, gate=None, col32=0, ldo32=0, act_from=0, cols=0) -> EpiArgs:
     """Epilogue arguments. ``bias``: optional fp32 [N] added to every output column (in packed
     column order); ``cos=None`` with EPI_QKV: no RoPE, natural q|k|v column order.
     ``ss_out`` / ``ss_in`` (gemm_sk): fp32 [>= M, H/64] row partial sums of squares - a RESID
     GEMM writes them for its outputs, a QKV / SWIGLU GEMM reading the raw residual stream as A
     applies the RMSNorm scale from them (the norm weight is folded into its W). ``out32``: fp32
     output of an EPI_STORE GEMM instead of ``out``. ``glu_limit`` > 0: EPI_SWIGLU computes the
-    clipped gated unit with these constants instead of silu(g) * u (epilogue.h glu)."""
+    clipped gated unit with these constants instead of silu(g) * u (epilogue.h glu).
+    An EPI_STORE GEMM of several parts: with both ``out`` and ``out32``, columns from ``col32`` on go to
+    out32 [M][ldo32]; ``act`` applies to columns from ``act_from`` on. ``gate`` [M, >= cols] (with out32
+    alone): out32[:, :cols] += sigmoid(gate) * y instead of the store."""
     _req(out32 is None or out32.dtype == torch.float32, "epilogue: out32 must be fp32")
+    if out is None:
+        col32, ldo32 = 0, ldo
+    _req(col32 % 16 == 0 and act_from % 16 == 0 and cols % 16 == 0 and ldo32 % 4 == 0, "epilogue: column parts of whole 16s")
+    _req(gate is None or (out is None and out32 is not None and 0 < cols <= min(ldo, gate.shape[1]) and act == ACT_NONE
+                          and gate.stride(1) == 1 and gate.stride(0) % 8 == 0 and gate.data_ptr() % 16 == 0),
+         "epilogue: gated accumulation")
     if bias is not None:
         _req(bias.dtype == torch.float32 and bias.is_contiguous(), "epilogue bias: contiguous fp32")
     # vectorised epilogues store 16-B runs: rows must start 16-B aligned
@@ -168,7 +184,8 @@ def make_epi(out=None, resid=None, k_cache=None, v_cache=None, slot=None, pos=No
     return EpiArgs(_p(out), _p(resid), _p(k_cache), _p(v_cache), _p(slot), _p(pos), _p(cos), _p(sin),
                    _p(keys), _p(bias), ldo, ldr, n_heads, n_kv, head_dim, t_max, col_offset, int(act),
                    _p(ss_out), _p(ss_in), 0 if ssb is None else ssb.shape[1], float(ss_eps), _p(out32),
-                   float(glu_alpha), float(glu_limit), float(glu_shift))
+                   float(glu_alpha), float(glu_limit), float(glu_shift), _p(gate), 0 if gate is None else gate.stride(0),
+                   col32, ldo32, act_from, cols)
 
 
 # ------------------------------------------------------------------------------ projections

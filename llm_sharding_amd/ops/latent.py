@@ -1,5 +1,4 @@
-"""Bindings and weights of the latent-attention kernels (csrc/kernels/latent*.hip), the fp32-stream
-kernels (stream_ops.hip) and the fp32 projections (linear_f32.hip).
+"""Bindings and weights of the latent-attention kernels (csrc/kernels/latent*.hip).
 
 The conventions of :mod:`.hip` hold: shapes are checked on the host, launches go to torch's current
 stream, nothing falls back to another implementation."""
@@ -12,7 +11,9 @@ import torch
 
 from . import hip
 from .hip import _check, _p, _req, _stream, lib
-from .packing import fuse_gate_up, pack_b
+from .packing import pack_b
+from .stream import (Linear, cast_rows, is_f32, logits_argmax, pad2, stream_add_norm, stream_embed,  # noqa: F401
+                     stream_norm)
 
 PAGE = 64  # tokens per cache page (LAT_PAGE in csrc/kernels/latent.h)
 
@@ -22,108 +23,6 @@ class LatentArgs(ctypes.Structure):
                 + [(n, ctypes.c_int) for n in ("max_pages", "n_pages", "heads", "dim", "rot_dim", "rot_dims", "vdim",
                                                "kv_rank", "q_rank", "dkp", "rp", "dvp", "krp")]
                 + [("scale", ctypes.c_float), ("eps", ctypes.c_float)])
-
-
-def is_f32(dt) -> int:
-    _req(dt in (torch.float32, torch.bfloat16), f"unsupported compute type {dt}")
-    return int(dt == torch.float32)
-
-
-# ------------------------------------------------------------------------------ projections
-def pad2(w: torch.Tensor, n: int, k: int) -> torch.Tensor:
-    """[N, K] -> [n, k], zeros behind."""
-    out = torch.zeros((n, k), dtype=w.dtype, device=w.device)
-    out[:w.shape[0], :w.shape[1]] = w
-    return out
-
-
-class Linear:
-    """One projection of a stack engine in the engine's type: N and K padded to whole 128-wide
-    blocks with zeros, so that every kernel configuration takes it; bf16 weights packed for
-    the MFMA kernels, fp32 ones row-major."""
-
-    def __init__(self, w: torch.Tensor, k: int = 0):
-        N, K = w.shape
-        self.n, self.k = -(-N // 128) * 128, k or -(-K // 128) * 128
-        wp = w if w.shape == (self.n, self.k) else pad2(w, self.n, self.k)
-        self.f32 = is_f32(w.dtype)
-        self.w = wp.contiguous() if self.f32 else pack_b(wp).contiguous()
-
-    @staticmethod
-    def glu(gate: torch.Tensor, up: torch.Tensor) -> "Linear":
-        """Gate and up projection, interleaved for the gated epilogue; ff padded to 128."""
-        ff, K = gate.shape
-        n = -(-ff // 128) * 128
-        return Linear(fuse_gate_up(pad2(gate, n, K), pad2(up, n, K)))
-
-    def tensors(self) -> list:
-        return [self.w]
-
-    def __call__(self, x: torch.Tensor, rows: int, out: torch.Tensor, ws=None, sk_ws=None, glu=None, keys=None,
-                 bias=None, col_offset: int = 0) -> None:
-        """out[:rows] = x[:rows] . W^T (``out`` bf16 or fp32), or with ``glu`` (a GluSpec) the gated
-        unit of the interleaved halves; ``keys``: argmax keys instead of an output."""
-        _req(x.dim() == 2 and x.shape[0] >= rows and x.shape[1] >= self.k and x.stride(1) == 1, "linear: input shape")
-        kw = {}
-        if keys is None:
-            n_out = self.n // 2 if glu is not None else self.n
-            _req(out.shape[0] >= rows and out.shape[1] >= n_out and out.stride(1) == 1, "linear: output shape")
-            kw["ldo"] = out.stride(0)
-            kw["out32" if out.dtype == torch.float32 else "out"] = out
-        if glu is not None:
-            kw.update(glu_alpha=glu.alpha, glu_limit=glu.limit, glu_shift=glu.shift)
-        epi = hip.EPI_SWIGLU if glu is not None else (hip.EPI_STORE if keys is None else hip.EPI_ARGMAX)
-        ep = hip.make_epi(keys=keys, bias=bias, col_offset=col_offset, **kw)
-        if self.f32:
-            _req(x.dtype == torch.float32 and x.is_cuda and keys is None, "linear: fp32 cuda input")
-            _check(lib().lsa_linear_f32(_p(x), x.stride(0), _p(self.w), rows, self.n, self.k, epi, ctypes.byref(ep),
-                                        _stream()), "lsa_linear_f32")
-        elif rows <= 128:
-            hip.gemv(x, self.w, rows, self.n, self.k, epi, ep, ws=ws)
-        else:
-            hip.gemm_sk(x, self.w, rows, self.n, self.k, epi, ep, ws=sk_ws)
-
-
-# ------------------------------------------------------------------------------ fp32 stream
-def stream_embed(ids, table, scale: float, x, xc, rows: int) -> None:
-    W = x.shape[1]
-    _req(ids.dtype == torch.int32 and ids.is_cuda and ids.numel() >= rows, "stream_embed: int32 ids")
-    _req(x.dtype == torch.float32 and table.dtype == xc.dtype and table.shape[1] >= W and xc.shape[1] >= W
-         and min(x.shape[0], xc.shape[0]) >= rows, "stream_embed: shapes")
-    _check(lib().lsa_stream_embed(is_f32(xc.dtype), _p(ids), rows, _p(table), table.stride(0), float(scale), W, _p(x),
-                                  x.stride(0), _p(xc), xc.stride(0), _stream()), "lsa_stream_embed")
-
-
-def cast_rows(x, xc, rows: int, x2=None) -> None:
-    """xc = x in the projections' type; ``x2`` (fp32): a copy as it is."""
-    _req(x.dtype == torch.float32 and x.stride(1) == 1 and xc.shape[1] >= x.shape[1]
-         and min(x.shape[0], xc.shape[0]) >= rows, "cast_rows: shapes")
-    _req(x2 is None or (x2.dtype == torch.float32 and x2.shape[0] >= rows and x2.shape[1] >= x.shape[1]), "cast_rows: x2")
-    _check(lib().lsa_cast_rows(is_f32(xc.dtype), _p(x), x.stride(0), rows, x.shape[1], _p(xc), xc.stride(0), _p(x2),
-                               0 if x2 is None else x2.stride(0), _stream()), "lsa_cast_rows")
-
-
-def stream_add_norm(y, gain, eps: float, x, xc, rows: int) -> None:
-    """x += rms(y) * gain; xc = x in the projections' type."""
-    W = gain.numel()
-    _req(all(t.dtype == torch.float32 for t in (y, gain, x)) and y.shape[1] >= W and x.shape[1] >= W and xc.shape[1] >= W
-         and min(t.shape[0] for t in (y, x, xc)) >= rows, "stream_add_norm: shapes")
-    _check(lib().lsa_stream_add_norm(is_f32(xc.dtype), _p(y), y.stride(0), _p(gain), float(eps), rows, W, _p(x),
-                                     x.stride(0), _p(xc), xc.stride(0), _stream()), "lsa_stream_add_norm")
-
-
-def stream_norm(x, gain, eps: float, out, rows: int) -> None:
-    W = gain.numel()
-    _req(x.dtype == torch.float32 and gain.dtype == torch.float32 and x.shape[1] >= W and out.shape[1] >= W
-         and min(x.shape[0], out.shape[0]) >= rows, "stream_norm: shapes")
-    _check(lib().lsa_stream_norm(is_f32(out.dtype), _p(x), x.stride(0), _p(gain), float(eps), rows, W, _p(out),
-                                 out.stride(0), _stream()), "lsa_stream_norm")
-
-
-def logits_argmax(lg, rows: int, vocab: int, keys, offset: int = 0) -> None:
-    _req(lg.dtype == torch.float32 and lg.shape[0] >= rows and lg.shape[1] >= vocab and keys.dtype == torch.int64
-         and keys.numel() >= rows, "logits_argmax: shapes")
-    _check(lib().lsa_logits_argmax(_p(lg), lg.stride(0), rows, vocab, offset, _p(keys), _stream()), "lsa_logits_argmax")
 
 
 # ------------------------------------------------------------------------------ latent attention
@@ -274,13 +173,7 @@ def declare(L: ctypes.CDLL) -> None:
     """Signatures of these entry points (called by hip.load_library)."""
     vp, i, f = ctypes.c_void_p, ctypes.c_int, ctypes.c_float
     la = ctypes.POINTER(LatentArgs)
-    sig = {
-        "lsa_stream_embed": [i, vp, i, vp, i, f, i, vp, i, vp, i, vp],
-        "lsa_cast_rows": [i, vp, i, i, i, vp, i, vp, i, vp],
-        "lsa_stream_add_norm": [i, vp, i, vp, f, i, i, vp, i, vp, i, vp],
-        "lsa_stream_norm": [i, vp, i, vp, f, i, i, vp, i, vp],
-        "lsa_logits_argmax": [vp, i, i, i, i, vp, vp],
-        "lsa_linear_f32": [vp, i, vp, i, i, i, i, ctypes.POINTER(hip.EpiArgs), vp],
+    hip.set_signatures(L, {
         "lsa_latent_append": [i, la, i, vp, i, i, i, vp, vp, vp, i, vp],
         "lsa_latent_absorb": [i, la, i, vp, i, vp, vp, vp],
         "lsa_latent_attend": [i, la, i, vp, i, vp, vp, vp],
@@ -290,7 +183,4 @@ def declare(L: ctypes.CDLL) -> None:
         "lsa_latent_value_mfma": [la, i, vp, vp, i, vp, vp, i, vp, i, vp],
         "lsa_latent_prefill": [la, vp, i, vp, i, vp, i, vp, vp, i, vp, i, vp],
         "lsa_latent_gather": [la, vp, i, vp, vp],
-    }
-    for name, args in sig.items():
-        fn = getattr(L, name)
-        fn.argtypes, fn.restype = args, ctypes.c_int
+    })

@@ -1,0 +1,133 @@
+"""Bindings of the paged grouped-query attention kernels (csrc/kernels/paged_attn*.hip).
+
+The conventions of :mod:`.hip` hold: shapes are checked on the host, launches go to torch's current
+stream, nothing falls back to another implementation."""
+from __future__ import annotations
+
+import ctypes
+
+import torch
+
+from . import hip
+from .hip import _check, _p, _req, _stream, lib
+from .stream import is_f32
+
+PAGE = 64        # tokens per cache page (ATT_PAGE in csrc/kernels/paged_attn.h)
+TILE_ROWS = 128  # query rows of one attn_tiles workgroup, at most
+ALL = (1 << 31) - 1
+
+
+class AttnArgs(ctypes.Structure):
+    _fields_ = ([(n, ctypes.c_void_p) for n in ("k", "v", "table", "slot", "pos", "index", "hscale")]
+                + [(n, ctypes.c_int) for n in ("max_pages", "n_pages", "heads", "kv_heads", "dim", "vdim", "dkp", "dvp",
+                                               "window", "keep")]
+                + [("softcap", ctypes.c_float)])
+
+
+def tuned_size(s) -> bool:
+    """The MFMA kernels take this size (others run the plain kernel)."""
+    return s.dkp in (64, 128, 256) and s.dvp in (64, 128, 256)
+
+
+def head_tiles(s) -> int:
+    """Workgroups per (row, split) of :func:`rows`: 16 heads of one kv head each."""
+    return s.kv_heads * -(-s.group // 16)
+
+
+def cache_shapes(s, pages: int) -> tuple:
+    return (pages, s.kv_heads, PAGE, s.dkp), (pages, s.kv_heads, s.dvp, PAGE)
+
+
+def value_order() -> torch.Tensor:
+    """Place of token r of a page in a value row (att_vidx)."""
+    r = torch.arange(PAGE)
+    return (r & 32) | ((r & 12) << 1) | ((r & 16) >> 2) | (r & 3)
+
+
+def make_args(s, cache: tuple, table, slot, pos, hscale, index=None) -> AttnArgs:
+    """``cache``: (keys, values) of :func:`cache_shapes`; ``table`` int32 [slots, max_pages]; ``slot`` / ``pos``
+    int32 [rows]; ``hscale`` fp32 [heads]; ``index`` int32 [entries]."""
+    k, v = cache
+    _req(tuple(k.shape[1:]) == (s.kv_heads, PAGE, s.dkp) and tuple(v.shape) == (k.shape[0], s.kv_heads, s.dvp, PAGE)
+         and k.is_contiguous() and v.is_contiguous() and k.is_cuda and k.dtype == v.dtype, "attention: cache shapes")
+    _req(table.dtype == torch.int32 and table.dim() == 2 and table.is_contiguous(), "attention: int32 page table")
+    _req(slot.dtype == torch.int32 and pos.dtype == torch.int32, "attention: int32 slot / pos")
+    _req(index is None or index.dtype == torch.int32, "attention: int32 index")
+    _req(hscale.dtype == torch.float32 and hscale.numel() == s.heads, "attention: head scales")
+    return AttnArgs(k.data_ptr(), v.data_ptr(), table.data_ptr(), slot.data_ptr(), pos.data_ptr(),
+                    None if index is None else index.data_ptr(), hscale.data_ptr(), table.shape[1], k.shape[0], s.heads,
+                    s.kv_heads, s.dim, s.vdim, s.dkp, s.dvp, s.window or ALL, s.keep_first, float(s.softcap))
+
+
+def _inputs(a: AttnArgs, inp, ok: int, ov: int) -> None:
+    _req(inp.stride(1) == 1 and inp.shape[1] >= max(ok + a.kv_heads * a.dkp, ov + a.kv_heads * a.dvp), "append: columns")
+
+
+def append(a: AttnArgs, n: int, inp, ok: int, ov: int) -> None:
+    """Keys at column ``ok`` and values at ``ov`` of n rows (or a.index' rows) -> their places in the cache."""
+    _inputs(a, inp, ok, ov)
+    _check(lib().lsa_attn_append(is_f32(inp.dtype), ctypes.byref(a), n, _p(inp), inp.stride(0), ok, ov, _stream()),
+           "lsa_attn_append")
+
+
+def check_tiles(tiles_host, rows: int, slots: int, max_pages: int) -> None:
+    r0, nr, sl, p0 = (tiles_host[:, i] for i in range(4))
+    _req(bool((nr >= 1).all() and (nr <= TILE_ROWS).all() and (r0 >= 0).all()) and int((r0 + nr).max()) <= rows,
+         "attention tiles: rows")
+    _req(bool((sl >= 0).all() and (p0 >= 0).all()) and int(sl.max()) < slots
+         and int((p0 + nr).max()) <= max_pages * PAGE, "attention tiles: positions")
+
+
+def append_tiles(a: AttnArgs, tiles, inp, ok: int, ov: int) -> None:
+    """As :func:`append` for the rows of checked tiles [row0, rows, slot, pos0]."""
+    _inputs(a, inp, ok, ov)
+    _check(lib().lsa_attn_append_tiles(is_f32(inp.dtype), ctypes.byref(a), _p(tiles), tiles.shape[0], _p(inp),
+                                       inp.stride(0), ok, ov, _stream()), "lsa_attn_append_tiles")
+
+
+def _shapes(a: AttnArgs, q, gate, out, dtype=None) -> tuple:
+    _req(q.dtype == out.dtype and (gate is None or gate.dtype == q.dtype) and (dtype is None or q.dtype == dtype),
+         "attention: types")
+    _req(q.stride(1) == 1 and q.shape[1] >= a.heads * a.dkp and out.stride(1) == 1 and out.shape[1] >= a.heads * a.dvp
+         and (gate is None or (gate.stride(1) == 1 and gate.shape[1] >= a.heads)), "attention: shapes")
+    return _p(q), q.stride(0), _p(gate), 0 if gate is None else gate.stride(0), _p(out), out.stride(0)
+
+
+def plain(a: AttnArgs, n: int, q, gate, out) -> None:
+    """Attention of n rows (or a.index' rows), any size, both types. ``gate`` [rows, >= heads] or None."""
+    _check(lib().lsa_attn_plain(is_f32(q.dtype), ctypes.byref(a), n, *_shapes(a, q, gate, out), _stream()),
+           "lsa_attn_plain")
+
+
+def rows(a: AttnArgs, n: int, q, gate, out, ns: int, po, pm) -> None:
+    """As :func:`plain` on MFMA, keys in ``ns`` splits (workspaces fp32, used when ns > 1)."""
+    e = n * a.heads * ns
+    _req(ns == 1 or (po.dtype == pm.dtype == torch.float32 and po.numel() >= e * a.dvp and pm.numel() >= 2 * e),
+         "attention: workspace")
+    io = _shapes(a, q, gate, out, torch.bfloat16)
+    _check(lib().lsa_attn_rows(ctypes.byref(a), n, *io, ns, _p(po), _p(pm), _stream()), "lsa_attn_rows")
+    if ns > 1:
+        _check(lib().lsa_attn_merge(ctypes.byref(a), n, _p(po), _p(pm), ns, *io[2:], _stream()), "lsa_attn_merge")
+
+
+def tiles(a: AttnArgs, tiles_dev, q, gate, out) -> None:
+    """Attention of the rows of checked tiles [row0, rows, slot, pos0], bf16."""
+    _req(tiles_dev.dtype == torch.int32 and tiles_dev.dim() == 2 and tiles_dev.shape[1] == 4 and tiles_dev.is_contiguous(),
+         "attention tiles: table")
+    _check(lib().lsa_attn_tiles(ctypes.byref(a), _p(tiles_dev), tiles_dev.shape[0],
+                                *_shapes(a, q, gate, out, torch.bfloat16), _stream()), "lsa_attn_tiles")
+
+
+def declare(L: ctypes.CDLL) -> None:
+    """Signatures of these entry points (called by hip.load_library)."""
+    vp, i = ctypes.c_void_p, ctypes.c_int
+    aa = ctypes.POINTER(AttnArgs)
+    io = [vp, i, vp, i, vp, i]
+    hip.set_signatures(L, {
+        "lsa_attn_append": [i, aa, i, vp, i, i, i, vp],
+        "lsa_attn_append_tiles": [i, aa, vp, i, vp, i, i, i, vp],
+        "lsa_attn_plain": [i, aa, i] + io + [vp],
+        "lsa_attn_rows": [aa, i] + io + [i, vp, vp, vp],
+        "lsa_attn_merge": [aa, i, vp, vp, i, vp, i, vp, i, vp],
+        "lsa_attn_tiles": [aa, vp, i] + io + [vp],
+    })

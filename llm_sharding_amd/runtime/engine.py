@@ -30,7 +30,7 @@ import torch
 import torch.nn.functional as F
 
 from ..config import LlamaConfig, ceil_div
-from ..models import deretar as DT
+from ..models import designs
 from ..models import gpt2 as G2
 from ..models import weights as W
 from ..models.rope import rope_table
@@ -130,31 +130,36 @@ class RandomSource(WeightSource):
 
 
 class StackFolderSource(WeightSource):
-    """A stack design's checkpoint folder (config.json + model.safetensors, models/deretar.py)."""
+    """A stack design's checkpoint folder (config.json + model.safetensors, models/designs.py)."""
 
     def __init__(self, path: str, cfg):
         self.path, self.cfg = path, cfg
-        self.tensors = DT.DeretarTensors(path)
+        self.design = designs.of(cfg)
+        self.tensors = designs.CheckpointTensors(path)
 
     def layer(self, i, device, dtype):
         o = self.cfg.layers[i].owner
-        shapes = DT.layer_shapes(self.cfg, o)
+        shapes = self.design.layer_shapes(self.cfg, o)
         t = self.tensors.get({k: f"l{o}.{k}" for k in shapes}, device, dtype)
         for k, shp in shapes.items():
             if tuple(t[k].shape) != shp:
                 raise ValueError(f"l{o}.{k} has shape {tuple(t[k].shape)}, config.json says {shp}")
         return t
 
-    def embedding(self, device, dtype):
-        t = self.tensors.get({"w": "embed"}, device, dtype)["w"]
+    def _table(self, name, device, dtype):
+        t = self.tensors.get({"w": name}, device, dtype)["w"]
         if tuple(t.shape) != (self.cfg.vocab_size, self.cfg.hidden_size):
-            raise ValueError(f"embed has shape {tuple(t.shape)}")
+            raise ValueError(f"{name} has shape {tuple(t.shape)}")
         return t
+
+    def embedding(self, device, dtype):
+        return self._table("embed", device, dtype)
 
     def final_norm(self, device, dtype):
         return self.tensors.get({"w": "final.norm"}, device, dtype)["w"]
 
-    lm_head = embedding  # tied
+    def lm_head(self, device, dtype):
+        return self._table("embed" if self.design.TIED_HEAD else "head", device, dtype)
 
 
 class StackRandomSource(WeightSource):
@@ -162,17 +167,20 @@ class StackRandomSource(WeightSource):
 
     def __init__(self, cfg, seed: int = 0):
         self.cfg, self.seed = cfg, seed
+        self.design = designs.of(cfg)
 
     def layer(self, i, device, dtype):
-        return DT.random_layer(self.cfg, i, dtype, device, self.seed)
+        return self.design.random_layer(self.cfg, i, dtype, device, self.seed)
 
     def embedding(self, device, dtype):
-        return DT.random_embedding(self.cfg, dtype, device, self.seed)
+        return self.design.random_embedding(self.cfg, dtype, device, self.seed)
 
     def final_norm(self, device, dtype):
-        return DT.random_final_norm(self.cfg, dtype, device, self.seed)
+        return self.design.random_final_norm(self.cfg, dtype, device, self.seed)
 
-    lm_head = embedding
+    def lm_head(self, device, dtype):
+        return self.embedding(device, dtype) if self.design.TIED_HEAD else self.design.random_head(
+            self.cfg, dtype, device, self.seed)
 
 
 @dataclass
@@ -542,6 +550,9 @@ class StageEngine:
     # Cache memory that sequences share (paged engines): units in all, units a sequence of ``tokens``
     # takes, and room for a slot's next decoded token. A static cache has no shared budget.
     cache_budget: Optional[int] = None
+
+    # whether running a token twice differs from once (recurrent layers)
+    carries_state = False
 
     def cache_need(self, tokens: int) -> int:
         return 0
@@ -1090,6 +1101,8 @@ class DecodeGraph:
         run (if any) is undone (positions restored) and never communicates."""
         pos0, tok0 = self.pos.clone(), self.tokens.clone()
         kin0 = self.keys_in.clone() if self.split_head else None
+        if self.eng.carries_state:  # rows without a position are idle: the warm-up moves no state on
+            self.pos.fill_(-1)
         s = torch.cuda.Stream(device=self.eng.device)
         s.wait_stream(torch.cuda.current_stream(self.eng.device))
         with torch.cuda.stream(s):

@@ -1,0 +1,136 @@
+"""Feed-forwards of a layer stack: the clipped gated unit, the dense gelu layer and the mixture of experts.
+
+A feed-forward that runs beside its mixer on the same input gives the block the rows it wants of the
+block's input projection (``input_parts``) and takes their columns."""
+from __future__ import annotations
+
+import torch
+import torch.nn.functional as F
+
+from ..models.stack import DenseSpec, GluSpec, MoeSpec
+
+
+class Glu:
+    """Gate / up / down projection of a clipped gated unit."""
+
+    def __init__(self, spec: GluSpec, t: dict, gpu: bool):
+        self.spec = spec
+        self.raw = None if gpu else t
+        if gpu:
+            from ..ops import stream as L
+            self.gate_up, self.down = L.Linear.glu(t["gate"], t["up"]), L.Linear(t["down"])
+
+    def tensors(self) -> list:
+        return list(self.raw.values()) if self.raw is not None else self.gate_up.tensors() + self.down.tensors()
+
+    def scratch(self) -> dict:
+        return {"act": self.down.k}
+
+    def projections(self) -> list:
+        return [self.gate_up, self.down]
+
+    def forward(self, eng, x, y, rows: int) -> None:
+        act = eng.scratch_view("act", rows, self.down.k)
+        eng.project(self.gate_up, x, rows, act, glu=self.spec)
+        eng.project(self.down, act, rows, y)
+
+    def forward_torch(self, x) -> torch.Tensor:
+        w, s = {k: v.float() for k, v in self.raw.items()}, self.spec
+        g = F.linear(x, w["gate"]).clamp(max=s.limit)
+        u = F.linear(x, w["up"]).clamp(-s.limit, s.limit)
+        return F.linear(g * torch.sigmoid(s.alpha * g) * (u + s.shift), w["down"])
+
+
+class Dense:
+    """W_down gelu(W_up h): the up rows ride in the block's input projection, gelu in its epilogue."""
+
+    def __init__(self, spec: DenseSpec, t: dict, gpu: bool):
+        self.spec = spec
+        self.raw = None if gpu else t
+        if gpu:
+            from ..ops import stream as L
+            self.down = L.Linear(t["down"])
+            self.up = F.pad(t["up"], (0, 0, 0, self.down.k - spec.ff))  # as wide as the down projection reads
+
+    def input_parts(self) -> list:
+        return [("up", self.up, None, "gelu")]
+
+    def tensors(self) -> list:
+        return list(self.raw.values()) if self.raw is not None else self.down.tensors()
+
+    def scratch(self) -> dict:
+        return {}
+
+    def projections(self) -> list:
+        return [self.down]
+
+    def forward(self, eng, h, inp, in32, col: dict, gate, rows: int) -> dict:
+        """The gated result joins the stream here, or is handed to the block's join."""
+        act = inp[:, col["up"]:col["up"] + self.down.k]
+        return eng.project_gated(self.down, act, rows, gate, "y2", "second")
+
+    def forward_torch(self, x) -> torch.Tensor:
+        w = {k: v.float() for k, v in self.raw.items()}
+        return F.linear(F.gelu(F.linear(x, w["up"]), approximate="tanh"), w["down"])
+
+
+class Moe:
+    """Experts: routing, grouping and both products (csrc/kernels/moe.h); the router's rows ride in the block's
+    input projection, the weighted sum of a row's experts is left to its join."""
+
+    def __init__(self, spec: MoeSpec, t: dict, gpu: bool):
+        self.spec = spec
+        self.raw = None if gpu else t
+        if gpu:
+            from ..ops import moe as X
+            e = range(spec.experts)
+            self.router = t["router"]
+            self.experts = X.Experts(*([t[f"e{i}.{k}"] for i in e] for k in ("gate", "up", "down")))
+
+    def input_parts(self) -> list:
+        return [("router", self.router, None, "f32")]
+
+    def tensors(self) -> list:
+        return list(self.raw.values()) if self.raw is not None else self.experts.tensors()
+
+    def scratch(self) -> dict:
+        top = self.spec.top
+        return {"act": top * self.experts.ff, "ye": top * self.experts.width, "pairs": (3 * top, torch.int32),
+                "tiles": (8 * top, torch.int32), "pair_w": (top, torch.float32)}
+
+    def projections(self) -> list:
+        return []
+
+    def forward(self, eng, h, inp, in32, col: dict, gate, rows: int) -> dict:
+        from ..ops import moe as X
+        s, x = self.spec, self.experts
+        pairs = rows * s.top
+        expert, order, place = eng.scratch_view("pairs", rows, 3 * s.top).reshape(3, pairs)
+        weight, tiles = eng.scratch_view("pair_w", rows, s.top).reshape(-1), eng.scratch_view("tiles", rows, 8 * s.top)
+        act, ye = eng.scratch_view("act", pairs, x.ff), eng.scratch_view("ye", pairs, x.width)
+        X.route(in32[:, col["router"]:], rows, s.experts, s.top, expert, weight)
+        tr = X.tile_rows(pairs, s.experts, x.f32)
+        nt = X.group(expert, pairs, s.experts, tr, order, place, tiles)
+        X.gemm(tiles, nt, tr, order, s.top, h, x.up, 2 * x.ff, x.width, act, pairs, glu=True)
+        X.gemm(tiles, nt, tr, order, s.top, act, x.down, x.width, x.ff, ye, pairs, glu=False)
+        return {"experts": (ye, weight, place, s.top), "gate2": gate}
+
+    def forward_torch(self, x) -> torch.Tensor:
+        w, s = {k: v.float() for k, v in self.raw.items()}, self.spec
+        best, at = F.linear(x, w["router"]).topk(s.top, -1)
+        weight = torch.softmax(best, -1)
+        out = torch.zeros_like(x)
+        for e in range(s.experts):
+            row, k = (at == e).nonzero(as_tuple=True)
+            if row.numel():
+                h = x[row]
+                a = F.silu(F.linear(h, w[f"e{e}.gate"])) * F.linear(h, w[f"e{e}.up"])
+                out.index_add_(0, row, F.linear(a, w[f"e{e}.down"]) * weight[row, k, None])
+        return out
+
+
+def feed_forward(spec, t: dict, gpu: bool):
+    return {GluSpec: Glu, DenseSpec: Dense, MoeSpec: Moe}[type(spec)](spec, t, gpu)
+
+
+__all__ = ["Glu", "Dense", "Moe", "feed_forward"]

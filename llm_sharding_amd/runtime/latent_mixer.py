@@ -16,12 +16,11 @@ flash kernel; everything else attends over the latents themselves.
 """
 from __future__ import annotations
 
-from typing import Optional
-
 import torch
 import torch.nn.functional as F
 
 from ..models.stack import LatentSpec, pad_to
+from .plan import Plan
 
 
 def rotation_tables(spec: LatentSpec, n: int, device) -> tuple:
@@ -88,6 +87,12 @@ class Weights:
             ts += lin.tensors() if lin is not None else []
         return ts
 
+    def scratch(self) -> dict:
+        return {"inp": self.inp.n, "cq": self.uq.k, "q": self.uq.n, "attn": self.out.k}
+
+    def projections(self) -> list:
+        return [p for p in (self.inp, self.uq, self.out, self.kv) if p is not None]
+
     # ------------------------------------------------------------------ GPU
     def forward(self, eng, x: torch.Tensor, y: torch.Tensor, cache: torch.Tensor, slot, pos, rows: int, plan) -> None:
         """``x`` [rows, padded width] -> ``y`` fp32 [rows, padded width]; appends to ``cache``."""
@@ -104,14 +109,14 @@ class Weights:
         gate = inp[:, self.og:]
         absorb, attend, value = ((L.absorb_mfma, L.attend_mfma, L.value_mfma) if self.tuned
                                  else (L.absorb, L.attend, L.value))
-        for idx, n in plan.absorbed_chunks(self):
+        for idx, n in absorbed_chunks(plan, self):
             b = a if idx is None else L.make_args(s, cache, table, slot, pos, cos, sin, eng.cfg.norm_eps, index=idx)
             qt, po, pm = eng.attend_scratch()
-            ns = max(1, min(plan.nsplit(eng, self), eng.ATTEND_ITEMS // n))
+            ns = max(1, min(key_splits(plan, self), eng.ATTEND_ITEMS // n))
             absorb(b, n, q, self.wk, qt)
             attend(b, n, qt, ns, po, pm)
             value(b, n, po, pm, ns, self.wv, gate, ao)
-        for g in plan.expanded_groups(self):
+        for g in _split(plan, self)[2]:
             lat, kv = eng.expand_scratch(s, g.tokens, self.kv.n)
             L.gather(a, g.src, g.tokens, lat)
             eng.project(self.kv, lat, g.tokens, kv)
@@ -172,74 +177,46 @@ class Group:
         self.tiles = self.tiles_host.to(device)
 
 
-class Plan:
-    """How one row batch's attention runs: built once per forward, used by every layer."""
-
-    GROUP_TOKENS = 1 << 16  # expanded tokens at a time (bounds the expanded keys' and values' memory)
-
-    def __init__(self, eng, rows: int, runs: Optional[list], nsplit: Optional[int] = None):
-        """``runs``: [(first row, rows, slot, first position)] covering the batch, or None when only
-        the device knows (a decode graph): everything absorbed."""
-        self.eng, self.rows, self.runs, self._ns = eng, rows, runs, nsplit
-        self._cache: dict = {}
-
-    @staticmethod
-    def find_runs(slot, pos) -> list:
-        """Stretches of one slot's consecutive positions in int64 tensors (host)."""
-        new = torch.ones(slot.numel(), dtype=torch.bool)
-        new[1:] = (slot[1:] != slot[:-1]) | (pos[1:] != pos[:-1] + 1)
-        at = new.nonzero().flatten()
-        ends = torch.cat([at[1:], torch.tensor([slot.numel()])])
-        return list(zip(at.tolist(), (ends - at).tolist(), slot[at].tolist(), pos[at].tolist()))
-
-    def _split(self, w: Weights):
-        key = w.spec if w.expand else None
-        if key not in self._cache:
-            if self.runs is None or not w.expand:
-                self._cache[key] = (self.rows, None, [])
-            else:
-                long = [r for r in self.runs if r[1] >= self.eng.expand_min]
-                if not long:
-                    self._cache[key] = (self.rows, None, [])
-                else:
-                    from ..ops import latent as L
-                    idx = [i for r in self.runs if r[1] < self.eng.expand_min for i in range(r[0], r[0] + r[1])]
-                    groups, cur, tok = [], [], 0
-                    rows = L.prefill_tile_rows(sum(r[1] for r in long), w.spec.heads)
-                    for r in long:
-                        if cur and tok + r[1] + r[3] > self.GROUP_TOKENS:
-                            groups.append(Group(cur, rows, self.eng.device))
-                            cur, tok = [], 0
-                        cur.append(r)
-                        tok += r[1] + r[3]
-                    groups.append(Group(cur, rows, self.eng.device))
-                    dev = torch.tensor(idx, dtype=torch.int32).to(self.eng.device) if idx else None
-                    self._cache[key] = (len(idx), dev, groups)
-        return self._cache[key]
-
-    def n_absorbed(self, w) -> int:
-        return self._split(w)[0]
-
-    def absorbed_chunks(self, w) -> list:
-        """[(row indices or None for all rows, count)] of the absorbed form, at most
-        ``ATTEND_ITEMS`` at a time (its buffers)."""
-        n, idx, _ = self._split(w)
-        cap = self.eng.ATTEND_ITEMS
-        if idx is None and n <= cap:
-            return [(None, n)] if n else []
-        if idx is None:
-            idx = torch.arange(n, dtype=torch.int32, device=self.eng.device)
-        return [(idx[c:c + cap], min(cap, n - c)) for c in range(0, n, cap)]
-
-    def expanded_groups(self, w) -> list:
-        return self._split(w)[2]
-
-    def nsplit(self, eng, w) -> int:
-        """Splits of a row's keys, so that a small batch still fills the chip."""
-        if self._ns is None:
-            longest = max(p0 + n for _, n, _, p0 in self.runs)
-            return eng.latent_nsplit(w.spec, self.n_absorbed(w), longest)
-        return self._ns
+GROUP_TOKENS = 1 << 16  # expanded tokens at a time (bounds the expanded keys' and values' memory)
 
 
-__all__ = ["Weights", "Plan", "Group", "rotation_tables"]
+def _split(plan: Plan, w: Weights) -> tuple:
+    """(row indices or None for all rows, their count, groups): what runs absorbed and what expanded."""
+    def make():
+        idx, n, long = plan.split_rows(plan.eng.expand_min) if w.expand else (None, plan.rows, [])
+        if not long:
+            return None, plan.rows, []
+        from ..ops import latent as L
+        groups, cur, tok = [], [], 0
+        rows = L.prefill_tile_rows(sum(r[1] for r in long), w.spec.heads)
+        for r in long:
+            if cur and tok + r[1] + r[3] > GROUP_TOKENS:
+                groups.append(Group(cur, rows, plan.eng.device))
+                cur, tok = [], 0
+            cur.append(r)
+            tok += r[1] + r[3]
+        groups.append(Group(cur, rows, plan.eng.device))
+        return idx, n, groups
+    return plan.memo(("latent", w.spec if w.expand else None), make)
+
+
+def absorbed_chunks(plan: Plan, w: Weights) -> list:
+    """[(row indices or None for all rows, count)] of the absorbed form, at most ``ATTEND_ITEMS`` at a
+    time (its buffers)."""
+    idx, n, _ = _split(plan, w)
+    cap = plan.eng.ATTEND_ITEMS
+    if idx is None and n <= cap:
+        return [(None, n)] if n else []
+    if idx is None:
+        idx = torch.arange(n, dtype=torch.int32, device=plan.eng.device)
+    return [(idx[c:c + cap], min(cap, n - c)) for c in range(0, n, cap)]
+
+
+def key_splits(plan: Plan, w: Weights) -> int:
+    """Splits of a row's keys, so that a small batch still fills the chip."""
+    if plan._ns is not None:
+        return plan._ns
+    return plan.eng.latent_nsplit(w.spec, _split(plan, w)[1], plan.longest)
+
+
+__all__ = ["Weights", "Group", "rotation_tables"]

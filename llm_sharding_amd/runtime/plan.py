@@ -1,0 +1,56 @@
+"""How one row batch runs: its stretches of consecutive positions, and what the layers' mixers derive
+from them once per forward (row lists, tile tables) and share."""
+from __future__ import annotations
+
+from typing import Callable, Optional
+
+import torch
+
+
+class Plan:
+    def __init__(self, eng, rows: int, runs: Optional[list], nsplit: Optional[int] = None):
+        """``runs``: [(first row, rows, slot, first position)] covering the batch, or None when only
+        the device knows (a decode graph: every row on its own)."""
+        self.eng, self.rows, self.runs, self._ns = eng, rows, runs, nsplit
+        self._memo: dict = {}
+
+    @staticmethod
+    def find_runs(slot, pos) -> list:
+        """Stretches of one slot's consecutive positions in int64 tensors (host)."""
+        new = torch.ones(slot.numel(), dtype=torch.bool)
+        new[1:] = (slot[1:] != slot[:-1]) | (pos[1:] != pos[:-1] + 1)
+        at = new.nonzero().flatten()
+        ends = torch.cat([at[1:], torch.tensor([slot.numel()])])
+        return list(zip(at.tolist(), (ends - at).tolist(), slot[at].tolist(), pos[at].tolist()))
+
+    def memo(self, key, make: Callable):
+        """make(), once per forward and key."""
+        if key not in self._memo:
+            self._memo[key] = make()
+        return self._memo[key]
+
+    @property
+    def longest(self) -> int:
+        """Tokens of the longest sequence in the batch (of any, in a decode graph)."""
+        if self.runs is None:
+            return self.eng.max_seq
+        return max(p0 + n for _, n, _, p0 in self.runs)
+
+    def i32(self, rows: list) -> torch.Tensor:
+        return torch.tensor(rows, dtype=torch.int32).to(self.eng.device)
+
+    def split_rows(self, least: int) -> tuple:
+        """(row indices or None for all rows, their count, runs of at least ``least`` rows): the rows outside
+        those runs, on the device."""
+        def make():
+            if self.runs is None:
+                return None, self.rows, []
+            long = [r for r in self.runs if r[1] >= least]
+            if not long:
+                return None, self.rows, []
+            idx = [i for r in self.runs if r[1] < least for i in range(r[0], r[0] + r[1])]
+            return (self.i32(idx) if idx else None), len(idx), long
+        return self.memo(("split", least), make)
+
+
+__all__ = ["Plan"]

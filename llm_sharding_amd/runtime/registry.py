@@ -10,7 +10,7 @@ import json
 import os
 
 from ..config import LlamaConfig
-from ..models import deretar
+from ..models import designs
 from ..models.stack import StackConfig
 from .engine import RandomSource, ShardFolderSource, StackFolderSource, StackRandomSource, StageEngine
 
@@ -20,8 +20,11 @@ def load_config(path: str):
     p = os.path.join(path, "config.json") if os.path.isdir(path) else path
     with open(p) as f:
         d = json.load(f)
-    if deretar.is_deretar(d):
-        return deretar.config_from_dict(d, name=os.path.basename(os.path.dirname(os.path.abspath(p))))
+    if d.get("architecture") in designs.DESIGNS:
+        folder = os.path.dirname(os.path.abspath(p))
+        have = os.path.exists(os.path.join(folder, "model.safetensors"))
+        return designs.DESIGNS[d["architecture"]].config_from_dict(
+            d, name=os.path.basename(folder), shapes=designs.CheckpointTensors(folder).shapes() if have else None)
     if "layers" in d and "architecture" in d:
         raise ValueError(f"unknown architecture {d['architecture']!r}")
     return LlamaConfig.from_pretrained(path)
@@ -59,7 +62,9 @@ def compute_dtype(cfg, device, dtype):
 
 def kernel_family(cfg) -> str:
     """The kernel library that serves this model alone (csrc/build.py FAMILIES; "" = the full one)."""
-    return "latent" if is_stack(cfg) else ""
+    if not is_stack(cfg):
+        return ""
+    return "latent" if cfg.model_type == "deretar" else "hybrid"
 
 
 __all__ = ["load_config", "is_stack", "engine_class", "make_engine", "folder_source", "random_source",

@@ -3,11 +3,13 @@
 The same step function, sequence API, decode graphs and serving as :class:`.engine.StageEngine`, for
 decoders that differ from Llama / GPT-2 in what a layer is made of:
 
-* the residual stream is fp32 (rows of ``hidden_dtype``), every sublayer reads it in the projections'
-  type and its result joins it through a norm of its own (stream_ops.hip, one launch);
-* mixers and feed-forwards come from the layer's spec; layers may share tensors;
+* the residual stream is fp32 (rows of ``hidden_dtype``); how the sublayers read and join it is the
+  layer's block (:mod:`.blocks`);
+* mixers and feed-forwards come from the layer's spec; layers may share tensors, or read another
+  layer's keys and values;
 * the cache is paged (:mod:`.paging`): one pool for all slots, one page table for all layers;
-* projections run the framework's GEMV / GEMM kernels on padded weights (ops/latent.Linear); fp32
+* recurrent layers keep a state per slot, which starts from zero at position 0;
+* projections run the framework's GEMV / GEMM kernels on padded weights (ops/stream.Linear); fp32
   engines run every product in true fp32.
 """
 from __future__ import annotations
@@ -18,10 +20,12 @@ import torch
 import torch.nn.functional as F
 
 from ..config import ceil_div
-from ..models.stack import StackConfig, pad_to
+from ..models.stack import AttentionSpec, DeltaSpec, LatentSpec, StackConfig, pad_to
+from .blocks import COPY, Layer, block
 from .engine import StageEngine, WeightSource
-from .latent_mixer import Plan, Weights, rotation_tables
+from .latent_mixer import rotation_tables
 from .paging import PagePool
+from .plan import Plan
 
 PAGE = 64
 
@@ -31,39 +35,9 @@ def embed_rows(cfg: StackConfig, table: torch.Tensor, ids: torch.Tensor) -> torc
     h = torch.empty((ids.numel(), cfg.hidden_size), dtype=torch.float32, device=table.device)
     if table.device.type != "cuda":
         return h.copy_(F.embedding(ids.long(), table).float() * cfg.embed_scale)
-    from ..ops import latent as L
+    from ..ops import stream as L
     L.stream_embed(ids.to(torch.int32), table, cfg.embed_scale, h, torch.empty_like(h, dtype=table.dtype), ids.numel())
     return h
-
-
-class _Layer:
-    def __init__(self, spec, mixer, mlp, gain1, gain2):
-        self.spec, self.mixer, self.mlp, self.gain1, self.gain2 = spec, mixer, mlp, gain1, gain2
-
-
-class _Glu:
-    """Gate / up / down projection of a clipped gated unit."""
-
-    def __init__(self, spec, t: dict, gpu: bool):
-        self.spec = spec
-        self.raw = None if gpu else t
-        if gpu:
-            from ..ops import latent as L
-            self.gate_up, self.down = L.Linear.glu(t["gate"], t["up"]), L.Linear(t["down"])
-
-    def tensors(self) -> list:
-        return list(self.raw.values()) if self.raw is not None else self.gate_up.tensors() + self.down.tensors()
-
-    def forward(self, eng, x, y, rows: int) -> None:
-        act = eng.scratch_view("act", rows, self.down.k)
-        eng.project(self.gate_up, x, rows, act, glu=self.spec)
-        eng.project(self.down, act, rows, y)
-
-    def forward_torch(self, x) -> torch.Tensor:
-        w, s = {k: v.float() for k, v in self.raw.items()}, self.spec
-        g = F.linear(x, w["gate"]).clamp(max=s.limit)
-        u = F.linear(x, w["up"]).clamp(-s.limit, s.limit)
-        return F.linear(g * torch.sigmoid(s.alpha * g) * (u + s.shift), w["down"])
 
 
 class StackEngine(StageEngine):
@@ -118,18 +92,17 @@ class StackEngine(StageEngine):
             spec = cfg.layers[i]
             if spec.owner not in shared:
                 self._log(f"[INFO] loading layer {i}")
-                shared[spec.owner] = self._prepare(spec, self.source.layer(i, dev, dt))
-            self.layers.append(_Layer(spec, *shared[spec.owner]))
-        table = None
-        if self.has_embed or self.has_head:
-            table = self.source.embedding(dev, dt).contiguous()
+                shared[spec.owner] = block(cfg, spec, self.source.layer(i, dev, dt), self.gpu)
+            self.layers.append(Layer(spec, shared[spec.owner]))
         if self.has_embed:
-            self.embed_w = table
+            self.embed_w = self.source.embedding(dev, dt).contiguous()
         if self.has_head:
-            self.final_norm = (self.source.final_norm(dev, dt).float() + cfg.norm_offset).contiguous()
-            head = F.pad(table, (0, 0, 0, cfg.head_rows - cfg.vocab_size))[self.head_v0:self.head_v1]
+            self.final_norm = (self.source.final_norm(dev, dt).float().reshape(-1)
+                               + cfg.norm_offset).expand(cfg.hidden_size).contiguous()
+            head = self.embed_w if cfg.tie_word_embeddings and self.has_embed else self.source.lm_head(dev, dt)
+            head = F.pad(head, (0, 0, 0, cfg.head_rows - cfg.vocab_size))[self.head_v0:self.head_v1]
             if self.gpu:
-                from ..ops import latent as L
+                from ..ops import stream as L
                 self.lm_head = L.Linear(head)
             else:
                 self.lm_head = head.contiguous()
@@ -139,51 +112,65 @@ class StackEngine(StageEngine):
                 self.head_bias[self.head_vocab:] = -3.0e38
         self._alloc_runtime()
 
-    def _prepare(self, spec, t: dict) -> tuple:
-        def part(p):
-            return {k[len(p):]: v for k, v in t.items() if k.startswith(p)}
-
-        def gain(n):  # norm weight times layer scale, fp32
-            return ((t[f"norm{n}"].float() + self.cfg.norm_offset) * t[f"ls{n}"].float()).contiguous()
-
-        mixer = Weights(spec.mixer, part("mix."), self.gpu)
-        if spec.mlp is None:
-            return mixer, None, gain(1), None
-        return mixer, _Glu(spec.mlp, part("mlp."), self.gpu), gain(1), gain(2)
-
     # ------------------------------------------------------------------------- memory
     def _alloc_runtime(self) -> None:
         cfg, dev, dt = self.cfg, self.device, self.dtype
         self.pool = PagePool(self.cache_pages, self.max_slots, self.max_seq, PAGE, dev)
 
-        def width(spec):
-            return spec.mixer.cache_width if self.gpu else spec.mixer.kv_rank + spec.mixer.rot_dim
-
-        self.k_cache = [torch.zeros((self.cache_pages, PAGE, width(l.spec)), dtype=dt, device=dev) for l in self.layers]
-        self.v_cache = []
-        for l in self.layers:
+        self.k_cache, self.v_cache, self.states = [], [], []
+        for i, l in enumerate(self.layers):
+            k, v, state = self._layer_memory(l.spec.mixer)
+            j = getattr(l.spec.mixer, "kv_from", None)
+            if j is not None:
+                if j < self.start:
+                    raise ValueError(f"layer {self.start + i} reads layer {j}'s keys and values: both belong on one stage")
+                k, v = self.k_cache[j - self.start], self.v_cache[j - self.start]
+            self.k_cache.append(k)
+            self.v_cache.append(v)
+            self.states.append(state)
             m = l.spec.mixer
-            if (m.rot_base, m.rot_dims) not in self._rot:
+            if isinstance(m, LatentSpec) and (m.rot_base, m.rot_dims) not in self._rot:
                 self._rot[(m.rot_base, m.rot_dims)] = rotation_tables(m, self.pool.max_pages * PAGE, dev)
         self.cos = self.sin = None
         if self.gpu:
-            # widest row of every intermediate over the layers
-            mx = {"inp": 0, "cq": 0, "q": 0, "attn": 0, "act": 0}
+            # widest row of every intermediate over the layers, and its type
+            self._widths = {"y2": (self.width_p if cfg.hidden_size % 16 else 0, torch.float32)}
             for l in self.layers:
-                w = l.mixer
-                for k, n in (("inp", w.inp.n), ("cq", w.uq.k), ("q", w.uq.n), ("attn", w.out.k),
-                             ("act", l.mlp.down.k if l.mlp is not None else 0)):
-                    mx[k] = max(mx[k], n)
-            self._widths = mx
+                for part in l.w.scratch():
+                    for k, n in part.items():
+                        n, t = n if isinstance(n, tuple) else (n, dt)
+                        self._widths[k] = (max(self._widths.get(k, (0,))[0], n), t)
             for k, v in self._scratch_set(max(self.max_prefill_rows, self.DECODE_MAX_ROWS)).items():
                 setattr(self, k, v)
+
+    def _layer_memory(self, m) -> tuple:
+        """(key cache, value cache, state) of one layer's mixer; latent attention has one cache."""
+        dev, dt, pages = self.device, self.dtype, self.cache_pages
+        if isinstance(m, LatentSpec):
+            width = m.cache_width if self.gpu else m.kv_rank + m.rot_dim
+            return torch.zeros((pages, PAGE, width), dtype=dt, device=dev), None, None
+        if isinstance(m, DeltaSpec):
+            from ..ops.delta import state_shapes
+            S, ring = state_shapes(m, self.max_slots)
+            if not self.gpu:
+                S = S[:2] + (m.dim, m.vdim)
+            return None, None, tuple(torch.zeros(n, dtype=torch.float32, device=dev) for n in (S, ring))
+        if m.kv_from is not None:
+            return None, None, None
+        from ..ops.paged_attn import cache_shapes
+        shapes = cache_shapes(m, pages) if self.gpu else ((pages, PAGE, m.kv_heads, m.dim), (pages, PAGE, m.kv_heads, m.vdim))
+        return tuple(torch.zeros(n, dtype=dt, device=dev) for n in shapes) + (None,)
+
+    @property
+    def carries_state(self) -> bool:
+        """Running a token twice is not the same as once (a recurrent layer's state moves on)."""
+        return any(s is not None for s in self.states)
 
     def _projections(self) -> list:
         out = []
         for l in self.layers:
-            out += [(p.n, p.k, False) for p in (l.mixer.inp, l.mixer.uq, l.mixer.out, l.mixer.kv) if p is not None]
-            if l.mlp is not None:
-                out += [(l.mlp.gate_up.n, l.mlp.gate_up.k, True), (l.mlp.down.n, l.mlp.down.k, False)]
+            gated = getattr(l.mlp, "gate_up", None)
+            out += [(p.n, p.k, p is gated) for p in l.w.projections()]
         if self.has_head:
             out.append((self.lm_head.n, self.lm_head.k, False))
         return sorted(set(out))
@@ -195,14 +182,17 @@ class StackEngine(StageEngine):
         out = {"buf_h": torch.zeros((R, self.cfg.hidden_size), dtype=torch.float32, device=dev),
                "buf_x": torch.zeros((R, W), dtype=dt, device=dev),
                "buf_y": torch.zeros((R, W), dtype=torch.float32, device=dev),
-               "flat": {k: torch.zeros(R * n, dtype=dt, device=dev) for k, n in self._widths.items() if n},
+               "flat": {k: torch.zeros(R * n, dtype=t, device=dev) for k, (n, t) in self._widths.items() if n},
                "keys": torch.zeros(R, dtype=torch.int64, device=dev),
                "tokens": torch.zeros(R, dtype=torch.int32, device=dev), "_x_ready": False, "coop_ws": None, "sk_ws": None}
-        # absorbed attention: queries and split partials of up to ATTEND_ITEMS (row, split) pairs at a time
+        # attention split over keys: absorbed queries and split partials of up to ATTEND_ITEMS (row, split)
+        # pairs at a time
         items = self.ATTEND_ITEMS
-        qn = max(l.spec.mixer.heads * l.spec.mixer.cache_width for l in self.layers)
-        on = max(l.spec.mixer.heads * l.spec.mixer.krp for l in self.layers)
-        hn = max(l.spec.mixer.heads for l in self.layers)
+        ms = [l.spec.mixer for l in self.layers]
+        latent, paged = ([m for m in ms if isinstance(m, t)] for t in (LatentSpec, AttentionSpec))
+        qn = max((m.heads * m.cache_width for m in latent), default=0)
+        on = max([m.heads * m.krp for m in latent] + [m.heads * m.dvp for m in paged], default=0)
+        hn = max((m.heads for m in latent + paged), default=0)
         out["qt"] = torch.zeros(items * qn, dtype=dt, device=dev)
         out["part_o"] = torch.zeros(items * on, dtype=torch.float32, device=dev)
         out["part_ml"] = torch.zeros(items * hn * 2, dtype=torch.float32, device=dev)
@@ -239,8 +229,9 @@ class StackEngine(StageEngine):
         key = torch.cuda.current_stream(self.device).cuda_stream
         lat, kv = self._expand_bufs.get(key, (None, None))
         if lat is None or lat.numel() < tokens * s.cache_width or kv.numel() < tokens * n:
-            m = max(l.spec.mixer.cache_width for l in self.layers)
-            kn = max(l.mixer.kv.n for l in self.layers if l.mixer.kv is not None)
+            latent = [l for l in self.layers if isinstance(l.spec.mixer, LatentSpec)]
+            m = max(l.spec.mixer.cache_width for l in latent)
+            kn = max(l.mixer.kv.n for l in latent if l.mixer.kv is not None)
             t = pad_to(tokens, 1024)
             lat = torch.empty(t * m, dtype=self.dtype, device=self.device)
             kv = torch.empty(t * kn, dtype=self.dtype, device=self.device)
@@ -251,10 +242,10 @@ class StackEngine(StageEngine):
         return self._rot[(s.rot_base, s.rot_dims)]
 
     def memory_bytes(self) -> int:
-        ts = [self.embed_w, self.final_norm] + self.k_cache
+        ts = [self.embed_w, self.final_norm] + self.k_cache + self.v_cache + [t for s in self.states if s for t in s]
         ts += (self.lm_head.tensors() if self.gpu else [self.lm_head]) if self.has_head else []
         for l in self.layers:
-            ts += l.mixer.tensors() + (l.mlp.tensors() if l.mlp is not None else []) + [l.gain1, l.gain2]
+            ts += l.w.tensors()
         seen, n = set(), 0
         for t in ts:
             if t is not None and t.data_ptr() not in seen:
@@ -286,8 +277,19 @@ class StackEngine(StageEngine):
         return out
 
     # ------------------------------------------------------------------------- forward
-    def project(self, lin, x, rows: int, out, glu=None) -> None:
-        lin(x, rows, out, ws=self.coop_ws, sk_ws=self.sk_ws, glu=glu)
+    def project(self, lin, x, rows: int, out, glu=None, **kw) -> None:
+        lin(x, rows, out, ws=self.coop_ws, sk_ws=self.sk_ws, glu=glu, **kw)
+
+    def project_gated(self, lin, x, rows: int, gate, name: str, key: str) -> dict:
+        """stream += sigmoid(gate) * (lin x), in the product's epilogue ({} is left to do); where the stream's
+        width does not allow that, what :func:`..ops.stream.stream_join` has to add."""
+        W = self.cfg.hidden_size
+        if W % 16 == 0:
+            self.project(lin, x, rows, None, out32=self.buf_h[:rows], gate=gate, cols=W)
+            return {}
+        y = self.buf_y[:rows] if name == "y1" else self.scratch_view(name, rows, self.width_p)
+        self.project(lin, x, rows, y)
+        return {key: (y, gate)} if key == "first" else {key: y, "gate2": gate}
 
     def embed_into(self, ids: torch.Tensor, h: torch.Tensor) -> None:
         if self.embed_w is None:
@@ -296,7 +298,7 @@ class StackEngine(StageEngine):
         if not self.gpu:
             h.copy_(F.embedding(ids.long(), self.embed_w).float() * self.cfg.embed_scale)
             return
-        from ..ops import latent as L
+        from ..ops import stream as L
         fits = rows <= self.buf_x.shape[0]
         xc = self.buf_x if fits else torch.empty((rows, self.width_p), dtype=self.dtype, device=self.device)
         L.stream_embed(ids, self.embed_w, self.cfg.embed_scale, h, xc, rows)
@@ -332,47 +334,48 @@ class StackEngine(StageEngine):
         return int(max(1, min(64, hip.N_CU // max(1, entries * L.head_groups(s)), ceil_div(longest, PAGE))))
 
     def decode_nsplit(self, rows: int) -> int:
-        m = max((l.spec.mixer for l in self.layers), key=lambda m: m.heads)
-        return self.latent_nsplit(m, rows, self.max_seq)
+        latent = [l.spec.mixer for l in self.layers if isinstance(l.spec.mixer, LatentSpec)]
+        return self.latent_nsplit(max(latent, key=lambda m: m.heads), rows, self.max_seq) if latent else 1
 
     def _forward_hip(self, h, slot, pos, kv_len, rows, nsplit: Optional[int] = None, tiles=None, runs=None):
-        from ..ops import latent as L
+        from ..ops import stream as L
         if rows > max(self.max_prefill_rows, self.DECODE_MAX_ROWS):
             raise ValueError(f"{rows} rows exceed max_prefill_rows={self.max_prefill_rows}")
         if h.dtype != torch.float32 or not h.is_contiguous():
             h = h.to(torch.float32).contiguous()
-        hbuf, x, y = self.buf_h[:rows], self.buf_x[:rows], self.buf_y[:rows]
+        hbuf, x = self.buf_h[:rows], self.buf_x[:rows]
         own = h.data_ptr() == hbuf.data_ptr()
-        if not (own and self._x_ready):
-            L.cast_rows(h, x, rows, x2=None if own else hbuf)
+        have = COPY if own and self._x_ready else None
         self._x_ready = False
+        if not own:
+            if self.layers[0].w.entry is COPY:
+                L.cast_rows(h, x, rows, x2=hbuf)
+                have = COPY
+            else:
+                hbuf.copy_(h)
         if runs is None and nsplit is None:
             nsplit = self.decode_nsplit(rows)
         plan = Plan(self, rows, runs, nsplit)
-        eps = self.cfg.norm_eps
-        for i, l in enumerate(self.layers):
-            l.mixer.forward(self, x, y, self.k_cache[i], slot, pos, rows, plan)
-            L.stream_add_norm(y, l.gain1, eps, hbuf, x, rows)
-            if l.mlp is not None:
-                l.mlp.forward(self, x, y, rows)
-                L.stream_add_norm(y, l.gain2, eps, hbuf, x, rows)
+        ws = [l.w for l in self.layers]
+        for i, w in enumerate(ws):
+            if have is not w.entry:
+                if w.entry is COPY:
+                    L.cast_rows(hbuf, x, rows)
+                else:
+                    L.stream_norm(hbuf, w.entry, self.cfg.norm_eps, x, rows)
+            have = w.forward(self, i, slot, pos, rows, plan, ws[i + 1].entry if i + 1 < len(ws) else None)
         return hbuf
 
     def _forward_stack_torch(self, h, slot, pos) -> torch.Tensor:
-        def join(x, y, gain):
-            return x + y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + self.cfg.norm_eps) * gain
-
         x = h.float()
         for i, l in enumerate(self.layers):
-            x = join(x, l.mixer.forward_torch(self, x, self.k_cache[i], slot, pos), l.gain1)
-            if l.mlp is not None:
-                x = join(x, l.mlp.forward_torch(x), l.gain2)
+            x = l.w.forward_torch(self, i, x, slot, pos)
         return x
 
     # ------------------------------------------------------------------------- head
     def _normed(self, h, rows: int, a_rows=None) -> torch.Tensor:
         """Final norm of the selected rows -> the head projection's input."""
-        from ..ops import latent as L
+        from ..ops import stream as L
         src = h[:rows] if a_rows is None else h.index_select(0, a_rows.long())
         xn = self.buf_x[:rows] if rows <= self.buf_x.shape[0] else torch.zeros(
             (rows, self.width_p), dtype=self.dtype, device=self.device)
@@ -380,7 +383,7 @@ class StackEngine(StageEngine):
         return xn
 
     def head_gemv(self, h: torch.Tensor, rows: int, keys: torch.Tensor, a_rows=None) -> None:
-        from ..ops import latent as L
+        from ..ops import stream as L
         xn = self._normed(h, rows, a_rows)
         if self.dtype == torch.float32:
             lg = torch.empty((rows, self.lm_head.n), dtype=torch.float32, device=self.device)
