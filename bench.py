@@ -88,12 +88,12 @@ def parse():
     ap.add_argument("--no-fallback", dest="fallback", action="store_false",
                     help="N > 1: do not restart with --transport ipc when the RCCL ring preflight fails")
     ap.add_argument("--compare", default="",
-                    help="instead of the headline: prefill and decode throughput of Deretar stacks of these sizes "
+                    help="instead of the headline: prefill and decode throughput of Deretar and Gupuvik stacks of these sizes "
                          "(2k,4k,8k: layers like a 2048-wide model's, Llama-2-7B's, Llama-2-70B's; random weights) "
                          "beside Llama layers of the same width, heads and ff")
     ap.add_argument("--compare-points", default="prefill:1x2048,prefill:4x2048,decode:1,decode:16,decode:64,decode:128",
                     help="prefill:SEQUENCESxTOKENS and decode:BATCH points of --compare")
-    ap.add_argument("--compare-models", default="deretar,llama", help="which of the two --compare runs")
+    ap.add_argument("--compare-models", default="deretar,gupuvik,llama", help="which of these --compare runs")
     ap.add_argument("--compare-context", type=int, default=1024, help="cached tokens per sequence of a decode point")
     ap.add_argument("--compare-layers", type=int, default=8)
     return ap.parse_args()
@@ -378,8 +378,10 @@ def compare_designs(a) -> list:
         ll = LlamaConfig(hidden_size=st.hidden_size, intermediate_size=ff, num_hidden_layers=a.compare_layers,
                          num_attention_heads=m.heads, num_key_value_heads=kv_heads[size], head_dim=128,
                          vocab_size=st.vocab_size, max_position_embeddings=1 << 15, name=f"llama-{size}")
-        for cfg in (st, ll):
-            kind = "deretar" if is_stack(cfg) else "llama"
+        gu = get_preset(f"gupuvik-{size}")
+        gu = dataclasses.replace(gu, layers=gu.layers[:a.compare_layers])
+        for cfg in (st, gu, ll):
+            kind = cfg.model_type if is_stack(cfg) else "llama"
             if kind not in a.compare_models.split(","):
                 continue
             for point in [x.strip() for x in a.compare_points.split(",") if x.strip()]:
@@ -411,6 +413,8 @@ def compare_designs(a) -> list:
                        "ms_per_layer": round(ms / a.compare_layers, 5),
                        "layer_mb": round(cfg.layer_bytes() / 1e6, 1),
                        "cache_bytes_per_token_layer": cfg.kv_bytes_per_token_per_layer()}
+                if is_stack(cfg) and eng.carries_state:
+                    rec["state_mb_per_sequence_layer"] = round(cfg.state_bytes_per_slot() / 1e6, 2)
                 print(json.dumps(rec), flush=True)
                 out.append(rec)
                 g = None

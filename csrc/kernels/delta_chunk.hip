@@ -1,0 +1,463 @@
+// The gated delta rule over prompt portions in chunks of 32 rows (delta.h), bf16 engine.
+//
+// With G_i the sum of the log decays of rows 0..i of a chunk (per key channel) and S the state before it,
+//
+//   u = U - W S             U = T (beta v), W = T (beta k e^G), T = (1 + A)^-1
+//   o = (q e^G) S + P u     A_ij = beta_i sum_d k_i k_j e^(G_i - G_j) (j < i),  P_ij the same of q_i, k_j (j <= i)
+//   S <- e^G_31 S + (k e^(G_31 - G))^T u
+//
+// delta_chunk_kernel makes W, U, q e^G, k e^(G_31 - G), P and e^G_31 of every (chunk, head) at once;
+// delta_scan_kernel then walks a run's chunks, one workgroup per (run, head). No exponent is ever
+// positive: the 16 x 16 blocks on the diagonal of A and P take e^(G_i - G_j) pair by pair, the block
+// below them splits it at row 15.
+//
+// Everything is fp32 or, where it is an operand of a matrix product, a pair of bf16 (the value's
+// rounding and the rounding of what that leaves): each product is the sum of three, hi hi + hi lo + lo hi.
+// The pairs lie in memory in operand order, the K index in the order in which the accumulators hold it,
+// so the state never leaves the scan's registers.
+#include "delta.h"
+
+namespace {
+
+constexpr int C = 32;
+
+struct DeltaChunk {  // rows row0 .. row0 + n of one run at positions pos0 ..; before: rows of that run ahead of row0
+  int row0, n, slot, pos0, before, pad0, pad1, pad2;
+};
+struct DeltaSpan {  // chunks [chunk0, chunk0 + chunks) of one run, its rows and first position
+  int chunk0, chunks, slot, pos0, row0, n, pad0, pad1;
+};
+
+template <int DK>
+struct Pieces {  // 1-KiB pieces of a (chunk, head) in the workspace; hi ones first
+  static constexpr int KF = DK / 32, W = 0, Q = 4 * KF, K = 8 * KF, P = 12 * KF, E = P + 4, U = E + 1;
+};
+
+// 8 values -> operand pieces
+LSA_DEVICE void put_pair(unsigned char* hi, unsigned char* lo, int at, const float* f) {
+  const u32x4_t h = pack8(f);
+  float b[8], r[8];
+  unpack8(h, b);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) r[j] = f[j] - b[j];
+  st16(hi + at * 16, h);
+  st16(lo + at * 16, pack8(r));
+}
+LSA_DEVICE void split_pair(const float* f, u32x4_t& h, u32x4_t& l) {
+  h = pack8(f);
+  float b[8], r[8];
+  unpack8(h, b);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) r[j] = f[j] - b[j];
+  l = pack8(r);
+}
+LSA_DEVICE f32x4_t mfma_pair(u32x4_t ah, u32x4_t al, u32x4_t bh, u32x4_t bl, f32x4_t c) {
+  return mfma16(al, bh, mfma16(ah, bl, mfma16(ah, bh, c)));
+}
+
+LSA_DEVICE float silu_fast(float x) { return x / (1.f + __expf(-x)); }
+
+// convolution and silu of one channel over the chunk's rows: f(row, value), zero past the last one
+template <typename F>
+LSA_DEVICE void conv_rows(const DeltaArgs& a, const DeltaChunk& ck, int ch, int col, int channels, F f) {
+  const bf16_raw* in = (const bf16_raw*)a.in + (size_t)ck.row0 * a.ldi + col;
+  const float* w = a.conv + (size_t)ch * a.taps + a.taps - 1;
+  auto past = [&](int t, int j) -> float {  // the input j rows before row t
+    const int back = j - t;  // rows before row0
+    if (back <= ck.before) return bf2f(in[(ptrdiff_t)(t - j) * a.ldi]);
+    const int p = ck.pos0 + t - j;
+    return p < 0 ? 0.f : a.ring[((size_t)ck.slot * a.taps + p % a.taps) * channels + ch];
+  };
+  if (a.taps <= 4) {
+    float w0 = w[0], w1 = a.taps > 1 ? w[-1] : 0.f, w2 = a.taps > 2 ? w[-2] : 0.f, w3 = a.taps > 3 ? w[-3] : 0.f;
+    float x1 = a.taps > 1 ? past(0, 1) : 0.f, x2 = a.taps > 2 ? past(0, 2) : 0.f, x3 = a.taps > 3 ? past(0, 3) : 0.f;
+#pragma unroll
+    for (int t = 0; t < C; ++t) {
+      const float x = t < ck.n ? bf2f(in[(size_t)t * a.ldi]) : 0.f;
+      const float y = silu_fast(fmaf(x3, w3, fmaf(x2, w2, fmaf(x1, w1, x * w0))));
+      f(t, t < ck.n ? y : 0.f);
+      x3 = x2;
+      x2 = x1;
+      x1 = x;
+    }
+  } else {
+#pragma unroll
+    for (int t = 0; t < C; ++t) {
+      float y = 0.f;
+      if (t < ck.n) {
+        for (int j = 0; j < a.taps; ++j) y = fmaf(past(t, j), w[-j], y);
+        y = silu_fast(y);
+      }
+      f(t, y);
+    }
+  }
+}
+
+template <int DK, int DV>
+__global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a, const DeltaChunk* __restrict__ chunks,
+                                                          unsigned char* __restrict__ ws) {
+  using PC = Pieces<DK>;
+  constexpr int KF = DK / 32, LD = DK + 4, LA = C + 4;
+  constexpr size_t STRIDE = (size_t)(PC::U + DV / 8) * 1024;
+  __shared__ __attribute__((aligned(16))) float sq[C][LD], sk[C][LD], sg[C][LD], sA[C][LA], sP[C][LA];
+  __shared__ float su[2 * C], sb[C];
+  const DeltaChunk ck = chunks[blockIdx.x];
+  const int h = blockIdx.y, kb = h / (a.heads / a.kv_heads), kc = a.kv_heads * a.dim;
+  const int channels = 2 * kc + a.heads * a.vdim;
+  const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, q4 = lane >> 4;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  unsigned char* out = ws + ((size_t)blockIdx.x * a.heads + h) * STRIDE;
+
+  for (int c = tid; c < 2 * DK; c += 256) {  // q and k
+    const int d = c % DK, isk = c / DK;
+    auto& dst = isk ? sk : sq;
+    if (d < a.dim)
+      conv_rows(a, ck, isk * kc + kb * a.dim + d, (isk ? a.ok : a.oq) + kb * a.dim + d, channels,
+                [&](int t, float y) { dst[t][d] = y; });
+    else
+      for (int t = 0; t < C; ++t) dst[t][d] = 0.f;
+  }
+  for (int c = tid; c < 2 * DK; c += 256) {  // sums of log2 decays, 16 rows at a time
+    const int d = c % DK, t0 = (c / DK) * 16;
+    const float A = d < a.dim ? -a.decay[h] * 1.4426950408889634f : 0.f, bias = d < a.dim ? a.dt_bias[h * a.dim + d] : 0.f;
+    const float* z = a.z + (size_t)ck.row0 * a.ldz + h * a.dim + d;
+    float g = 0.f;
+#pragma unroll
+    for (int t = t0; t < t0 + 16; ++t) {
+      if (d < a.dim && t < ck.n) g = fmaf(A, delta_softplus(z[(size_t)t * a.ldz] + bias), g);
+      sg[t][d] = g;
+    }
+  }
+  if (tid < C) sb[tid] = tid < ck.n ? 1.f / (1.f + __expf(-a.in32[(size_t)(ck.row0 + tid) * a.ld32 + a.ob + h])) : 0.f;
+  for (int e = tid; e < C * LA; e += 256) (&sA[0][0])[e] = (&sP[0][0])[e] = 0.f;
+  __syncthreads();
+  {  // unit vectors: four threads per vector
+    const int v = tid >> 2, t = v & (C - 1);
+    const float* x = v < C ? sq[t] : sk[t];
+    float ss = 0.f;
+    for (int d = tid & 3; d < DK; d += 4) ss = fmaf(x[d], x[d], ss);
+    ss += __shfl_xor(ss, 1, 64);
+    ss += __shfl_xor(ss, 2, 64);
+    if ((tid & 3) == 0) su[v] = (v < C ? a.q_scale : 1.f) / sqrtf(ss + a.unit_eps);
+  }
+  for (int e = tid; e < 16 * DK; e += 256) sg[16 + e / DK][e % DK] += sg[15][e % DK];
+  __syncthreads();
+  for (int e = tid; e < C * DK; e += 256) {
+    const int t = e / DK, d = e % DK;
+    sq[t][d] *= su[t];
+    sk[t][d] *= su[C + t];
+  }
+  __syncthreads();
+
+  {  // A and P: the two blocks on the diagonal, one pair of rows per thread
+    const int r0 = tid >> 4, r1 = tid & 15;
+    const int i = r0 >= r1 ? r0 : 16 + r1, j = r0 >= r1 ? r1 : 16 + r0;
+    float x = 0.f, y = 0.f;
+#pragma unroll 4
+    for (int d = 0; d < DK; d += 4) {
+      const f32x4_t gi = *reinterpret_cast<const f32x4_t*>(&sg[i][d]), gj = *reinterpret_cast<const f32x4_t*>(&sg[j][d]);
+      const f32x4_t ki = *reinterpret_cast<const f32x4_t*>(&sk[i][d]), kj = *reinterpret_cast<const f32x4_t*>(&sk[j][d]);
+      const f32x4_t qi = *reinterpret_cast<const f32x4_t*>(&sq[i][d]);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float z = kj[e] * __builtin_amdgcn_exp2f(gi[e] - gj[e]);
+        x = fmaf(ki[e], z, x);
+        y = fmaf(qi[e], z, y);
+      }
+    }
+    if (i != j) sA[i][j] = sb[i] * x;
+    sP[i][j] = y;
+    if (tid < 16) {  // the second block's diagonal
+      float p = 0.f;
+      for (int d = 0; d < DK; ++d) p = fmaf(sq[16 + tid][d], sk[16 + tid][d], p);
+      sP[16 + tid][16 + tid] = p;
+    }
+  }
+  if (w < 2) {  // the block below, through row 15: wave 0 A, wave 1 P
+    f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+    const auto& sx = w ? sq : sk;
+#pragma unroll
+    for (int kf = 0; kf < KF; ++kf) {
+      float x[8], y[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int d = kf * 32 + q4 * 8 + e;
+        const float g = sg[15][d];
+        x[e] = sx[16 + l16][d] * __builtin_amdgcn_exp2f(sg[16 + l16][d] - g);
+        y[e] = sk[l16][d] * __builtin_amdgcn_exp2f(g - sg[l16][d]);
+      }
+      u32x4_t xh, xl, yh, yl;
+      split_pair(x, xh, xl);
+      split_pair(y, yh, yl);
+      acc = mfma_pair(xh, xl, yh, yl, acc);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = 16 + q4 * 4 + r;
+      if (w) sP[i][l16] = acc[r];
+      else sA[i][l16] = sb[i] * acc[r];
+    }
+  }
+  // q e^G (rows x key channels) and k e^(G_31 - G) (key channels x rows)
+  for (int e = tid; e < 2 * KF * 64; e += 256) {
+    const int ln = e & 63, kf = (e >> 6) % KF, t = (e >> 6) / KF * 16 + (ln & 15), d0 = kf * 32 + (ln >> 4) * 4;
+    float f[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const int d = d0 + (j & 4) * 4 + (j & 3);
+      f[j] = sq[t][d] * __builtin_amdgcn_exp2f(sg[t][d]);
+    }
+    put_pair(out + PC::Q * 1024, out + (PC::Q + 2 * KF) * 1024, e, f);
+  }
+  for (int e = tid; e < 2 * KF * 64; e += 256) {
+    const int ln = e & 63, d = (e >> 6) * 16 + (ln & 15), t0 = (ln >> 4) * 4;
+    float f[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const int t = t0 + (j & 4) * 4 + (j & 3);
+      f[j] = sk[t][d] * __builtin_amdgcn_exp2f(sg[C - 1][d] - sg[t][d]);
+    }
+    put_pair(out + PC::K * 1024, out + (PC::K + 2 * KF) * 1024, e, f);
+  }
+  for (int d = tid; d < DK; d += 256) reinterpret_cast<float*>(out + PC::E * 1024)[d] = __builtin_amdgcn_exp2f(sg[C - 1][d]);
+  __syncthreads();
+  if (tid < 128) {  // P (rows x rows)
+    const int t = (tid >> 6) * 16 + l16;
+    float f[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) f[j] = sP[t][q4 * 4 + (j & 4) * 4 + (j & 3)];
+    put_pair(out + PC::P * 1024, out + (PC::P + 2) * 1024, tid, f);
+  }
+  // (1 + A) x = b, one column per thread: beta v -> U, beta k e^G -> W
+  for (int c = tid; c < DV + DK; c += 256) {
+    float x[C];
+    if (c < DV) {
+      if (c < a.vdim) {
+        conv_rows(a, ck, 2 * kc + h * a.vdim + c, a.ov + h * a.vdim + c, channels, [&](int t, float y) { x[t] = y * sb[t]; });
+      } else {
+#pragma unroll
+        for (int t = 0; t < C; ++t) x[t] = 0.f;
+      }
+    } else {
+#pragma unroll
+      for (int t = 0; t < C; ++t) x[t] = sb[t] * sk[t][c - DV] * __builtin_amdgcn_exp2f(sg[t][c - DV]);
+    }
+#pragma unroll
+    for (int i = 1; i < C; ++i) {
+      float s = x[i];
+#pragma unroll
+      for (int j = 0; j < i; j += 4) {
+        const f32x4_t r = *reinterpret_cast<const f32x4_t*>(&sA[i][j]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (j + e < i) s = fmaf(-r[e], x[j + e], s);
+      }
+      x[i] = s;
+    }
+    if (c < DV) {
+      f32x4_t* u = reinterpret_cast<f32x4_t*>(out + (PC::U + (c / 16) * 2) * 1024);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) u[e * 16 + (c & 15)] = f32x4_t{x[4 * e], x[4 * e + 1], x[4 * e + 2], x[4 * e + 3]};
+    } else {
+#pragma unroll
+      for (int t = 0; t < C; ++t) sq[t][c - DV] = x[t];  // q is in memory already
+    }
+  }
+  __syncthreads();
+  for (int e = tid; e < 2 * KF * 64; e += 256) {
+    const int ln = e & 63, kf = (e >> 6) % KF, t = (e >> 6) / KF * 16 + (ln & 15), d0 = kf * 32 + (ln >> 4) * 4;
+    float f[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) f[j] = sq[t][d0 + (j & 4) * 4 + (j & 3)];
+    put_pair(out, out + 2 * KF * 1024, e, f);
+  }
+}
+
+LSA_DEVICE void glds16(const void* src, unsigned char* lds_base) {
+  __builtin_amdgcn_global_load_lds(src, (__attribute__((address_space(3))) void*)lds_base, 16, 0, 0);
+}
+
+// One workgroup per (run, head): the state in registers (wave w: value channels w NC 16 ..), a chunk's
+// operands by LDS-DMA into a double buffer. Read-outs are normed over the head's value channels one
+// chunk later, behind the barrier that the next chunk needs anyway.
+template <int DK, int DV, int NC>
+__global__ __launch_bounds__(DV / NC * 4) void delta_scan_kernel(DeltaArgs a, const DeltaSpan* __restrict__ spans,
+                                                                 const unsigned char* __restrict__ ws) {
+  using PC = Pieces<DK>;
+  constexpr int KF = DK / 32, MT = DK / 16, NW = DV / 16 / NC, NP = PC::U;
+  constexpr size_t STRIDE = (size_t)(PC::U + DV / 8) * 1024;
+  __shared__ __attribute__((aligned(16))) unsigned char smem[2 * NP * 1024 + 2 * NW * C * 4];
+  float* s_ss = reinterpret_cast<float*>(smem + 2 * NP * 1024);  // [2][NW][C]
+  const DeltaSpan sp = spans[blockIdx.x];
+  const int h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, q4 = lane >> 4;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const unsigned char* src = ws + ((size_t)sp.chunk0 * a.heads + h) * STRIDE;
+  const size_t step = (size_t)a.heads * STRIDE;
+
+  f32x4_t S[NC][MT];
+  float* st = a.state + ((size_t)sp.slot * a.heads + h) * DK * DV + w * NC * 16 + l16;
+#pragma unroll
+  for (int n = 0; n < NC; ++n)
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) S[n][m][r] = sp.pos0 ? st[(size_t)(m * 16 + q4 * 4 + r) * DV + n * 16] : 0.f;
+  float nw[NC];
+#pragma unroll
+  for (int n = 0; n < NC; ++n) {
+    const int v = (w * NC + n) * 16 + l16;
+    nw[n] = v < a.vdim ? a.norm[v] : 0.f;
+  }
+
+  f32x4_t U[NC][2], O[NC][2];
+  float gl[NC][8];
+  auto stage = [&](int c, int buf) {
+    const unsigned char* p = src + c * step;
+    for (int i = w; i < NP; i += NW) glds16(p + i * 1024 + lane * 16, smem + (buf * NP + i) * 1024);
+  };
+  auto load_u = [&](int c) {
+    const unsigned char* p = src + c * step + PC::U * 1024;
+#pragma unroll
+    for (int n = 0; n < NC; ++n)
+#pragma unroll
+      for (int m = 0; m < 2; ++m)
+        U[n][m] = *reinterpret_cast<const f32x4_t*>(p + ((w * NC + n) * 2 + m) * 1024 + lane * 16);
+  };
+  // gate logits of chunk c in accumulator order
+  auto load_gate = [&](int c) {
+#pragma unroll
+    for (int n = 0; n < NC; ++n)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int t = c * C + (e >> 2) * 16 + q4 * 4 + (e & 3), v = (w * NC + n) * 16 + l16;
+        gl[n][e] = a.gate && t < sp.n && v < a.vdim
+                       ? bf2f(((const bf16_raw*)a.gate)[(size_t)(sp.row0 + t) * a.ldg + h * a.vdim + v]) : 0.f;
+      }
+  };
+  auto finish = [&](int c) {  // chunk c's read-outs
+    const float* ss = s_ss + (c & 1) * NW * C;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const int r = (e >> 2) * 16 + q4 * 4 + (e & 3), t = c * C + r;
+      float sum = 0.f;
+#pragma unroll
+      for (int x = 0; x < NW; ++x) sum += ss[x * C + r];
+      const float rs = 1.f / sqrtf(sum / (float)a.vdim + a.eps);
+#pragma unroll
+      for (int n = 0; n < NC; ++n) {
+        const int v = (w * NC + n) * 16 + l16;
+        if (t < sp.n && v < a.vdim)
+          ((bf16_raw*)a.out)[(size_t)(sp.row0 + t) * a.ldo + h * a.vdim + v] =
+              f2bf(O[n][e >> 2][e & 3] * rs * nw[n] * (a.gate ? sigmoid(gl[n][e]) : 1.f));
+      }
+    }
+  };
+
+  stage(0, 0);
+  load_u(0);
+  for (int c = 0; c < sp.chunks; ++c) {
+    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+    if (c) finish(c - 1);
+    if (c + 1 < sp.chunks) stage(c + 1, (c + 1) & 1);
+    load_gate(c);
+    const unsigned char* p = smem + (c & 1) * NP * 1024 + lane * 16;
+    auto piece = [&](int i) { return *reinterpret_cast<const u32x4_t*>(p + i * 1024); };
+    u32x4_t sh[NC][KF], sl[NC][KF];
+#pragma unroll
+    for (int n = 0; n < NC; ++n)
+#pragma unroll
+      for (int kf = 0; kf < KF; ++kf) {
+        float f[8];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          f[j] = S[n][2 * kf][j];
+          f[4 + j] = S[n][2 * kf + 1][j];
+        }
+        split_pair(f, sh[n][kf], sl[n][kf]);
+      }
+    f32x4_t V[NC][2];
+#pragma unroll
+    for (int m = 0; m < 2; ++m) {
+#pragma unroll
+      for (int n = 0; n < NC; ++n) V[n][m] = O[n][m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kf = 0; kf < KF; ++kf) {
+        const u32x4_t wh = piece(PC::W + m * KF + kf), wl = piece(PC::W + (2 + m) * KF + kf);
+        const u32x4_t qh = piece(PC::Q + m * KF + kf), ql = piece(PC::Q + (2 + m) * KF + kf);
+#pragma unroll
+        for (int n = 0; n < NC; ++n) {
+          V[n][m] = mfma_pair(wh, wl, sh[n][kf], sl[n][kf], V[n][m]);
+          O[n][m] = mfma_pair(qh, ql, sh[n][kf], sl[n][kf], O[n][m]);
+        }
+      }
+    }
+    u32x4_t vh[NC], vl[NC];
+#pragma unroll
+    for (int n = 0; n < NC; ++n) {
+      float f[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) f[j] = U[n][j >> 2][j & 3] - V[n][j >> 2][j & 3];
+      split_pair(f, vh[n], vl[n]);
+    }
+    if (c + 1 < sp.chunks) load_u(c + 1);
+#pragma unroll
+    for (int m = 0; m < 2; ++m) {
+      const u32x4_t ph = piece(PC::P + m), pl = piece(PC::P + 2 + m);
+#pragma unroll
+      for (int n = 0; n < NC; ++n) O[n][m] = mfma_pair(ph, pl, vh[n], vl[n], O[n][m]);
+    }
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+      const u32x4_t kh = piece(PC::K + m), kl = piece(PC::K + MT + m);
+      const f32x4_t e = *reinterpret_cast<const f32x4_t*>(smem + ((c & 1) * NP + PC::E) * 1024 + (m * 16 + q4 * 4) * 4);
+#pragma unroll
+      for (int n = 0; n < NC; ++n) S[n][m] = mfma_pair(kh, kl, vh[n], vl[n], S[n][m] * e);
+    }
+    float* ss = s_ss + ((c & 1) * NW + w) * C;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float x = 0.f;
+#pragma unroll
+      for (int n = 0; n < NC; ++n) x = fmaf(O[n][e >> 2][e & 3], O[n][e >> 2][e & 3], x);
+      x = group_sum<16>(x);
+      if (l16 == 0) ss[(e >> 2) * 16 + q4 * 4 + (e & 3)] = x;
+    }
+  }
+  __syncthreads();
+  finish(sp.chunks - 1);
+#pragma unroll
+  for (int n = 0; n < NC; ++n)
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) st[(size_t)(m * 16 + q4 * 4 + r) * DV + n * 16] = S[n][m][r];
+}
+
+}  // namespace
+
+// bytes of one (chunk, head) in the workspace, 0: size not built
+extern "C" int lsa_delta_chunk_bytes(int dk, int dv) {
+  if ((dk != 32 && dk != 64 && dk != 128) || (dv != 32 && dv != 64 && dv != 128)) return 0;
+  return (12 * (dk / 32) + 5 + dv / 8) * 1024;
+}
+
+// chunks: n_chunks DeltaChunk; spans: n_spans DeltaSpan over them; ws: n_chunks * heads * lsa_delta_chunk_bytes
+extern "C" int lsa_delta_chunked(const DeltaArgs* a, const void* chunks, int n_chunks, const void* spans, int n_spans,
+                                 void* ws, hipStream_t s) {
+  if (!a || bad_delta(a) || n_chunks < 1 || n_spans < 1 || !chunks || !spans || !ws || (uintptr_t)ws % 16) return LSA_BAD_SHAPE;
+#define LSA_C(K, V, NC)                                                                                                     \
+  if (a->dk == K && a->dv == V) {                                                                                           \
+    delta_chunk_kernel<K, V><<<dim3(n_chunks, a->heads), 256, 0, s>>>(*a, (const DeltaChunk*)chunks, (unsigned char*)ws);   \
+    LSA_CHECK_LAUNCH();                                                                                                     \
+    delta_scan_kernel<K, V, NC><<<dim3(n_spans, a->heads), V / NC * 4, 0, s>>>(*a, (const DeltaSpan*)spans,                 \
+                                                                               (const unsigned char*)ws);                   \
+    LSA_CHECK_LAUNCH();                                                                                                     \
+    return LSA_OK;                                                                                                          \
+  }
+  LSA_C(32, 32, 1) LSA_C(32, 64, 1) LSA_C(32, 128, 2) LSA_C(64, 32, 1) LSA_C(64, 64, 1) LSA_C(64, 128, 2) LSA_C(128, 32, 1)
+  LSA_C(128, 64, 1) LSA_C(128, 128, 2)
+#undef LSA_C
+  return LSA_UNSUPPORTED;
+}

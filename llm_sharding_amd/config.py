@@ -239,7 +239,33 @@ def _deretar(width: int, heads: int, ff: int, layers: int, vocab: int, kv_rank: 
     return cfg
 
 
+def _gupuvik(width: int, heads: int, kv_heads: int, ff: int, layers: int, vocab: int, experts: int, top: int, eff: int,
+             dim: int = 128, vdim: int = 128, window: int = 2048, keep: int = 4, dheads: int = 0, dkv: int = 0,
+             ddim: int = 128, rank: int = 128, max_pos: int = 1 << 17, name: str = "gupuvik"):
+    """A Gupuvik stack (random-init presets): per eight layers two of attention, the second reading the
+    first's keys, and six of the delta rule; two dense feed-forwards, six mixtures of experts."""
+    from .models import gupuvik as G
+    dheads = dheads or heads
+    entries = []
+    for i in range(layers):
+        mlp = G.dense(ff) if i % 8 in (0, 7) else G.moe(experts, top, eff)
+        if i % 4 == 0:
+            entries.append(G.attention_entry(heads, kv_heads, dim, vdim, window, keep, mlp, kv_from=i - 4 if i % 8 else None))
+        else:
+            entries.append(G.delta_entry(dheads, dkv or dheads, ddim, vdim, 4, mlp))
+    cfg = G.make_config(width, vocab, entries, name=name, rank=rank)
+    cfg.max_position_embeddings = max_pos
+    return cfg
+
+
 PRESETS = {
+    # Gupuvik with the widths of a 2048-wide model / Llama-2-7B / Llama-2-70B; a token's experts
+    # together are as wide as the dense feed-forward
+    "gupuvik-2k": lambda: _gupuvik(2048, 16, 4, 8192, 24, 32000, 32, 8, 1024, name="gupuvik-2k"),
+    "gupuvik-4k": lambda: _gupuvik(4096, 32, 8, 11008, 32, 32000, 32, 8, 1408, name="gupuvik-4k"),
+    "gupuvik-8k": lambda: _gupuvik(8192, 64, 8, 28672, 80, 32000, 16, 4, 7168, dkv=32, name="gupuvik-8k"),
+    "tiny-gupuvik": lambda: _gupuvik(112, 4, 2, 150, 9, 330, 5, 2, 40, dim=24, vdim=40, window=50, keep=3, dheads=3, dkv=1,
+                                     ddim=20, rank=9, max_pos=1024, name="tiny-gupuvik"),
     # Deretar with the layer sizes of Llama-2-7B / a 2048-wide model / Llama-2-70B
     "deretar-4k": lambda: _deretar(4096, 32, 11008, 32, 32000, 512, 1536, name="deretar-4k"),
     "deretar-2k": lambda: _deretar(2048, 16, 8192, 24, 32000, 256, 768, name="deretar-2k"),

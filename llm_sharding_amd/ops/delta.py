@@ -72,6 +72,42 @@ def ring(a: DeltaArgs, dtype, n: int) -> None:
     _check(lib().lsa_delta_ring(is_f32(dtype), ctypes.byref(a), n, _stream()), "lsa_delta_ring")
 
 
+CHUNK = 32  # rows per chunk (C in csrc/kernels/delta_chunk.hip)
+
+
+def chunk_bytes(s) -> int:
+    """Workspace bytes of one (chunk, head); 0: the chunked kernels do not take this size."""
+    return int(lib().lsa_delta_chunk_bytes(*s.state_dims))
+
+
+def chunk_groups(runs: list, most: int) -> list:
+    """Long runs (row0, rows, slot, pos0) cut into groups of at most ``most`` chunks, each run going on in the next
+    group where it stopped: [(chunks int32 [n, 8], spans int32 [m, 8])], host."""
+    at, groups = [0] * len(runs), []
+    while True:
+        live = [i for i, r in enumerate(runs) if at[i] < r[1]][:most]
+        if not live:
+            return groups
+        share, chunks, spans = max(1, most // len(live)), [], []
+        for i in live:
+            row0, n, slot, pos0 = runs[i]
+            take = min(n - at[i], share * CHUNK)
+            spans.append([len(chunks), -(-take // CHUNK), slot, pos0 + at[i], row0 + at[i], take, 0, 0])
+            for c in range(0, take, CHUNK):
+                b = at[i] + c
+                chunks.append([row0 + b, min(CHUNK, take - c), slot, pos0 + b, b, 0, 0, 0])
+            at[i] += take
+        groups.append((torch.tensor(chunks, dtype=torch.int32), torch.tensor(spans, dtype=torch.int32)))
+
+
+def chunked(a: DeltaArgs, chunks, spans, ws, nbytes: int) -> None:
+    """One group of :func:`chunk_groups` of checked runs (tables on the device), bf16."""
+    _req(all(t.dtype == torch.int32 and t.is_contiguous() and t.shape[1] == 8 for t in (chunks, spans)), "delta: tables")
+    _req(ws.dtype == torch.uint8 and ws.numel() >= chunks.shape[0] * a.heads * nbytes and nbytes > 0, "delta: workspace")
+    _check(lib().lsa_delta_chunked(ctypes.byref(a), _p(chunks), chunks.shape[0], _p(spans), spans.shape[0], _p(ws),
+                                   _stream()), "lsa_delta_chunked")
+
+
 def declare(L: ctypes.CDLL) -> None:
     """Signatures of these entry points (called by hip.load_library)."""
     vp, i = ctypes.c_void_p, ctypes.c_int
@@ -79,4 +115,6 @@ def declare(L: ctypes.CDLL) -> None:
     hip.set_signatures(L, {
         "lsa_delta_steps": [i, da, i, i, vp],
         "lsa_delta_ring": [i, da, i, vp],
+        "lsa_delta_chunk_bytes": [i, i],
+        "lsa_delta_chunked": [da, vp, i, vp, i, vp, vp],
     })

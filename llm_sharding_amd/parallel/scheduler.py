@@ -131,12 +131,18 @@ def plan_stages(cfg: LlamaConfig, devices: Sequence[DeviceSpec] | int, *,
         return stage_mem(k, a, b) <= d.mem_bytes - d.reserve_bytes
 
     INF = float("inf")
+    # where a stage may start (a stack's layers that read another layer's cache stay with it)
+    cuts_ok = set(cfg.stage_cuts()) | {L} if hasattr(cfg, "stage_cuts") else set(range(L + 1))
+    if len(cuts_ok) <= n:
+        raise ValueError(f"cannot place {cfg.name} on {n} stages: its layers come apart at {len(cuts_ok) - 1} places only")
     # best[k][i] = min bottleneck placing layers [0, i) on stages 0..k-1 (stage k-1 ends at i)
     best = [[INF] * (L + 1) for _ in range(n + 1)]
     arg = [[-1] * (L + 1) for _ in range(n + 1)]
     best[0][0] = 0.0
     for k in range(1, n + 1):
         for i in range(k * min_layers, L - (n - k) * min_layers + 1):
+            if i not in cuts_ok:
+                continue
             for j in range((k - 1) * min_layers, i - min_layers + 1):
                 if best[k - 1][j] == INF or not fits(k - 1, j, i):
                     continue
@@ -160,6 +166,11 @@ def plan_stages(cfg: LlamaConfig, devices: Sequence[DeviceSpec] | int, *,
     return plan
 
 
+def _state_bytes(cfg) -> int:
+    """Per sequence and layer, whatever its length (recurrent layers of a stack)."""
+    return cfg.state_bytes_per_slot() if hasattr(cfg, "state_bytes_per_slot") else 0
+
+
 def kv_slots_for_memory(cfg: LlamaConfig, n_layers: int, max_seq: int, mem_bytes: float,
                         weight_bytes: float, reserve_bytes: float = 8e9, elem_bytes: int = 2,
                         microbatches: int = 1, max_per_microbatch: int = 128) -> int:
@@ -167,7 +178,7 @@ def kv_slots_for_memory(cfg: LlamaConfig, n_layers: int, max_seq: int, mem_bytes
     ``n_layers`` layers next to its weights: the static KV cache is sized from the device's
     HBM (288 GB on MI355X) instead of a fixed guess. Capped at
     ``max_per_microbatch`` (the largest hipGraph decode batch)."""
-    per_slot = float(cfg.kv_bytes_per_token_per_layer(elem_bytes)) * n_layers * max_seq
+    per_slot = (float(cfg.kv_bytes_per_token_per_layer(elem_bytes)) * max_seq + _state_bytes(cfg)) * n_layers
     free = mem_bytes - reserve_bytes - weight_bytes
     if per_slot <= 0 or free < per_slot * microbatches:
         raise ValueError(f"no room for a KV cache of {max_seq} tokens x {n_layers} layers "
@@ -217,7 +228,7 @@ def stage_memory(cfg: LlamaConfig, n_layers: int, *, slots: int, max_seq: int, p
         w += cfg.vocab_size * H * elem_bytes
     if head_rows:
         w += head_rows * H * elem_bytes + H * elem_bytes          # lm_head part + final norm
-    kv = n_layers * cfg.kv_bytes_per_token_per_layer(elem_bytes) * slots * max_seq
+    kv = n_layers * slots * (cfg.kv_bytes_per_token_per_layer(elem_bytes) * max_seq + _state_bytes(cfg))
     scratch = scratch_bytes(cfg, prefill_rows, scratch_sets, max_seq, head_rows)
     io = io_rows * (H * elem_bytes + 4 + 8)
     return {"weights": float(w), "kv": float(kv), "scratch": float(scratch), "io": float(io),

@@ -18,6 +18,9 @@ from ..models.stack import DeltaSpec, pad_to
 
 
 class Delta:
+    chunk_min = 48           # rows from which a run goes chunk by chunk (bf16) instead of step by step
+    CHUNK_BYTES = 256 << 20  # workspace of one group of chunks (about what the last-level cache holds)
+
     def __init__(self, spec: DeltaSpec, t: dict, gpu: bool):
         self.spec, self.gpu = spec, gpu
         s = spec
@@ -40,6 +43,8 @@ class Delta:
         self.low = L.Linear(w2)
         self.out = L.Linear(t["o"])
         self.dtype = t["q"].dtype
+        from ..ops import delta as D
+        self.nbytes = D.chunk_bytes(s) if self.dtype == torch.bfloat16 else 0
 
     def input_parts(self) -> list:
         return self.parts
@@ -68,23 +73,34 @@ class Delta:
         if plan.runs is None:
             D.steps(args(slot=slot, pos=pos), self.dtype, rows, keep=True)
             return ao
-        single, n1, short, n2 = plan.memo("delta", lambda: self._runs(plan, rows, state))
-        if n1:
-            D.steps(args(runs=single), self.dtype, n1, keep=True)
-        if n2:
+        single, short, groups, long = plan.memo(("delta", s if self.nbytes else None), lambda: self._runs(plan, rows, state))
+        if single is not None:
+            D.steps(args(runs=single), self.dtype, single.shape[0], keep=True)
+        if short is not None:
             a = args(runs=short)
-            D.steps(a, self.dtype, n2, keep=False)
-            D.ring(a, self.dtype, n2)
+            D.steps(a, self.dtype, short.shape[0], keep=False)
+            D.ring(a, self.dtype, short.shape[0])
+        if long is not None:
+            a = args(runs=long)
+            ws = eng.workspace("delta", max(c.shape[0] for c, _ in groups) * s.heads * self.nbytes)
+            for chunks, spans in groups:
+                D.chunked(a, chunks, spans, ws, self.nbytes)
+            D.ring(a, self.dtype, long.shape[0])
         return ao
 
-    @staticmethod
-    def _runs(plan, rows: int, state: tuple) -> tuple:
-        """Tables of the runs of one row and of the longer ones, longest first."""
+    def _runs(self, plan, rows: int, state: tuple) -> tuple:
+        """Tables of the runs of one row, of the ones that go step by step (longest first), and the groups of
+        chunks and the table of those that go in chunks; None for what the batch does not have."""
         from ..ops import delta as D
-        host = torch.tensor(plan.runs, dtype=torch.int32)
-        D.check_runs(host, rows, state[0].shape[0])
-        one, more = [r for r in plan.runs if r[1] == 1], sorted((r for r in plan.runs if r[1] > 1), key=lambda r: -r[1])
-        return plan.i32(one), len(one), plan.i32(more), len(more)
+        D.check_runs(torch.tensor(plan.runs, dtype=torch.int32), rows, state[0].shape[0])
+        least = self.chunk_min if self.nbytes else 1 << 30
+        one, more, long = [], [], []
+        for r in sorted(plan.runs, key=lambda r: -r[1]):
+            (one if r[1] == 1 else more if r[1] < least else long).append(r)
+        groups = D.chunk_groups(long, max(1, self.CHUNK_BYTES // (self.spec.heads * self.nbytes))) if long else []
+        dev = plan.eng.device
+        return tuple(plan.i32(t) if t else None for t in (one, more)) + (
+            [(c.to(dev), p.to(dev)) for c, p in groups], plan.i32(long) if long else None)
 
     # ------------------------------------------------------------------ CPU
     def forward_torch(self, eng, x, cache, state: tuple, slot, pos) -> torch.Tensor:

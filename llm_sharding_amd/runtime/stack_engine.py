@@ -62,6 +62,7 @@ class StackEngine(StageEngine):
         self.cache_pages = pages if cache_tokens is None else ceil_div(cache_tokens, PAGE)
         self._rot: dict = {}
         self._expand_bufs: dict = {}
+        self._workspaces: dict = {}
         super().__init__(cfg, start, end, device, dtype, has_embed=has_embed, has_head=has_head, source=source,
                          max_slots=max_slots, max_seq=max_seq, max_prefill_rows=max_prefill_rows, causal=causal,
                          load=load, verbose=verbose, head_cols=head_cols, weight_dtype=weight_dtype)
@@ -237,6 +238,15 @@ class StackEngine(StageEngine):
             kv = torch.empty(t * kn, dtype=self.dtype, device=self.device)
             self._expand_bufs[key] = (lat, kv)
         return lat[:tokens * s.cache_width].view(tokens, -1), kv[:tokens * n].view(tokens, n)
+
+    def workspace(self, name: str, nbytes: int) -> torch.Tensor:
+        """Memory that long portions need (grown on demand: they run eagerly; one per stream of concurrent
+        micro-batches)."""
+        key = (name, torch.cuda.current_stream(self.device).cuda_stream)
+        if key not in self._workspaces or self._workspaces[key].numel() < nbytes:
+            self._workspaces[key] = None
+            self._workspaces[key] = torch.empty(nbytes, dtype=torch.uint8, device=self.device)
+        return self._workspaces[key]
 
     def rotation(self, s) -> tuple:
         return self._rot[(s.rot_base, s.rot_dims)]
