@@ -61,12 +61,13 @@ LSA_DEVICE void delta_store(const DeltaArgs& a, int row, int h, int d, float o, 
 
 template <typename T, int DK, int DV>
 __global__ __launch_bounds__(256) void delta_steps_kernel(DeltaArgs a, int keep) {
-  constexpr int NG = 256 / DV, RPT = DK / NG;  // row groups; state rows per thread
-  static_assert(RPT % 4 == 0, "geometry");
-  __shared__ __attribute__((aligned(16))) float sq[DK], sk[DK], sg[DK], sv[DV], s_a[256], s_b[256];
+  // a thread holds RPT rows x 4 value channels of the state
+  constexpr int NG = 1024 / DV, RPT = DK / NG;
+  static_assert(RPT >= 1 && NG * RPT == DK, "geometry");
+  __shared__ __attribute__((aligned(16))) float sq[DK], sk[DK], sg[DK], sv[DV], s_a[NG][DV], s_b[NG][DV];
   __shared__ float s_unit[2], s_ss[4];
   const DeltaRun r = delta_run(a, blockIdx.x);
-  const int h = blockIdx.y, tid = threadIdx.x, v = tid % DV, d0 = (tid / DV) * RPT;
+  const int h = blockIdx.y, tid = threadIdx.x, v = (tid % (DV / 4)) * 4, grp = tid / (DV / 4), d0 = grp * RPT;
   const int channels = 2 * a.kv_heads * a.dim + a.heads * a.vdim;
   if (r.n == 0) {
     if (!a.runs)
@@ -74,56 +75,53 @@ __global__ __launch_bounds__(256) void delta_steps_kernel(DeltaArgs a, int keep)
     return;
   }
   float* st = a.state + ((size_t)r.slot * a.heads + h) * DK * DV + (size_t)d0 * DV + v;
-  float S[RPT];
+  f32x4_t S[RPT];
 #pragma unroll
-  for (int j = 0; j < RPT; ++j) S[j] = r.pos0 ? st[(size_t)j * DV] : 0.f;
+  for (int j = 0; j < RPT; ++j) S[j] = *reinterpret_cast<const f32x4_t*>(st + (size_t)j * DV);
+  if (r.pos0 == 0) {
+#pragma unroll
+    for (int j = 0; j < RPT; ++j) S[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  }
   for (int t = 0; t < r.n; ++t) {
     const int row = r.row0 + t;
     delta_row<T>(a, r, t, h, channels, DK, DV, sq, sk, sv, sg);
     __syncthreads();
     delta_unit(a, DK, sq, sk, s_unit);
-    float part = 0.f;
+    f32x4_t part = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int j = 0; j < RPT; j += 4) {
-      const f32x4_t g4 = *reinterpret_cast<const f32x4_t*>(sg + d0 + j), k4 = *reinterpret_cast<const f32x4_t*>(sk + d0 + j);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        S[j + e] *= g4[e];
-        part = fmaf(S[j + e], k4[e], part);
-      }
+    for (int j = 0; j < RPT; ++j) {
+      S[j] *= sg[d0 + j];
+      part += S[j] * sk[d0 + j];
     }
-    s_a[tid] = part;
+    *reinterpret_cast<f32x4_t*>(&s_a[grp][v]) = part;
     __syncthreads();
     const float ku = s_unit[1], beta = 1.f / (1.f + expf(-a.in32[(size_t)row * a.ld32 + a.ob + h]));
-    float dot = 0.f;
+    f32x4_t dot = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int g = 0; g < NG; ++g) dot += s_a[g * DV + v];
-    const float u = beta * (sv[v] - dot * ku) * ku;  // times the scale of k
-    float o = 0.f;
+    for (int g = 0; g < NG; ++g) dot += *reinterpret_cast<const f32x4_t*>(&s_a[g][v]);
+    // beta (v - S^T k), times the scale of k
+    const f32x4_t u = (*reinterpret_cast<const f32x4_t*>(&sv[v]) - dot * ku) * (beta * ku);
+    f32x4_t o = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int j = 0; j < RPT; j += 4) {
-      const f32x4_t q4 = *reinterpret_cast<const f32x4_t*>(sq + d0 + j), k4 = *reinterpret_cast<const f32x4_t*>(sk + d0 + j);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        S[j + e] = fmaf(k4[e], u, S[j + e]);
-        o = fmaf(S[j + e], q4[e], o);
-      }
+    for (int j = 0; j < RPT; ++j) {
+      S[j] += u * sk[d0 + j];
+      o += S[j] * sq[d0 + j];
     }
-    s_b[tid] = o;
+    *reinterpret_cast<f32x4_t*>(&s_b[grp][v]) = o;
     __syncthreads();
-    o = 0.f;
+    float x = 0.f;
     if (tid < DV) {
 #pragma unroll
-      for (int g = 0; g < NG; ++g) o += s_b[g * DV + v];
-      o *= s_unit[0];
+      for (int g = 0; g < NG; ++g) x += s_b[g][tid];
+      x *= s_unit[0];
     }
-    const float ss = wave_sum(o * o);
+    const float ss = wave_sum(x * x);
     if ((tid & 63) == 0) s_ss[tid >> 6] = ss;
     __syncthreads();
-    if (tid < a.vdim) delta_store<T>(a, row, h, tid, o, 1.f / sqrtf((s_ss[0] + s_ss[1] + s_ss[2] + s_ss[3]) / (float)a.vdim + a.eps));
+    if (tid < a.vdim) delta_store<T>(a, row, h, tid, x, 1.f / sqrtf((s_ss[0] + s_ss[1] + s_ss[2] + s_ss[3]) / (float)a.vdim + a.eps));
   }
 #pragma unroll
-  for (int j = 0; j < RPT; ++j) st[(size_t)j * DV] = S[j];
+  for (int j = 0; j < RPT; ++j) *reinterpret_cast<f32x4_t*>(st + (size_t)j * DV) = S[j];
   if (keep) delta_keep<T>(a, r, h, channels);
 }
 

@@ -55,43 +55,67 @@ LSA_DEVICE f32x4_t mfma_pair(u32x4_t ah, u32x4_t al, u32x4_t bh, u32x4_t bl, f32
   return mfma16(al, bh, mfma16(ah, bl, mfma16(ah, bh, c)));
 }
 
-LSA_DEVICE float silu_fast(float x) { return x / (1.f + __expf(-x)); }
+// log(1 + e^x) in fp32 on the hardware's exponential and logarithm
+LSA_DEVICE float softplus_fast(float x) {
+  const float e = __expf(-fabsf(x));
+  return fmaxf(x, 0.f) + (e < 0x1p-9f ? e * (1.f - e * (0.5f - e * 0.33333333f)) : __logf(1.f + e));
+}
+LSA_DEVICE float silu_fast(float x) {
+  return x * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * -1.4426950408889634f));
+}
 
-// convolution and silu of one channel over the chunk's rows: f(row, value), zero past the last one
-template <typename F>
-LSA_DEVICE void conv_rows(const DeltaArgs& a, const DeltaChunk& ck, int ch, int col, int channels, F f) {
-  const bf16_raw* in = (const bf16_raw*)a.in + (size_t)ck.row0 * a.ldi + col;
-  const float* w = a.conv + (size_t)ch * a.taps + a.taps - 1;
-  auto past = [&](int t, int j) -> float {  // the input j rows before row t
-    const int back = j - t;  // rows before row0
-    if (back <= ck.before) return bf2f(in[(ptrdiff_t)(t - j) * a.ldi]);
+// Convolution and silu of one channel over the chunk's rows. load() requests its inputs (up to four taps), so
+// that a thread can ask for everything it needs before it waits for any of it; run(f) calls f(row, value),
+// zero past the last row.
+struct ConvRows {
+  bf16_raw raw[C];
+  float x1, x2, x3;
+  int ch, col;
+
+  // the input j rows before row t
+  LSA_DEVICE float past(const DeltaArgs& a, const DeltaChunk& ck, int channels, int t, int j) const {
+    if (j - t <= ck.before) return bf2f(((const bf16_raw*)a.in)[(size_t)(ck.row0 + t - j) * a.ldi + col]);
     const int p = ck.pos0 + t - j;
     return p < 0 ? 0.f : a.ring[((size_t)ck.slot * a.taps + p % a.taps) * channels + ch];
-  };
-  if (a.taps <= 4) {
-    float w0 = w[0], w1 = a.taps > 1 ? w[-1] : 0.f, w2 = a.taps > 2 ? w[-2] : 0.f, w3 = a.taps > 3 ? w[-3] : 0.f;
-    float x1 = a.taps > 1 ? past(0, 1) : 0.f, x2 = a.taps > 2 ? past(0, 2) : 0.f, x3 = a.taps > 3 ? past(0, 3) : 0.f;
+  }
+  LSA_DEVICE void load(const DeltaArgs& a, const DeltaChunk& ck, int channels, int ch_, int col_) {
+    ch = ch_;
+    col = col_;
+    if (a.taps > 4) return;
+    const bf16_raw* in = (const bf16_raw*)a.in + (size_t)ck.row0 * a.ldi + col;
 #pragma unroll
-    for (int t = 0; t < C; ++t) {
-      const float x = t < ck.n ? bf2f(in[(size_t)t * a.ldi]) : 0.f;
-      const float y = silu_fast(fmaf(x3, w3, fmaf(x2, w2, fmaf(x1, w1, x * w0))));
-      f(t, t < ck.n ? y : 0.f);
-      x3 = x2;
-      x2 = x1;
-      x1 = x;
-    }
-  } else {
+    for (int t = 0; t < C; ++t) raw[t] = in[(size_t)min(t, ck.n - 1) * a.ldi];
+    x1 = a.taps > 1 ? past(a, ck, channels, 0, 1) : 0.f;
+    x2 = a.taps > 2 ? past(a, ck, channels, 0, 2) : 0.f;
+    x3 = a.taps > 3 ? past(a, ck, channels, 0, 3) : 0.f;
+  }
+  template <typename F>
+  LSA_DEVICE void run(const DeltaArgs& a, const DeltaChunk& ck, int channels, F f) {
+    const float* w = a.conv + (size_t)ch * a.taps + a.taps - 1;
+    if (a.taps <= 4) {
+      const float w0 = w[0], w1 = a.taps > 1 ? w[-1] : 0.f, w2 = a.taps > 2 ? w[-2] : 0.f, w3 = a.taps > 3 ? w[-3] : 0.f;
 #pragma unroll
-    for (int t = 0; t < C; ++t) {
-      float y = 0.f;
-      if (t < ck.n) {
-        for (int j = 0; j < a.taps; ++j) y = fmaf(past(t, j), w[-j], y);
-        y = silu_fast(y);
+      for (int t = 0; t < C; ++t) {
+        const float x = bf2f(raw[t]);
+        const float y = silu_fast(fmaf(x3, w3, fmaf(x2, w2, fmaf(x1, w1, x * w0))));
+        f(t, t < ck.n ? y : 0.f);
+        x3 = x2;
+        x2 = x1;
+        x1 = x;
       }
-      f(t, y);
+    } else {
+#pragma unroll
+      for (int t = 0; t < C; ++t) {
+        float y = 0.f;
+        if (t < ck.n) {
+          for (int j = 0; j < a.taps; ++j) y = fmaf(past(a, ck, channels, t, j), w[-j], y);
+          y = silu_fast(y);
+        }
+        f(t, y);
+      }
     }
   }
-}
+};
 
 template <int DK, int DV>
 __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a, const DeltaChunk* __restrict__ chunks,
@@ -108,24 +132,30 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a, const Del
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
   unsigned char* out = ws + ((size_t)blockIdx.x * a.heads + h) * STRIDE;
 
-  for (int c = tid; c < 2 * DK; c += 256) {  // q and k
-    const int d = c % DK, isk = c / DK;
-    auto& dst = isk ? sk : sq;
-    if (d < a.dim)
-      conv_rows(a, ck, isk * kc + kb * a.dim + d, (isk ? a.ok : a.oq) + kb * a.dim + d, channels,
-                [&](int t, float y) { dst[t][d] = y; });
-    else
-      for (int t = 0; t < C; ++t) dst[t][d] = 0.f;
-  }
-  for (int c = tid; c < 2 * DK; c += 256) {  // sums of log2 decays, 16 rows at a time
-    const int d = c % DK, t0 = (c / DK) * 16;
-    const float A = d < a.dim ? -a.decay[h] * 1.4426950408889634f : 0.f, bias = d < a.dim ? a.dt_bias[h * a.dim + d] : 0.f;
+  static_assert(2 * DK <= 256 && DK + DV <= 256, "one channel per thread");
+  const int cd = tid % DK, isk = tid / DK;  // thread < 2 DK: channel cd of q / k, and 16 rows of its decay
+  ConvRows qk, vc;
+  float zz[16];
+  if (tid < 2 * DK) {
+    const int d = min(cd, a.dim - 1);
+    qk.load(a, ck, channels, isk * kc + kb * a.dim + d, (isk ? a.ok : a.oq) + kb * a.dim + d);
     const float* z = a.z + (size_t)ck.row0 * a.ldz + h * a.dim + d;
-    float g = 0.f;
 #pragma unroll
-    for (int t = t0; t < t0 + 16; ++t) {
-      if (d < a.dim && t < ck.n) g = fmaf(A, delta_softplus(z[(size_t)t * a.ldz] + bias), g);
-      sg[t][d] = g;
+    for (int t = 0; t < 16; ++t) zz[t] = z[(size_t)min(isk * 16 + t, ck.n - 1) * a.ldz];
+  }
+  if (tid < DV) {
+    const int d = min(tid, a.vdim - 1);
+    vc.load(a, ck, channels, 2 * kc + h * a.vdim + d, a.ov + h * a.vdim + d);
+  }
+  if (tid < 2 * DK) {
+    auto& dst = isk ? sk : sq;
+    qk.run(a, ck, channels, [&](int t, float y) { dst[t][cd] = cd < a.dim ? y : 0.f; });
+    const float A = cd < a.dim ? -a.decay[h] * 1.4426950408889634f : 0.f, bias = cd < a.dim ? a.dt_bias[h * a.dim + cd] : 0.f;
+    float g = 0.f;  // sums of log2 decays, 16 rows at a time
+#pragma unroll
+    for (int t = 0; t < 16; ++t) {
+      g = isk * 16 + t < ck.n ? fmaf(A, softplus_fast(zz[t] + bias), g) : g;
+      sg[isk * 16 + t][cd] = g;
     }
   }
   if (tid < C) sb[tid] = tid < ck.n ? 1.f / (1.f + __expf(-a.in32[(size_t)(ck.row0 + tid) * a.ld32 + a.ob + h])) : 0.f;
@@ -229,15 +259,11 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a, const Del
     put_pair(out + PC::P * 1024, out + (PC::P + 2) * 1024, tid, f);
   }
   // (1 + A) x = b, one column per thread: beta v -> U, beta k e^G -> W
-  for (int c = tid; c < DV + DK; c += 256) {
+  if (tid < DV + DK) {
+    const int c = tid;
     float x[C];
     if (c < DV) {
-      if (c < a.vdim) {
-        conv_rows(a, ck, 2 * kc + h * a.vdim + c, a.ov + h * a.vdim + c, channels, [&](int t, float y) { x[t] = y * sb[t]; });
-      } else {
-#pragma unroll
-        for (int t = 0; t < C; ++t) x[t] = 0.f;
-      }
+      vc.run(a, ck, channels, [&](int t, float y) { x[t] = c < a.vdim ? y * sb[t] : 0.f; });
     } else {
 #pragma unroll
       for (int t = 0; t < C; ++t) x[t] = sb[t] * sk[t][c - DV] * __builtin_amdgcn_exp2f(sg[t][c - DV]);
@@ -301,7 +327,13 @@ __global__ __launch_bounds__(DV / NC * 4) void delta_scan_kernel(DeltaArgs a, co
 #pragma unroll
     for (int m = 0; m < MT; ++m)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) S[n][m][r] = sp.pos0 ? st[(size_t)(m * 16 + q4 * 4 + r) * DV + n * 16] : 0.f;
+      for (int r = 0; r < 4; ++r) S[n][m][r] = st[(size_t)(m * 16 + q4 * 4 + r) * DV + n * 16];
+  if (sp.pos0 == 0) {
+#pragma unroll
+    for (int n = 0; n < NC; ++n)
+#pragma unroll
+      for (int m = 0; m < MT; ++m) S[n][m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  }
   float nw[NC];
 #pragma unroll
   for (int n = 0; n < NC; ++n) {
@@ -310,7 +342,7 @@ __global__ __launch_bounds__(DV / NC * 4) void delta_scan_kernel(DeltaArgs a, co
   }
 
   f32x4_t U[NC][2], O[NC][2];
-  float gl[NC][8];
+  bf16_raw gl[NC][8];
   auto stage = [&](int c, int buf) {
     const unsigned char* p = src + c * step;
     for (int i = w; i < NP; i += NW) glds16(p + i * 1024 + lane * 16, smem + (buf * NP + i) * 1024);
@@ -323,17 +355,18 @@ __global__ __launch_bounds__(DV / NC * 4) void delta_scan_kernel(DeltaArgs a, co
       for (int m = 0; m < 2; ++m)
         U[n][m] = *reinterpret_cast<const f32x4_t*>(p + ((w * NC + n) * 2 + m) * 1024 + lane * 16);
   };
-  // gate logits of chunk c in accumulator order
+  // gate logits of chunk c in accumulator order, as they are: a conversion here would wait for them
   auto load_gate = [&](int c) {
+    const bf16_raw* gp = (const bf16_raw*)a.gate + (size_t)sp.row0 * a.ldg + h * a.vdim;
 #pragma unroll
-    for (int n = 0; n < NC; ++n)
+    for (int e = 0; e < 8; ++e) {
+      const int t = min(c * C + (e >> 2) * 16 + q4 * 4 + (e & 3), sp.n - 1);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const int t = c * C + (e >> 2) * 16 + q4 * 4 + (e & 3), v = (w * NC + n) * 16 + l16;
-        gl[n][e] = a.gate && t < sp.n && v < a.vdim
-                       ? bf2f(((const bf16_raw*)a.gate)[(size_t)(sp.row0 + t) * a.ldg + h * a.vdim + v]) : 0.f;
-      }
+      for (int n = 0; n < NC; ++n) gl[n][e] = gp[(size_t)t * a.ldg + min((w * NC + n) * 16 + l16, a.vdim - 1)];
+    }
   };
+  const float inv_v = 1.f / (float)a.vdim;
+  bf16_raw* op = (bf16_raw*)a.out + (size_t)sp.row0 * a.ldo + h * a.vdim + w * NC * 16 + l16;
   auto finish = [&](int c) {  // chunk c's read-outs
     const float* ss = s_ss + (c & 1) * NW * C;
 #pragma unroll
@@ -342,13 +375,12 @@ __global__ __launch_bounds__(DV / NC * 4) void delta_scan_kernel(DeltaArgs a, co
       float sum = 0.f;
 #pragma unroll
       for (int x = 0; x < NW; ++x) sum += ss[x * C + r];
-      const float rs = 1.f / sqrtf(sum / (float)a.vdim + a.eps);
+      const float rs = __builtin_amdgcn_rsqf(fmaf(sum, inv_v, a.eps));
 #pragma unroll
       for (int n = 0; n < NC; ++n) {
         const int v = (w * NC + n) * 16 + l16;
-        if (t < sp.n && v < a.vdim)
-          ((bf16_raw*)a.out)[(size_t)(sp.row0 + t) * a.ldo + h * a.vdim + v] =
-              f2bf(O[n][e >> 2][e & 3] * rs * nw[n] * (a.gate ? sigmoid(gl[n][e]) : 1.f));
+        const float g = __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(bf2f(gl[n][e]) * -1.4426950408889634f));
+        if (t < sp.n && v < a.vdim) op[t * a.ldo + n * 16] = f2bf(O[n][e >> 2][e & 3] * rs * nw[n] * g);
       }
     }
   };
@@ -359,6 +391,11 @@ __global__ __launch_bounds__(DV / NC * 4) void delta_scan_kernel(DeltaArgs a, co
     asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
     __builtin_amdgcn_s_barrier();
     asm volatile("" ::: "memory");
+    // U has arrived here, not at its first use below (whose wait would also drain the next chunk's DMA)
+#pragma unroll
+    for (int n = 0; n < NC; ++n)
+#pragma unroll
+      for (int m = 0; m < 2; ++m) asm volatile("" : "+v"(U[n][m]));
     if (c) finish(c - 1);
     if (c + 1 < sp.chunks) stage(c + 1, (c + 1) & 1);
     load_gate(c);
@@ -446,7 +483,7 @@ extern "C" int lsa_delta_chunk_bytes(int dk, int dv) {
 // chunks: n_chunks DeltaChunk; spans: n_spans DeltaSpan over them; ws: n_chunks * heads * lsa_delta_chunk_bytes
 extern "C" int lsa_delta_chunked(const DeltaArgs* a, const void* chunks, int n_chunks, const void* spans, int n_spans,
                                  void* ws, hipStream_t s) {
-  if (!a || bad_delta(a) || n_chunks < 1 || n_spans < 1 || !chunks || !spans || !ws || (uintptr_t)ws % 16) return LSA_BAD_SHAPE;
+  if (!a || bad_delta(a) || !a->gate || n_chunks < 1 || n_spans < 1 || !chunks || !spans || !ws || (uintptr_t)ws % 16) return LSA_BAD_SHAPE;
 #define LSA_C(K, V, NC)                                                                                                     \
   if (a->dk == K && a->dv == V) {                                                                                           \
     delta_chunk_kernel<K, V><<<dim3(n_chunks, a->heads), 256, 0, s>>>(*a, (const DeltaChunk*)chunks, (unsigned char*)ws);   \
@@ -457,7 +494,7 @@ extern "C" int lsa_delta_chunked(const DeltaArgs* a, const void* chunks, int n_c
     return LSA_OK;                                                                                                          \
   }
   LSA_C(32, 32, 1) LSA_C(32, 64, 1) LSA_C(32, 128, 2) LSA_C(64, 32, 1) LSA_C(64, 64, 1) LSA_C(64, 128, 2) LSA_C(128, 32, 1)
-  LSA_C(128, 64, 1) LSA_C(128, 128, 2)
+  LSA_C(128, 64, 1) LSA_C(128, 128, 1)
 #undef LSA_C
   return LSA_UNSUPPORTED;
 }

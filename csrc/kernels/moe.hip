@@ -6,14 +6,14 @@ namespace {
 
 // one wave per row: ``top`` times the largest logit left (ties: the smaller index), softmax over them
 constexpr int MAX_E = 1024;
-__global__ __launch_bounds__(256) void route_kernel(const float* __restrict__ logits, int ldl, int rows, int E, int top,
-                                                    int* __restrict__ expert, float* __restrict__ weight) {
-  const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (row >= rows) return;
+template <int NE>  // logits per lane: at most 64 NE experts
+LSA_DEVICE void route_row(const float* __restrict__ logits, int ldl, int row, int E, int top, int* __restrict__ expert,
+                          float* __restrict__ weight) {
+  const int lane = threadIdx.x & 63;
   const float* z = logits + (size_t)row * ldl;
-  float v[MAX_E / 64];
+  float v[NE];
 #pragma unroll
-  for (int j = 0; j < MAX_E / 64; ++j) {
+  for (int j = 0; j < NE; ++j) {
     const int e = j * 64 + lane;
     v[j] = e < E ? z[e] : 0.f;
   }
@@ -22,7 +22,7 @@ __global__ __launch_bounds__(256) void route_kernel(const float* __restrict__ lo
   for (int k = 0; k < top; ++k) {
     unsigned long long best = 0ull;
 #pragma unroll
-    for (int j = 0; j < MAX_E / 64; ++j) {
+    for (int j = 0; j < NE; ++j) {
       const int e = j * 64 + lane;
       if (e < E && !(taken >> j & 1)) {
         const unsigned long long key = argmax_key(v[j], (unsigned)e);
@@ -51,15 +51,37 @@ __global__ __launch_bounds__(256) void route_kernel(const float* __restrict__ lo
   for (int k = lane; k < top; k += 64) weight[(size_t)row * top + k] *= inv;  // this lane's own stores
 }
 
-// one workgroup: counting sort of the pairs by expert, and the tile table
-__global__ __launch_bounds__(1024) void group_kernel(const int* __restrict__ expert, int pairs, int E, int tile_rows,
-                                                     int max_tiles, int* __restrict__ order, int* __restrict__ place,
-                                                     MoeTile* __restrict__ tiles) {
+template <int NE>
+__global__ __launch_bounds__(256) void route_kernel(const float* __restrict__ logits, int ldl, int rows, int E, int top,
+                                                    int* __restrict__ expert, float* __restrict__ weight) {
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (row < rows) route_row<NE>(logits, ldl, row, E, top, expert, weight);
+}
+
+// One workgroup: counting sort of the pairs by expert, and the tile table. NE > 0: few rows, whose routing
+// comes first.
+template <int NE>
+__global__ __launch_bounds__(1024) void group_kernel(const float* __restrict__ logits, int ldl, int top,
+                                                     float* __restrict__ weight, int* expert, int pairs, int E,
+                                                     int tile_rows, int max_tiles, int* __restrict__ order,
+                                                     int* __restrict__ place, MoeTile* __restrict__ tiles) {
   __shared__ int s_cnt[MAX_E], s_off[MAX_E], s_tile[MAX_E], s_n[1], s_w[2][16];
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
   s_cnt[tid] = 0;
+  if constexpr (NE > 0) {
+    for (int row = w; row < pairs / top; row += 16) route_row<NE>(logits, ldl, row, E, top, expert, weight);
+    __threadfence_block();
+  }
   __syncthreads();
-  for (int i = tid; i < pairs; i += 1024) place[i] = atomicAdd(&s_cnt[expert[i]], 1);  // rank within its expert
+  constexpr int U = 8;  // loads in flight per thread
+  for (int i0 = tid; i0 < pairs; i0 += 1024 * U) {
+    int e[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) e[u] = i0 + u * 1024 < pairs ? expert[i0 + u * 1024] : 0;
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (i0 + u * 1024 < pairs) place[i0 + u * 1024] = atomicAdd(&s_cnt[e[u]], 1);  // rank within its expert
+  }
   __syncthreads();
   // exclusive sums over experts of pairs and of tiles
   const int c = tid < E ? s_cnt[tid] : 0, nt = (c + tile_rows - 1) / tile_rows;
@@ -91,10 +113,22 @@ __global__ __launch_bounds__(1024) void group_kernel(const int* __restrict__ exp
       if (s_tile[tid] + t < max_tiles)
         tiles[s_tile[tid] + t] = MoeTile{tid, s_off[tid] + t * tile_rows, min(tile_rows, c - t * tile_rows), 0};
   for (int t = s_n[0] + tid; t < max_tiles; t += 1024) tiles[t] = MoeTile{-1, 0, 0, 0};
-  for (int i = tid; i < pairs; i += 1024) {  // this thread's own ranks
-    const int at = s_off[expert[i]] + place[i];
-    place[i] = at;
-    order[at] = i;
+  for (int i0 = tid; i0 < pairs; i0 += 1024 * U) {
+    int e[U], rank[U];  // this thread's own ranks
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int i = min(i0 + u * 1024, pairs - 1);
+      e[u] = expert[i];
+      rank[u] = place[i];
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int i = i0 + u * 1024;
+      if (i >= pairs) break;
+      const int at = s_off[e[u]] + rank[u];
+      place[i] = at;
+      order[at] = i;
+    }
   }
 }
 
@@ -229,7 +263,11 @@ __global__ __launch_bounds__(256) void moe_f32_kernel(const MoeTile* __restrict_
 extern "C" int lsa_moe_route(const float* logits, int ldl, int rows, int E, int top, int* expert, float* weight,
                              hipStream_t s) {
   if (rows < 1 || E < 1 || E > MAX_E || top < 1 || top > E || ldl < E) return LSA_BAD_SHAPE;
-  route_kernel<<<(rows + 3) / 4, 256, 0, s>>>(logits, ldl, rows, E, top, expert, weight);
+#define LSA_RT(NE) route_kernel<NE><<<(rows + 3) / 4, 256, 0, s>>>(logits, ldl, rows, E, top, expert, weight)
+  if (E <= 64) LSA_RT(1);
+  else if (E <= 256) LSA_RT(4);
+  else LSA_RT(MAX_E / 64);
+#undef LSA_RT
   LSA_CHECK_LAUNCH();
   return LSA_OK;
 }
@@ -239,7 +277,24 @@ extern "C" int lsa_moe_group(const int* expert, int pairs, int E, int tile_rows,
                              void* tiles, hipStream_t s) {
   if (pairs < 1 || E < 1 || E > MAX_E || tile_rows < 1 || max_tiles < (E < pairs ? E : pairs) + pairs / tile_rows)
     return LSA_BAD_SHAPE;
-  group_kernel<<<1, 1024, 0, s>>>(expert, pairs, E, tile_rows, max_tiles, order, place, (MoeTile*)tiles);
+  group_kernel<0><<<1, 1024, 0, s>>>(nullptr, 0, 1, nullptr, const_cast<int*>(expert), pairs, E, tile_rows, max_tiles,
+                                     order, place, (MoeTile*)tiles);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+// lsa_moe_route and lsa_moe_group of few rows in one launch
+extern "C" int lsa_moe_route_group(const float* logits, int ldl, int rows, int E, int top, int* expert, float* weight,
+                                   int tile_rows, int max_tiles, int* order, int* place, void* tiles, hipStream_t s) {
+  const int pairs = rows * top;
+  if (rows < 1 || rows > 64 || E < 1 || E > 256 || top < 1 || top > E || ldl < E || tile_rows < 1 ||
+      max_tiles < (E < pairs ? E : pairs) + pairs / tile_rows)
+    return LSA_BAD_SHAPE;
+#define LSA_RG(NE) \
+  group_kernel<NE><<<1, 1024, 0, s>>>(logits, ldl, top, weight, expert, pairs, E, tile_rows, max_tiles, order, place, (MoeTile*)tiles)
+  if (E <= 64) LSA_RG(1);
+  else LSA_RG(4);
+#undef LSA_RG
   LSA_CHECK_LAUNCH();
   return LSA_OK;
 }

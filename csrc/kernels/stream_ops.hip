@@ -183,12 +183,18 @@ LSA_DEVICE void join_at(const JoinArgs& a, int row, int c, float* x) {
     } else {
 #pragma unroll
       for (int k = 0; k < V; ++k) y[k] = 0.f;
-      for (int e = 0; e < a.top; ++e) {
-        float z[V];
-        get((const T*)a.ye + (size_t)a.place[row * a.top + e] * a.ldye + c, z);
-        const float w = a.weight[row * a.top + e];
+      for (int e0 = 0; e0 < a.top; e0 += 4) {  // four results requested at a time
+        float z[4][V], w[4];
 #pragma unroll
-        for (int k = 0; k < V; ++k) y[k] = fmaf(w, z[k], y[k]);
+        for (int e = 0; e < 4; ++e) {
+          const int i = row * a.top + min(e0 + e, a.top - 1);
+          w[e] = e0 + e < a.top ? a.weight[i] : 0.f;
+          get((const T*)a.ye + (size_t)a.place[i] * a.ldye + c, z[e]);
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+          for (int k = 0; k < V; ++k) y[k] = fmaf(w[e], z[e][k], y[k]);
       }
     }
 #pragma unroll

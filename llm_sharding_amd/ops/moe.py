@@ -39,8 +39,8 @@ def tile_rows(pairs: int, experts: int, f32: bool) -> int:
     """Pairs per tile: what an expert gets on average, rounded to a kernel's size."""
     if f32:
         return 64
-    mean = pairs / experts
-    return 16 if mean <= 16 else (32 if mean <= 32 else 64)
+    mean = pairs / experts  # (a second tile of an expert reads its weights again)
+    return next((n for n in (16, 32, 64) if mean <= 0.75 * n), 128 if mean <= 320 else 256)
 
 
 def max_tiles(pairs: int, experts: int, rows: int) -> int:
@@ -67,6 +67,22 @@ def group(expert, pairs: int, experts: int, rows: int, order, place, tiles) -> i
     return n
 
 
+def route_group(logits, rows: int, experts: int, top: int, tile: int, expert, weight, order, place, tiles) -> int:
+    """:func:`route` and :func:`group`, in one launch where there are few rows."""
+    pairs = rows * top
+    if rows > 64 or experts > 256:
+        route(logits, rows, experts, top, expert, weight)
+        return group(expert, pairs, experts, tile, order, place, tiles)
+    n = max_tiles(pairs, experts, tile)
+    _req(logits.dtype == torch.float32 and logits.stride(1) == 1 and logits.shape[0] >= rows
+         and logits.shape[1] >= experts and weight.dtype == torch.float32 and weight.numel() >= pairs, "route: shapes")
+    _req(all(t.dtype == torch.int32 for t in (expert, order, place, tiles)) and tiles.numel() >= 4 * n
+         and min(expert.numel(), order.numel(), place.numel()) >= pairs, "group: shapes")
+    _check(lib().lsa_moe_route_group(_p(logits), logits.stride(0), rows, experts, top, _p(expert), _p(weight), tile, n,
+                                     _p(order), _p(place), _p(tiles), _stream()), "lsa_moe_route_group")
+    return n
+
+
 def gemm(tiles, n_tiles: int, rows: int, order, top: int, a, w, n: int, k: int, out, pairs: int, glu: bool) -> None:
     """One product of every tile's expert: ``glu`` up from rows of h (``a``) to out [pairs, n / 2], else down from
     out rows of the sorted pairs (``a`` [pairs, k]) to out [pairs, n]."""
@@ -74,6 +90,10 @@ def gemm(tiles, n_tiles: int, rows: int, order, top: int, a, w, n: int, k: int, 
          and out.shape[0] >= pairs and out.shape[1] >= (n // 2 if glu else n) and order.numel() >= pairs
          and (a.shape[0] * top >= pairs if glu else a.shape[0] >= pairs), "moe: shapes")
     _req(w[0].numel() == n * k and w.is_contiguous(), "moe: weights")
+    if rows > 64:
+        _check(lib().lsa_moe_gemm_big(int(glu), _p(tiles), n_tiles, rows, _p(order), top, _p(a), a.shape[0] if glu else 0,
+                                      a.stride(0), _p(w), n, k, _p(out), out.stride(0), _stream()), "lsa_moe_gemm_big")
+        return
     _check(lib().lsa_moe_gemm(is_f32(a.dtype), int(glu), _p(tiles), n_tiles, rows, _p(order), top, _p(a), a.stride(0), _p(w),
                               n, k, _p(out), out.stride(0), _stream()), "lsa_moe_gemm")
 
@@ -84,5 +104,7 @@ def declare(L: ctypes.CDLL) -> None:
     hip.set_signatures(L, {
         "lsa_moe_route": [vp, i, i, i, i, vp, vp, vp],
         "lsa_moe_group": [vp, i, i, i, i, vp, vp, vp, vp],
+        "lsa_moe_route_group": [vp, i, i, i, i, vp, vp, i, i, vp, vp, vp, vp],
+        "lsa_moe_gemm_big": [i, vp, i, i, vp, i, vp, i, i, vp, i, i, vp, i, vp],
         "lsa_moe_gemm": [i, i, vp, i, i, vp, i, vp, i, vp, i, i, vp, i, vp],
     })

@@ -108,9 +108,8 @@ class Moe:
         expert, order, place = eng.scratch_view("pairs", rows, 3 * s.top).reshape(3, pairs)
         weight, tiles = eng.scratch_view("pair_w", rows, s.top).reshape(-1), eng.scratch_view("tiles", rows, 8 * s.top)
         act, ye = eng.scratch_view("act", pairs, x.ff), eng.scratch_view("ye", pairs, x.width)
-        X.route(in32[:, col["router"]:], rows, s.experts, s.top, expert, weight)
         tr = X.tile_rows(pairs, s.experts, x.f32)
-        nt = X.group(expert, pairs, s.experts, tr, order, place, tiles)
+        nt = X.route_group(in32[:, col["router"]:], rows, s.experts, s.top, tr, expert, weight, order, place, tiles)
         X.gemm(tiles, nt, tr, order, s.top, h, x.up, 2 * x.ff, x.width, act, pairs, glu=True)
         X.gemm(tiles, nt, tr, order, s.top, act, x.down, x.width, x.ff, ye, pairs, glu=False)
         return {"experts": (ye, weight, place, s.top), "gate2": gate}
