@@ -214,6 +214,8 @@ class PipelineServer:
               and all(a < b for a, b in st) and all(x[1] == y[0] for x, y in zip(st, st[1:])))
         if not ok:
             raise ValueError(f"replan: {st} is not a contiguous split of {L} layers over {self.world} stages")
+        if hasattr(self.cfg, "stage_cuts") and not set(a for a, _ in st) <= set(self.cfg.stage_cuts()):
+            raise ValueError(f"replan: {st} parts a layer from the one whose keys and values it reads")
         with self._lock:
             self._replan = [a for a, _ in st] + [L]
 

@@ -72,12 +72,18 @@ def short_conv(x, taps):
     out = torch.zeros_like(x)
     for j in range(t):
         back = t - 1 - j  # how far back this column looks
-        out[back:] += x[:x.shape[0] - back] * taps[:, j]
+        if back < x.shape[0]:
+            out[back:] += x[:x.shape[0] - back] * taps[:, j]
     return out
 
 
+def unit_eps(x, eps):
+    """x over its length, eps inside the root."""
+    return x / torch.sqrt((x * x).sum(dim=-1, keepdim=True) + eps)
+
+
 def unit(x):
-    return x / torch.sqrt((x * x).sum(dim=-1, keepdim=True) + 1e-6)
+    return unit_eps(x, 1e-6)
 
 
 def log_decay(h, w, m):

@@ -14,7 +14,8 @@ from llm_sharding_amd.parallel.scheduler import plan_stages
 from llm_sharding_amd.runtime.registry import random_source
 
 M, B, P, NEW = 2, 2, 5, 6
-MODELS = {"llama": lambda: tiny(layers=5), "gpt2": lambda: tiny_gpt2(layers=5), "deretar": lambda: get_preset("tiny-deretar")}
+MODELS = {"llama": lambda: tiny(layers=5), "gpt2": lambda: tiny_gpt2(layers=5), "deretar": lambda: get_preset("tiny-deretar"),
+          "gupuvik": lambda: get_preset("tiny-gupuvik")}
 
 
 def _free_port() -> int:
@@ -92,11 +93,12 @@ def test_gpt2_pipeline_matches_single():
     assert _run_world(2, "gpt2") == ref
 
 
-def test_stack_pipeline_matches_single():
-    """A Deretar stack (fp32 residual stream handed over, paged cache per stage) over 2 gloo ranks."""
-    ref = _single("deretar")
+@pytest.mark.parametrize("name", ["deretar", "gupuvik"])
+def test_stack_pipeline_matches_single(name):
+    """A stack (fp32 residual stream handed over, paged cache and states per stage) over 2 gloo ranks."""
+    ref = _single(name)
     assert len(set(sum(sum(ref, []), []))) > 3
-    assert _run_world(2, "deretar") == ref
+    assert _run_world(2, name) == ref
 
 
 def test_plan_covers_all_layers():
