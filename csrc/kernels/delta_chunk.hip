@@ -303,173 +303,187 @@ LSA_DEVICE void glds16(const void* src, unsigned char* lds_base) {
   __builtin_amdgcn_global_load_lds(src, (__attribute__((address_space(3))) void*)lds_base, 16, 0, 0);
 }
 
-// One workgroup per (run, head): the state in registers (wave w: value channels w NC 16 ..), a chunk's
-// operands by LDS-DMA into a double buffer. Read-outs are normed over the head's value channels one
-// chunk later, behind the barrier that the next chunk needs anyway.
-template <int DK, int DV, int NC>
-__global__ __launch_bounds__(DV / NC * 4) void delta_scan_kernel(DeltaArgs a, const DeltaSpan* __restrict__ spans,
-                                                                 const unsigned char* __restrict__ ws) {
+// One workgroup per (run, head, NW 16 value channels): the state in registers (a wave has 16 channels of it), a
+// chunk's operands by LDS-DMA into a double buffer. Leaves the read-outs in fp32 for delta_norm_kernel.
+template <int DK, int DV, int NW>
+__global__ __launch_bounds__(NW * 64) void delta_scan_kernel(DeltaArgs a, const DeltaSpan* __restrict__ spans,
+                                                             const unsigned char* __restrict__ ws,
+                                                             float* __restrict__ o32) {
   using PC = Pieces<DK>;
-  constexpr int KF = DK / 32, MT = DK / 16, NW = DV / 16 / NC, NP = PC::U;
+  constexpr int KF = DK / 32, MT = DK / 16, NP = PC::U;
+  constexpr int NDMA = (NP + NW - 1) / NW, LESS = NP % NW;  // DMA instructions per wave; waves >= LESS > 0: one less
   constexpr size_t STRIDE = (size_t)(PC::U + DV / 8) * 1024;
-  __shared__ __attribute__((aligned(16))) unsigned char smem[2 * NP * 1024 + 2 * NW * C * 4];
-  float* s_ss = reinterpret_cast<float*>(smem + 2 * NP * 1024);  // [2][NW][C]
+  __shared__ __attribute__((aligned(16))) unsigned char smem[3 * NP * 1024];
   const DeltaSpan sp = spans[blockIdx.x];
   const int h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, q4 = lane >> 4;
-  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6), vt = blockIdx.z * NW + w;  // this wave's channels: 16 vt ..
   const unsigned char* src = ws + ((size_t)sp.chunk0 * a.heads + h) * STRIDE;
   const size_t step = (size_t)a.heads * STRIDE;
 
-  f32x4_t S[NC][MT];
-  float* st = a.state + ((size_t)sp.slot * a.heads + h) * DK * DV + w * NC * 16 + l16;
+  f32x4_t S[MT], U0[2], U1[2];
+  float* st = a.state + ((size_t)sp.slot * a.heads + h) * DK * DV + vt * 16 + l16;
 #pragma unroll
-  for (int n = 0; n < NC; ++n)
+  for (int m = 0; m < MT; ++m)
 #pragma unroll
-    for (int m = 0; m < MT; ++m)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) S[n][m][r] = st[(size_t)(m * 16 + q4 * 4 + r) * DV + n * 16];
+    for (int r = 0; r < 4; ++r) S[m][r] = st[(size_t)(m * 16 + q4 * 4 + r) * DV];
   if (sp.pos0 == 0) {
 #pragma unroll
-    for (int n = 0; n < NC; ++n)
-#pragma unroll
-      for (int m = 0; m < MT; ++m) S[n][m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int m = 0; m < MT; ++m) S[m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   }
-  float nw[NC];
-#pragma unroll
-  for (int n = 0; n < NC; ++n) {
-    const int v = (w * NC + n) * 16 + l16;
-    nw[n] = v < a.vdim ? a.norm[v] : 0.f;
-  }
-
-  f32x4_t U[NC][2], O[NC][2];
-  bf16_raw gl[NC][8];
   auto stage = [&](int c, int buf) {
-    const unsigned char* p = src + c * step;
-    for (int i = w; i < NP; i += NW) glds16(p + i * 1024 + lane * 16, smem + (buf * NP + i) * 1024);
+    const unsigned char* p = src + c * step + lane * 16;
+#pragma unroll
+    for (int i = 0; i < NDMA; ++i)
+      if (LESS == 0 || i * NW + w < NP) glds16(p + (i * NW + w) * 1024, smem + (buf * NP + i * NW + w) * 1024);
   };
-  auto load_u = [&](int c) {
-    const unsigned char* p = src + c * step + PC::U * 1024;
+  auto load_u = [&](int c, f32x4_t (&U)[2]) {
+    const unsigned char* p = src + c * step + (PC::U + vt * 2) * 1024 + lane * 16;
 #pragma unroll
-    for (int n = 0; n < NC; ++n)
-#pragma unroll
-      for (int m = 0; m < 2; ++m)
-        U[n][m] = *reinterpret_cast<const f32x4_t*>(p + ((w * NC + n) * 2 + m) * 1024 + lane * 16);
+    for (int m = 0; m < 2; ++m) U[m] = *reinterpret_cast<const f32x4_t*>(p + m * 1024);
   };
-  // gate logits of chunk c in accumulator order, as they are: a conversion here would wait for them
-  auto load_gate = [&](int c) {
-    const bf16_raw* gp = (const bf16_raw*)a.gate + (size_t)sp.row0 * a.ldg + h * a.vdim;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const int t = min(c * C + (e >> 2) * 16 + q4 * 4 + (e & 3), sp.n - 1);
-#pragma unroll
-      for (int n = 0; n < NC; ++n) gl[n][e] = gp[(size_t)t * a.ldg + min((w * NC + n) * 16 + l16, a.vdim - 1)];
-    }
-  };
-  const float inv_v = 1.f / (float)a.vdim;
-  bf16_raw* op = (bf16_raw*)a.out + (size_t)sp.row0 * a.ldo + h * a.vdim + w * NC * 16 + l16;
-  auto finish = [&](int c) {  // chunk c's read-outs
-    const float* ss = s_ss + (c & 1) * NW * C;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const int r = (e >> 2) * 16 + q4 * 4 + (e & 3), t = c * C + r;
-      float sum = 0.f;
-#pragma unroll
-      for (int x = 0; x < NW; ++x) sum += ss[x * C + r];
-      const float rs = __builtin_amdgcn_rsqf(fmaf(sum, inv_v, a.eps));
-#pragma unroll
-      for (int n = 0; n < NC; ++n) {
-        const int v = (w * NC + n) * 16 + l16;
-        const float g = __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(bf2f(gl[n][e]) * -1.4426950408889634f));
-        if (t < sp.n && v < a.vdim) op[t * a.ldo + n * 16] = f2bf(O[n][e >> 2][e & 3] * rs * nw[n] * g);
-      }
-    }
-  };
+  const int v = vt * 16 + l16;
+  float* op = o32 + (size_t)sp.row0 * a.heads * a.vdim + h * a.vdim + min(v, a.vdim - 1);
+  const int ldo = a.heads * a.vdim;
 
-  stage(0, 0);
-  load_u(0);
-  for (int c = 0; c < sp.chunks; ++c) {
-    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+  // Chunk c + 2 is requested while chunk c runs: operands into the buffer chunk c - 1 used, U into the
+  // registers chunk c's has left. The counted wait leaves those of chunk c + 1 in flight (the read-outs'
+  // stores come after them, so it waits for a few of them at most).
+  int buf = 0, buf2 = 2;
+  auto chunk = [&](int c, f32x4_t (&U)[2]) {
+    if (c + 1 < sp.chunks) {
+      if (LESS == 0 || w < LESS) asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" ::"i"(NDMA + 2) : "memory");
+      else asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" ::"i"(NDMA + 1) : "memory");
+    } else {
+      asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+    }
     __builtin_amdgcn_s_barrier();
     asm volatile("" ::: "memory");
-    // U has arrived here, not at its first use below (whose wait would also drain the next chunk's DMA)
+    const unsigned char* p = smem + buf * NP * 1024 + lane * 16;
+    // operands are read a whole group ahead of their products; pin() is where the wait for a group goes
+    auto fetch = [&](auto& r, int first) {
 #pragma unroll
-    for (int n = 0; n < NC; ++n)
+      for (int i = 0; i < (int)(sizeof(r) / sizeof(r[0])); ++i) r[i] = *reinterpret_cast<const u32x4_t*>(p + (first + i) * 1024);
+    };
+    auto pin = [](auto& r) {
 #pragma unroll
-      for (int m = 0; m < 2; ++m) asm volatile("" : "+v"(U[n][m]));
-    if (c) finish(c - 1);
-    if (c + 1 < sp.chunks) stage(c + 1, (c + 1) & 1);
-    load_gate(c);
-    const unsigned char* p = smem + (c & 1) * NP * 1024 + lane * 16;
-    auto piece = [&](int i) { return *reinterpret_cast<const u32x4_t*>(p + i * 1024); };
-    u32x4_t sh[NC][KF], sl[NC][KF];
+      for (int i = 0; i < (int)(sizeof(r) / sizeof(r[0])); ++i) asm volatile("" : "+v"(r[i]));
+    };
+    u32x4_t wf[4 * KF], qf[4 * KF], kf_[4 * KF], pf[4];
+    f32x4_t ef[MT];
+    fetch(wf, PC::W);
+    fetch(qf, PC::Q);
+    float u[8];
 #pragma unroll
-    for (int n = 0; n < NC; ++n)
+    for (int j = 0; j < 8; ++j) u[j] = U[j >> 2][j & 3];
 #pragma unroll
-      for (int kf = 0; kf < KF; ++kf) {
-        float f[8];
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          f[j] = S[n][2 * kf][j];
-          f[4 + j] = S[n][2 * kf + 1][j];
-        }
-        split_pair(f, sh[n][kf], sl[n][kf]);
-      }
-    f32x4_t V[NC][2];
-#pragma unroll
-    for (int m = 0; m < 2; ++m) {
-#pragma unroll
-      for (int n = 0; n < NC; ++n) V[n][m] = O[n][m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int kf = 0; kf < KF; ++kf) {
-        const u32x4_t wh = piece(PC::W + m * KF + kf), wl = piece(PC::W + (2 + m) * KF + kf);
-        const u32x4_t qh = piece(PC::Q + m * KF + kf), ql = piece(PC::Q + (2 + m) * KF + kf);
-#pragma unroll
-        for (int n = 0; n < NC; ++n) {
-          V[n][m] = mfma_pair(wh, wl, sh[n][kf], sl[n][kf], V[n][m]);
-          O[n][m] = mfma_pair(qh, ql, sh[n][kf], sl[n][kf], O[n][m]);
-        }
-      }
+    for (int j = 0; j < 8; ++j) asm volatile("" : "+v"(u[j]));
+    if (c + 2 < sp.chunks) {
+      stage(c + 2, buf2);
+      load_u(c + 2, U);
     }
-    u32x4_t vh[NC], vl[NC];
+    u32x4_t sh[KF], sl[KF];
 #pragma unroll
-    for (int n = 0; n < NC; ++n) {
+    for (int kf = 0; kf < KF; ++kf) {
       float f[8];
 #pragma unroll
-      for (int j = 0; j < 8; ++j) f[j] = U[n][j >> 2][j & 3] - V[n][j >> 2][j & 3];
-      split_pair(f, vh[n], vl[n]);
+      for (int j = 0; j < 4; ++j) {
+        f[j] = S[2 * kf][j];
+        f[4 + j] = S[2 * kf + 1][j];
+      }
+      split_pair(f, sh[kf], sl[kf]);
     }
-    if (c + 1 < sp.chunks) load_u(c + 1);
+    f32x4_t V[2], O[2];
 #pragma unroll
-    for (int m = 0; m < 2; ++m) {
-      const u32x4_t ph = piece(PC::P + m), pl = piece(PC::P + 2 + m);
+    for (int m = 0; m < 2; ++m) V[m] = O[m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    pin(wf);
 #pragma unroll
-      for (int n = 0; n < NC; ++n) O[n][m] = mfma_pair(ph, pl, vh[n], vl[n], O[n][m]);
-    }
+    for (int kf = 0; kf < KF; ++kf)
 #pragma unroll
-    for (int m = 0; m < MT; ++m) {
-      const u32x4_t kh = piece(PC::K + m), kl = piece(PC::K + MT + m);
-      const f32x4_t e = *reinterpret_cast<const f32x4_t*>(smem + ((c & 1) * NP + PC::E) * 1024 + (m * 16 + q4 * 4) * 4);
-#pragma unroll
-      for (int n = 0; n < NC; ++n) S[n][m] = mfma_pair(kh, kl, vh[n], vl[n], S[n][m] * e);
-    }
-    float* ss = s_ss + ((c & 1) * NW + w) * C;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      float x = 0.f;
-#pragma unroll
-      for (int n = 0; n < NC; ++n) x = fmaf(O[n][e >> 2][e & 3], O[n][e >> 2][e & 3], x);
-      x = group_sum<16>(x);
-      if (l16 == 0) ss[(e >> 2) * 16 + q4 * 4 + (e & 3)] = x;
-    }
-  }
-  __syncthreads();
-  finish(sp.chunks - 1);
-#pragma unroll
-  for (int n = 0; n < NC; ++n)
+      for (int m = 0; m < 2; ++m) V[m] = mfma_pair(wf[m * KF + kf], wf[(2 + m) * KF + kf], sh[kf], sl[kf], V[m]);
+    fetch(kf_, PC::K);
+    fetch(pf, PC::P);
 #pragma unroll
     for (int m = 0; m < MT; ++m)
+      ef[m] = *reinterpret_cast<const f32x4_t*>(smem + (buf * NP + PC::E) * 1024 + (m * 16 + q4 * 4) * 4);
+    pin(qf);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) st[(size_t)(m * 16 + q4 * 4 + r) * DV + n * 16] = S[n][m][r];
+    for (int kf = 0; kf < KF; ++kf)
+#pragma unroll
+      for (int m = 0; m < 2; ++m) O[m] = mfma_pair(qf[m * KF + kf], qf[(2 + m) * KF + kf], sh[kf], sl[kf], O[m]);
+    u32x4_t vh, vl;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) u[j] -= V[j >> 2][j & 3];
+    split_pair(u, vh, vl);
+    pin(kf_);
+    pin(ef);
+#pragma unroll
+    for (int m = 0; m < MT; ++m) S[m] = mfma_pair(kf_[m], kf_[MT + m], vh, vl, S[m] * ef[m]);
+#pragma unroll
+    for (int m = 0; m < 2; ++m) {
+      O[m] = mfma_pair(pf[m], pf[2 + m], vh, vl, O[m]);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = c * C + m * 16 + q4 * 4 + r;
+        if (t < sp.n && v < a.vdim) op[(size_t)t * ldo] = O[m][r];
+      }
+    }
+    buf = buf == 2 ? 0 : buf + 1;
+    buf2 = buf2 == 2 ? 0 : buf2 + 1;
+  };
+  stage(0, 0);
+  load_u(0, U0);
+  if (sp.chunks > 1) {
+    stage(1, 1);
+    load_u(1, U1);
+  }
+  for (int c = 0; c < sp.chunks; c += 2) {
+    chunk(c, U0);
+    if (c + 1 < sp.chunks) chunk(c + 1, U1);
+  }
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) st[(size_t)(m * 16 + q4 * 4 + r) * DV] = S[m][r];
+}
+
+// Read-outs -> RMS norm over the head's value channels, weight, output gate. One workgroup per (chunk, head), 16
+// lanes per row.
+__global__ __launch_bounds__(256) void delta_norm_kernel(DeltaArgs a, const DeltaChunk* __restrict__ chunks,
+                                                         const float* __restrict__ o32) {
+  const DeltaChunk ck = chunks[blockIdx.x];
+  const int h = blockIdx.y, l16 = threadIdx.x & 15;
+  for (int t = threadIdx.x >> 4; t < ck.n; t += 16) {
+    const size_t row = ck.row0 + t;
+    const float* o = o32 + (row * a.heads + h) * a.vdim;
+    const bf16_raw* g = (const bf16_raw*)a.gate + row * a.ldg + h * a.vdim;
+    bf16_raw* out = (bf16_raw*)a.out + row * a.ldo + h * a.vdim;
+    float x[8], ss = 0.f;  // vdim <= 128
+    if (a.vdim == 128 && !((a.ldg | a.ldo) & 7) && !(((uintptr_t)a.gate | (uintptr_t)a.out) & 15)) {
+      *reinterpret_cast<f32x4_t*>(x) = *reinterpret_cast<const f32x4_t*>(o + l16 * 8);
+      *reinterpret_cast<f32x4_t*>(x + 4) = *reinterpret_cast<const f32x4_t*>(o + l16 * 8 + 4);
+      float z[8];
+      unpack8(ld16(g + l16 * 8), z);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss = fmaf(x[j], x[j], ss);
+      const float rs = 1.f / sqrtf(group_sum<16>(ss) / 128.f + a.eps);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] *= rs * a.norm[l16 * 8 + j] * sigmoid(z[j]);
+      st16(out + l16 * 8, pack8(x));
+      continue;
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const int d = j * 16 + l16;
+      x[j] = d < a.vdim ? o[d] : 0.f;
+      ss = fmaf(x[j], x[j], ss);
+    }
+    const float rs = 1.f / sqrtf(group_sum<16>(ss) / (float)a.vdim + a.eps);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const int d = j * 16 + l16;
+      if (d < a.vdim) out[d] = f2bf(x[j] * rs * a.norm[d] * sigmoid(bf2f(g[d])));
+    }
+  }
 }
 
 }  // namespace
@@ -480,21 +494,28 @@ extern "C" int lsa_delta_chunk_bytes(int dk, int dv) {
   return (12 * (dk / 32) + 5 + dv / 8) * 1024;
 }
 
-// chunks: n_chunks DeltaChunk; spans: n_spans DeltaSpan over them; ws: n_chunks * heads * lsa_delta_chunk_bytes
+// chunks: n_chunks DeltaChunk; spans: n_spans DeltaSpan over them; ws: n_chunks * heads * lsa_delta_chunk_bytes;
+// o32: [rows][heads * vdim]
 extern "C" int lsa_delta_chunked(const DeltaArgs* a, const void* chunks, int n_chunks, const void* spans, int n_spans,
-                                 void* ws, hipStream_t s) {
-  if (!a || bad_delta(a) || !a->gate || n_chunks < 1 || n_spans < 1 || !chunks || !spans || !ws || (uintptr_t)ws % 16) return LSA_BAD_SHAPE;
-#define LSA_C(K, V, NC)                                                                                                     \
-  if (a->dk == K && a->dv == V) {                                                                                           \
-    delta_chunk_kernel<K, V><<<dim3(n_chunks, a->heads), 256, 0, s>>>(*a, (const DeltaChunk*)chunks, (unsigned char*)ws);   \
-    LSA_CHECK_LAUNCH();                                                                                                     \
-    delta_scan_kernel<K, V, NC><<<dim3(n_spans, a->heads), V / NC * 4, 0, s>>>(*a, (const DeltaSpan*)spans,                 \
-                                                                               (const unsigned char*)ws);                   \
-    LSA_CHECK_LAUNCH();                                                                                                     \
-    return LSA_OK;                                                                                                          \
+                                 void* ws, float* o32, hipStream_t s) {
+  if (!a || bad_delta(a) || !a->gate || n_chunks < 1 || n_spans < 1 || !chunks || !spans || !ws || !o32 || (uintptr_t)ws % 16)
+    return LSA_BAD_SHAPE;
+#define LSA_S(K, V, NW)                                                                                                  \
+  delta_scan_kernel<K, V, NW><<<dim3(n_spans, a->heads, V / (NW * 16)), NW * 64, 0, s>>>(*a, (const DeltaSpan*)spans,     \
+                                                                                       (const unsigned char*)ws, o32)
+#define LSA_C(K, V)                                                                                                       \
+  if (a->dk == K && a->dv == V) {                                                                                         \
+    delta_chunk_kernel<K, V><<<dim3(n_chunks, a->heads), 256, 0, s>>>(*a, (const DeltaChunk*)chunks, (unsigned char*)ws); \
+    LSA_CHECK_LAUNCH();                                                                                                   \
+    LSA_S(K, V, (V == 32 ? 2 : 4));                                                                                       \
+    LSA_CHECK_LAUNCH();                                                                                                   \
+    delta_norm_kernel<<<dim3(n_chunks, a->heads), 256, 0, s>>>(*a, (const DeltaChunk*)chunks, o32);                       \
+    LSA_CHECK_LAUNCH();                                                                                                   \
+    return LSA_OK;                                                                                                        \
   }
-  LSA_C(32, 32, 1) LSA_C(32, 64, 1) LSA_C(32, 128, 2) LSA_C(64, 32, 1) LSA_C(64, 64, 1) LSA_C(64, 128, 2) LSA_C(128, 32, 1)
-  LSA_C(128, 64, 1) LSA_C(128, 128, 1)
+  LSA_C(32, 32) LSA_C(32, 64) LSA_C(32, 128) LSA_C(64, 32) LSA_C(64, 64) LSA_C(64, 128) LSA_C(128, 32) LSA_C(128, 64)
+  LSA_C(128, 128)
 #undef LSA_C
+#undef LSA_S
   return LSA_UNSUPPORTED;
 }

@@ -100,12 +100,15 @@ def chunk_groups(runs: list, most: int) -> list:
         groups.append((torch.tensor(chunks, dtype=torch.int32), torch.tensor(spans, dtype=torch.int32)))
 
 
-def chunked(a: DeltaArgs, chunks, spans, ws, nbytes: int) -> None:
-    """One group of :func:`chunk_groups` of checked runs (tables on the device), bf16."""
+def chunked(a: DeltaArgs, chunks, spans, ws, nbytes: int, o32) -> None:
+    """One group of :func:`chunk_groups` of checked runs (tables on the device), bf16. ``ws``: bytes; ``o32`` fp32
+    [rows, heads vdim]."""
+    _req(o32.dtype == torch.float32 and o32.is_contiguous() and o32.dim() == 2 and o32.shape[1] == a.heads * a.vdim,
+         "delta: read-outs")
     _req(all(t.dtype == torch.int32 and t.is_contiguous() and t.shape[1] == 8 for t in (chunks, spans)), "delta: tables")
     _req(ws.dtype == torch.uint8 and ws.numel() >= chunks.shape[0] * a.heads * nbytes and nbytes > 0, "delta: workspace")
     _check(lib().lsa_delta_chunked(ctypes.byref(a), _p(chunks), chunks.shape[0], _p(spans), spans.shape[0], _p(ws),
-                                   _stream()), "lsa_delta_chunked")
+                                   _p(o32), _stream()), "lsa_delta_chunked")
 
 
 def declare(L: ctypes.CDLL) -> None:
@@ -116,5 +119,5 @@ def declare(L: ctypes.CDLL) -> None:
         "lsa_delta_steps": [i, da, i, i, vp],
         "lsa_delta_ring": [i, da, i, vp],
         "lsa_delta_chunk_bytes": [i, i],
-        "lsa_delta_chunked": [da, vp, i, vp, i, vp, vp],
+        "lsa_delta_chunked": [da, vp, i, vp, i, vp, vp, vp],
     })

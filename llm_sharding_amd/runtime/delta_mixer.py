@@ -83,8 +83,10 @@ class Delta:
         if long is not None:
             a = args(runs=long)
             ws = eng.workspace("delta", max(c.shape[0] for c, _ in groups) * s.heads * self.nbytes)
+            wide = s.heads * s.vdim
+            o32 = eng.workspace("delta_o", 4 * rows * wide).view(torch.float32)[:rows * wide].view(rows, wide)
             for chunks, spans in groups:
-                D.chunked(a, chunks, spans, ws, self.nbytes)
+                D.chunked(a, chunks, spans, ws, self.nbytes, o32)
             D.ring(a, self.dtype, long.shape[0])
         return ao
 

@@ -363,8 +363,9 @@ class DeltaCase:
             nb = D.chunk_bytes(s)
             ws = torch.full((5 * s.heads * nb,), 255, dtype=torch.uint8, device=DEV)
             held = [(c.to(DEV), p.to(DEV)) for c, p in D.chunk_groups(runs, 5)]
+            o32 = torch.full((row, s.heads * s.vdim), float("nan"), device=DEV)
             for c, p in held:
-                D.chunked(a, c, p, ws, nb)
+                D.chunked(a, c, p, ws, nb, o32)
             D.ring(a, self.dtype, len(runs))
         out = out.cpu().float()
         for (i, p), o in zip(pick, out):
