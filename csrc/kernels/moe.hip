@@ -160,18 +160,31 @@ __global__ __launch_bounds__(256) void moe_small_kernel(const MoeTile* __restric
 #pragma unroll
     for (int n = 0; n < NT; ++n) acc[m][n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   const int k1 = KT * (w + 1) / 4;
-#pragma unroll 4
-  for (int kt = KT * w / 4; kt < k1; ++kt) {
-    u32x4_t b[NT], x[MT];
+  // the next step's operands are requested before this one's products
+  auto load = [&](int kt, u32x4_t (&b)[NT], u32x4_t (&x)[MT]) {
 #pragma unroll
     for (int n = 0; n < NT; ++n) b[n] = ld16(wp + ((size_t)min(n, ntn - 1) * KT + kt) * 512);
 #pragma unroll
     for (int m = 0; m < MT; ++m) x[m] = ld16(ar[m] + kt * 32);
+  };
+  auto mul = [&](const u32x4_t (&b)[NT], const u32x4_t (&x)[MT]) {
 #pragma unroll
     for (int m = 0; m < MT; ++m)
 #pragma unroll
       for (int n = 0; n < NT; ++n) acc[m][n] = mfma16(x[m], b[n], acc[m][n]);
+  };
+  u32x4_t b0[NT], x0[MT], b1[NT], x1[MT];
+  int kt = KT * w / 4;
+  if (kt < k1) load(kt, b0, x0);
+  for (; kt + 2 < k1; kt += 2) {
+    load(kt + 1, b1, x1);
+    mul(b0, x0);
+    load(kt + 2, b0, x0);
+    mul(b1, x1);
   }
+  if (kt + 1 < k1) load(kt + 1, b1, x1);
+  if (kt < k1) mul(b0, x0);
+  if (kt + 1 < k1) mul(b1, x1);
 #pragma unroll
   for (int m = 0; m < MT; ++m)
 #pragma unroll

@@ -202,11 +202,11 @@ LSA_DEVICE void join_at(const JoinArgs& a, int row, int c, float* x) {
   }
 }
 
-// NV > 0: rows of up to 1024 NV values in registers, four at a time; 0: any width
-template <typename T, int NV>
-__global__ __launch_bounds__(256) void join_kernel(JoinArgs a, int W, float* __restrict__ x, int ldx, T* __restrict__ xc,
+// NT threads per row. NV > 0: rows of up to 4 NT NV values in registers, four at a time; 0: any width
+template <typename T, int NV, int NT>
+__global__ __launch_bounds__(NT) void join_kernel(JoinArgs a, int W, float* __restrict__ x, int ldx, T* __restrict__ xc,
                                                    int ldc) {
-  __shared__ float s_part[4];
+  __shared__ float s_part[NT / 64];
   const int row = blockIdx.x, tid = threadIdx.x;
   float* xr = x + (size_t)row * ldx;
   float s = 0.f;
@@ -214,7 +214,7 @@ __global__ __launch_bounds__(256) void join_kernel(JoinArgs a, int W, float* __r
   if constexpr (NV > 0) {
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
-      const int c = (tid + j * 256) * 4;
+      const int c = (tid + j * NT) * 4;
       v[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
       if (c >= W) continue;
       float f[4];
@@ -228,7 +228,7 @@ __global__ __launch_bounds__(256) void join_kernel(JoinArgs a, int W, float* __r
       for (int k = 0; k < 4; ++k) s += f[k] * f[k];
     }
   } else {
-    for (int c = tid; c < W; c += 256) {
+    for (int c = tid; c < W; c += NT) {
       float f = xr[c];
       join_at<T, 1>(a, row, c, &f);
       xr[c] = f;
@@ -239,16 +239,19 @@ __global__ __launch_bounds__(256) void join_kernel(JoinArgs a, int W, float* __r
   s = wave_sum(s);
   if ((tid & 63) == 0) s_part[tid >> 6] = s;
   __syncthreads();
-  const float rs = 1.f / sqrtf((s_part[0] + s_part[1] + s_part[2] + s_part[3]) / (float)W + a.eps);
+  float sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < NT / 64; ++i) sum += s_part[i];
+  const float rs = 1.f / sqrtf(sum / (float)W + a.eps);
   T* cr = xc + (size_t)row * ldc;
   if constexpr (NV > 0) {
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
-      const int c = (tid + j * 256) * 4;
+      const int c = (tid + j * NT) * 4;
       if (c < W) st4(cr + c, v[j] * rs * *reinterpret_cast<const f32x4_t*>(a.gain + c));
     }
   } else {
-    for (int c = tid; c < W; c += 256) st1(cr + c, xr[c] * rs * a.gain[c]);  // this thread's own stores
+    for (int c = tid; c < W; c += NT) st1(cr + c, xr[c] * rs * a.gain[c]);  // this thread's own stores
   }
 }
 
@@ -258,11 +261,15 @@ void launch_join(const JoinArgs& a, int rows, int W, float* x, int ldx, T* xc, i
                    !(((uintptr_t)x | (uintptr_t)xc | (uintptr_t)a.y1 | (uintptr_t)a.g1 | (uintptr_t)a.g2 |
                       (uintptr_t)a.y2 | (uintptr_t)a.ye | (uintptr_t)a.gain) % 16);
   const int nv = vec ? (W + 1023) / 1024 : 0;
-#define LSA_J(NV) join_kernel<T, NV><<<rows, 256, 0, s>>>(a, W, x, ldx, xc, ldc)
-  if (nv >= 1 && nv <= 2) LSA_J(2);
-  else if (nv >= 3 && nv <= 4) LSA_J(4);
-  else if (nv >= 5 && nv <= 8) LSA_J(8);
-  else LSA_J(0);
+#define LSA_J(NV, NT) join_kernel<T, NV, NT><<<rows, NT, 0, s>>>(a, W, x, ldx, xc, ldc)
+  if (nv >= 1 && nv <= 8 && rows <= 256) {  // few rows: their latency counts
+    if (nv == 1) LSA_J(1, 256);
+    else if (nv <= 4) LSA_J(1, 1024);
+    else LSA_J(2, 1024);
+  } else if (nv >= 1 && nv <= 2) LSA_J(2, 256);
+  else if (nv >= 3 && nv <= 4) LSA_J(4, 256);
+  else if (nv >= 5 && nv <= 8) LSA_J(8, 256);
+  else LSA_J(0, 256);
 #undef LSA_J
 }
 

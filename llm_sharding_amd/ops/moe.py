@@ -70,7 +70,7 @@ def group(expert, pairs: int, experts: int, rows: int, order, place, tiles) -> i
 def route_group(logits, rows: int, experts: int, top: int, tile: int, expert, weight, order, place, tiles) -> int:
     """:func:`route` and :func:`group`, in one launch where there are few rows."""
     pairs = rows * top
-    if rows > 64 or experts > 256:
+    if rows > 16 or experts > 256:
         route(logits, rows, experts, top, expert, weight)
         return group(expert, pairs, experts, tile, order, place, tiles)
     n = max_tiles(pairs, experts, tile)
