@@ -90,14 +90,15 @@ class Attention:
         return host.to(plan.eng.device)
 
     def key_splits(self, eng, entries: int, longest: int) -> int:
-        """Splits of a row's keys: about two workgroups per CU, four pages each at least."""
+        """Splits of a row's keys: about one workgroup per CU, four pages each at least, at most 16 (the merge
+        reads one partial sum per split)."""
         from ..ops import hip
         from ..ops import paged_attn as A
         s = self.spec
         seen = longest if not s.window else min(longest, s.window + 64 + -(-s.keep_first // 64) * 64)
-        want = 2 * hip.N_CU // max(1, entries * A.head_tiles(s))
+        want = hip.N_CU // max(1, entries * A.head_tiles(s))
         cap = eng.part_o.numel() // max(1, entries * s.heads * s.dvp)
-        return int(max(1, min(want, cap, -(-seen // (4 * A.PAGE)))))
+        return int(max(1, min(16, want, cap, -(-seen // (4 * A.PAGE)))))
 
     # ------------------------------------------------------------------ CPU
     def forward_torch(self, eng, x, cache: tuple, state, slot, pos) -> torch.Tensor:
