@@ -39,6 +39,8 @@ FAMILIES = {
                "linear_f32.hip", "stream_ops.hip", "paged_attn", "delta", "moe"),
     "looped": ("elementwise.hip", "gemm_sk.hip", "gemv.hip", "gemv_coop.hip-0", "gemv_coop.hip-4", "gemv_coop.hip-7",
                "linear_f32.hip", "stream_ops.hip", "paged_attn", "retention", "moe"),
+    "streams": ("elementwise.hip", "gemm_sk.hip", "gemv.hip", "gemv_coop.hip-0", "gemv_coop.hip-2", "gemv_coop.hip-4",
+                "gemv_coop.hip-7", "linear_f32.hip", "stream_ops.hip", "stream_mix.hip", "latent", "mlstm", "moe"),
 }
 
 

@@ -6,7 +6,7 @@
 //               columns to either; or out32 += sigmoid(gate) * y (a result joins an fp32 stream)
 //   EPI_RESID   out = resid + y (+ bias)        (o_proj / down_proj + residual add)
 //   EPI_SWIGLU  out = silu(gate) * up           (gate/up fused GEMM, tiles interleaved), or the
-//               clipped GLU of glu() when glu_limit > 0
+//               clipped GLU of glu() when glu_limit > 0, or gelu(gate) * up with act 1
 //   EPI_QKV     half-split RoPE on q/k + direct write of k/v into the static KV cache
 //               (replaces apply_rotary_pos_emb + DynamicCache.update's torch.cat); with
 //               cos_t == nullptr (GPT-2: learned absolute positions) no rotation and the
@@ -41,7 +41,7 @@ struct EpiArgs {
   int head_dim;
   int t_max;
   int col_offset;           // ARGMAX: vocabulary index of column 0 (vocab-parallel chunks)
-  int act;                  // STORE: 0 identity, 1 gelu (tanh form, GPT-2 "gelu_new"), 2 relu squared
+  int act;                  // STORE: 0 identity, 1 gelu (tanh form, GPT-2 "gelu_new"), 2 relu squared; SWIGLU: 1 gelu
   // fused RMSNorm across GEMMs (gemm_sk only; layout [M][ss_n] fp32, one partial sum of squares
   // per 64 columns of the residual stream): RESID writes the partials of its rounded outputs to
   // ss_out; QKV / SWIGLU scale row m by rsqrt(sum(ss_in[m][:]) / (64 ss_n) + ss_eps) first
@@ -75,20 +75,20 @@ static inline bool bad_store(const EpiArgs& e, int N) {
 
 LSA_DEVICE float silu(float g) { return g / (1.0f + __expf(-g)); }
 
-// The gated unit of an EPI_SWIGLU GEMM: silu(g) * u, or with glu_limit L > 0 the clipped unit
+// 0.5 x (1 + tanh(sqrt(2/pi) (x + 0.044715 x^3))), tanh(u) = 1 - 2 / (exp(2u) + 1)
+LSA_DEVICE float gelu_tanh(float x) {
+  const float u = 0.7978845608028654f * (x + 0.044715f * x * x * x);
+  return 0.5f * x * (2.0f - 2.0f / (__expf(2.0f * u) + 1.0f));
+}
+
+// The gated unit of an EPI_SWIGLU GEMM: silu(g) * u, with act 1 gelu(g) * u, or with glu_limit L > 0 the clipped unit
 //   g' = min(g, L), u' = clamp(u, -L, L):  g' * sigmoid(alpha * g') * (u' + shift)
 LSA_DEVICE float glu(const EpiArgs& ep, float g, float u) {
   if (ep.glu_limit > 0.f) {
     const float gc = fminf(g, ep.glu_limit), uc = fminf(fmaxf(u, -ep.glu_limit), ep.glu_limit);
     return gc / (1.0f + __expf(-ep.glu_alpha * gc)) * (uc + ep.glu_shift);
   }
-  return silu(g) * u;
-}
-
-// 0.5 x (1 + tanh(sqrt(2/pi) (x + 0.044715 x^3))), tanh(u) = 1 - 2 / (exp(2u) + 1)
-LSA_DEVICE float gelu_tanh(float x) {
-  const float u = 0.7978845608028654f * (x + 0.044715f * x * x * x);
-  return 0.5f * x * (2.0f - 2.0f / (__expf(2.0f * u) + 1.0f));
+  return (ep.act ? gelu_tanh(g) : silu(g)) * u;
 }
 
 // activation of an EPI_STORE product (act 1 or 2)

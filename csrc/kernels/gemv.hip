@@ -181,8 +181,8 @@ __global__ __launch_bounds__(NW * 64) void gemv_packed_kernel(
       const int tp = e / (MR * 16), mm = (e >> 4) % MR, n = e & 15;
       if (mm >= M) continue;
       const float r = rstd(mm);
-      const float g = rsum(2 * tp, mm, n) * r, u = rsum(2 * tp + 1, mm, n) * r;
-      const int col = (nt0 / 2 + tp) * 16 + n;
+      const int col = (nt0 / 2 + tp) * 16 + n, gc = (nt0 + 2 * tp) * 16 + n;
+      const float g = rsum(2 * tp, mm, n) * r + epi_bias(ep, gc), u = rsum(2 * tp + 1, mm, n) * r + epi_bias(ep, gc + 16);
       ep.out[(size_t)mm * ep.ldo + col] = f2bf(glu(ep, g, u));
     }
   } else {

@@ -489,6 +489,8 @@ __global__ __launch_bounds__(NW * KW * 64) void gemv_coop_kernel(
       float gg[16], uu[16];
       load16(2 * tp, mm, r, gg);
       load16(2 * tp + 1, mm, r, uu);
+      epi_bias16(ep, (ntg0 + 2 * tp) * 16, gg);
+      epi_bias16(ep, (ntg0 + 2 * tp + 1) * 16, uu);
 #pragma unroll
       for (int j = 0; j < 16; ++j) gg[j] = glu(ep, gg[j], uu[j]);
       bf16_raw* o = ep.out + (size_t)mm * ep.ldo + (ntg0 / 2 + tp) * 16;

@@ -8,6 +8,9 @@
 //             (decode and short portions; latent.hip, latent_decode.hip)
 //   expanded  keys and values of the visible tokens are multiplied out once per portion and an
 //             ordinary flash attention runs over them (long portions; latent_prefill.hip)
+//
+// A row sees all keys up to its own or the last ``window`` of them; with ``sink`` the denominator has one
+// more term per head, which belongs to no key.
 #pragma once
 #include "elem.h"
 
@@ -22,8 +25,10 @@ struct LatentArgs {
   const int* index;    // optional: entry i of the launch is row index[i]
   const float* cos_t;  // [max_pages * LAT_PAGE][rot_dims / 2]
   const float* sin_t;
+  const float* sink;   // [heads] log2 of a term in the softmax's denominator, null: none
   int max_pages;
   int n_pages;
+  int window;             // keys a row sees, its own among them (0: all)
   int heads;
   int dim, rot_dim, rot_dims, vdim, kv_rank, q_rank;  // the model's sizes (rot_dims <= rot_dim)
   int dkp, rp, dvp, krp;  // padded: unrotated / rotated query part, value, latent (zeros behind)
@@ -44,6 +49,14 @@ LSA_DEVICE int lat_keys(const LatentArgs& a, int row) {
 LSA_DEVICE int lat_page(const LatentArgs& a, int slot, int b) {
   const int pg = a.table[(size_t)slot * a.max_pages + b];
   return pg < 0 || pg >= a.n_pages ? 0 : pg;
+}
+
+// first key of a row that sees ``len`` keys without a window
+LSA_DEVICE int lat_first(const LatentArgs& a, int len) { return a.window > 0 && len > a.window ? len - a.window : 0; }
+
+// the sink's part of a denominator whose terms are 2^(score - m) (m finite: of a row that sees a key)
+LSA_DEVICE float lat_sink(const LatentArgs& a, int head, float m) {
+  return a.sink ? __builtin_amdgcn_exp2f(a.sink[head] - m) : 0.f;
 }
 
 // entry i of a rotated vector v (rot_dim values) at position p

@@ -157,8 +157,9 @@ __global__ __launch_bounds__(256) void attend_kernel(LatentArgs a, const T* __re
   float* part = sp + 256;
   const int e = blockIdx.x, h = blockIdx.y, s = blockIdx.z, row = a.index ? a.index[e] : e;
   const size_t out = ((size_t)e * a.heads + h) * ns + s;
-  const int len = lat_keys(a, row), nb = (len + LAT_PAGE - 1) / LAT_PAGE, slot = a.slot[row];
-  const int k0 = nb * s / ns * LAT_PAGE, k1 = min(len, nb * (s + 1) / ns * LAT_PAGE);
+  const int len = lat_keys(a, row), first = lat_first(a, len), slot = a.slot[row];
+  const int fb = first / LAT_PAGE, nb = (len + LAT_PAGE - 1) / LAT_PAGE - fb;
+  const int k0 = max(first, (fb + nb * s / ns) * LAT_PAGE), k1 = min(len, (fb + nb * (s + 1) / ns) * LAT_PAGE);
   const T* qh = qt + ((size_t)e * a.heads + h) * cw;
   const float sl2 = a.scale * 1.4426950408889634f;
   for (int c = tid; c < cw; c += 256) sq[c] = ld1(qh + c) * sl2;
@@ -210,6 +211,7 @@ __global__ __launch_bounds__(256) void value_kernel(LatentArgs a, const float* _
   for (int s = 0; s < ns; ++s) M = fmaxf(M, pm[(b + s) * 2]);
   if (M == -INFINITY) M = 0.f;
   for (int s = 0; s < ns; ++s) L += pm[(b + s) * 2 + 1] * __builtin_amdgcn_exp2f(pm[(b + s) * 2] - M);
+  L += lat_sink(a, h, M);
   const float inv = L > 0.f ? 1.f / L : 0.f;
   for (int d = threadIdx.x; d < a.krp; d += 256) {
     float o = 0.f;
@@ -238,7 +240,7 @@ __global__ __launch_bounds__(256) void gather_kernel(LatentArgs a, const int* __
 }
 
 bool args_ok(const LatentArgs* a, int n) {
-  return a && n >= 1 && a->cache && a->table && a->slot && a->pos && a->max_pages >= 1 && a->n_pages >= 1 && a->heads >= 1 &&
+  return a && n >= 1 && a->window >= 0 && a->cache && a->table && a->slot && a->pos && a->max_pages >= 1 && a->n_pages >= 1 && a->heads >= 1 &&
          a->dim >= 1 && a->dim <= a->dkp && a->rot_dim >= 2 && a->rot_dim <= a->rp && a->rot_dims >= 2 &&
          a->rot_dims % 2 == 0 && a->rot_dims <= a->rot_dim && a->vdim >= 1 && a->vdim <= a->dvp && a->kv_rank >= 1 &&
          a->kv_rank <= a->krp && a->q_rank >= 1 && a->cos_t && a->sin_t && a->dkp % 64 == 0 && a->rp % 64 == 0 &&

@@ -63,7 +63,8 @@ __global__ __launch_bounds__((attend_waves<KRP, HT>() * 64), (attend_waves<KRP, 
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6), kg = w & 3, t0 = (w >> 2) * QT;
   const int slot = __builtin_amdgcn_readfirstlane(a.slot[row]);
   const int len = __builtin_amdgcn_readfirstlane(lat_keys(a, row));
-  const int nb = (len + LAT_PAGE - 1) / LAT_PAGE, b0 = nb * sp / ns, b1 = nb * (sp + 1) / ns;
+  const int first = lat_first(a, len), fb = first / LAT_PAGE, nb = (len + LAT_PAGE - 1) / LAT_PAGE - fb;
+  const int b0 = fb + nb * sp / ns, b1 = fb + nb * (sp + 1) / ns;
   const bf16_raw* cache = static_cast<const bf16_raw*>(a.cache);
   const float sl2 = a.scale * 1.4426950408889634f;
 
@@ -147,7 +148,7 @@ __global__ __launch_bounds__((attend_waves<KRP, HT>() * 64), (attend_waves<KRP, 
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int key = b * LAT_PAGE + kg * 16 + g * 4 + r;
-        const float v = key < len ? (s[t][r] + s2[t][r]) * sl2 : -INFINITY;
+        const float v = key < len && key >= first ? (s[t][r] + s2[t][r]) * sl2 : -INFINITY;
         s[t][r] = v;
         mx = fmaxf(mx, v);
       }
@@ -321,7 +322,7 @@ __global__ __launch_bounds__(512) void value_mfma_kernel(LatentArgs a, int n, co
       const float m = lane < ns ? p[2 * lane] : -INFINITY, l = lane < ns ? p[2 * lane + 1] : 0.f;
       float M = wave_max(m);
       if (M == -INFINITY) M = 0.f;
-      const float f = __builtin_amdgcn_exp2f(m - M), L = wave_sum(l * f);
+      const float f = __builtin_amdgcn_exp2f(m - M), L = wave_sum(l * f) + lat_sink(a, h, M);
       wgt[r][lane] = L > 0.f ? f / L : 0.f;
     }
   }
@@ -333,7 +334,7 @@ __global__ __launch_bounds__(512) void value_mfma_kernel(LatentArgs a, int n, co
       const size_t b = ((size_t)e * a.heads + h) * ns;
       const float* p = po + b * KRP + c;
       if (ns == 1) {
-        const float L = pm[b * 2 + 1];
+        const float m = pm[b * 2], L = pm[b * 2 + 1] + (m == -INFINITY ? 0.f : lat_sink(a, h, m));
         v = *reinterpret_cast<const f32x4_t*>(p) * (L > 0.f ? 1.f / L : 0.f);
       } else {
         int s = 0;
@@ -366,7 +367,7 @@ __global__ __launch_bounds__(512) void value_mfma_kernel(LatentArgs a, int n, co
 }
 
 bool size_ok(const LatentArgs* a, int n) {
-  return a && n >= 1 && a->cache && a->table && a->slot && a->pos && a->max_pages >= 1 && a->n_pages >= 1 && a->heads >= 1 &&
+  return a && n >= 1 && a->window >= 0 && a->cache && a->table && a->slot && a->pos && a->max_pages >= 1 && a->n_pages >= 1 && a->heads >= 1 &&
          a->dim >= 1 && a->dim <= a->dkp && a->dkp % 64 == 0 && a->rp == RP && a->rot_dim >= 2 && a->rot_dim <= RP &&
          a->rot_dims >= 2 && a->rot_dims % 2 == 0 && a->rot_dims <= a->rot_dim && a->vdim >= 1 && a->vdim <= a->dvp &&
          a->dvp % 64 == 0 && a->kv_rank >= 1 && a->kv_rank <= a->krp && a->cos_t && a->sin_t &&

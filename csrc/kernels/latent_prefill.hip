@@ -14,8 +14,9 @@ namespace {
 
 constexpr int BKV = 64, NWV = 8, NTHR = NWV * 64, NBUF = 2, RP = 64;
 
-struct LatTile {  // as PrefillTile: kv0 = first gathered row of the sequence (its position 0)
-  int row0, nrows, kv0, pos0, kvlen, pad0, pad1, pad2;
+// as PrefillTile: kv0 = first gathered row of the sequence, of position ``base``; kvlen counts from there
+struct LatTile {
+  int row0, nrows, kv0, pos0, kvlen, base, pad1, pad2;
 };
 
 typedef short v4s_t __attribute__((ext_vector_type(4)));
@@ -62,7 +63,7 @@ __global__ __launch_bounds__(NTHR, 4) void latent_prefill_kernel(LatentArgs a, c
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int my_row = w * 16 + l16;
   const bool row_ok = my_row < tile.nrows;
-  const int my_pos = tile.pos0 + my_row;
+  const int rel0 = tile.pos0 - tile.base, my_pos = rel0 + my_row;  // positions among the gathered rows
 
   u32x4_t qf[KF];
   {
@@ -85,10 +86,14 @@ __global__ __launch_bounds__(NTHR, 4) void latent_prefill_kernel(LatentArgs a, c
 #pragma unroll
     for (int kf = 0; kf < KF; ++kf) asm volatile("" : "+v"(qf[kf]));
   }
-  const int lim = min(tile.pos0 + tile.nrows, tile.kvlen);
+  const int lim = min(rel0 + tile.nrows, tile.kvlen);
   const int my_lim = min(my_pos + 1, tile.kvlen);
-  const int wave_lim = min(tile.pos0 + min(w * 16 + 16, tile.nrows), tile.kvlen);
-  const int wave_min_lim = min(tile.pos0 + w * 16 + 1, tile.kvlen);
+  const int wave_lim = min(rel0 + min(w * 16 + 16, tile.nrows), tile.kvlen);
+  const int wave_min_lim = min(rel0 + w * 16 + 1, tile.kvlen);
+  // first visible key: of this lane's row, of the wave's first and last row, of the tile
+  const int win = a.window > 0 ? a.window : 0x3fffffff;
+  const int my_first = my_pos + 1 - win, wave_first = rel0 + w * 16 + 1 - win, wave_max_first = wave_first + 15;
+  const int kb_first = max(0, rel0 + 1 - win) / BKV;
   const int nkb = (lim + BKV - 1) / BKV;
   const int cw = a.krp + RP;
   const bf16_raw* kvb = kv + (size_t)tile.kv0 * ldkv + (size_t)head * (DK + DV);
@@ -123,13 +128,13 @@ __global__ __launch_bounds__(NTHR, 4) void latent_prefill_kernel(LatentArgs a, c
 #pragma unroll
   for (int d = 0; d < DT; ++d) v_off[d] = sw_off<NCV>(key_lo, 2 * d + ((l16 & 3) >> 1)) + 8 * (l16 & 1);
 
-  if (nkb > 0) stage(0, 0);
-  for (int kb = 0; kb < nkb; ++kb) {
+  if (nkb > kb_first) stage(kb_first, kb_first & 1);
+  for (int kb = kb_first; kb < nkb; ++kb) {
     asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
     __builtin_amdgcn_s_barrier();
     asm volatile("" ::: "memory");
     if (kb + 1 < nkb) stage(kb + 1, (kb + 1) & 1);
-    if (kb * BKV >= wave_lim) continue;
+    if (kb * BKV >= wave_lim || (kb + 1) * BKV <= wave_first) continue;
     const unsigned char* ks = smem + (kb & 1) * (KBLK + VBLK);
     const unsigned char* vs = ks + KBLK;
     f32x4_t s[4];
@@ -143,7 +148,7 @@ __global__ __launch_bounds__(NTHR, 4) void latent_prefill_kernel(LatentArgs a, c
       }
     }
     float mx = -INFINITY;
-    if ((kb + 1) * BKV <= wave_min_lim) {
+    if ((kb + 1) * BKV <= wave_min_lim && kb * BKV >= wave_max_first) {
 #pragma unroll
       for (int kt = 0; kt < 4; ++kt)
 #pragma unroll
@@ -157,7 +162,7 @@ __global__ __launch_bounds__(NTHR, 4) void latent_prefill_kernel(LatentArgs a, c
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int key = kb * BKV + kt * 16 + g * 4 + r;
-          const float v = key < my_lim ? s[kt][r] * sl2 : -INFINITY;
+          const float v = key < my_lim && key >= my_first ? s[kt][r] * sl2 : -INFINITY;
           s[kt][r] = v;
           mx = fmaxf(mx, v);
         }
@@ -210,6 +215,7 @@ __global__ __launch_bounds__(NTHR, 4) void latent_prefill_kernel(LatentArgs a, c
   l_run += __shfl_xor(l_run, 16, 64);
   l_run += __shfl_xor(l_run, 32, 64);
   if (!row_ok) return;
+  if (m_run > -INFINITY) l_run += lat_sink(a, head, m_run);
   const float inv = l_run > 0.f ? 1.f / l_run : 0.f;
   const size_t row = tile.row0 + my_row;
   const bf16_raw* gr = gate ? gate + row * ldg + (size_t)head * DV : nullptr;
@@ -230,11 +236,11 @@ __global__ __launch_bounds__(NTHR, 4) void latent_prefill_kernel(LatentArgs a, c
 
 }  // namespace
 
-// tiles: n_tiles LatTile {row0, nrows <= 128, kv0, pos0, kvlen, pad x3} with kv0 + kvlen inside kv and lat
+// tiles: n_tiles LatTile {row0, nrows <= 128, kv0, pos0, kvlen, base, pad x2} with kv0 + kvlen inside kv and lat
 extern "C" int lsa_latent_prefill(const LatentArgs* a, const void* tiles, int n_tiles, const void* q, int ldq,
                                   const void* kv, int ldkv, const void* lat, const void* gate, int ldg, void* out,
                                   int ldo, hipStream_t s) {
-  if (!a || n_tiles < 1 || a->heads < 1 || a->rp != RP || a->rot_dim < 2 || a->rot_dim > RP || a->rot_dims < 2 ||
+  if (!a || n_tiles < 1 || a->window < 0 || a->heads < 1 || a->rp != RP || a->rot_dim < 2 || a->rot_dim > RP || a->rot_dims < 2 ||
       a->rot_dims % 2 || a->rot_dims > a->rot_dim || !a->cos_t || !a->sin_t || a->krp % 64)
     return LSA_BAD_SHAPE;
   if (ldq < a->heads * (a->dkp + RP) || ldq % 8 || ldkv < a->heads * (a->dkp + a->dvp) || ldkv % 8 ||

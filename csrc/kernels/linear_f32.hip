@@ -68,7 +68,10 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict
 #pragma unroll
       for (int p = 0; p < 2; ++p) {
         const int c = n0 + 32 * p;
-        if (c < N) ep.out32[(size_t)m * ep.ldo + c / 2 + tx] = glu(ep, acc[i][2 * p], acc[i][2 * p + 1]);
+        if (c >= N) continue;
+        const int n = c + tx;
+        ep.out32[(size_t)m * ep.ldo + c / 2 + tx] =
+            glu(ep, acc[i][2 * p] + epi_bias(ep, n), acc[i][2 * p + 1] + epi_bias(ep, n + 16));
       }
     } else {
 #pragma unroll

@@ -11,6 +11,7 @@
 //
 // The products run on MFMA with every fp32 operand (rotated q and k, weights, state) as a pair of bf16, its rounding
 // and the rounding of what that leaves; v is bf16 already. No exponent of a decay is negative.
+#include "mfma_pair.h"
 #include "retention.h"
 
 namespace {
@@ -22,23 +23,6 @@ struct RetItem {  // Mirrored by llm_sharding_amd/ops/retention.py::segments
   int ws;                   // the run's first entry in the workspace: its initial state, then its segments' sums
   int seg, n_seg, len;      // which segment; all but the last have len rows
 };
-
-LSA_DEVICE int vidx(int r) { return (r & 32) | ((r & 12) << 1) | ((r & 16) >> 2) | (r & 3); }  // accumulator order
-
-// 8 values -> their rounding and the rounding of what that leaves
-LSA_DEVICE void split8(const float* f, u32x4_t& h, u32x4_t& l) {
-  float r[8], t[8];
-  h = pack8(f);
-  unpack8(h, r);
-#pragma unroll
-  for (int j = 0; j < 8; ++j) t[j] = f[j] - r[j];
-  l = pack8(t);
-}
-// two values, one above the other
-LSA_DEVICE void split2(float f, float g, unsigned& h, unsigned& l) {
-  h = (unsigned)f2bf(f) | ((unsigned)f2bf(g) << 16);
-  l = (unsigned)f2bf(f - __uint_as_float(h << 16)) | ((unsigned)f2bf(g - __uint_as_float(h & 0xffff0000u)) << 16);
-}
 
 constexpr int NT = 512;  // eight waves: four tiles of 16 queries x two halves of the value slice
 

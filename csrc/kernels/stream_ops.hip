@@ -1,6 +1,7 @@
 // Kernels of a decoder whose residual stream is fp32 and whose norms sit on the sublayers' OUTPUTS
 // (the sublayers read the stream itself):
-//   lsa_stream_embed     x = table[id] * scale in fp32, plus the copy the projections read
+//   lsa_stream_embed     x = table[id] * scale in fp32 (or several copies side by side: a decoder with several
+//                        streams, stream_mix.hip), plus, where asked for, the copy the projections read
 //   lsa_stream_add_norm  x += rms(y) * gain: a sublayer's result, RMS-normed, joins the stream (gain
 //                        = norm weight times layer scale, fp32), plus the copy the projections read
 //   lsa_stream_norm      rms(x) * gain -> the head projection's input
@@ -10,31 +11,32 @@
 // and of one with norms on both sides of its sublayers:
 //   lsa_stream_renorm    v = y + the weighted sum of a row's expert results; x (+)= rms(v) * post (or v as it
 //                        is), then (optionally) rms(x) * gain -> the next sublayer's input, or x itself
+//   lsa_softcap_rows     logits -> cap tanh(logits / cap)
 //   lsa_logits_argmax    argmax keys of fp32 logits (the fp32 engine; the bf16 one fuses this
 //                        into the head GEMM)
 //   lsa_cast_rows        fp32 rows -> the projections' type (a stage's input stream)
 // T is the projections' type (bf16, or fp32 for the fp32 engine). Rows of the copies may be wider
 // than the stream (GEMM padding): those columns are left as they are (zero).
-#include "elem.h"
+#include "stream_row.h"
 
 namespace {
 
 template <typename T>
 __global__ __launch_bounds__(256) void stream_embed_kernel(const int* __restrict__ ids, const T* __restrict__ table,
-                                                           int ldt, float scale, int W, float* __restrict__ x, int ldx,
-                                                           T* __restrict__ xc, int ldc) {
+                                                           int ldt, float scale, int W, int copies,
+                                                           float* __restrict__ x, int ldx, T* __restrict__ xc, int ldc) {
   const int row = blockIdx.x;
   const T* src = table + (size_t)ids[row] * ldt;
   for (int c = threadIdx.x; c < W; c += 256) {
     const float v = ld1(src + c) * scale;
-    x[(size_t)row * ldx + c] = v;
-    st1(xc + (size_t)row * ldc + c, v);
+    for (int s = 0; s < copies; ++s) x[(size_t)row * ldx + (size_t)s * W + c] = v;
+    if (xc) st1(xc + (size_t)row * ldc + c, v);
   }
 }
 // bf16, 8 values per thread and step
 __global__ __launch_bounds__(256) void stream_embed8_kernel(const int* __restrict__ ids, const bf16_raw* __restrict__ table,
-                                                            int ldt, float scale, int W, float* __restrict__ x, int ldx,
-                                                            bf16_raw* __restrict__ xc, int ldc) {
+                                                            int ldt, float scale, int W, int copies,
+                                                            float* __restrict__ x, int ldx, bf16_raw* __restrict__ xc, int ldc) {
   const int row = blockIdx.x;
   const bf16_raw* src = table + (size_t)ids[row] * ldt;
   for (int c = threadIdx.x * 8; c < W; c += 2048) {
@@ -42,10 +44,12 @@ __global__ __launch_bounds__(256) void stream_embed8_kernel(const int* __restric
     unpack8(ld16(src + c), f);
 #pragma unroll
     for (int k = 0; k < 8; ++k) f[k] *= scale;
-    float* d = x + (size_t)row * ldx + c;
-    *reinterpret_cast<f32x4_t*>(d) = f32x4_t{f[0], f[1], f[2], f[3]};
-    *reinterpret_cast<f32x4_t*>(d + 4) = f32x4_t{f[4], f[5], f[6], f[7]};
-    st16(xc + (size_t)row * ldc + c, pack8(f));
+    for (int s = 0; s < copies; ++s) {
+      float* d = x + (size_t)row * ldx + (size_t)s * W + c;
+      *reinterpret_cast<f32x4_t*>(d) = f32x4_t{f[0], f[1], f[2], f[3]};
+      *reinterpret_cast<f32x4_t*>(d + 4) = f32x4_t{f[4], f[5], f[6], f[7]};
+    }
+    if (xc) st16(xc + (size_t)row * ldc + c, pack8(f));
   }
 }
 
@@ -149,56 +153,24 @@ struct JoinArgs {  // Mirrored by llm_sharding_amd/ops/stream.py::JoinArgs
   float eps;
 };
 
-template <typename T>
-LSA_DEVICE f32x4_t load4(const T* p) {
-  if constexpr (sizeof(T) == 4) {
-    return *reinterpret_cast<const f32x4_t*>(p);
-  } else {
-    const u32x2_t v = *reinterpret_cast<const u32x2_t*>(p);
-    return f32x4_t{__uint_as_float(v[0] << 16), __uint_as_float(v[0] & 0xffff0000u), __uint_as_float(v[1] << 16),
-                   __uint_as_float(v[1] & 0xffff0000u)};
-  }
-}
-
 // what the results add to x[row][c .. c + V)
 template <typename T, int V>
 LSA_DEVICE void join_at(const JoinArgs& a, int row, int c, float* x) {
-  auto get = [&](const auto* p, float* f) {
-    if constexpr (V == 4) {
-      const f32x4_t v = load4(p);
-#pragma unroll
-      for (int k = 0; k < 4; ++k) f[k] = v[k];
-    } else {
-      f[0] = ld1(p);
-    }
-  };
   float y[V], g[V];
   if (a.y1) {
-    get(a.y1 + (size_t)row * a.ldy1 + c, y);
-    get((const T*)a.g1 + (size_t)row * a.ldg1 + c, g);
+    get<V>(a.y1 + (size_t)row * a.ldy1 + c, y);
+    get<V>((const T*)a.g1 + (size_t)row * a.ldg1 + c, g);
 #pragma unroll
     for (int k = 0; k < V; ++k) x[k] += sigmoid(g[k]) * y[k];
   }
   if (a.y2 || a.ye) {
-    get((const T*)a.g2 + (size_t)row * a.ldg2 + c, g);
+    get<V>((const T*)a.g2 + (size_t)row * a.ldg2 + c, g);
     if (a.y2) {
-      get(a.y2 + (size_t)row * a.ldy2 + c, y);
+      get<V>(a.y2 + (size_t)row * a.ldy2 + c, y);
     } else {
 #pragma unroll
       for (int k = 0; k < V; ++k) y[k] = 0.f;
-      for (int e0 = 0; e0 < a.top; e0 += 4) {  // four results requested at a time
-        float z[4][V], w[4];
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const int i = row * a.top + min(e0 + e, a.top - 1);
-          w[e] = e0 + e < a.top ? a.weight[i] : 0.f;
-          get((const T*)a.ye + (size_t)a.place[i] * a.ldye + c, z[e]);
-        }
-#pragma unroll
-        for (int e = 0; e < 4; ++e)
-#pragma unroll
-          for (int k = 0; k < V; ++k) y[k] = fmaf(w[e], z[e][k], y[k]);
-      }
+      add_pairs<V>((const T*)a.ye, a.ldye, a.weight, a.place, a.top, row, c, y);
     }
 #pragma unroll
     for (int k = 0; k < V; ++k) x[k] += sigmoid(g[k]) * y[k];
@@ -291,47 +263,13 @@ struct RenormArgs {  // Mirrored by llm_sharding_amd/ops/stream.py::RenormArgs
 // the result at [row][c .. c + V)
 template <typename T, int V>
 LSA_DEVICE void renorm_at(const RenormArgs& a, int row, int c, float* y) {
-  auto get = [&](const auto* p, float* f) {
-    if constexpr (V == 4) {
-      const f32x4_t v = load4(p);
-#pragma unroll
-      for (int k = 0; k < 4; ++k) f[k] = v[k];
-    } else {
-      f[0] = ld1(p);
-    }
-  };
   if (a.y) {
-    get(a.y + (size_t)row * a.ldy + c, y);
+    get<V>(a.y + (size_t)row * a.ldy + c, y);
   } else {
 #pragma unroll
     for (int k = 0; k < V; ++k) y[k] = 0.f;
   }
-  if (!a.ye) return;
-  for (int e0 = 0; e0 < a.top; e0 += 4) {  // four results requested at a time
-    float z[4][V], w[4];
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int i = row * a.top + min(e0 + e, a.top - 1);
-      w[e] = e0 + e < a.top ? a.weight[i] : 0.f;
-      get((const T*)a.ye + (size_t)a.place[i] * a.ldye + c, z[e]);
-    }
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-#pragma unroll
-      for (int k = 0; k < V; ++k) y[k] = fmaf(w[e], z[e][k], y[k]);
-  }
-}
-
-template <int NT>
-LSA_DEVICE float row_sum(float s, float* s_part) {
-  s = wave_sum(s);
-  __syncthreads();  // the sum before this one has been read
-  if ((threadIdx.x & 63) == 0) s_part[threadIdx.x >> 6] = s;
-  __syncthreads();
-  float sum = 0.f;
-#pragma unroll
-  for (int i = 0; i < NT / 64; ++i) sum += s_part[i];
-  return sum;
+  if (a.ye) add_pairs<V>((const T*)a.ye, a.ldye, a.weight, a.place, a.top, row, c, y);
 }
 
 // NT threads per row. NV > 0: rows of up to 4 NT NV values in registers, four at a time; 0: any width
@@ -423,6 +361,11 @@ void launch_renorm(const RenormArgs& a, int rows, int W, float* x, int ldx, T* x
 #undef LSA_J
 }
 
+__global__ __launch_bounds__(256) void softcap_kernel(float* __restrict__ lg, int ldl, int n, float cap) {
+  float* r = lg + (size_t)blockIdx.y * ldl;
+  for (int c = blockIdx.x * 1024 + threadIdx.x; c < min(n, (int)(blockIdx.x + 1) * 1024); c += 256) r[c] = cap * tanhf(r[c] / cap);
+}
+
 // grid (rows, blocks): every workgroup one stretch of the vocabulary
 __global__ __launch_bounds__(256) void logits_argmax_kernel(const float* __restrict__ lg, int ldl, int V, int offset,
                                                             unsigned long long* __restrict__ keys) {
@@ -441,15 +384,16 @@ __global__ __launch_bounds__(256) void logits_argmax_kernel(const float* __restr
 
 }  // namespace
 
-extern "C" int lsa_stream_embed(int f32, const int* ids, int rows, const void* table, int ldt, float scale, int W,
+extern "C" int lsa_stream_embed(int f32, const int* ids, int rows, const void* table, int ldt, float scale, int W, int copies,
                                 float* x, int ldx, void* xc, int ldc, hipStream_t s) {
-  if (rows < 1 || W < 1 || ldt < W || ldx < W || ldc < W) return LSA_BAD_SHAPE;
+  if (rows < 1 || W < 1 || copies < 1 || ldt < W || ldx < W * copies || (xc && ldc < W)) return LSA_BAD_SHAPE;
   if (f32)
-    stream_embed_kernel<float><<<rows, 256, 0, s>>>(ids, (const float*)table, ldt, scale, W, x, ldx, (float*)xc, ldc);
+    stream_embed_kernel<float><<<rows, 256, 0, s>>>(ids, (const float*)table, ldt, scale, W, copies, x, ldx, (float*)xc, ldc);
   else if (!((W | ldt | ldx | ldc) % 8) && !(((uintptr_t)table | (uintptr_t)x | (uintptr_t)xc) % 16))
-    stream_embed8_kernel<<<rows, 256, 0, s>>>(ids, (const bf16_raw*)table, ldt, scale, W, x, ldx, (bf16_raw*)xc, ldc);
+    stream_embed8_kernel<<<rows, 256, 0, s>>>(ids, (const bf16_raw*)table, ldt, scale, W, copies, x, ldx, (bf16_raw*)xc, ldc);
   else
-    stream_embed_kernel<bf16_raw><<<rows, 256, 0, s>>>(ids, (const bf16_raw*)table, ldt, scale, W, x, ldx, (bf16_raw*)xc, ldc);
+    stream_embed_kernel<bf16_raw><<<rows, 256, 0, s>>>(ids, (const bf16_raw*)table, ldt, scale, W, copies, x, ldx, (bf16_raw*)xc,
+                                                       ldc);
   LSA_CHECK_LAUNCH();
   return LSA_OK;
 }
@@ -506,6 +450,13 @@ extern "C" int lsa_stream_renorm(int f32, const RenormArgs* a, int rows, int W, 
   if (a->ye && (a->ldye < W || a->top < 1 || !a->weight || !a->place)) return LSA_BAD_SHAPE;
   if (f32) launch_renorm<float>(*a, rows, W, x, ldx, (float*)xc, ldc, s);
   else launch_renorm<bf16_raw>(*a, rows, W, x, ldx, (bf16_raw*)xc, ldc, s);
+  LSA_CHECK_LAUNCH();
+  return LSA_OK;
+}
+
+extern "C" int lsa_softcap_rows(float* lg, int ldl, int rows, int n, float cap, hipStream_t s) {
+  if (!lg || rows < 1 || rows > 65535 || n < 1 || ldl < n || !(cap > 0.f)) return LSA_BAD_SHAPE;
+  softcap_kernel<<<dim3((n + 1023) / 1024, rows), 256, 0, s>>>(lg, ldl, n, cap);
   LSA_CHECK_LAUNCH();
   return LSA_OK;
 }

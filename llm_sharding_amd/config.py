@@ -48,6 +48,11 @@ class LlamaConfig:
 
     # ------------------------------------------------------------------ derived
     @property
+    def stream_width(self) -> int:
+        """Values of one row of hidden states between layers and stages."""
+        return self.hidden_size
+
+    @property
     def q_size(self) -> int:
         return self.num_attention_heads * self.head_dim
 

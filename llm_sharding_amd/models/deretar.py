@@ -43,6 +43,8 @@ def _mlp(entry: dict) -> Optional[GluSpec]:
         return None
     if m.get("kind", "dense") != "dense":
         raise ValueError(f"unknown feed-forward kind {m.get('kind')!r}")
+    if not float(m["limit"]) > 0:
+        raise ValueError("gated unit: limit must be positive")
     return GluSpec(ff=int(m["ff"]), limit=float(m["limit"]), alpha=GLU_ALPHA, shift=GLU_SHIFT)
 
 

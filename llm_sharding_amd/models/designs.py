@@ -9,10 +9,10 @@ import json
 import os
 import struct
 
-from . import deretar, dumizen, gupuvik
+from . import deretar, dumizen, gupuvik, runidra
 
-DESIGNS = {m.ARCHITECTURE: m for m in (deretar, gupuvik, dumizen)}
-_BY_TYPE = {"deretar": deretar, "gupuvik": gupuvik, "dumizen": dumizen}
+DESIGNS = {m.ARCHITECTURE: m for m in (deretar, gupuvik, dumizen, runidra)}
+_BY_TYPE = {"deretar": deretar, "gupuvik": gupuvik, "dumizen": dumizen, "runidra": runidra}
 
 
 def of(cfg):

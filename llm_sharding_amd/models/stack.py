@@ -5,7 +5,7 @@ feed-forward with every size and constant of its own and how they are arranged a
 stream, and may use the tensors of another layer (``owner``, with a cache of its own) or another
 layer's cached keys and values (``AttentionSpec.kv_from``). A stretch of layers that runs several times in
 a row is listed once per run (``LayerSpec.enters`` marks where a pass begins). Designs
-(``models/deretar.py``, ``gupuvik.py``, ``dumizen.py``) only translate their config.json and tensor names
+(``models/deretar.py``, ``gupuvik.py``, ``dumizen.py``, ``runidra.py``) only translate their config.json and tensor names
 into this description; the mechanisms and their constants are parameters here, so that another design can
 combine them differently.
 
@@ -59,7 +59,10 @@ class RotarySpec:
 
 @dataclass(frozen=True)
 class LatentSpec:
-    """Latent attention with a latent query, a shared rotated key part and an output gate."""
+    """Latent attention with a latent query and a shared rotated key part. A row at position i sees the last
+    ``window`` keys up to its own (0: all). ``gate``: every output value is multiplied by the sigmoid of a projected
+    one; ``sink``: the softmax's denominator has one more term, exp of a number per head. Pairs of the rotated part
+    are (i, i + rot_dims / 2), or ``interleaved`` (2i, 2i + 1)."""
     heads: int
     dim: int        # unrotated query / key dimensions per head
     rot_dim: int    # rotated part: per head for the query, one for all heads for the key
@@ -67,11 +70,15 @@ class LatentSpec:
     kv_rank: int
     q_rank: int
     rot_base: float
-    rot_dims: int   # leading entries of the rotated part that turn (rotate-half pairs)
+    rot_dims: int   # leading entries of the rotated part that turn
     scale: float
+    gate: bool = True
+    window: int = 0
+    sink: bool = False
+    interleaved: bool = False
 
     def __post_init__(self):
-        if min(self.heads, self.dim, self.rot_dim, self.vdim, self.kv_rank, self.q_rank) < 1:
+        if min(self.heads, self.dim, self.rot_dim, self.vdim, self.kv_rank, self.q_rank) < 1 or self.window < 0:
             raise ValueError(f"latent attention: sizes must be positive: {self}")
         if self.rot_dims % 2 or not 2 <= self.rot_dims <= self.rot_dim:
             raise ValueError(f"latent attention: rot dims {self.rot_dims} must be even and at most {self.rot_dim}")
@@ -106,7 +113,7 @@ class LatentSpec:
     @property
     def scratch_width(self) -> int:
         """Values per row that a forward keeps besides the stream (every intermediate of the mixer)."""
-        return self.q_rank * 2 + self.kv_rank + self.rot_dim + self.heads * (2 * self.dvp + self.dkp + self.rp)
+        return self.q_rank * 2 + self.kv_rank + self.rot_dim + self.heads * ((1 + self.gate) * self.dvp + self.dkp + self.rp)
 
     def part_bytes(self, items: int, elem_bytes: int) -> int:
         """Split partials of ``items`` (row, key split) pairs."""
@@ -115,27 +122,30 @@ class LatentSpec:
     def params(self, width: int) -> int:
         q = self.q_rank * width + self.heads * (self.dim + self.rot_dim) * self.q_rank + self.q_rank
         kv = (self.kv_rank + self.rot_dim) * width + self.heads * (self.dim + self.vdim) * self.kv_rank + self.kv_rank
-        return q + kv + 2 * self.heads * self.vdim * width
+        return q + kv + (1 + self.gate) * self.heads * self.vdim * width + self.sink * self.heads
 
 
 @dataclass(frozen=True)
 class GluSpec:
-    """Clipped gated unit: g = min(gate, limit), u = clamp(up, -limit, limit),
-    g * sigmoid(alpha g) * (u + shift)."""
+    """Gated unit act(gate) * up, act silu or with ``gelu`` the tanh form of gelu. With ``limit`` the clipped unit:
+    g = min(gate, limit), u = clamp(up, -limit, limit), g * sigmoid(alpha g) * (u + shift). ``bias``: all three
+    projections have one."""
     ff: int
-    limit: float
-    alpha: float
-    shift: float
+    limit: float = 0.0
+    alpha: float = 1.0
+    shift: float = 0.0
+    gelu: bool = False
+    bias: bool = False
 
     def __post_init__(self):
-        if self.ff < 1 or not self.limit > 0:
-            raise ValueError(f"gated unit: ff and limit must be positive: {self}")
+        if self.ff < 1 or self.limit < 0 or (self.gelu and self.limit):
+            raise ValueError(f"gated unit: bad values: {self}")
 
     def scratch_width(self, width: int) -> int:
-        return self.ff
+        return pad_to(self.ff, 128)
 
     def params(self, width: int) -> int:
-        return 3 * self.ff * width
+        return 3 * self.ff * width + self.bias * (2 * self.ff + width)
 
     active_params = params
 
@@ -371,6 +381,55 @@ class RetentionSpec:
 
 
 @dataclass(frozen=True)
+class MlstmSpec:
+    """Matrix memory (mLSTM): per head a state S [dim, vdim], n [dim] and a running maximum m, all from zero. With
+    log gates i = gate_cap tanh(. / gate_cap) and f = log sigmoid(gate_cap tanh(. / gate_cap)) of projected numbers,
+
+        m' = max(f + m, i);  S <- exp(f + m - m') S + exp(i - m') k v^T;  n <- the same with k alone;  m <- m'
+        o = S^T q / (max(|n . q|, exp(-m)) + 1e-6)
+
+    q times ``q_scale``; o is RMS-normed per head, weighted and multiplied by the sigmoid of a projected gate."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+    q_scale: float
+
+    cache_width = 0
+
+    def __post_init__(self):
+        if min(self.heads, self.dim, self.vdim) < 1 or not self.gate_cap > 0:
+            raise ValueError(f"matrix memory: bad values: {self}")
+
+    @property
+    def state_dims(self) -> tuple:
+        return pad_state(self.dim, self.vdim)
+
+    @property
+    def copies(self) -> int:
+        """Times n and m are stored: once per slice of the value channels that a workgroup of its own advances
+        (csrc/kernels/mlstm.h)."""
+        return 2 if self.state_dims[1] == 128 and self.state_dims[0] <= 128 else 1
+
+    @property
+    def state_bytes(self) -> int:
+        dk, dv = self.state_dims
+        return 4 * self.heads * (dk * dv + self.copies * (dk + 1))
+
+    @property
+    def scratch_width(self) -> int:
+        dk, dv = self.state_dims
+        return self.heads * (2 * dk + 3 * dv) + 4 * pad_to(self.heads, 16) + 256
+
+    def part_bytes(self, items: int, elem_bytes: int) -> int:
+        return 0
+
+    def params(self, width: int) -> int:
+        H = self.heads
+        return H * (2 * self.dim + 3 * self.vdim) * width + 2 * H * (width + 1) + H * self.vdim
+
+
+@dataclass(frozen=True)
 class PairSpec:
     """Attention and a recurrent mixer side by side on one input: left_scale * left + right_scale * right."""
     left: AttentionSpec
@@ -433,7 +492,8 @@ class MoeSpec:
     logits, weighted by the softmax over these; or with ``sigmoid`` those with the largest sigmoid of the
     logit plus a ``correction`` per expert, among the ``keep`` of ``groups`` equal groups of neighbours whose
     two best choices sum highest, weighted by the sigmoids over their sum, times ``scale``. ``shared_ff``: one
-    more expert of this size that every token uses."""
+    more expert of this size that every token uses, with ``shared_gate`` times the sigmoid of one projected number.
+    ``bias``: the router has one."""
     experts: int
     top: int
     ff: int
@@ -444,11 +504,13 @@ class MoeSpec:
     keep: int = 1
     scale: float = 1.0
     shared_ff: int = 0
+    shared_gate: bool = False
+    bias: bool = False
 
     def __post_init__(self):
         if min(self.experts, self.top, self.ff) < 1 or self.top > self.experts or self.shared_ff < 0:
             raise ValueError(f"experts: bad sizes: {self}")
-        if self.act not in (SILU_GLU, RELU2) or (self.shared_ff and self.act != RELU2):
+        if self.act not in (SILU_GLU, RELU2) or (self.shared_gate and not self.shared_ff):
             raise ValueError(f"experts: unknown kind: {self}")
         if not 1 <= self.keep <= self.groups or self.experts % self.groups \
                 or self.top > self.keep * (self.experts // self.groups):
@@ -462,26 +524,28 @@ class MoeSpec:
         return 3 if self.act == SILU_GLU else 2
 
     def scratch_width(self, width: int) -> int:
-        return 2 * pad_to(self.experts, 16) + self.top * (pad_to(self.ff, 128) + 2 * pad_to(width, 128) + 8) \
+        return 2 * pad_to(self.experts + self.shared_gate, 128) + self.top * (pad_to(self.ff, 128) + 2 * pad_to(width, 128) + 8) \
             + pad_to(self.shared_ff, 128) + (2 * pad_to(width, 128) if self.shared_ff else 0)
 
     def params(self, width: int) -> int:
-        return (self.experts * (self.mats * self.ff + 1) + self.mats * self.shared_ff) * width
+        return (self.experts * (self.mats * self.ff + 1) + self.mats * self.shared_ff + self.shared_gate) * width \
+            + self.experts * self.bias
 
     def active_params(self, width: int) -> int:
         """Weights one token uses."""
-        return (self.mats * (self.ff * self.top + self.shared_ff) + self.experts) * width
+        return (self.mats * (self.ff * self.top + self.shared_ff) + self.experts + self.shared_gate) * width
 
 
 # How a layer's sublayers meet the residual stream
 POST_NORM = "post_norm"  # each sublayer reads the stream; its result is normed, scaled per element and added
 PARALLEL = "parallel"    # both read one norm of the stream; each result is added through a sigmoid gate per element
 SANDWICH = "sandwich"    # each sublayer reads a norm of the stream; its result is normed again and added
+HYPER = "hyper"          # several streams: each sublayer reads a norm of a weighted sum of them; a matrix mixes them anew
 
 
 @dataclass(frozen=True)
 class LayerSpec:
-    mixer: Any  # LatentSpec | AttentionSpec | DeltaSpec | RetentionSpec | PairSpec
+    mixer: Any  # LatentSpec | AttentionSpec | DeltaSpec | RetentionSpec | MlstmSpec | PairSpec
     mlp: Any    # GluSpec | DenseSpec | MoeSpec | None
     owner: int  # number, in the tensors' names, of the layer whose tensors this one uses
     block: str = POST_NORM
@@ -502,6 +566,9 @@ class StackConfig:
     model_type: str = "stack"
     name: str = "stack"
     tie_word_embeddings: bool = True
+    streams: int = 1           # copies of the residual stream; the head reads their sum
+    logit_scale: float = 1.0
+    logit_softcap: float = 0.0  # logits become softcap tanh(logits / softcap) (0: as they are)
     raw: Optional[dict] = None  # the config.json it was read from
 
     is_gpt2 = False
@@ -510,6 +577,11 @@ class StackConfig:
     @property
     def num_hidden_layers(self) -> int:
         return len(self.layers)
+
+    @property
+    def stream_width(self) -> int:
+        """Values of one row between layers and stages."""
+        return self.streams * self.hidden_size
 
     @property
     def rms_norm_eps(self) -> float:
@@ -537,6 +609,9 @@ class StackConfig:
         if s.block == PARALLEL:
             n = s.mixer.params(W) + 1 + W * W + W
             extra = W * W + W
+        elif s.block == HYPER:
+            coef = self.streams * (self.streams + 2)
+            n, extra = s.mixer.params(W) + W + coef, W + coef
         elif s.enters is not None:
             n, extra = s.mixer.params(W) + 2 * W + 2 * W * W + W, 2 * W
         else:
@@ -577,7 +652,7 @@ class StackConfig:
         """What a stage engine allocates besides weights and cache for ``rows`` rows (the largest layer
         sets every buffer): StackEngine._scratch_set."""
         W = pad_to(self.hidden_size, 128)
-        n = rows * (self.hidden_size * 4 + W * (4 + elem_bytes) + 12)
+        n = rows * (self.stream_width * 4 + W * (4 + elem_bytes) + 12)
         inter = part = 0
         for l in self.layers:
             gates = 2 * pad_to(self.hidden_size, 16) if l.block == PARALLEL else 0
@@ -589,7 +664,7 @@ class StackConfig:
 
     def stream_bytes(self) -> int:
         """Bytes of one row of the residual stream between pipeline stages (fp32)."""
-        return 4 * self.hidden_size
+        return 4 * self.stream_width
 
     def to_dict(self) -> dict:
         if self.raw is None:
@@ -597,6 +672,6 @@ class StackConfig:
         return self.raw
 
 
-__all__ = ["StackConfig", "LayerSpec", "LatentSpec", "AttentionSpec", "DeltaSpec", "RetentionSpec", "PairSpec", "RotarySpec",
-           "GluSpec", "DenseSpec", "MoeSpec", "POST_NORM", "PARALLEL", "SANDWICH", "HEAD", "WHOLE", "SILU_GLU", "RELU2",
+__all__ = ["StackConfig", "LayerSpec", "LatentSpec", "AttentionSpec", "DeltaSpec", "RetentionSpec", "MlstmSpec", "PairSpec", "RotarySpec",
+           "GluSpec", "DenseSpec", "MoeSpec", "POST_NORM", "PARALLEL", "SANDWICH", "HYPER", "HEAD", "WHOLE", "SILU_GLU", "RELU2",
            "leaves", "pad_to", "pad_part"]

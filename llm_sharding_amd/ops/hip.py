@@ -107,8 +107,8 @@ def load_library(path: str, mode: int = ctypes.RTLD_LOCAL) -> ctypes.CDLL:
         "lsa_version": [],
     }
     set_signatures(L, sig)
-    from . import delta, latent, moe, paged_attn, retention, stream
-    for m in (stream, latent, paged_attn, delta, retention, moe):
+    from . import delta, latent, mlstm, moe, paged_attn, retention, stream
+    for m in (stream, latent, paged_attn, delta, retention, mlstm, moe):
         m.declare(L)
     if os.environ.get("LSA_ATTN_SMALL_MAX_WGS"):  # A/B runs of the small-grid decode attention's range
         L.lsa_attn_set_small_max_wgs.argtypes = [i]

@@ -19,8 +19,8 @@ PAGE = 64  # tokens per cache page (LAT_PAGE in csrc/kernels/latent.h)
 
 
 class LatentArgs(ctypes.Structure):
-    _fields_ = ([(n, ctypes.c_void_p) for n in ("cache", "table", "slot", "pos", "index", "cos_t", "sin_t")]
-                + [(n, ctypes.c_int) for n in ("max_pages", "n_pages", "heads", "dim", "rot_dim", "rot_dims", "vdim",
+    _fields_ = ([(n, ctypes.c_void_p) for n in ("cache", "table", "slot", "pos", "index", "cos_t", "sin_t", "sink")]
+                + [(n, ctypes.c_int) for n in ("max_pages", "n_pages", "window", "heads", "dim", "rot_dim", "rot_dims", "vdim",
                                                "kv_rank", "q_rank", "dkp", "rp", "dvp", "krp")]
                 + [("scale", ctypes.c_float), ("eps", ctypes.c_float)])
 
@@ -57,9 +57,9 @@ def prefill_tile_rows(rows: int, heads: int) -> int:
     return t
 
 
-def make_args(spec, cache, table, slot, pos, cos, sin, eps: float, index=None) -> LatentArgs:
+def make_args(spec, cache, table, slot, pos, cos, sin, eps: float, index=None, sink=None) -> LatentArgs:
     """``cache`` [pages, PAGE, krp + rp], ``table`` int32 [slots, max_pages], ``slot`` / ``pos`` int32
-    [rows], ``cos`` / ``sin`` fp32 [>= max_pages * PAGE, rot_dims / 2], ``index`` int32 [entries]."""
+    [rows], ``cos`` / ``sin`` fp32 [>= max_pages * PAGE, rot_dims / 2], ``index`` int32 [entries], ``sink`` fp32 [heads] in log2 units."""
     _req(cache.dim() == 3 and cache.shape[1] == PAGE and cache.shape[2] == spec.cache_width and cache.is_contiguous()
          and cache.is_cuda, "latent: cache [pages, 64, width]")
     _req(table.dtype == torch.int32 and table.dim() == 2 and table.is_contiguous(), "latent: int32 page table")
@@ -67,9 +67,11 @@ def make_args(spec, cache, table, slot, pos, cos, sin, eps: float, index=None) -
     _req(index is None or index.dtype == torch.int32, "latent: int32 index")
     _req(cos.dtype == torch.float32 and cos.shape == sin.shape and cos.shape[0] >= table.shape[1] * PAGE
          and cos.shape[1] == spec.rot_dims // 2, "latent: rotation tables")
+    _req((sink is not None) == spec.sink and (sink is None or (sink.dtype == torch.float32 and sink.numel() == spec.heads
+                                                               and sink.is_contiguous())), "latent: sink")
     return LatentArgs(cache.data_ptr(), table.data_ptr(), slot.data_ptr(), pos.data_ptr(),
-                      None if index is None else index.data_ptr(), cos.data_ptr(), sin.data_ptr(), table.shape[1],
-                      cache.shape[0], spec.heads, spec.dim, spec.rot_dim, spec.rot_dims, spec.vdim, spec.kv_rank,
+                      None if index is None else index.data_ptr(), cos.data_ptr(), sin.data_ptr(), _p(sink),
+                      table.shape[1], cache.shape[0], spec.window, spec.heads, spec.dim, spec.rot_dim, spec.rot_dims, spec.vdim, spec.kv_rank,
                       spec.q_rank, spec.dkp, spec.rp, spec.dvp, spec.krp, float(spec.scale), float(eps))
 
 
@@ -146,8 +148,9 @@ _TILES_OK = None  # the last tile table prefill() validated: a forward checks it
 
 
 def prefill(a: LatentArgs, tiles, tiles_host, q, kv, lat, gate, out, rows: int, tokens: int) -> None:
-    """Attention of the query tiles [row0, nrows, kv0, pos0, kvlen, 0, 0, 0] over expanded keys and
-    values ``kv`` [tokens, heads (dkp + dvp)] and the gathered entries ``lat`` [tokens, krp + rp]."""
+    """Attention of the query tiles [row0, nrows, kv0, pos0, kvlen, base, 0, 0] over expanded keys and
+    values ``kv`` [tokens, heads (dkp + dvp)] and the gathered entries ``lat`` [tokens, krp + rp], the
+    sequence's from row kv0 (position ``base``) on."""
     _req(all(t.dtype == torch.bfloat16 for t in (q, kv, lat, out)) and tiles.dtype == torch.int32
          and tiles.shape == tiles_host.shape and tiles.shape[1] == 8 and tiles.is_contiguous(), "prefill: types")
     _req(min(q.shape[0], out.shape[0]) >= rows and out.shape[1] >= a.heads * a.dvp
@@ -158,11 +161,12 @@ def prefill(a: LatentArgs, tiles, tiles_host, q, kv, lat, gate, out, rows: int, 
     global _TILES_OK
     key = (tiles.data_ptr(), rows, tokens, a.max_pages)
     if not (_TILES_OK is not None and _TILES_OK[0] is tiles_host and _TILES_OK[1] == key):
-        r0, nr, k0, p0, kl = (tiles_host[:, i] for i in range(5))
+        r0, nr, k0, p0, kl, base = (tiles_host[:, i] for i in range(6))
         _req(bool((nr >= 1).all() and (nr <= 128).all() and (r0 >= 0).all()) and int((r0 + nr).max()) <= rows,
              "prefill: tile rows")
         _req(bool((k0 >= 0).all() and (kl >= 1).all() and (p0 >= 0).all()) and int((k0 + kl).max()) <= tokens
-             and bool((p0 + nr <= kl).all()) and int(kl.max()) <= a.max_pages * PAGE, "prefill: tile keys")
+             and bool((base >= 0).all() and (p0 >= base).all() and (p0 + nr <= base + kl).all())
+             and int((base + kl).max()) <= a.max_pages * PAGE, "prefill: tile keys")
         _TILES_OK = (tiles_host, key)
     _check(lib().lsa_latent_prefill(ctypes.byref(a), _p(tiles), tiles.shape[0], _p(q), q.stride(0), _p(kv), kv.stride(0),
                                     _p(lat), _p(gate), 0 if gate is None else gate.stride(0), _p(out), out.stride(0),

@@ -47,6 +47,12 @@ class Linear:
         n = -(-ff // 128) * 128
         return Linear(fuse_gate_up(pad2(gate, n, K), pad2(up, n, K)))
 
+    @staticmethod
+    def glu_bias(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
+        """Biases [ff] of both, in the order of :meth:`glu`'s columns."""
+        n = -(-gate.numel() // 128) * 128
+        return fuse_gate_up(pad2(gate[:, None], n, 1), pad2(up[:, None], n, 1)).reshape(-1).contiguous()
+
     def tensors(self) -> list:
         return [self.w]
 
@@ -82,7 +88,7 @@ class Linear:
         if act_from is not None:
             kw.update(act=act, act_from=act_from)
         if glu is not None:
-            kw.update(glu_alpha=glu.alpha, glu_limit=glu.limit, glu_shift=glu.shift)
+            kw.update(glu_alpha=glu.alpha, glu_limit=glu.limit, glu_shift=glu.shift, act=hip.ACT_GELU if glu.gelu else hip.ACT_NONE)
         _req(bias is None or bias.numel() >= self.n, "linear: bias")
         epi = hip.EPI_SWIGLU if glu is not None else (hip.EPI_STORE if keys is None else hip.EPI_ARGMAX)
         ep = hip.make_epi(keys=keys, bias=bias, col_offset=col_offset, **kw)
@@ -97,13 +103,14 @@ class Linear:
 
 
 # ------------------------------------------------------------------------------ fp32 stream
-def stream_embed(ids, table, scale: float, x, xc, rows: int) -> None:
-    W = x.shape[1]
+def stream_embed(ids, table, scale: float, x, xc, rows: int, copies: int = 1) -> None:
+    """x = table[ids] * scale, ``copies`` of it side by side; ``xc`` (or None): one in the projections' type."""
+    W = x.shape[1] // copies
     _req(ids.dtype == torch.int32 and ids.is_cuda and ids.numel() >= rows, "stream_embed: int32 ids")
-    _req(x.dtype == torch.float32 and table.dtype == xc.dtype and table.shape[1] >= W and xc.shape[1] >= W
-         and min(x.shape[0], xc.shape[0]) >= rows, "stream_embed: shapes")
-    _check(lib().lsa_stream_embed(is_f32(xc.dtype), _p(ids), rows, _p(table), table.stride(0), float(scale), W, _p(x),
-                                  x.stride(0), _p(xc), xc.stride(0), _stream()), "lsa_stream_embed")
+    _req(x.dtype == torch.float32 and x.shape[0] >= rows and x.shape[1] == W * copies and table.shape[1] >= W, "stream_embed: shapes")
+    _req(xc is None or (table.dtype == xc.dtype and xc.shape[1] >= W and xc.shape[0] >= rows), "stream_embed: copy")
+    _check(lib().lsa_stream_embed(is_f32(table.dtype), _p(ids), rows, _p(table), table.stride(0), float(scale), W, copies, _p(x),
+                                  x.stride(0), _p(xc), 0 if xc is None else xc.stride(0), _stream()), "lsa_stream_embed")
 
 
 def cast_rows(x, xc, rows: int, x2=None) -> None:
@@ -201,6 +208,56 @@ def stream_renorm(x, rows: int, y=None, experts=None, post=None, gain=None, eps:
            "lsa_stream_renorm")
 
 
+class MixArgs(ctypes.Structure):
+    _fields_ = ([(n, ctypes.c_void_p) for n in ("coef", "y", "ygate", "ye", "weight", "place", "read", "gain")]
+                + [(n, ctypes.c_int) for n in ("streams", "ldy", "ldyg", "ldye", "top")] + [("eps", ctypes.c_float)])
+
+
+MAX_STREAMS = 8  # of stream_mix (MAXS in csrc/kernels/stream_mix.hip)
+
+
+def stream_mix(x, rows: int, streams: int, coef=None, y=None, ygate=None, experts=None, read=None, eps: float = 0.0,
+               out=None) -> None:
+    """Rows of ``streams`` streams x_s side by side. With ``coef`` = [out | mix] (fp32): x_t <- sum_s mix[s, t] x_s +
+    out[t] v, v = ``y`` (fp32), times the sigmoid of ``ygate`` [rows, 1..] (fp32) where given, plus with ``experts`` =
+    (results of the sorted pairs, weights, places, top) a row's weighted sum. With ``read`` (its ``weights`` and
+    ``gain``, fp32) then out = rms(sum_s weights[s] x_s) * gain in the projections' type."""
+    _req(1 <= streams <= MAX_STREAMS and x.shape[1] % streams == 0, f"mix: 1 to {MAX_STREAMS} streams")
+    W = x.shape[1] // streams
+    ye, weight, place, top = experts if experts is not None else (None, None, None, 0)
+    _req(x.dtype == torch.float32 and x.stride(1) == 1 and x.shape[0] >= rows, "mix: streams")
+    _req((coef is None) == (y is None and ye is None) and (coef is not None or read is not None), "mix: nothing to do")
+    _req(coef is None or (coef.dtype == torch.float32 and coef.numel() == streams * (streams + 1) and coef.is_contiguous()),
+         "mix: coefficients")
+    _req(y is None or (y.dtype == torch.float32 and y.shape[0] >= rows and y.shape[1] >= W and y.stride(1) == 1), "mix: y")
+    _req(ygate is None or (y is not None and ygate.dtype == torch.float32 and ygate.shape[0] >= rows), "mix: gate")
+    _req(ye is None or (ye.stride(1) == 1 and ye.shape[1] >= W and ye.shape[0] >= rows * top
+                        and min(weight.numel(), place.numel()) >= rows * top and weight.dtype == torch.float32
+                        and place.dtype == torch.int32), "mix: experts")
+    wts, gain = (read.weights, read.gain) if read is not None else (None, None)
+    if read is None:
+        out = None
+    else:
+        _req(wts.dtype == gain.dtype == torch.float32 and wts.numel() == streams and gain.numel() == W
+             and wts.is_contiguous() and gain.is_contiguous(), "mix: read")
+        _req(out is not None and out.stride(1) == 1 and out.shape[1] >= W and out.shape[0] >= rows
+             and (ye is None or ye.dtype == out.dtype), "mix: copy")
+
+    def ld(t):
+        return 0 if t is None else t.stride(0)
+    a = MixArgs(_p(coef), _p(y), _p(ygate), _p(ye), _p(weight), _p(place), _p(wts), _p(gain), streams, ld(y), ld(ygate), ld(ye),
+                top, float(eps))
+    dt = ye.dtype if ye is not None else out.dtype if out is not None else torch.float32
+    _check(lib().lsa_stream_mix(is_f32(dt), ctypes.byref(a), rows, W, _p(x), x.stride(0), _p(out), ld(out), _stream()),
+           "lsa_stream_mix")
+
+
+def softcap_rows(lg, rows: int, n: int, cap: float) -> None:
+    """lg[:rows, :n] becomes cap * tanh(lg / cap)."""
+    _req(lg.dtype == torch.float32 and lg.stride(1) == 1 and lg.shape[0] >= rows and lg.shape[1] >= n and cap > 0, "softcap_rows: shapes")
+    _check(lib().lsa_softcap_rows(_p(lg), lg.stride(0), rows, n, float(cap), _stream()), "lsa_softcap_rows")
+
+
 def logits_argmax(lg, rows: int, vocab: int, keys, offset: int = 0) -> None:
     _req(lg.dtype == torch.float32 and lg.shape[0] >= rows and lg.shape[1] >= vocab and keys.dtype == torch.int64
          and keys.numel() >= rows, "logits_argmax: shapes")
@@ -211,7 +268,9 @@ def declare(L: ctypes.CDLL) -> None:
     """Signatures of these entry points (called by hip.load_library)."""
     vp, i, f = ctypes.c_void_p, ctypes.c_int, ctypes.c_float
     hip.set_signatures(L, {
-        "lsa_stream_embed": [i, vp, i, vp, i, f, i, vp, i, vp, i, vp],
+        "lsa_stream_embed": [i, vp, i, vp, i, f, i, i, vp, i, vp, i, vp],
+        "lsa_stream_mix": [i, ctypes.POINTER(MixArgs), i, i, vp, i, vp, i, vp],
+        "lsa_softcap_rows": [vp, i, i, i, f, vp],
         "lsa_cast_rows": [i, vp, i, i, i, vp, i, vp, i, vp],
         "lsa_stream_add_norm": [i, vp, i, vp, f, i, i, vp, i, vp, i, vp],
         "lsa_stream_norm": [i, vp, i, vp, f, i, i, vp, i, vp],

@@ -272,7 +272,7 @@ class PipelineStage:
                                    max_slots=batch * microbatches, max_seq=max_seq,
                                    max_prefill_rows=max(max_prefill_rows, batch), head_cols=head_cols,
                                    weight_dtype=weight_dtype)
-        H = cfg.hidden_size
+        H = cfg.stream_width
         self.h_out = [torch.zeros((batch, H), dtype=self.eng.hidden_dtype, device=self.device) for _ in range(microbatches)]
         self.tok_out = [torch.zeros(batch, dtype=torch.int32, device=self.device) for _ in range(microbatches)]
         if self.split:
@@ -328,7 +328,7 @@ class PipelineStage:
     def prefill_mb(self, mb: int, prompts, prompt_len: int, recv_token: bool = True):
         """Prefill one micro-batch on this stage. Returns the first generated ids on the stage
         that ends up holding them (rank 0 after the back-edge, or a single-stage pipeline)."""
-        eng, B, P, H = self.eng, self.B, prompt_len, self.cfg.hidden_size
+        eng, B, P, H = self.eng, self.B, prompt_len, self.cfg.stream_width
         sl = self.slots(mb)
         slot, pos = eng.prefill_rows(sl, [P] * B)
         if self.first:
@@ -363,7 +363,7 @@ class PipelineStage:
 
     def recv_first_token(self, mb: int = 0) -> torch.Tensor:
         if self.split:
-            hf = torch.zeros((self.B, self.cfg.hidden_size), dtype=self.eng.hidden_dtype, device=self.device)
+            hf = torch.zeros((self.B, self.cfg.stream_width), dtype=self.eng.hidden_dtype, device=self.device)
             keys = torch.zeros(self.B, dtype=torch.int64, device=self.device)
             self._recv(hf, self.world - 1)
             self._recv(keys, self.world - 1)
@@ -421,7 +421,7 @@ class PipelineStage:
                 and getattr(self.p2p, "graph_capturable", False)
                 and os.environ.get("LSA_GRAPH_COMM", "1") == "1"):
             return False
-        H = self.cfg.hidden_size
+        H = self.cfg.stream_width
         probe = [torch.empty((self.B, H), dtype=self.eng.hidden_dtype, device=self.device),
                  torch.empty(self.B, dtype=torch.int64, device=self.device),
                  torch.empty(self.B, dtype=torch.int32, device=self.device)]

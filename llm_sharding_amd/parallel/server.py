@@ -307,7 +307,7 @@ class PipelineServer:
             return self._exec_body(cmd, mb, items, resets, ids)
 
     def _exec_body(self, cmd, mb, items, resets, ids=None):
-        eng, H = self.eng, self.cfg.hidden_size
+        eng, H = self.eng, self.cfg.stream_width
         for s in resets:
             self._clear(s)
         if cmd == CMD_PREFILL:

@@ -11,6 +11,8 @@ returns which of these buf_x then holds, or None. :class:`.stack_engine.StackEng
   for the next block.
 * ``Sandwich``: each sublayer reads a norm of the stream through one input projection; its result is normed
   again and added, in one kernel that also norms for the next sublayer.
+* ``Hyper``: several streams; each sublayer reads a norm of a weighted sum of them, and its result and a matrix
+  make every stream anew, in one kernel that also sums and norms for the next sublayer (``Sum``).
 
 ``Entry`` is what happens before a pass of layers that run several times in a row.
 """
@@ -19,15 +21,18 @@ from __future__ import annotations
 import torch
 import torch.nn.functional as F
 
-from ..models.stack import (PARALLEL, SANDWICH, AttentionSpec, DeltaSpec, LatentSpec, PairSpec, RetentionSpec, pad_to)
+from ..models.stack import (HYPER, PARALLEL, SANDWICH, AttentionSpec, DeltaSpec, LatentSpec, MlstmSpec, PairSpec, RetentionSpec,
+                            pad_to)
 from .attn_mixer import Attention
 from .delta_mixer import Delta
 from .feed_forward import feed_forward
 from .latent_mixer import Weights
+from .mlstm_mixer import Mlstm
 from .retention_mixer import Pair, Retention
 
 COPY = "copy"
-MIXERS = {LatentSpec: Weights, AttentionSpec: Attention, DeltaSpec: Delta, RetentionSpec: Retention, PairSpec: Pair}
+MIXERS = {LatentSpec: Weights, AttentionSpec: Attention, DeltaSpec: Delta, RetentionSpec: Retention, MlstmSpec: Mlstm,
+          PairSpec: Pair}
 
 
 def _part(t: dict, prefix: str) -> dict:
@@ -53,11 +58,12 @@ class Layer:
 class InputProjection:
     """One product of the sublayers' input for everything they compute from it. ``parts``: [(name, weight, bias or
     None, kind)], kind None: a result in the engine's type, "gelu" / "relu2": with that activation, "f32": in fp32.
-    They lie in this order; ``col`` has their first columns (of the fp32 result for the last kind)."""
+    They lie in this order; ``col`` has their first columns (of the fp32 result for the last kind). ``whole``: the
+    width is a multiple of it (default: of 128, above 2048 of 256)."""
 
     KINDS = (None, "gelu", "relu2", "f32")
 
-    def __init__(self, parts: list, name: str):
+    def __init__(self, parts: list, name: str, whole: int = 0):
         from ..ops import hip
         from ..ops import stream as L
         parts = sorted(parts, key=lambda p: self.KINDS.index(p[3]))
@@ -73,7 +79,7 @@ class InputProjection:
                 self.col32 = n
             self.col[key] = n - (self.col32 or 0)
             n += pad_to(w.shape[0], 16)
-        n = pad_to(n, 128 if n <= 2048 else 256)
+        n = pad_to(n, whole or (128 if n <= 2048 else 256))
         dev, dt, o = parts[0][1].device, parts[0][1].dtype, 0
         win, bias = torch.zeros((n, parts[0][1].shape[1]), dtype=dt, device=dev), torch.zeros(n, device=dev)
         for _, w, b, _ in parts:
@@ -113,30 +119,34 @@ class PostNorm:
         self.mixer = MIXERS[type(spec.mixer)](spec.mixer, _part(t, "mix."), gpu)
         self.mlp = None if spec.mlp is None else feed_forward(spec.mlp, _part(t, "mlp."), gpu)
         self.gain1, self.gain2 = gain(1), None if spec.mlp is None else gain(2)
+        self.inp = InputProjection(self.mixer.input_parts(), "inp", 128) if gpu else None
 
     def tensors(self) -> list:
-        return self.mixer.tensors() + (self.mlp.tensors() if self.mlp is not None else []) + [self.gain1, self.gain2]
+        subs = [p for p in (self.inp, self.mixer, self.mlp) if p is not None]
+        return [t for p in subs for t in p.tensors()] + [self.gain1, self.gain2]
 
     def scratch(self) -> list:
-        return [self.mixer.scratch()] + ([self.mlp.scratch()] if self.mlp is not None else [])
+        return [self.inp.scratch(), self.mixer.scratch()] + ([self.mlp.scratch()] if self.mlp is not None else [])
 
     def projections(self) -> list:
-        return self.mixer.projections() + (self.mlp.projections() if self.mlp is not None else [])
+        return [self.inp.lin] + self.mixer.projections() + (self.mlp.projections() if self.mlp is not None else [])
 
     def forward(self, eng, i: int, slot, pos, rows: int, plan, nxt):
         from ..ops import stream as L
         h, x, y, eps = eng.buf_h[:rows], eng.buf_x[:rows], eng.buf_y[:rows], eng.cfg.norm_eps
-        self.mixer.forward(eng, x, y, eng.k_cache[i], slot, pos, rows, plan)
+        inp, in32 = self.inp(eng, x, rows)
+        ao = self.mixer.forward(eng, inp, in32, self.inp.col, eng.cache(i), eng.states[i], slot, pos, rows, plan)
+        eng.project(self.mixer.out, ao, rows, y, bias=self.mixer.out_bias)
         L.stream_add_norm(y, self.gain1, eps, h, x, rows)
         if self.mlp is not None:
-            self.mlp.forward(eng, x, y, rows)
+            y = self.mlp.forward(eng, x, None, None, {}, None, rows)["y"]
             L.stream_add_norm(y, self.gain2, eps, h, x, rows)
         return COPY
 
     def forward_torch(self, eng, i: int, x, slot, pos) -> torch.Tensor:
         def join(x, y, gain):
             return x + y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eng.cfg.norm_eps) * gain
-        x = join(x, self.mixer.forward_torch(eng, x, eng.k_cache[i], slot, pos), self.gain1)
+        x = join(x, self.mixer.forward_torch(eng, x, eng.cache(i), eng.states[i], slot, pos), self.gain1)
         return x if self.mlp is None else join(x, self.mlp.forward_torch(x), self.gain2)
 
 
@@ -237,6 +247,84 @@ class Sandwich:
         return x if self.mlp is None else x + norm(self.mlp.forward_torch(norm(x, self.norm2)), self.post2)
 
 
+class Sum:
+    """What a sublayer reads of several streams: a norm of their weighted sum."""
+
+    def __init__(self, weights, gain):
+        self.weights, self.gain = weights, gain  # fp32 [streams], [width]
+
+    def read(self, eng, x, out, rows: int) -> None:
+        from ..ops import stream as L
+        L.stream_mix(x, rows, self.weights.numel(), read=self, eps=eng.cfg.norm_eps, out=out)
+
+    def read_torch(self, eng, xs) -> torch.Tensor:
+        u = torch.einsum("nsw,s->nw", xs, self.weights)
+        return u * torch.rsqrt(u.pow(2).mean(-1, keepdim=True) + eng.cfg.norm_eps) * self.gain
+
+
+class Hyper:
+    """x_t <- sum_s mix[s, t] x_s + out[t] sublayer(norm(sum_s in[s] x_s)), for the mixer and the feed-forward."""
+
+    def __init__(self, cfg, spec, t: dict, gpu: bool):
+        self.mixer = MIXERS[type(spec.mixer)](spec.mixer, _part(t, "mix."), gpu)
+        self.mlp = None if spec.mlp is None else feed_forward(spec.mlp, _part(t, "mlp."), gpu)
+
+        def sub(n):  # (what it reads, [out | mix] of its streams)
+            hc = {k: t[f"hc{n}.{k}"].float() for k in ("in", "out", "mix")}
+            return (Sum(hc["in"].contiguous(), (t[f"norm{n}"].float() + cfg.norm_offset).contiguous()),
+                    torch.cat([hc["out"], hc["mix"].reshape(-1)]).contiguous())
+        self.entry, self.coef1 = sub(1)
+        self.entry2, self.coef2 = sub(2) if self.mlp is not None else (None, None)
+        self.inputs = []
+        if gpu:
+            self.inp = InputProjection(self.mixer.input_parts(), "inp")
+            parts = self.mlp.input_parts() if self.mlp is not None else []
+            self.ffin = InputProjection(parts, "ffin") if parts else None
+            self.inputs = [p for p in (self.inp, self.ffin) if p is not None]
+
+    def _subs(self) -> list:
+        return [self.mixer] + ([self.mlp] if self.mlp is not None else [])
+
+    def tensors(self) -> list:
+        own = [self.coef1, self.entry.weights, self.entry.gain]
+        if self.mlp is not None:
+            own += [self.coef2, self.entry2.weights, self.entry2.gain]
+        return own + [t for p in self.inputs + self._subs() for t in p.tensors()]
+
+    def scratch(self) -> list:
+        return [p.scratch() for p in self.inputs + self._subs()]
+
+    def projections(self) -> list:
+        return [p.lin for p in self.inputs] + [lin for p in self._subs() for lin in p.projections()]
+
+    def forward(self, eng, i: int, slot, pos, rows: int, plan, nxt):
+        from ..ops import stream as L
+        x, h, y, eps, n = eng.buf_h[:rows], eng.buf_x[:rows], eng.buf_y[:rows], eng.cfg.norm_eps, eng.cfg.streams
+        nxt = nxt if isinstance(nxt, Sum) else None
+        inp, in32 = self.inp(eng, h, rows)
+        ao = self.mixer.forward(eng, inp, in32, self.inp.col, eng.cache(i), eng.states[i], slot, pos, rows, plan)
+        eng.project(self.mixer.out, ao, rows, y, bias=self.mixer.out_bias)
+        second = self.entry2 if self.mlp is not None else nxt
+        L.stream_mix(x, rows, n, coef=self.coef1, y=y, read=second, eps=eps, out=h)
+        if self.mlp is not None:
+            inp, in32 = self.ffin(eng, h, rows) if self.ffin is not None else (None, None)
+            left = self.mlp.forward(eng, h, inp, in32, self.ffin.col if self.ffin is not None else {}, None, rows)
+            L.stream_mix(x, rows, n, coef=self.coef2, **left, read=nxt, eps=eps, out=h)
+        return nxt
+
+    def forward_torch(self, eng, i: int, x, slot, pos) -> torch.Tensor:
+        n = eng.cfg.streams
+        xs = x.view(x.shape[0], n, -1)
+
+        def join(coef, y):
+            return torch.einsum("nsw,st->ntw", xs, coef[n:].view(n, n)) + coef[:n, None] * y[:, None]
+        xs = join(self.coef1, self.mixer.forward_torch(eng, self.entry.read_torch(eng, xs), eng.cache(i), eng.states[i],
+                                                       slot, pos))
+        if self.mlp is not None:
+            xs = join(self.coef2, self.mlp.forward_torch(self.entry2.read_torch(eng, xs)))
+        return xs.reshape(x.shape)
+
+
 class Entry:
     """What a pass of layers that run several times in a row starts from: x <- W_in [x; x0] + step[pass], x0 the
     embedding output. The stream's and x0's copies in the projections' type lie side by side, x0's from the start of
@@ -280,11 +368,11 @@ class Entry:
         return F.linear(torch.cat([x, x0], -1), w["loop.in"]) + w["loop.step"][t]
 
 
-BLOCKS = {PARALLEL: Parallel, SANDWICH: Sandwich}
+BLOCKS = {PARALLEL: Parallel, SANDWICH: Sandwich, HYPER: Hyper}
 
 
 def block(cfg, spec, t: dict, gpu: bool):
     return BLOCKS.get(spec.block, PostNorm)(cfg, spec, t, gpu)
 
 
-__all__ = ["COPY", "Layer", "InputProjection", "PostNorm", "Parallel", "Sandwich", "Entry", "block"]
+__all__ = ["COPY", "Layer", "InputProjection", "PostNorm", "Parallel", "Sandwich", "Sum", "Hyper", "Entry", "block"]

@@ -1052,7 +1052,7 @@ class DecodeGraph:
         self.pos = torch.tensor([eng.seq_len[s] for s in self.slots], dtype=torch.int32, device=dev)
         self.tokens = torch.zeros(rows, dtype=torch.int32, device=dev)
         self.keys = torch.zeros(rows, dtype=torch.int64, device=dev)
-        self.h_in = torch.zeros((rows, eng.cfg.hidden_size), dtype=eng.hidden_dtype, device=dev)
+        self.h_in = torch.zeros((rows, eng.cfg.stream_width), dtype=eng.hidden_dtype, device=dev)
         self._host_pos = [eng.seq_len[s] for s in self.slots]  # paged caches: where the next tokens go
         self.history = torch.zeros((max(1, history_len), rows), dtype=torch.int32, device=dev) if history_len else None
         self.step_ctr = torch.zeros(1, dtype=torch.int32, device=dev)
@@ -1069,7 +1069,7 @@ class DecodeGraph:
         if split_head:
             if mode not in ("first", "last"):
                 raise ValueError("split_head needs mode 'first' or 'last'")
-            self.h_fin = torch.zeros((rows, eng.cfg.hidden_size), dtype=eng.hidden_dtype, device=dev)
+            self.h_fin = torch.zeros((rows, eng.cfg.stream_width), dtype=eng.hidden_dtype, device=dev)
             self.keys_in = torch.zeros(rows, dtype=torch.int64, device=dev)
 
     def _body(self) -> None:
@@ -1166,13 +1166,13 @@ class EagerDecode:
         self.eng, self.rows, self.mode = eng, rows, mode
         self.slots = list(range(rows)) if slots is None else list(slots)
         self.tokens = torch.zeros(rows, dtype=torch.int32)
-        self.h_in = torch.zeros((rows, eng.cfg.hidden_size), dtype=eng.hidden_dtype)
+        self.h_in = torch.zeros((rows, eng.cfg.stream_width), dtype=eng.hidden_dtype)
         self.history = torch.zeros((history_len, rows), dtype=torch.int32) if history_len else None
         self.step = 0
         self._out = None
         self.split_head = split_head
         self.keys = torch.zeros(rows, dtype=torch.int64)
-        self.h_fin = torch.zeros((rows, eng.cfg.hidden_size), dtype=eng.hidden_dtype)
+        self.h_fin = torch.zeros((rows, eng.cfg.stream_width), dtype=eng.hidden_dtype)
         self.keys_in = torch.zeros(rows, dtype=torch.int64)
 
     def _body(self) -> None:

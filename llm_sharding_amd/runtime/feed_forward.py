@@ -1,7 +1,7 @@
-"""Feed-forwards of a layer stack: the clipped gated unit, the dense gelu layer and the mixture of experts.
+"""Feed-forwards of a layer stack: gated units, the dense gelu layer and the mixture of experts.
 
-A feed-forward that runs beside its mixer on the same input gives the block the rows it wants of the
-block's input projection (``input_parts``) and takes their columns."""
+A feed-forward gives the block the rows it wants of the block's input projection (``input_parts``) and takes
+their columns."""
 from __future__ import annotations
 
 import torch
@@ -11,7 +11,7 @@ from ..models.stack import SILU_GLU, DenseSpec, GluSpec, MoeSpec
 
 
 class Glu:
-    """Gate / up / down projection of a clipped gated unit."""
+    """Gate / up / down projection of a gated unit; gate and up are one product with the unit in its epilogue."""
 
     def __init__(self, spec: GluSpec, t: dict, gpu: bool):
         self.spec = spec
@@ -19,9 +19,18 @@ class Glu:
         if gpu:
             from ..ops import stream as L
             self.gate_up, self.down = L.Linear.glu(t["gate"], t["up"]), L.Linear(t["down"])
+            self.bias = self.down_bias = None
+            if spec.bias:
+                self.bias = L.Linear.glu_bias(t["gate.b"].float(), t["up.b"].float())
+                self.down_bias = F.pad(t["down.b"].float(), (0, self.down.n - t["down.b"].numel())).contiguous()
+
+    def input_parts(self) -> list:
+        return []
 
     def tensors(self) -> list:
-        return list(self.raw.values()) if self.raw is not None else self.gate_up.tensors() + self.down.tensors()
+        if self.raw is not None:
+            return list(self.raw.values())
+        return self.gate_up.tensors() + self.down.tensors() + ([self.bias, self.down_bias] if self.spec.bias else [])
 
     def scratch(self) -> dict:
         return {"act": self.down.k}
@@ -29,13 +38,17 @@ class Glu:
     def projections(self) -> list:
         return [self.gate_up, self.down]
 
-    def forward(self, eng, x, y, rows: int) -> None:
-        act = eng.scratch_view("act", rows, self.down.k)
-        eng.project(self.gate_up, x, rows, act, glu=self.spec)
-        eng.project(self.down, act, rows, y)
+    def forward(self, eng, h, inp, in32, col: dict, gate, rows: int) -> dict:
+        act, y = eng.scratch_view("act", rows, self.down.k), eng.buf_y[:rows]
+        eng.project(self.gate_up, h, rows, act, glu=self.spec, bias=self.bias)
+        eng.project(self.down, act, rows, y, bias=self.down_bias)
+        return {"y": y}
 
     def forward_torch(self, x) -> torch.Tensor:
         w, s = {k: v.float() for k, v in self.raw.items()}, self.spec
+        if not s.limit:
+            g, u = (F.linear(x, w[k], w.get(k + ".b")) for k in ("gate", "up"))
+            return F.linear((F.gelu(g, approximate="tanh") if s.gelu else F.silu(g)) * u, w["down"], w.get("down.b"))
         g = F.linear(x, w["gate"]).clamp(max=s.limit)
         u = F.linear(x, w["up"]).clamp(-s.limit, s.limit)
         return F.linear(g * torch.sigmoid(s.alpha * g) * (u + s.shift), w["down"])
@@ -75,8 +88,9 @@ class Dense:
 
 
 class Moe:
-    """Experts: routing, grouping and both products (csrc/kernels/moe.h); the router's rows and the shared expert's up
-    rows ride in the block's input projection, the weighted sum of a row's experts is left to its join."""
+    """Experts: routing, grouping and both products (csrc/kernels/moe.h); the router's rows, the shared expert's gate
+    and, where it is no gated unit, its up rows ride in the block's input projection, the weighted sum of a row's
+    experts is left to its join."""
 
     def __init__(self, spec: MoeSpec, t: dict, gpu: bool):
         self.spec = spec
@@ -85,36 +99,43 @@ class Moe:
             from ..ops import moe as X
             from ..ops import stream as L
             e = range(spec.experts)
-            self.router = t["router"]
+            self.router, self.bias = t["router"], t["router.b"].float() if spec.bias else None
+            self.gate = t["shared.sg"] if spec.shared_gate else None
             gates = [t[f"e{i}.gate"] for i in e] if spec.act == SILU_GLU else None
             self.experts = X.Experts(gates, *([t[f"e{i}.{k}"] for i in e] for k in ("up", "down")))
             self.correction = t["correction"].float().contiguous() if spec.correction else None
             self.how = X.route_args(spec, self.correction)
-            self.shared = None
+            self.shared = self.shared_up = self.shared_glu = None
             if spec.shared_ff:
                 self.shared = L.Linear(t["shared.down"])
+            if spec.shared_ff and spec.act == SILU_GLU:
+                self.shared_glu, self.unit = L.Linear.glu(t["shared.gate"], t["shared.up"]), GluSpec(spec.shared_ff)
+            elif spec.shared_ff:
                 self.shared_up = F.pad(t["shared.up"], (0, 0, 0, self.shared.k - spec.shared_ff))  # as wide as it reads
 
     def input_parts(self) -> list:
-        own = [("shared", self.shared_up, None, "relu2")] if self.shared is not None else []
-        return own + [("router", self.router, None, "f32")]
+        own = [("shared", self.shared_up, None, "relu2")] if self.shared_up is not None else []
+        own += [("sg", self.gate, None, "f32")] if self.gate is not None else []
+        return own + [("router", self.router, self.bias, "f32")]
 
     def tensors(self) -> list:
         if self.raw is not None:
             return list(self.raw.values())
         own = [self.correction] if self.correction is not None else []
-        return self.experts.tensors() + own + (self.shared.tensors() if self.shared is not None else [])
+        return self.experts.tensors() + own + [t for lin in self.projections() for t in lin.tensors()]
 
     def scratch(self) -> dict:
         top = self.spec.top
-        return {"act": top * self.experts.ff, "ye": top * self.experts.width, "pairs": (3 * top, torch.int32),
+        own = {"sact": self.shared.k} if self.shared_glu is not None else {}
+        return {**own, "act": top * self.experts.ff, "ye": top * self.experts.width, "pairs": (3 * top, torch.int32),
                 "tiles": (8 * top, torch.int32), "pair_w": (top, torch.float32)}
 
     def projections(self) -> list:
-        return [self.shared] if self.shared is not None else []
+        return [lin for lin in (self.shared_glu, self.shared) if lin is not None]
 
     def forward(self, eng, h, inp, in32, col: dict, gate, rows: int) -> dict:
-        """What the block's join adds: the experts' results, the shared one's (``y``), and the gate's logits."""
+        """What the block's join adds: the experts' results, the shared one's (``y``) and the logits of its gate
+        (``ygate``), and the logits of the block's gate."""
         from ..ops import moe as X
         s, x = self.spec, self.experts
         pairs = rows * s.top
@@ -131,18 +152,27 @@ class Moe:
             out["gate2"] = gate
         if self.shared is not None:
             out["y"] = eng.buf_y[:rows]
-            eng.project(self.shared, inp[:, col["shared"]:], rows, out["y"])
+            if self.shared_glu is not None:
+                a = eng.scratch_view("sact", rows, self.shared.k)
+                eng.project(self.shared_glu, h, rows, a, glu=self.unit)
+            else:
+                a = inp[:, col["shared"]:]
+            eng.project(self.shared, a, rows, out["y"])
+            if self.gate is not None:
+                out["ygate"] = in32[:, col["sg"]:]
         return out
 
     def forward_torch(self, x) -> torch.Tensor:
         w, s = {k: v.float() for k, v in self.raw.items()}, self.spec
-        at, weight = self._route(F.linear(x, w["router"]), w.get("correction"))
+        at, weight = self._route(F.linear(x, w["router"], w.get("router.b")), w.get("correction"))
 
         def expert(h, name):
             up = F.linear(h, w[name + ".up"])
             a = F.silu(F.linear(h, w[name + ".gate"])) * up if s.act == SILU_GLU else F.relu(up).square()
             return F.linear(a, w[name + ".down"])
         out = expert(x, "shared") if s.shared_ff else torch.zeros_like(x)
+        if s.shared_gate:
+            out = out * torch.sigmoid(F.linear(x, w["shared.sg"]))
         for e in range(s.experts):
             row, k = (at == e).nonzero(as_tuple=True)
             if row.numel():

@@ -64,7 +64,7 @@ def kernel_family(cfg) -> str:
     """The kernel library that serves this model alone (csrc/build.py FAMILIES; "" = the full one)."""
     if not is_stack(cfg):
         return ""
-    return {"deretar": "latent", "gupuvik": "hybrid", "dumizen": "looped"}[cfg.model_type]
+    return {"deretar": "latent", "gupuvik": "hybrid", "dumizen": "looped", "runidra": "streams"}[cfg.model_type]
 
 
 __all__ = ["load_config", "is_stack", "engine_class", "make_engine", "folder_source", "random_source",

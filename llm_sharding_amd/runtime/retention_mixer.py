@@ -17,6 +17,21 @@ from .attn_mixer import Attention, turned
 from .latent_mixer import _head_pad
 
 
+def split_runs(plan, rows: int, slots: int, spec, least: int) -> tuple:
+    """Table of the runs that go step by step (longest first), segments of those of at least ``least`` rows (0: none),
+    which go in chunks; None for what the batch does not have."""
+    from ..ops import hip
+    from ..ops import retention as X
+    X.check_runs(torch.tensor(plan.runs, dtype=torch.int32), rows, slots)
+    runs = sorted(plan.runs, key=lambda r: -r[1])
+    long = [r for r in runs if least and r[1] >= least]
+    short = runs[len(long):]
+    if long:
+        items, *rest = X.segments(spec, long, hip.N_CU)
+        long = (items.to(plan.eng.device), *rest)
+    return plan.i32(short) if short else None, long or None
+
+
 class Retention:
     chunk_min = 48  # rows from which a run goes chunk by chunk (bf16) instead of step by step
 
@@ -65,7 +80,8 @@ class Retention:
         if plan.runs is None:
             X.steps(args(slot=slot, pos=pos), self.dtype, rows)
             return ao
-        short, long = plan.memo(("retention", s, self.chunks), lambda: self._runs(plan, rows, state))
+        short, long = plan.memo(("retention", s, self.chunks),
+                                lambda: split_runs(plan, rows, state[0].shape[0], s, self.chunk_min if self.chunks else 0))
         if short is not None:
             X.steps(args(runs=short), self.dtype, short.shape[0])
         if long is not None:
@@ -75,20 +91,6 @@ class Retention:
             ws = eng.workspace("ret", 4 * entries * s.heads * dk * dv).view(f32) if several else None
             X.chunked(args(runs=items), s, items, longest, several, ws, o32)
         return ao
-
-    def _runs(self, plan, rows: int, state: tuple) -> tuple:
-        """Table of the runs that go step by step (longest first), segments of those that go in chunks; None for what
-        the batch does not have."""
-        from ..ops import hip
-        from ..ops import retention as X
-        X.check_runs(torch.tensor(plan.runs, dtype=torch.int32), rows, state[0].shape[0])
-        least = self.chunk_min if self.chunks else 1 << 30
-        runs = sorted(plan.runs, key=lambda r: -r[1])
-        short, long = [r for r in runs if r[1] < least], [r for r in runs if r[1] >= least]
-        if long:
-            items, *rest = X.segments(self.spec, long, hip.N_CU)
-            long = (items.to(plan.eng.device), *rest)
-        return plan.i32(short) if short else None, long or None
 
     # ------------------------------------------------------------------ CPU
     def forward_torch(self, eng, x, cache, state: tuple, slot, pos) -> torch.Tensor:
@@ -152,4 +154,4 @@ class Pair:
         return sum(m.forward_torch(eng, x, cache, state, slot, pos) for m in self.sides.values())
 
 
-__all__ = ["Retention", "Pair"]
+__all__ = ["Retention", "Pair", "split_runs"]

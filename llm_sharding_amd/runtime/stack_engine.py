@@ -3,8 +3,8 @@
 The same step function, sequence API, decode graphs and serving as :class:`.engine.StageEngine`, for
 decoders that differ from Llama / GPT-2 in what a layer is made of:
 
-* the residual stream is fp32 (rows of ``hidden_dtype``); how the sublayers read and join it is the
-  layer's block (:mod:`.blocks`);
+* the residual stream is fp32 (rows of ``hidden_dtype``), or several streams side by side; how the sublayers read
+  and join it is the layer's block (:mod:`.blocks`);
 * mixers and feed-forwards come from the layer's spec; layers may share tensors, or read another
   layer's keys and values;
 * the cache is paged (:mod:`.paging`): one pool for all slots, one page table for all layers;
@@ -22,9 +22,10 @@ import torch
 import torch.nn.functional as F
 
 from ..config import ceil_div
-from ..models.stack import AttentionSpec, DeltaSpec, LatentSpec, PairSpec, RetentionSpec, StackConfig, leaves, pad_to
+from ..models.stack import (AttentionSpec, DeltaSpec, LatentSpec, MlstmSpec, PairSpec, RetentionSpec, StackConfig, leaves,
+                            pad_to)
 from .attn_mixer import rotary_tables
-from .blocks import COPY, Entry, Layer, block
+from .blocks import COPY, Entry, Layer, Sum, block
 from .engine import StageEngine, WeightSource
 from .latent_mixer import rotation_tables
 from .paging import PagePool
@@ -35,11 +36,11 @@ PAGE = 64
 
 def embed_rows(cfg: StackConfig, table: torch.Tensor, ids: torch.Tensor) -> torch.Tensor:
     """Rows of the stream for ``ids`` [n], without an engine (an ingress that holds the table only)."""
-    h = torch.empty((ids.numel(), cfg.hidden_size), dtype=torch.float32, device=table.device)
+    h = torch.empty((ids.numel(), cfg.stream_width), dtype=torch.float32, device=table.device)
     if table.device.type != "cuda":
-        return h.copy_(F.embedding(ids.long(), table).float() * cfg.embed_scale)
+        return h.copy_((F.embedding(ids.long(), table).float() * cfg.embed_scale).repeat(1, cfg.streams))
     from ..ops import stream as L
-    L.stream_embed(ids.to(torch.int32), table, cfg.embed_scale, h, torch.empty_like(h, dtype=table.dtype), ids.numel())
+    L.stream_embed(ids.to(torch.int32), table, cfg.embed_scale, h, None, ids.numel(), cfg.streams)
     return h
 
 
@@ -108,6 +109,9 @@ class StackEngine(StageEngine):
         if self.has_head:
             self.final_norm = (self.source.final_norm(dev, dt).float().reshape(-1)
                                + cfg.norm_offset).expand(cfg.hidden_size).contiguous()
+            if cfg.logit_scale != 1.0:  # the head is linear: its input is scaled
+                self.final_norm = self.final_norm * cfg.logit_scale
+            self.head_read = Sum(torch.ones(cfg.streams, device=dev), self.final_norm)
             head = self.embed_w if cfg.tie_word_embeddings and self.has_embed else self.source.lm_head(dev, dt)
             head = F.pad(head, (0, 0, 0, cfg.head_rows - cfg.vocab_size))[self.head_v0:self.head_v1]
             if self.gpu:
@@ -172,6 +176,10 @@ class StackEngine(StageEngine):
         if isinstance(m, RetentionSpec):
             dims = m.state_dims if self.gpu else (m.dim, m.vdim)
             return None, None, (torch.zeros((self.max_slots, m.heads) + dims, dtype=torch.float32, device=dev),), ()
+        if isinstance(m, MlstmSpec):
+            dims, n = (m.state_dims, m.copies) if self.gpu else ((m.dim, m.vdim), 1)
+            shapes = (dims, (n, dims[0]), (n,))
+            return None, None, tuple(torch.zeros((self.max_slots, m.heads) + s, dtype=torch.float32, device=dev) for s in shapes), ()
         if isinstance(m, DeltaSpec):
             from ..ops.delta import state_shapes
             S, ring = state_shapes(m, self.max_slots)
@@ -204,8 +212,8 @@ class StackEngine(StageEngine):
     def _projections(self) -> list:
         out = []
         for l in self.layers:
-            gated = getattr(l.mlp, "gate_up", None)
-            out += [(p.n, p.k, p is gated) for p in l.w.projections()]
+            gated = [p for p in (getattr(l.mlp, k, None) for k in ("gate_up", "shared_glu")) if p is not None]
+            out += [(p.n, p.k, any(p is g for g in gated)) for p in l.w.projections()]
         if self.loop is not None:
             out.append((self.loop.lin.n, self.loop.lin.k, False))
         if self.has_head:
@@ -216,7 +224,7 @@ class StackEngine(StageEngine):
         """Everything a forward of up to R rows writes besides the cache."""
         from ..ops import hip, packing
         dev, dt, W = self.device, self.dtype, self.width_p
-        out = {"buf_h": torch.zeros((R, self.cfg.hidden_size), dtype=torch.float32, device=dev),
+        out = {"buf_h": torch.zeros((R, self.cfg.stream_width), dtype=torch.float32, device=dev),
                "buf_x": torch.zeros((R, W), dtype=dt, device=dev),
                "buf_y": torch.zeros((R, W), dtype=torch.float32, device=dev),
                "flat": {k: torch.zeros(R * n, dtype=t, device=dev) for k, (n, t) in self._widths.items() if n},
@@ -350,9 +358,12 @@ class StackEngine(StageEngine):
             raise RuntimeError("[ERROR] this stage has no embedding layer")
         rows = ids.numel()
         if not self.gpu:
-            h.copy_(F.embedding(ids.long(), self.embed_w).float() * self.cfg.embed_scale)
+            h.copy_((F.embedding(ids.long(), self.embed_w).float() * self.cfg.embed_scale).repeat(1, self.cfg.streams))
             return
         from ..ops import stream as L
+        if self.cfg.streams > 1:
+            L.stream_embed(ids, self.embed_w, self.cfg.embed_scale, h, None, rows, self.cfg.streams)
+            return
         fits = rows <= self.buf_x.shape[0]
         xc = self.buf_x if fits else torch.empty((rows, self.width_p), dtype=self.dtype, device=self.device)
         L.stream_embed(ids, self.embed_w, self.cfg.embed_scale, h, xc, rows)
@@ -360,7 +371,7 @@ class StackEngine(StageEngine):
 
     def embed(self, ids: torch.Tensor) -> torch.Tensor:
         ids = ids.reshape(-1)
-        h = torch.empty((ids.numel(), self.cfg.hidden_size), dtype=torch.float32, device=self.device)
+        h = torch.empty((ids.numel(), self.cfg.stream_width), dtype=torch.float32, device=self.device)
         self.embed_into(self._i32(ids), h)
         return h
 
@@ -382,9 +393,11 @@ class StackEngine(StageEngine):
 
     def latent_nsplit(self, s, entries: int, longest: int) -> int:
         """Key splits of the absorbed attention: about one workgroup per CU (each fills a CU's
-        LDS with its two pages), no more splits than pages."""
+        LDS with its two pages), no more splits than pages with visible keys."""
         from ..ops import hip
         from ..ops import latent as L
+        if s.window:
+            longest = min(longest, s.window + PAGE - 1)  # a window may begin inside a page
         return int(max(1, min(64, hip.N_CU // max(1, entries * L.head_groups(s)), ceil_div(longest, PAGE))))
 
     def decode_nsplit(self, rows: int) -> int:
@@ -421,6 +434,8 @@ class StackEngine(StageEngine):
             elif have is not w.entry:
                 if w.entry is COPY:
                     L.cast_rows(hbuf, x, rows)
+                elif isinstance(w.entry, Sum):
+                    w.entry.read(self, hbuf, x, rows)
                 else:
                     L.stream_norm(hbuf, w.entry, self.cfg.norm_eps, x, rows)
             have = w.forward(self, i, slot, pos, rows, plan, reads[i + 1])
@@ -441,10 +456,14 @@ class StackEngine(StageEngine):
         src = h[:rows] if a_rows is None else h.index_select(0, a_rows.long())
         xn = self.buf_x[:rows] if rows <= self.buf_x.shape[0] else torch.zeros(
             (rows, self.width_p), dtype=self.dtype, device=self.device)
-        L.stream_norm(src, self.final_norm, self.cfg.norm_eps, xn, rows)
+        if self.cfg.streams > 1:
+            self.head_read.read(self, src, xn, rows)
+        else:
+            L.stream_norm(src, self.final_norm, self.cfg.norm_eps, xn, rows)
         return xn
 
     def head_gemv(self, h: torch.Tensor, rows: int, keys: torch.Tensor, a_rows=None) -> None:
+        # (a soft cap keeps the order of logits: the largest is the largest before it)
         from ..ops import stream as L
         xn = self._normed(h, rows, a_rows)
         if self.dtype == torch.float32:
@@ -458,16 +477,21 @@ class StackEngine(StageEngine):
     def logits(self, h: torch.Tensor, rows_idx=None) -> torch.Tensor:
         if not self.gpu:
             return super().logits(h, rows_idx)
+        from ..ops import stream as L
         idx = None if rows_idx is None else self._i32(rows_idx)
         rows = h.shape[0] if idx is None else idx.numel()
         lg = torch.empty((rows, self.lm_head.n), dtype=torch.float32, device=self.device)
         self.lm_head(self._normed(h, rows, idx), rows, lg, ws=self.coop_ws, sk_ws=self.sk_ws)
+        if self.cfg.logit_softcap:
+            L.softcap_rows(lg, rows, self.head_vocab, self.cfg.logit_softcap)
         return lg[:, :self.head_vocab]
 
     def logits_torch(self, hs: torch.Tensor) -> torch.Tensor:
-        x = hs.float()
+        x = hs.float().view(hs.shape[0], self.cfg.streams, -1).sum(1)
         x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + self.cfg.norm_eps) * self.final_norm
         lg = F.linear(x, self.lm_head.float())
+        if self.cfg.logit_softcap:
+            lg = self.cfg.logit_softcap * torch.tanh(lg / self.cfg.logit_softcap)
         return lg if self.head_bias is None else lg + self.head_bias
 
 

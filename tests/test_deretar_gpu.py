@@ -285,16 +285,19 @@ def test_append_norms_turns_and_places(dtype, name):
     case = Case(s, [130, 70], dtype)
     slot, pos = [0, 1, 0, 0, 1], [129, 64, 63, 0, 127]
     w = case.w
-    inp = _rand(6, w.inp.n, seed=3, dtype=dtype).to(DEV)
+    from llm_sharding_amd.runtime.blocks import InputProjection
+    proj = InputProjection(w.input_parts(), "inp", 128)
+    ok = proj.col["dkv"]
+    inp = _rand(6, proj.lin.n, seed=3, dtype=dtype).to(DEV)
     cq = torch.zeros(6, w.uq.k, dtype=dtype, device=DEV)
     before = case.cache.clone()
     slot, pos = slot + [1], pos + [case.max_pages * 64]  # outside the table: nothing is written
     a = case.args(slot, pos)
-    L.append(a, 6, inp, 0, w.ok, w.gq, w.gk, cq)
+    L.append(a, 6, inp, proj.col["dq"], ok, w.gq, w.gk, cq)
     x = inp.double().cpu()
     tol = 5e-3 if dtype == BF else 2e-6
     close(cq[:, :s.q_rank], P.gain_norm(x[:, :s.q_rank], case.t["dq.norm"].double(), 1e-4), tol, "query latent")
-    d = x[:, w.ok:w.ok + s.kv_rank + s.rot_dim]
+    d = x[:, ok:ok + s.kv_rank + s.rot_dim]
     c = P.gain_norm(d[:, :s.kv_rank], case.t["dkv.norm"].double(), 1e-4)
     kr = P.rotate(d[:, s.kv_rank:], torch.tensor(pos), s.rot_base, s.rot_dims)
     touched = torch.zeros(case.cache.shape[:2], dtype=torch.bool)
