@@ -88,12 +88,12 @@ def parse():
     ap.add_argument("--no-fallback", dest="fallback", action="store_false",
                     help="N > 1: do not restart with --transport ipc when the RCCL ring preflight fails")
     ap.add_argument("--compare", default="",
-                    help="instead of the headline: prefill and decode throughput of Deretar, Gupuvik and Dumizen stacks of these sizes "
+                    help="instead of the headline: prefill and decode throughput of Deretar, Gupuvik, Dumizen and Runidra stacks of these sizes "
                          "(2k,4k,8k: layers like a 2048-wide model's, Llama-2-7B's, Llama-2-70B's; random weights) "
                          "beside Llama layers of the same width, heads and ff")
     ap.add_argument("--compare-points", default="prefill:1x2048,prefill:4x2048,decode:1,decode:16,decode:64,decode:128",
                     help="prefill:SEQUENCESxTOKENS and decode:BATCH points of --compare")
-    ap.add_argument("--compare-models", default="deretar,gupuvik,dumizen,llama", help="which of these --compare runs")
+    ap.add_argument("--compare-models", default="deretar,gupuvik,dumizen,runidra,llama", help="which of these --compare runs")
     ap.add_argument("--compare-context", type=int, default=1024, help="cached tokens per sequence of a decode point")
     ap.add_argument("--compare-layers", type=int, default=8, help="layer runs of a stack")
     return ap.parse_args()
@@ -382,7 +382,9 @@ def compare_designs(a) -> list:
         gu = dataclasses.replace(gu, layers=gu.layers[:a.compare_layers])
         du = get_preset(f"dumizen-{size}")
         du = dataclasses.replace(du, layers=du.layers[:a.compare_layers])
-        for cfg in (st, gu, du, ll):
+        ru = get_preset(f"runidra-{size}")
+        ru = dataclasses.replace(ru, layers=ru.layers[:a.compare_layers])
+        for cfg in (st, gu, du, ru, ll):
             kind = cfg.model_type if is_stack(cfg) else "llama"
             if kind not in a.compare_models.split(","):
                 continue

@@ -283,7 +283,30 @@ def _dumizen(width: int, heads: int, kv_heads: int, layers: int, vocab: int, exp
     return cfg
 
 
+def _runidra(width: int, heads: int, ff: int, layers: int, vocab: int, kv_rank: int, q_rank: int, experts: int, top: int, eff: int,
+             shared: int, dim: int = 128, rot: int = 64, vdim: int = 128, window: int = 1024, mheads: int = 0, mdim: int = 128,
+             mvdim: int = 128, streams: int = 4, loop: tuple = (0, 2, 2), max_pos: int = 1 << 17, name: str = "runidra"):
+    """A Runidra stack (random-init presets): matrix memory and windowed latent attention in turn, dense and expert
+    feed-forwards by two."""
+    from .models import runidra as N
+    entries = []
+    for i in range(layers):
+        mlp = N.dense(ff) if i % 4 in (0, 3) else N.moe(experts, top, eff, shared)
+        entries.append(N.latent_entry(heads, dim, rot, vdim, kv_rank, q_rank, window, mlp) if i % 2
+                       else N.mlstm_entry(mheads or heads, mdim, mvdim, mlp))
+    cfg = N.make_config(width, vocab, entries, streams, loop, name=name)
+    cfg.max_position_embeddings = max_pos
+    return cfg
+
+
 PRESETS = {
+    # Runidra with the widths of a 2048-wide model / Llama-2-7B / Llama-2-70B; what a token uses of the experts and the
+    # shared one has about as many weights as the dense feed-forward
+    "runidra-2k": lambda: _runidra(2048, 16, 8192, 24, 32000, 256, 768, 32, 6, 1024, 2048, name="runidra-2k"),
+    "runidra-4k": lambda: _runidra(4096, 32, 11008, 32, 32000, 512, 1536, 32, 6, 1408, 2816, name="runidra-4k"),
+    "runidra-8k": lambda: _runidra(8192, 64, 28672, 80, 32000, 512, 1536, 16, 3, 7168, 7168, name="runidra-8k"),
+    "tiny-runidra": lambda: _runidra(112, 5, 150, 5, 330, 56, 88, 6, 2, 40, 56, dim=24, rot=16, vdim=40, window=50, mheads=3,
+                                     mdim=20, mvdim=28, streams=3, loop=(1, 3, 2), max_pos=1024, name="tiny-runidra"),
     # Dumizen with the widths of a 2048-wide model / Llama-2-7B / Llama-2-70B; what a token uses of the experts and
     # the shared one has as many weights as the dense feed-forward
     "dumizen-2k": lambda: _dumizen(2048, 16, 4, 24, 32000, 32, 8, 1024, 4096, name="dumizen-2k"),

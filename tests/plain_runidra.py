@@ -56,6 +56,10 @@ def leave(xs):
 
 
 # ------------------------------------------------------------------------------ matrix memory
+def denominator(nq, m):
+    return torch.maximum(nq.abs(), torch.exp(-m)) + 1e-6
+
+
 def memory(q, k, v, i, f, state=None):
     """One head: q, k [n, dim], v [n, vdim], log gates i and f [n] -> (outputs [n, vdim], state (S, n, m))."""
     if state is None:
@@ -68,7 +72,7 @@ def memory(q, k, v, i, f, state=None):
         keep, add = torch.exp(f[t] + m - top), torch.exp(i[t] - top)
         S = keep * S + add * k[t][:, None] * v[t][None, :]
         z, m = keep * z + add * k[t], top
-        out[t] = (S.T @ q[t]) / (torch.maximum((z @ q[t]).abs(), torch.exp(-m)) + 1e-6)
+        out[t] = (S.T @ q[t]) / denominator(z @ q[t], m)
     return out, (S, z, m)
 
 

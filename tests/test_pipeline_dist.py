@@ -15,7 +15,7 @@ from llm_sharding_amd.runtime.registry import random_source
 
 M, B, P, NEW = 2, 2, 5, 6
 MODELS = {"llama": lambda: tiny(layers=5), "gpt2": lambda: tiny_gpt2(layers=5), "deretar": lambda: get_preset("tiny-deretar"),
-          "gupuvik": lambda: get_preset("tiny-gupuvik"), "dumizen": lambda: get_preset("tiny-dumizen")}
+          "gupuvik": lambda: get_preset("tiny-gupuvik"), "dumizen": lambda: get_preset("tiny-dumizen"), "runidra": lambda: get_preset("tiny-runidra")}
 
 
 def _free_port() -> int:
@@ -93,7 +93,7 @@ def test_gpt2_pipeline_matches_single():
     assert _run_world(2, "gpt2") == ref
 
 
-@pytest.mark.parametrize("name", ["deretar", "gupuvik", "dumizen"])
+@pytest.mark.parametrize("name", ["deretar", "gupuvik", "dumizen", "runidra"])
 def test_stack_pipeline_matches_single(name):
     """A stack (fp32 residual stream handed over, paged cache and states per stage) over 2 gloo ranks."""
     ref = _single(name)
