@@ -25,9 +25,9 @@ struct MlItem {  // Mirrored by llm_sharding_amd/ops/retention.py::segments
   int seg, n_seg, len;      // which segment; all but the last have len rows
 };
 
-// Gates of every row, [heads][rows]: sums of log forget gates within the chunk, i less these, maxima of that so far
+// Gates of every row, [g, M, F][heads][rows]: F sums of log forget gates within the chunk, g = i - F, M maxima of g so far
 struct MlGates {
-  float *F, *g, *M;
+  float* all;
   int rows;
 };
 
@@ -60,10 +60,11 @@ __global__ __launch_bounds__(256) void ml_gates_kernel(MlArgs a, const MlItem* _
     M = lane >= o ? fmaxf(M, x) : M;
   }
   if (!in) return;
-  const size_t at = (size_t)h * G.rows + row;
-  G.F[at] = F;
-  G.g[at] = g;
-  G.M[at] = M;
+  const size_t one = (size_t)a.heads * G.rows;
+  float* at = G.all + (size_t)h * G.rows + row;
+  at[0] = g;
+  at[one] = M;
+  at[2 * one] = F;
 }
 
 template <int DK, int VS>
@@ -83,8 +84,8 @@ __global__ __launch_bounds__(NT, 2) void ml_chunk_kernel(MlArgs a, const MlItem*
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int w4 = w & 3, wh = w >> 2;  // tile of queries; half of the value slice, and what the wave stages: q and v, k
   const bf16_raw* in = (const bf16_raw*)a.in + (size_t)it.row0 * a.ldi;
-  const float *gF = G.F + (size_t)h * G.rows + it.row0, *gg = G.g + (size_t)h * G.rows + it.row0,
-              *gM = G.M + (size_t)h * G.rows + it.row0;
+  const size_t one = (size_t)a.heads * G.rows;
+  const float *gg = G.all + (size_t)h * G.rows + it.row0, *gM = gg + one, *gF = gM + one;
   const size_t entry = (size_t)a.heads * DK * a.dv, part = (size_t)h * DK * a.dv + v0;
   const size_t nentry = (size_t)a.heads * a.copies, npart = (size_t)h * a.copies + slice;
   const int dv = a.dv;
@@ -106,19 +107,20 @@ __global__ __launch_bounds__(NT, 2) void ml_chunk_kernel(MlArgs a, const MlItem*
   const bool fresh = it.pos0 == it.seg * it.len;  // the run starts at position 0
   float *st = a.S + (size_t)it.slot * entry + part, *stn = a.n + ((size_t)it.slot * nentry + npart) * DK + rt * 16 + q4 * 4,
         *stm = a.m + (size_t)it.slot * nentry + npart;
-  auto parts_n = [&](int e) { return P.n + ((size_t)(it.ws + e) * nentry + npart) * DK + rt * 16 + q4 * 4; };
-  auto parts_m = [&](int e) { return P.m + ((size_t)(it.ws + e) * nentry + npart) * 2; };
+  // this workgroup's part of the workspace; entry e of the run lies e entries behind
+  float *ws = P.S + (size_t)it.ws * entry + part, *wn = P.n + ((size_t)it.ws * nentry + npart) * DK + rt * 16 + q4 * 4,
+        *wm = P.m + ((size_t)it.ws * nentry + npart) * 2;
   if (local) {
     if (it.seg == 0) {  // the state before the run, for the second launch
       each([&](f32x4_t&, size_t o) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) P.S[(size_t)it.ws * entry + part + o + (size_t)r * dv] = fresh ? 0.f : st[o + (size_t)r * dv];
+        for (int r = 0; r < 4; ++r) ws[o + (size_t)r * dv] = fresh ? 0.f : st[o + (size_t)r * dv];
       });
       if (owner && l16 == 0) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) parts_n(0)[r] = fresh ? 0.f : stn[r];
+        for (int r = 0; r < 4; ++r) wn[r] = fresh ? 0.f : stn[r];
       }
-      if (tid == 0) parts_m(0)[0] = fresh ? 0.f : *stm;
+      if (tid == 0) wm[0] = fresh ? 0.f : *stm;
     }
   } else if (it.n_seg == 1) {
     if (!fresh) {
@@ -131,14 +133,14 @@ __global__ __launch_bounds__(NT, 2) void ml_chunk_kernel(MlArgs a, const MlItem*
     }
   } else {
     for (int e = 0; e <= it.seg; ++e) {  // entry 0: before the run, e: what segment e - 1 added
-      const float me = parts_m(e)[0], fm = e ? m0 + parts_m(e)[1] : -INFINITY, mn = fmaxf(fm, me);
+      const float me = wm[e * nentry * 2], fm = e ? m0 + wm[e * nentry * 2 + 1] : -INFINITY, mn = fmaxf(fm, me);
       const float keep = e ? __expf(fm - mn) : 0.f, add = __expf(me - mn);
-      const float* src = P.S + (size_t)(it.ws + e) * entry + part;
+      const float* src = ws + e * entry;
       each([&](f32x4_t& s, size_t o) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) s[r] = fmaf(src[o + (size_t)r * dv], add, s[r] * keep);
       });
-      if (mine) N = N * keep + *reinterpret_cast<const f32x4_t*>(parts_n(e)) * add;
+      if (mine) N = N * keep + *reinterpret_cast<const f32x4_t*>(wn + e * nentry * DK) * add;
       m0 = mn;
     }
   }
@@ -174,8 +176,7 @@ __global__ __launch_bounds__(NT, 2) void ml_chunk_kernel(MlArgs a, const MlItem*
     fend = gF[e];
     mend = gM[e];
     if (tid < 3 * C) {  // waves 0, 1, 2: g, M, F of the chunk's rows
-      const float* p = w == 0 ? gg : w == 1 ? gM : gF;
-      r1 = c0 + lane < it.n ? p[c0 + lane] : w == 0 ? -INFINITY : 0.f;
+      r1 = c0 + lane < it.n ? gg[w * one + c0 + lane] : w == 0 ? -INFINITY : 0.f;
     }
   };
   auto put = [&](float Me) {  // what was fetched -> LDS; Me: M of the chunk's last row
@@ -345,19 +346,20 @@ __global__ __launch_bounds__(NT, 2) void ml_chunk_kernel(MlArgs a, const MlItem*
     }
   }
   if (local || it.seg == it.n_seg - 1) {
-    float* dst = local ? P.S + (size_t)(it.ws + 1 + it.seg) * entry + part : st;
+    const size_t e = 1 + it.seg;
+    if (local) {
+      st = ws + e * entry;
+      stn = wn + e * nentry * DK;
+      stm = wm + e * nentry * 2;
+    }
     each([&](f32x4_t& s, size_t o) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) dst[o + (size_t)r * dv] = s[r];
+      for (int r = 0; r < 4; ++r) st[o + (size_t)r * dv] = s[r];
     });
-    if (owner && l16 == 0) *reinterpret_cast<f32x4_t*>(local ? parts_n(1 + it.seg) : stn) = N;
+    if (owner && l16 == 0) *reinterpret_cast<f32x4_t*>(stn) = N;
     if (tid == 0) {
-      if (local) {
-        parts_m(1 + it.seg)[0] = m0;
-        parts_m(1 + it.seg)[1] = fsum;
-      } else {
-        *stm = m0;
-      }
+      stm[0] = m0;
+      if (local) stm[1] = fsum;
     }
   }
 }
@@ -399,8 +401,7 @@ extern "C" int lsa_ml_chunked(const MlArgs* a, const void* items, int n_items, i
       ((uintptr_t)a->in | (uintptr_t)a->out | (uintptr_t)a->norm | (uintptr_t)a->n | (uintptr_t)n | (uintptr_t)o32) % 16)
     return LSA_BAD_SHAPE;
   const MlItem* it = (const MlItem*)items;
-  const size_t one = (size_t)a->heads * rows;
-  const MlGates G{gates, gates + one, gates + 2 * one, rows};
+  const MlGates G{gates, rows};
   const MlParts P{S, n, m};
 #define LSA_C(K, V)                                                                                                  \
   if (a->dk == K && (a->dv == V || (V == 64 && a->dv == 128)) && a->copies == a->dv / V) {                           \

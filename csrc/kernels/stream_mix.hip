@@ -9,7 +9,7 @@
 
 namespace {
 
-constexpr int MAXS = 8;
+constexpr int MAXS = 16;
 
 struct MixArgs {  // Mirrored by llm_sharding_amd/ops/stream.py::MixArgs
   const float* coef;     // [streams] out, [streams][streams] mix (from, to); null: the streams stay

@@ -213,7 +213,7 @@ class MixArgs(ctypes.Structure):
                 + [(n, ctypes.c_int) for n in ("streams", "ldy", "ldyg", "ldye", "top")] + [("eps", ctypes.c_float)])
 
 
-MAX_STREAMS = 8  # of stream_mix (MAXS in csrc/kernels/stream_mix.hip)
+MAX_STREAMS = 16  # of stream_mix (MAXS in csrc/kernels/stream_mix.hip)
 
 
 def stream_mix(x, rows: int, streams: int, coef=None, y=None, ygate=None, experts=None, read=None, eps: float = 0.0,

@@ -96,7 +96,7 @@ class Read:
 
 @pytest.mark.parametrize("dtype", [BF, F32])
 @pytest.mark.parametrize("W", [88, 250, 4096, 9001])
-@pytest.mark.parametrize("streams", [1, 2, 3, 4, 5, 8])
+@pytest.mark.parametrize("streams", [1, 2, 3, 4, 5, 16])
 @pytest.mark.parametrize("rows", [5, 300])
 def test_streams_mix(dtype, W, streams, rows):
     from llm_sharding_amd.ops import stream as L
@@ -134,7 +134,7 @@ def test_streams_refuse_what_does_not_fit():
     from llm_sharding_amd.ops import stream as L
     x, y, read = torch.zeros(2, 64, device=DEV), torch.zeros(2, 32, device=DEV), Read(torch.ones(2), torch.ones(32))
     with pytest.raises(ValueError):
-        L.stream_mix(torch.zeros(2, 9 * 32, device=DEV), 2, 9, read=read, out=y)  # more streams than it takes
+        L.stream_mix(torch.zeros(2, 17 * 32, device=DEV), 2, 17, read=read, out=y)  # more streams than it takes
     with pytest.raises(ValueError):
         L.stream_mix(x, 2, 2, coef=torch.zeros(6, device=DEV))  # nothing joins
     with pytest.raises(ValueError):
