@@ -287,7 +287,8 @@ __global__ __launch_bounds__(NT, 2) void ml_chunk_kernel(MlArgs a, const MlItem*
         const f32x4_t g = *reinterpret_cast<const f32x4_t*>(s_c + kt * 16 + q4 * 4);
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float p = kt * 16 + q4 * 4 + r <= qi ? s[kt][r] * a.q_scale * __expf(g[r] - Mq) : 0.f;
+          // (what the row does not see: exp(-inf))
+          const float p = s[kt][r] * a.q_scale * __expf(kt * 16 + q4 * 4 + r <= qi ? g[r] - Mq : -INFINITY);
           s[kt][r] = p;
           nq += p;
         }
