@@ -27,20 +27,20 @@ OBJ = os.path.join(ROOT, "build", "obj")
 ROCM = os.environ.get("ROCM_PATH", "/opt/rocm")
 
 
-# gemv_coop.hip is compiled once per unit (LSA_COOP_UNIT in the file): epilogues 0-5, fp8, entry
-COOP_UNITS = tuple(range(8))
+# gemv_coop.hip is compiled once per unit (LSA_COOP_UNIT in the file): epilogues 0-6, fp8, entry
+COOP_UNITS = tuple(range(9))
 
 # object name (without .o) prefixes a family's library is linked from:
 # ops/hip.py loads liblsa_kernels-<family>.so where the full library is not built
 FAMILIES = {
     "latent": ("elementwise.hip", "gemm_sk.hip", "gemv.hip", "gemv_coop.hip-0", "gemv_coop.hip-2", "gemv_coop.hip-4",
-               "gemv_coop.hip-7", "latent", "linear_f32.hip", "stream_ops.hip"),
-    "hybrid": ("elementwise.hip", "gemm_sk.hip", "gemv.hip", "gemv_coop.hip-0", "gemv_coop.hip-4", "gemv_coop.hip-7",
+               "gemv_coop.hip-8", "latent", "linear_f32.hip", "stream_ops.hip"),
+    "hybrid": ("elementwise.hip", "gemm_sk.hip", "gemv.hip", "gemv_coop.hip-0", "gemv_coop.hip-4", "gemv_coop.hip-8",
                "linear_f32.hip", "stream_ops.hip", "paged_attn", "delta", "moe"),
-    "looped": ("elementwise.hip", "gemm_sk.hip", "gemv.hip", "gemv_coop.hip-0", "gemv_coop.hip-4", "gemv_coop.hip-7",
+    "looped": ("elementwise.hip", "gemm_sk.hip", "gemv.hip", "gemv_coop.hip-0", "gemv_coop.hip-4", "gemv_coop.hip-8",
                "linear_f32.hip", "stream_ops.hip", "paged_attn", "retention", "moe"),
     "streams": ("elementwise.hip", "gemm_sk.hip", "gemv.hip", "gemv_coop.hip-0", "gemv_coop.hip-2", "gemv_coop.hip-4",
-                "gemv_coop.hip-7", "linear_f32.hip", "stream_ops.hip", "stream_mix.hip", "latent", "mlstm", "moe"),
+                "gemv_coop.hip-6", "gemv_coop.hip-8", "linear_f32.hip", "stream_ops.hip", "stream_mix.hip", "latent", "mlstm", "moe"),
 }
 
 

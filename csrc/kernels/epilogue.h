@@ -6,7 +6,8 @@
 //               columns to either; or out32 += sigmoid(gate) * y (a result joins an fp32 stream)
 //   EPI_RESID   out = resid + y (+ bias)        (o_proj / down_proj + residual add)
 //   EPI_SWIGLU  out = silu(gate) * up           (gate/up fused GEMM, tiles interleaved), or the
-//               clipped GLU of glu() when glu_limit > 0, or gelu(gate) * up with act 1
+//               clipped GLU of glu() when glu_limit > 0
+//   EPI_GEGLU   out = gelu(gate) * up           (the same interleaved GEMM; bf16 weights only)
 //   EPI_QKV     half-split RoPE on q/k + direct write of k/v into the static KV cache
 //               (replaces apply_rotary_pos_emb + DynamicCache.update's torch.cat); with
 //               cos_t == nullptr (GPT-2: learned absolute positions) no rotation and the
@@ -20,7 +21,9 @@
 // EPI_PARTIAL (gemm_sk only): every K-split workgroup stores its fp32 partial tile to
 // ((float*)out)[split][M][ldo]; the following norm kernel adds the partials to the residual
 // stream (lsa_resid_rmsnorm_partials) instead of an in-GEMM fixup.
-enum EpiMode { EPI_STORE = 0, EPI_RESID = 1, EPI_SWIGLU = 2, EPI_QKV = 3, EPI_ARGMAX = 4, EPI_PARTIAL = 5 };
+enum EpiMode { EPI_STORE = 0, EPI_RESID = 1, EPI_SWIGLU = 2, EPI_QKV = 3, EPI_ARGMAX = 4, EPI_PARTIAL = 5, EPI_GEGLU = 6 };
+
+constexpr bool epi_gated(int epi) { return epi == EPI_SWIGLU || epi == EPI_GEGLU; }  // gate and up tiles in turn
 
 // Mirrored by llm_sharding_amd/ops/hip.py::EpiArgs (ctypes) - keep field order in sync.
 struct EpiArgs {
@@ -41,7 +44,7 @@ struct EpiArgs {
   int head_dim;
   int t_max;
   int col_offset;           // ARGMAX: vocabulary index of column 0 (vocab-parallel chunks)
-  int act;                  // STORE: 0 identity, 1 gelu (tanh form, GPT-2 "gelu_new"), 2 relu squared; SWIGLU: 1 gelu
+  int act;                  // STORE: 0 identity, 1 gelu (tanh form, GPT-2 "gelu_new"), 2 relu squared
   // fused RMSNorm across GEMMs (gemm_sk only; layout [M][ss_n] fp32, one partial sum of squares
   // per 64 columns of the residual stream): RESID writes the partials of its rounded outputs to
   // ss_out; QKV / SWIGLU scale row m by rsqrt(sum(ss_in[m][:]) / (64 ss_n) + ss_eps) first
@@ -75,20 +78,26 @@ static inline bool bad_store(const EpiArgs& e, int N) {
 
 LSA_DEVICE float silu(float g) { return g / (1.0f + __expf(-g)); }
 
-// 0.5 x (1 + tanh(sqrt(2/pi) (x + 0.044715 x^3))), tanh(u) = 1 - 2 / (exp(2u) + 1)
-LSA_DEVICE float gelu_tanh(float x) {
-  const float u = 0.7978845608028654f * (x + 0.044715f * x * x * x);
-  return 0.5f * x * (2.0f - 2.0f / (__expf(2.0f * u) + 1.0f));
-}
-
-// The gated unit of an EPI_SWIGLU GEMM: silu(g) * u, with act 1 gelu(g) * u, or with glu_limit L > 0 the clipped unit
+// The gated unit of an EPI_SWIGLU GEMM: silu(g) * u, or with glu_limit L > 0 the clipped unit
 //   g' = min(g, L), u' = clamp(u, -L, L):  g' * sigmoid(alpha * g') * (u' + shift)
 LSA_DEVICE float glu(const EpiArgs& ep, float g, float u) {
   if (ep.glu_limit > 0.f) {
     const float gc = fminf(g, ep.glu_limit), uc = fminf(fmaxf(u, -ep.glu_limit), ep.glu_limit);
     return gc / (1.0f + __expf(-ep.glu_alpha * gc)) * (uc + ep.glu_shift);
   }
-  return (ep.act ? gelu_tanh(g) : silu(g)) * u;
+  return silu(g) * u;
+}
+
+// 0.5 x (1 + tanh(sqrt(2/pi) (x + 0.044715 x^3))), tanh(u) = 1 - 2 / (exp(2u) + 1)
+LSA_DEVICE float gelu_tanh(float x) {
+  const float u = 0.7978845608028654f * (x + 0.044715f * x * x * x);
+  return 0.5f * x * (2.0f - 2.0f / (__expf(2.0f * u) + 1.0f));
+}
+
+// the gated unit of a product with epilogue EPI
+template <int EPI>
+LSA_DEVICE float epi_glu(const EpiArgs& ep, float g, float u) {
+  return EPI == EPI_GEGLU ? gelu_tanh(g) * u : glu(ep, g, u);
 }
 
 // activation of an EPI_STORE product (act 1 or 2)
@@ -169,7 +178,7 @@ LSA_DEVICE void epi_qkv_store(const EpiArgs& ep, int m, int n, float v, float vp
 // Vectorised epilogue of one finished 16-column tile row: v[j] = C[m][c0 + j], c0 % 16 == 0
 // (packed column order). One thread per (tile, row) instead of one per element: 16-B stores,
 // 16-B residual / bias / cos / sin loads, the index math (shifts: head_dim is a power of two)
-// done once per 16 outputs. EPI_SWIGLU and EPI_ARGMAX are handled by the callers.
+// done once per 16 outputs. Gated units and EPI_ARGMAX are handled by the callers.
 // 16-B store; WT: write-through to memory (two 8-B agent-scope relaxed atomic stores = sc1), so a
 // consumer on another CU / XCD may read the bytes after an arrival counter with no release
 // fence on this side (MI355X_MICROARCH.md 'Valid forms'; scripts/probes/qkv_attn.hip)

@@ -197,7 +197,7 @@ extern "C" int lsa_gemm_sk(const void* a, int lda, const void* wp, int M, int N,
   const int BM = bm;
   if (nb == 0) nb = (bn == 128 || (bm == 128 && bn == 256)) ? 3 : 2;
   if (nb != 2 && !(nb == 3 && (bn == 128 || (bm == 128 && bn == 256)))) return LSA_UNSUPPORTED;
-  if (bn == 192 ? (N % 16 || (epi == EPI_SWIGLU && N % 32)) : N % bn) return LSA_BAD_SHAPE;
+  if (bn == 192 ? (N % 16 || (epi_gated(epi) && N % 32)) : N % bn) return LSA_BAD_SHAPE;
   if (grid < 1 || grid > 1024 || group_m < 1) return LSA_BAD_SHAPE;
   if (epi == EPI_RESID && !ep->resid) return LSA_BAD_SHAPE;
   if (epi == EPI_QKV && (!ep->k_cache || !ep->v_cache || !ep->slot || !ep->pos)) return LSA_BAD_SHAPE;
@@ -257,6 +257,7 @@ extern "C" int lsa_gemm_sk(const void* a, int lda, const void* wp, int M, int N,
     case EPI_SWIGLU: return LSA_G(EPI_SWIGLU);
     case EPI_PARTIAL: return LSA_G(EPI_PARTIAL);
     case EPI_ARGMAX: return LSA_G(EPI_ARGMAX);
+    case EPI_GEGLU: return LSA_G(EPI_GEGLU);
     default: return LSA_UNSUPPORTED;
   }
 #undef LSA_G

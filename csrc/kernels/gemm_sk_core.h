@@ -490,7 +490,7 @@ struct Kern {
       __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
       const int row_base = m0 + wr * TM + ps * EROWS;
       const int col_base = nt * BN + wc * TN;
-      if (EPI == EPI_SWIGLU) {
+      if (epi_gated(EPI)) {
         // units: EROWS rows x FN/2 gate|up tile pairs
         constexpr int UNITS = EROWS * (FN / 2);
 #pragma unroll
@@ -517,7 +517,7 @@ struct Kern {
             epi_bias16(ep, c0, g);
             epi_bias16(ep, c0 + 16, uu);
 #pragma unroll
-            for (int q = 0; q < 16; ++q) v[q] = glu(ep, g[q], uu[q]);
+            for (int q = 0; q < 16; ++q) v[q] = epi_glu<EPI>(ep, g[q], uu[q]);
             bf16_raw* o = ep.out + (size_t)m * ep.ldo + (c0 >> 1);
             st16(o, pack8(v));
             st16(o + 8, pack8(v + 8));

@@ -176,14 +176,18 @@ __global__ __launch_bounds__(NW * 64) void gemv_packed_kernel(
     return rsqrtf(t / (float)K + eps);
   };
 
-  if (EPI == EPI_SWIGLU) {
+  if (epi_gated(EPI)) {
     for (int e = tid; e < (TN / 2) * MR * 16; e += NTHR) {
       const int tp = e / (MR * 16), mm = (e >> 4) % MR, n = e & 15;
       if (mm >= M) continue;
       const float r = rstd(mm);
-      const int col = (nt0 / 2 + tp) * 16 + n, gc = (nt0 + 2 * tp) * 16 + n;
-      const float g = rsum(2 * tp, mm, n) * r + epi_bias(ep, gc), u = rsum(2 * tp + 1, mm, n) * r + epi_bias(ep, gc + 16);
-      ep.out[(size_t)mm * ep.ldo + col] = f2bf(glu(ep, g, u));
+      float g = rsum(2 * tp, mm, n) * r, u = rsum(2 * tp + 1, mm, n) * r;
+      const int col = (nt0 / 2 + tp) * 16 + n;
+      if (EPI == EPI_GEGLU) {
+        g += epi_bias(ep, (nt0 + 2 * tp) * 16 + n);
+        u += epi_bias(ep, (nt0 + 2 * tp + 1) * 16 + n);
+      }
+      ep.out[(size_t)mm * ep.ldo + col] = f2bf(epi_glu<EPI>(ep, g, u));
     }
   } else {
     for (int e = tid; e < TN * MR * 16; e += NTHR) {
@@ -238,7 +242,7 @@ int launch_epi(int tn, int nw, int u, bool norm, const bf16_raw* x, int ldx, con
   const int mb = M <= 16 ? 1 : (M <= 32 ? 2 : 4);
 #define LSA_CFG(T, B, W, UU)                                                            \
   if (tn == T && mb == B && nw == W && u == UU) {                                      \
-    if constexpr (EPI == EPI_SWIGLU && (T % 2)) return LSA_BAD_SHAPE;                  \
+    if constexpr (epi_gated(EPI) && (T % 2)) return LSA_BAD_SHAPE;                  \
     else return launch_cfg<T, B, W, UU, EPI>(norm, x, ldx, a_rows, wp, M, N, K, eps, ep, s); \
   }
   LSA_GEMV_CONFIGS(LSA_CFG)
@@ -255,7 +259,7 @@ extern "C" int lsa_gemv(const void* x, int ldx, const int* a_rows, const void* w
                         int K, int norm, float eps, int epi, const EpiArgs* ep, int tn, int nw,
                         int u, hipStream_t stream) {
   if (M < 1 || M > 64 || tn < 1 || u < 1 || N % (16 * tn) || K % 32 || ldx < K) return LSA_BAD_SHAPE;
-  if (epi == EPI_SWIGLU && (tn % 2)) return LSA_BAD_SHAPE;
+  if (epi_gated(epi) && (tn % 2)) return LSA_BAD_SHAPE;
   if ((K >> 5) % u) return LSA_BAD_SHAPE;  // waves take whole chunks (idle waves are fine)
   const bf16_raw* xx = static_cast<const bf16_raw*>(x);
   const bf16_raw* w = static_cast<const bf16_raw*>(wp);
@@ -266,6 +270,7 @@ extern "C" int lsa_gemv(const void* x, int ldx, const int* a_rows, const void* w
     case EPI_SWIGLU: return launch_epi<EPI_SWIGLU>(tn, nw, u, nrm, xx, ldx, a_rows, w, M, N, K, eps, *ep, stream);
     case EPI_QKV: return launch_epi<EPI_QKV>(tn, nw, u, nrm, xx, ldx, a_rows, w, M, N, K, eps, *ep, stream);
     case EPI_ARGMAX: return launch_epi<EPI_ARGMAX>(tn, nw, u, nrm, xx, ldx, a_rows, w, M, N, K, eps, *ep, stream);
+    case EPI_GEGLU: return launch_epi<EPI_GEGLU>(tn, nw, u, nrm, xx, ldx, a_rows, w, M, N, K, eps, *ep, stream);
     default: return LSA_UNSUPPORTED;
   }
 }

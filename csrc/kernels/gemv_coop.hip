@@ -113,7 +113,7 @@ __global__ __launch_bounds__(NW * KW * 64) void gemv_coop_kernel(
   const int SKe = ragged ? 1 : SK;
   int g = 0, s = 0, tlo, tcnt;
   if (ragged) {
-    constexpr int P = EPI == EPI_SWIGLU ? 2 : 1;
+    constexpr int P = epi_gated(EPI) ? 2 : 1;
     const int units = N / 16 / P;
     tlo = P * (int)(((long long)blockIdx.x * units) / gridDim.x);
     tcnt = P * (int)((((long long)blockIdx.x + 1) * units) / gridDim.x) - tlo;
@@ -480,7 +480,7 @@ __global__ __launch_bounds__(NW * KW * 64) void gemv_coop_kernel(
       }
     }
   };
-  if (EPI == EPI_SWIGLU) {
+  if (epi_gated(EPI)) {
     // gate tile 2tp / up tile 2tp+1 -> 16 outputs per thread, two 16-B stores
     for (int e = tid; e < (tcnt / 2) * MR; e += NTHR) {
       const int tp = e / MR, mm = e % MR;
@@ -489,10 +489,12 @@ __global__ __launch_bounds__(NW * KW * 64) void gemv_coop_kernel(
       float gg[16], uu[16];
       load16(2 * tp, mm, r, gg);
       load16(2 * tp + 1, mm, r, uu);
-      epi_bias16(ep, (ntg0 + 2 * tp) * 16, gg);
-      epi_bias16(ep, (ntg0 + 2 * tp + 1) * 16, uu);
+      if (EPI == EPI_GEGLU) {
+        epi_bias16(ep, (ntg0 + 2 * tp) * 16, gg);
+        epi_bias16(ep, (ntg0 + 2 * tp + 1) * 16, uu);
+      }
 #pragma unroll
-      for (int j = 0; j < 16; ++j) gg[j] = glu(ep, gg[j], uu[j]);
+      for (int j = 0; j < 16; ++j) gg[j] = epi_glu<EPI>(ep, gg[j], uu[j]);
       bf16_raw* o = ep.out + (size_t)mm * ep.ldo + (ntg0 / 2 + tp) * 16;
       st16(o, pack8(gg));
       st16(o + 8, pack8(gg + 8));
@@ -630,11 +632,11 @@ struct CoopCall {
 
 // The kernels of one (epilogue, weight format) are the slowest code of the library to compile,
 // so csrc/build.py compiles this file once per unit, side by side: LSA_COOP_UNIT = EPI_* (bf16
-// weights), LSA_COOP_UNIT_FP8 (every epilogue with fp8 weights) or LSA_COOP_UNIT_ENTRY (the
+// weights), LSA_COOP_UNIT_FP8 (the epilogues with fp8 weights) or LSA_COOP_UNIT_ENTRY (the
 // extern "C" entry points). Without LSA_COOP_UNIT the one object holds everything. A library
 // linked without a unit answers LSA_UNSUPPORTED for it (weak references).
-#define LSA_COOP_UNIT_FP8 6
-#define LSA_COOP_UNIT_ENTRY 7
+#define LSA_COOP_UNIT_FP8 7
+#define LSA_COOP_UNIT_ENTRY 8
 #ifdef LSA_COOP_UNIT
 #define COOP_HAS(U) (LSA_COOP_UNIT == (U))
 #else
@@ -646,6 +648,7 @@ struct CoopCall {
   __attribute__((weak)) int lsa_coop_unit_##name(const CoopCall& c);               \
   __attribute__((weak)) int lsa_coop_unit_fp8_##name(const CoopCall& c);
 LSA_COOP_EPIS(LSA_COOP_DECL)
+__attribute__((weak)) int lsa_coop_unit_geglu(const CoopCall& c);
 #define LSA_COOP_DEF(E, FP8, fn)                                                                                       \
   int fn(const CoopCall& c) {                                                                                          \
     return dispatch<E, FP8>(c.mb, c.tnw, c.nw, c.kf, c.kw, c.d, c.norm, c.x, c.ldx, c.a_rows, c.wp, c.M, c.N, c.K,     \
@@ -669,6 +672,9 @@ LSA_COOP_DEF(EPI_ARGMAX, false, lsa_coop_unit_argmax)
 #if COOP_HAS(5)
 LSA_COOP_DEF(EPI_PARTIAL, false, lsa_coop_unit_partial)
 #endif
+#if COOP_HAS(6)
+LSA_COOP_DEF(EPI_GEGLU, false, lsa_coop_unit_geglu)
+#endif
 #if COOP_HAS(LSA_COOP_UNIT_FP8)
 #define LSA_COOP_DEF_FP8(E, name) LSA_COOP_DEF(E, true, lsa_coop_unit_fp8_##name)
 LSA_COOP_EPIS(LSA_COOP_DEF_FP8)
@@ -690,14 +696,14 @@ int coop_entry(const void* x, int ldx, const int* a_rows, const void* wp, int M,
   const int mb = M <= 32 ? 2 : (M <= 64 ? 4 : 8);
   const int tg = nw * tnw;
   if (sk == 0) {  // ragged: tiles (SwiGLU: pairs) dealt to one workgroup per CU, at most tg each
-    const int P = epi == EPI_SWIGLU ? 2 : 1, cu = n_cu();
+    const int P = epi_gated(epi) ? 2 : 1, cu = n_cu();
     if (FP8 || epi == EPI_PARTIAL || N % (16 * P) || P % tnw) return LSA_BAD_SHAPE;
     const int units = N / 16 / P;
     if (units < cu || P * ((units + cu - 1) / cu) > tg) return LSA_BAD_SHAPE;
   } else if (N % (16 * tg) || sk > K / (32 * kf)) {
     return LSA_BAD_SHAPE;
   }
-  if (epi == EPI_SWIGLU && tg % 2) return LSA_BAD_SHAPE;  // gate / up tile pairs stay in one workgroup
+  if (epi_gated(epi) && tg % 2) return LSA_BAD_SHAPE;  // gate / up tile pairs stay in one workgroup
   if (sk > 1 && (!slab || !counters)) return LSA_BAD_SHAPE;
   const CoopCall c{mb, tnw, nw, kf, kw, d, norm != 0, static_cast<const bf16_raw*>(x), ldx, a_rows,
                    static_cast<const bf16_raw*>(wp), M, N, K, sk, eps, ep, slab, counters, wscale, stream};
@@ -706,6 +712,7 @@ int coop_entry(const void* x, int ldx, const int* a_rows, const void* wp, int M,
   case E: unit = FP8 ? lsa_coop_unit_fp8_##name : lsa_coop_unit_##name; break;
   switch (epi) {
     LSA_COOP_EPIS(LSA_D)
+    case EPI_GEGLU: unit = FP8 ? nullptr : lsa_coop_unit_geglu; break;
     default: return LSA_UNSUPPORTED;
   }
   return unit ? unit(c) : LSA_UNSUPPORTED;

@@ -1,7 +1,7 @@
 // Projections of the fp32 engine: C[M][N] = A[M][K] . W[N][K]^T with true fp32 products and sums
 // (VALU FMA; no reduced-precision matrix mode). 64 x 64 tiles, 16-deep K steps through LDS, 4 x 4
 // outputs per thread. Epilogues: store, or the gated unit over interleaved 16-row gate / up
-// blocks (ops/packing.py fuse_gate_up), as EPI_STORE / EPI_SWIGLU of the bf16 GEMMs.
+// blocks (ops/packing.py fuse_gate_up), as EPI_STORE / EPI_SWIGLU / EPI_GEGLU of the bf16 GEMMs.
 #include "epilogue.h"
 
 namespace {
@@ -21,7 +21,7 @@ LSA_DEVICE void store_f32(const EpiArgs& ep, int m, int n, float v) {
   else if (n < ep.cols) *o += sigmoid(((const float*)ep.gate)[(size_t)m * ep.ldg + n]) * v;
 }
 
-template <bool GLU>
+template <int EPI>
 __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict__ A, int lda,
                                                          const float* __restrict__ W, int M, int N, int K, EpiArgs ep) {
   __shared__ float sa[TK][TM + 4], sw[TK][TN + 4];
@@ -64,14 +64,14 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict
   for (int i = 0; i < 4; ++i) {
     const int m = m0 + ty + 16 * i;
     if (m >= M) continue;
-    if constexpr (GLU) {
+    if constexpr (epi_gated(EPI)) {
 #pragma unroll
       for (int p = 0; p < 2; ++p) {
         const int c = n0 + 32 * p;
         if (c >= N) continue;
         const int n = c + tx;
         ep.out32[(size_t)m * ep.ldo + c / 2 + tx] =
-            glu(ep, acc[i][2 * p] + epi_bias(ep, n), acc[i][2 * p + 1] + epi_bias(ep, n + 16));
+            epi_glu<EPI>(ep, acc[i][2 * p] + epi_bias(ep, n), acc[i][2 * p + 1] + epi_bias(ep, n + 16));
       }
     } else {
 #pragma unroll
@@ -90,12 +90,13 @@ extern "C" int lsa_linear_f32(const float* a, int lda, const float* w, int M, in
   if (M < 1 || N < 1 || K < 16 || K % 16 || lda < K || lda % 4 || !ep || !(ep->out32 || ep->out)) return LSA_BAD_SHAPE;
   if (((uintptr_t)a | (uintptr_t)w) % 16) return LSA_BAD_SHAPE;
   dim3 grid((N + TN - 1) / TN, (M + TM - 1) / TM);
-  if (epi == EPI_SWIGLU) {
+  if (epi_gated(epi)) {
     if (N % 32 || ep->ldo < N / 2 || !ep->out32) return LSA_BAD_SHAPE;
-    linear_f32_kernel<true><<<grid, 256, 0, stream>>>(a, lda, w, M, N, K, *ep);
+    if (epi == EPI_GEGLU) linear_f32_kernel<EPI_GEGLU><<<grid, 256, 0, stream>>>(a, lda, w, M, N, K, *ep);
+    else linear_f32_kernel<EPI_SWIGLU><<<grid, 256, 0, stream>>>(a, lda, w, M, N, K, *ep);
   } else if (epi == EPI_STORE) {
     if (bad_store(*ep, N)) return LSA_BAD_SHAPE;
-    linear_f32_kernel<false><<<grid, 256, 0, stream>>>(a, lda, w, M, N, K, *ep);
+    linear_f32_kernel<EPI_STORE><<<grid, 256, 0, stream>>>(a, lda, w, M, N, K, *ep);
   } else {
     return LSA_UNSUPPORTED;
   }

@@ -128,8 +128,8 @@ class LatentSpec:
 @dataclass(frozen=True)
 class GluSpec:
     """Gated unit act(gate) * up, act silu or with ``gelu`` the tanh form of gelu. With ``limit`` the clipped unit:
-    g = min(gate, limit), u = clamp(up, -limit, limit), g * sigmoid(alpha g) * (u + shift). ``bias``: all three
-    projections have one."""
+    g = min(gate, limit), u = clamp(up, -limit, limit), g * sigmoid(alpha g) * (u + shift). ``bias`` (with
+    gelu): all three projections have one."""
     ff: int
     limit: float = 0.0
     alpha: float = 1.0
@@ -138,7 +138,7 @@ class GluSpec:
     bias: bool = False
 
     def __post_init__(self):
-        if self.ff < 1 or self.limit < 0 or (self.gelu and self.limit):
+        if self.ff < 1 or self.limit < 0 or (self.gelu and self.limit) or (self.bias and not self.gelu):
             raise ValueError(f"gated unit: bad values: {self}")
 
     def scratch_width(self, width: int) -> int:

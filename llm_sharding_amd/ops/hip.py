@@ -27,7 +27,8 @@ NATIVE_DIR = os.path.join(os.path.dirname(os.path.dirname(os.path.abspath(__file
 # product and every test use the in-tree _native/liblsa_kernels.so)
 KERNELS_SO = os.environ.get("LSA_KERNELS_SO") or os.path.join(NATIVE_DIR, "liblsa_kernels.so")
 
-EPI_STORE, EPI_RESID, EPI_SWIGLU, EPI_QKV, EPI_ARGMAX, EPI_PARTIAL = range(6)
+EPI_STORE, EPI_RESID, EPI_SWIGLU, EPI_QKV, EPI_ARGMAX, EPI_PARTIAL, EPI_GEGLU = range(7)
+GATED_EPIS = (EPI_SWIGLU, EPI_GEGLU)  # gate and up tiles in turn
 _STATUS = {0: "ok", 1: "bad shape", 2: "unsupported", 3: "launch failed"}
 _UNSUPPORTED = 2  # LSA_UNSUPPORTED: no kernel instantiation for the shape
 
@@ -160,7 +161,7 @@ def make_epi(out=None, resid=None, k_cache=None, v_cache=None, slot=None, pos=No
     GEMM writes them for its outputs, a QKV / SWIGLU GEMM reading the raw residual stream as A
     applies the RMSNorm scale from them (the norm weight is folded into its W). ``out32``: fp32
     output of an EPI_STORE GEMM instead of ``out``. ``glu_limit`` > 0: EPI_SWIGLU computes the
-    clipped gated unit with these constants instead of silu(g) * u (epilogue.h glu).
+    clipped gated unit with these constants instead of silu(g) * u (epilogue.h glu); EPI_GEGLU: gelu(g) * u.
     An EPI_STORE GEMM of several parts: with both ``out`` and ``out32``, columns from ``col32`` on go to
     out32 [M][ldo32]; ``act`` applies to columns from ``act_from`` on. ``gate`` [M, >= cols] (with out32
     alone): out32[:, :cols] += sigmoid(gate) * y instead of the store."""
@@ -246,7 +247,7 @@ def gemv(x: torch.Tensor, wp: torch.Tensor, M: int, N: int, K: int, epi: int, ep
     else:
         _req(a_rows.dtype == torch.int32 and a_rows.is_cuda and a_rows.numel() >= M, "gemv: a_rows")
     if tn == 0 and coop is None:
-        algo, cfg = proj_config(N // 16, M, need_even=(epi == EPI_SWIGLU), k=K)
+        algo, cfg = proj_config(N // 16, M, need_even=epi in GATED_EPIS, k=K)
         if algo == "coop":
             coop = cfg
         else:
@@ -258,7 +259,7 @@ def gemv(x: torch.Tensor, wp: torch.Tensor, M: int, N: int, K: int, epi: int, ep
         if epi == EPI_PARTIAL:
             _req(out_numel >= sk * M * ep.ldo, f"gemv partial: output holds {out_numel} floats, "
                  f"{sk} splits x {M} rows x ldo {ep.ldo} needed")
-        _req(coop in coop_candidates(N // 16, K, M, epi == EPI_SWIGLU),
+        _req(coop in coop_candidates(N // 16, K, M, epi in GATED_EPIS),
              f"gemv: coop config {coop} invalid for N={N} K={K} M={M}")
         if ws is None:
             ws = default_workspace(x.device)
@@ -574,7 +575,7 @@ def gemm_sk(a: torch.Tensor, wp: torch.Tensor, M: int, N: int, K: int, epi: int,
          "gemm_sk: A must be [>=M, >=K] row-major with 16-B aligned rows")
     _req(a.data_ptr() % 16 == 0, "gemm_sk: A must be 16-byte aligned")
     _check_epi(epi, ep, N)
-    _req(epi in (EPI_STORE, EPI_RESID, EPI_SWIGLU, EPI_QKV, EPI_PARTIAL, EPI_ARGMAX), f"gemm_sk: epilogue {epi} not supported")
+    _req(epi in (EPI_STORE, EPI_RESID, *GATED_EPIS, EPI_QKV, EPI_PARTIAL, EPI_ARGMAX), f"gemm_sk: epilogue {epi} not supported")
     if epi == EPI_PARTIAL:  # exactly `split` K ranges per tile, every tile in one round
         _req(bn in (128, 192, 256) and split >= 1 and grid >= 1, "gemm_sk partial: explicit bn, grid and split required")
         _req(out_numel >= split * M * ep.ldo, f"gemm_sk partial: output holds {out_numel} floats, "
@@ -595,7 +596,7 @@ def gemm_sk(a: torch.Tensor, wp: torch.Tensor, M: int, N: int, K: int, epi: int,
     grid = grid or pg
     if split < 0:
         split = 0
-    _req(bn in (128, 192, 256) and N % (16 if bn == 192 else bn) == 0 and (bn != 192 or epi != EPI_SWIGLU or N % 32 == 0),
+    _req(bn in (128, 192, 256) and N % (16 if bn == 192 else bn) == 0 and (bn != 192 or epi not in GATED_EPIS or N % 32 == 0),
          f"gemm_sk: N={N} does not tile by bn={bn}")
     _req(1 <= grid <= 1024, "gemm_sk: grid")
     if ws is None:

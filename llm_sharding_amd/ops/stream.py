@@ -88,9 +88,10 @@ class Linear:
         if act_from is not None:
             kw.update(act=act, act_from=act_from)
         if glu is not None:
-            kw.update(glu_alpha=glu.alpha, glu_limit=glu.limit, glu_shift=glu.shift, act=hip.ACT_GELU if glu.gelu else hip.ACT_NONE)
+            _req(bias is None or glu.gelu, "linear: biases of a gated product go with gelu")
+            kw.update(glu_alpha=glu.alpha, glu_limit=glu.limit, glu_shift=glu.shift)
         _req(bias is None or bias.numel() >= self.n, "linear: bias")
-        epi = hip.EPI_SWIGLU if glu is not None else (hip.EPI_STORE if keys is None else hip.EPI_ARGMAX)
+        epi = (hip.EPI_GEGLU if glu.gelu else hip.EPI_SWIGLU) if glu is not None else (hip.EPI_STORE if keys is None else hip.EPI_ARGMAX)
         ep = hip.make_epi(keys=keys, bias=bias, col_offset=col_offset, **kw)
         if self.f32:
             _req(x.dtype == torch.float32 and x.is_cuda and keys is None, "linear: fp32 cuda input")

@@ -98,6 +98,12 @@ def test_placement_counts_streams_and_states():
         assert cfg.layer_params(i) == sum(v.numel() for k, v in t.items() if k.startswith(f"l{l.owner}.")), i
 
 
+def test_gated_units_refuse_what_no_kernel_has():
+    for kw in (dict(gelu=True, limit=1.0), dict(bias=True), dict(limit=-1.0)):
+        with pytest.raises(ValueError):
+            GluSpec(8, **kw)
+
+
 # ------------------------------------------------------------------------------ engine (CPU)
 def test_whole_portions_and_decoding_agree(model):
     cfg, t = model

@@ -79,13 +79,14 @@ def test_gated_gelu_with_biases(dtype, rows, ff, K):
     xp[:, :K] = x.to(DEV, dtype)
     out = torch.full((rows, lin.n // 2), 7.0, dtype=dtype, device=DEV)
     g, u = (P.linear(x.double(), {k: v.double() for k, v in w.items()}, n) for n in ("gate", "up"))
-    for bias in (True, False):
-        for gelu in (True, False):
-            lin(xp, rows, out, glu=GluSpec(ff, gelu=gelu, bias=bias),
-                bias=L.Linear.glu_bias(d["gate.b"].float(), d["up.b"].float()) if bias else None)
-            a, b = (g, u) if bias else (g - w["gate.b"].double(), u - w["up.b"].double())
-            rows_close(out[:, :ff], (P.gelu(a) if gelu else P.silu(a)) * b, 1e-2 if dtype == BF else 2e-6, (bias, gelu))
-            assert not out[:, ff:].any()
+    both = L.Linear.glu_bias(d["gate.b"].float(), d["up.b"].float())
+    for bias, gelu in ((True, True), (False, True), (False, False)):
+        lin(xp, rows, out, glu=GluSpec(ff, gelu=gelu, bias=bias), bias=both if bias else None)
+        a, b = (g, u) if bias else (g - w["gate.b"].double(), u - w["up.b"].double())
+        rows_close(out[:, :ff], (P.gelu(a) if gelu else P.silu(a)) * b, 1e-2 if dtype == BF else 2e-6, (bias, gelu))
+        assert not out[:, ff:].any()
+    with pytest.raises(ValueError):
+        lin(xp, rows, out, glu=GluSpec(ff), bias=both)
 
 
 # ------------------------------------------------------------------------------ streams
